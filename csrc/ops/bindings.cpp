@@ -2,9 +2,7 @@
 // Every entry point validates shapes/dtypes/devices on the host (so a bad call
 // fails loudly instead of faulting the GPU) and launches on the caller's
 // current HIP stream, which keeps them hipGraph-capturable.
-#include <torch/extension.h>
-#include <c10/hip/HIPStream.h>
-#include <hip/hip_runtime_api.h>
+#include "bind_common.h"
 
 extern "C" {
 int pa_rmsnorm(void* out, const void* x, const void* w, int T, int D, float eps, hipStream_t st);
@@ -22,7 +20,7 @@ int pa_paged_attention(void* out, float* part_o, float* part_ml, const void* q, 
                        hipStream_t st);
 int pa_sample_workspace_floats(int rows, int V);
 int pa_patch_pending_ids(int* ids, const int* sampled, int T, int n_sampled, hipStream_t st);
-int pa_sample(int* out_tokens, float* out_keys, float* workspace, const void* logits, int rows,
+int pa_sample(int fp32, int* out_tokens, float* out_keys, float* workspace, const void* logits, int rows,
               int V, int ld, int vocab_offset, const float* temperature, const int* mask_class,
               const uint32_t* class_masks, int mask_words, const int64_t* seeds,
               const int* offsets, const int* forced, const float* tau, hipStream_t st);
@@ -38,9 +36,6 @@ int pa_skinny_gemm(void* y, const void* x, const void* w, int M, int N, int K, i
 void pa_decode_set_variant(int v);
 void pa_handoff_set_acquire(int v);
 void pa_handoff_set_modes(int gemm, int attn);
-int pa_decode_gemm(void* y, const void* x, const void* wp, const void* resid, int M, int N, int K,
-                   int ldx, int ldy, int ldr, int epi, int norm, float eps, int nt, int waves, int splits,
-                   float* ws, long long ws_floats, int* counters, int n_counters, hipStream_t st);
 int pa_decode_qkv_rope(const void* x, const void* wp, int M, int N, int K, int ldx, float eps, void* q_out,
                        void* k_cache, void* v_cache, const int* positions, const int* slots,
                        const float* cos_sin, int H, int KV, int nt, int waves, int splits, float* ws,
@@ -66,11 +61,6 @@ void pa_prefill_gemm_plan(int M, int N, int K, int bn, int* full, int* S);
 int pa_prefill_pick_bn(int M, int N);
 void pa_prefill_set_variant(int v);
 long long pa_prefill_gemm_ws_floats(int M, int N, int bn, int full, int S);
-int pa_prefill_gemm(void* y, const void* x, const void* wp, const void* resid, float* ws, long long ws_floats,
-                    int* counters, int n_counters, int M, int N, int K, int ldx, int ldy, int ldr, int epi,
-                    const float* ss_in, float* ss_out, float* ss_zero, float eps, int full, int splits, int bn,
-                    void* q_out, void* k_cache, void* v_cache, const int* positions, const int* slots,
-                    const float* cos_sin, int H, int KV, int kernel_variant, hipStream_t st);
 long long pa_cosine_topk_workspace_bytes(int Q, int N, int K);
 int pa_cosine_topk(float* out_scores, int* out_rows, void* workspace, const void* queries,
                    const void* index, int Q, int N, int D, int K, const int* row_priority,
@@ -97,20 +87,6 @@ int pa_car_all_reduce(void* const* bases, int W, int rank0, int nranks_local, co
 }
 
 namespace {
-
-hipStream_t cur_stream() { return c10::hip::getCurrentHIPStream().stream(); }
-
-void check_gpu(const at::Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda(), name, " must be a GPU tensor");
-  TORCH_CHECK(t.is_contiguous(), name, " must be contiguous");
-}
-void check_dtype(const at::Tensor& t, at::ScalarType dt, const char* name) {
-  TORCH_CHECK(t.scalar_type() == dt, name, " has dtype ", t.scalar_type(), ", expected ", dt);
-}
-void check_rc(int rc, const char* what) {
-  TORCH_CHECK(rc == 0, what, " launch failed with code ", rc, " (",
-              rc > 0 ? hipGetErrorString((hipError_t)rc) : "bad arguments", ")");
-}
 
 void rmsnorm(at::Tensor out, at::Tensor x, at::Tensor w, double eps) {
   check_gpu(out, "out"); check_gpu(x, "x"); check_gpu(w, "w");
@@ -229,49 +205,6 @@ bool skinny_gemm(at::Tensor y, at::Tensor x, at::Tensor w) {
   return rc == 0;
 }
 
-// y = epi(rownorm(x) . W^T) on fragment-major packed weights wp [N/16, K/32, 64, 8]
-// (csrc/ops/gemm_decode.hip). epi 0 plain, 1 silu(gate)*up (y has N/2 columns),
-// 2 y = resid + acc. Returns false if the shape is not handled.
-bool decode_gemm(at::Tensor y, at::Tensor x, at::Tensor wp, c10::optional<at::Tensor> resid, int64_t epi,
-                 bool norm, double eps, int64_t nt, int64_t waves, int64_t splits, c10::optional<at::Tensor> ws,
-                 c10::optional<at::Tensor> counters) {
-  check_gpu(wp, "wp");
-  TORCH_CHECK(x.is_cuda() && x.dim() == 2 && x.stride(1) == 1, "x must be a 2-D GPU tensor, unit inner stride");
-  TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.stride(1) == 1, "y must be a 2-D GPU tensor, unit inner stride");
-  check_dtype(x, at::kBFloat16, "x"); check_dtype(wp, at::kBFloat16, "wp"); check_dtype(y, at::kBFloat16, "y");
-  TORCH_CHECK(wp.dim() == 4 && wp.size(2) == 64 && wp.size(3) == 8, "wp must be packed [N/16, K/32, 64, 8]");
-  const int M = x.size(0), K = x.size(1), N = wp.size(0) * 16;
-  TORCH_CHECK(wp.size(1) * 32 == K, "packed weight K ", wp.size(1) * 32, " != x K ", K);
-  TORCH_CHECK(x.stride(0) % 8 == 0 && K % 8 == 0, "x rows must be 16-byte aligned");
-  const int NO = epi == 1 ? N / 2 : N;
-  TORCH_CHECK(y.size(0) == M && y.size(1) == NO, "y shape [", y.size(0), ", ", y.size(1), "] != [", M, ", ", NO, "]");
-  const void* rp = nullptr;
-  int ldr = 0;
-  if (epi == 2) {
-    TORCH_CHECK(resid.has_value(), "epi=2 needs resid");
-    const auto& r = *resid;
-    TORCH_CHECK(r.is_cuda() && r.dim() == 2 && r.stride(1) == 1 && r.size(0) == M && r.size(1) == N,
-                "resid must be [M, N] with unit inner stride");
-    check_dtype(r, at::kBFloat16, "resid");
-    rp = r.data_ptr();
-    ldr = r.stride(0);
-  }
-  float* wsp = nullptr;
-  long long wsn = 0;
-  int* cp = nullptr;
-  int cn = 0;
-  if (ws.has_value() && counters.has_value()) {
-    check_gpu(*ws, "ws"); check_gpu(*counters, "counters");
-    check_dtype(*ws, at::kFloat, "ws"); check_dtype(*counters, at::kInt, "counters");
-    wsp = ws->data_ptr<float>(); wsn = ws->numel(); cp = counters->data_ptr<int>(); cn = counters->numel();
-  }
-  const int rc = pa_decode_gemm(y.data_ptr(), x.data_ptr(), wp.data_ptr(), rp, M, N, K, x.stride(0), y.stride(0),
-                                ldr, (int)epi, norm ? 1 : 0, (float)eps, (int)nt, (int)waves, (int)splits, wsp, wsn,
-                                cp, cn, cur_stream());
-  TORCH_CHECK(rc >= 0, "decode_gemm launch failed");
-  return rc == 0;
-}
-
 // Decode QKV projection + RoPE + paged KV write (csrc/ops/gemm_decode.hip, EPI_ROPE).
 void decode_qkv_rope(at::Tensor x, at::Tensor wp, double eps, at::Tensor q_out, at::Tensor k_cache,
                      at::Tensor v_cache, at::Tensor positions, at::Tensor slots, at::Tensor cos_sin, int64_t H,
@@ -308,14 +241,6 @@ void decode_qkv_rope(at::Tensor x, at::Tensor wp, double eps, at::Tensor q_out, 
                                     slots.data_ptr<int>(), cos_sin.data_ptr<float>(), (int)H, (int)KV, 0, 0,
                                     (int)splits, wsp, wsn, cp, cn, cur_stream());
   check_rc(rc < 0 ? rc : (rc > 0 ? -1 : 0), "decode_qkv_rope");
-}
-
-const float* opt_rows(const c10::optional<at::Tensor>& t, int M, const char* name) {
-  if (!t.has_value()) return nullptr;
-  check_gpu(*t, name);
-  check_dtype(*t, at::kFloat, name);
-  TORCH_CHECK(t->numel() >= M, name, " must hold >= M floats");
-  return t->data_ptr<float>();
 }
 
 // y = epi(rowscale(x) . W^T) for mid-size token counts on packed weights (csrc/ops/gemm_mid.hip).
@@ -489,51 +414,6 @@ std::vector<int64_t> stream_gemm_plan(int64_t M, int64_t N, int64_t K, int64_t e
   return {p[0], p[1], p[2], p[3], p[4], p[5], p[6], (int64_t)ws};
 }
 
-// Large-M projections (csrc/ops/gemm_prefill.hip): 256x256 MFMA tiles on the packed
-// weights with the same epilogues as mid_gemm (0 plain, 1 SwiGLU, 2 residual, 3 rope-perm).
-bool prefill_gemm(at::Tensor y, at::Tensor x, at::Tensor wp, c10::optional<at::Tensor> resid, at::Tensor ws,
-                  at::Tensor counters, int64_t epi, c10::optional<at::Tensor> ss_in, c10::optional<at::Tensor> ss_out,
-                  c10::optional<at::Tensor> ss_zero, double eps, int64_t full, int64_t splits, int64_t bn,
-                  int64_t variant) {
-  check_gpu(wp, "wp"); check_gpu(ws, "ws"); check_gpu(counters, "counters");
-  TORCH_CHECK(x.is_cuda() && x.dim() == 2 && x.stride(1) == 1, "x must be a 2-D GPU tensor, unit inner stride");
-  TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.stride(1) == 1, "y must be a 2-D GPU tensor, unit inner stride");
-  check_dtype(x, at::kBFloat16, "x"); check_dtype(wp, at::kBFloat16, "wp"); check_dtype(y, at::kBFloat16, "y");
-  check_dtype(ws, at::kFloat, "ws"); check_dtype(counters, at::kInt, "counters");
-  TORCH_CHECK(epi >= 0 && epi <= 3, "prefill_gemm epi must be 0..3 (RoPE + KV write: prefill_qkv_rope)");
-  TORCH_CHECK(wp.dim() == 4 && wp.size(2) == 64 && wp.size(3) == 8, "wp must be packed [N/16, K/32, 64, 8]");
-  const int M = x.size(0), K = x.size(1), N = wp.size(0) * 16;
-  TORCH_CHECK(wp.size(1) * 32 == K, "packed weight K mismatch");
-  TORCH_CHECK(x.stride(0) % 8 == 0 && y.stride(0) % 4 == 0, "x rows must be 16-byte, y rows 8-byte aligned");
-  // the non-pair epilogues (plain, residual) of the ping-pong kernels store -- and read the
-  // residual -- 16 B per lane (packed_epi.h store_pair_wide): y and resid rows 16-byte aligned
-  const bool wide = epi == 0 || epi == 2;
-  auto rows16 = [](const at::Tensor& t) { return t.stride(0) % 8 == 0 && ((uintptr_t)t.data_ptr() & 15) == 0; };
-  TORCH_CHECK(!wide || rows16(y), "y rows must be 16-byte aligned for the plain / residual epilogue");
-  TORCH_CHECK(((uintptr_t)y.data_ptr() & 7) == 0, "y must be 8-byte aligned");
-  const int NO = epi == 1 ? N / 2 : N;
-  TORCH_CHECK(y.size(0) == M && y.size(1) == NO, "y shape mismatch");
-  const void* rp = nullptr;
-  int ldr = 0;
-  if (epi == 2) {
-    TORCH_CHECK(resid.has_value(), "epi=2 needs resid");
-    const auto& r = *resid;
-    TORCH_CHECK(r.is_cuda() && r.dim() == 2 && r.stride(1) == 1 && r.size(0) == M && r.size(1) == N && rows16(r),
-                "resid must be [M, N] with unit inner stride and 16-byte aligned rows");
-    check_dtype(r, at::kBFloat16, "resid");
-    rp = r.data_ptr();
-    ldr = r.stride(0);
-  }
-  const int rc = pa_prefill_gemm(y.data_ptr(), x.data_ptr(), wp.data_ptr(), rp, ws.data_ptr<float>(), ws.numel(),
-                                 counters.data_ptr<int>(), counters.numel(), M, N, K, x.stride(0), y.stride(0), ldr,
-                                 (int)epi, opt_rows(ss_in, M, "ss_in"), const_cast<float*>(opt_rows(ss_out, M, "ss_out")),
-                                 const_cast<float*>(opt_rows(ss_zero, M, "ss_zero")), (float)eps, (int)full,
-                                 (int)splits, (int)bn, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0,
-                                 (int)variant, cur_stream());
-  TORCH_CHECK(rc >= 0, "prefill_gemm launch failed");
-  return rc == 0;
-}
-
 bool prefill_qkv_rope(at::Tensor x, at::Tensor wp, at::Tensor ss_in, double eps, at::Tensor q_out, at::Tensor k_cache,
                       at::Tensor v_cache, at::Tensor positions, at::Tensor slots, at::Tensor cos_sin, int64_t H,
                       int64_t KV, at::Tensor ws, at::Tensor counters, int64_t full, int64_t splits, int64_t bn,
@@ -616,7 +496,9 @@ void sample(at::Tensor out_tokens, c10::optional<at::Tensor> out_keys, at::Tenso
   check_gpu(class_masks, "class_masks"); check_gpu(seeds, "seeds"); check_gpu(offsets, "offsets");
   TORCH_CHECK(logits.is_cuda() && logits.dim() == 2 && logits.stride(1) == 1,
               "logits must be a 2-D GPU tensor with unit inner stride");
-  check_dtype(logits, at::kBFloat16, "logits"); check_dtype(out_tokens, at::kInt, "out_tokens");
+  const bool f32 = logits.scalar_type() == at::kFloat;
+  if (!f32) check_dtype(logits, at::kBFloat16, "logits");
+  check_dtype(out_tokens, at::kInt, "out_tokens");
   check_dtype(workspace, at::kFloat, "workspace"); check_dtype(temperature, at::kFloat, "temperature");
   check_dtype(mask_class, at::kInt, "mask_class"); check_dtype(class_masks, at::kInt, "class_masks");
   check_dtype(seeds, at::kLong, "seeds"); check_dtype(offsets, at::kInt, "offsets");
@@ -643,7 +525,7 @@ void sample(at::Tensor out_tokens, c10::optional<at::Tensor> out_keys, at::Tenso
     TORCH_CHECK(tau->numel() >= rows, "tau too short");
     tp = tau->data_ptr<float>();
   }
-  check_rc(pa_sample(out_tokens.data_ptr<int>(), keys, workspace.data_ptr<float>(),
+  check_rc(pa_sample(f32 ? 1 : 0, out_tokens.data_ptr<int>(), keys, workspace.data_ptr<float>(),
                      logits.data_ptr(), rows, V, logits.stride(0), vocab_offset,
                      temperature.data_ptr<float>(), mask_class.data_ptr<int>(),
                      reinterpret_cast<const uint32_t*>(class_masks.data_ptr<int>()),
@@ -899,28 +781,6 @@ void car_collective(std::vector<int64_t> bases, int64_t rank0, std::vector<at::T
                              reinterpret_cast<uint32_t*>(epochs.data_ptr<int>()), err.data_ptr<int>(), (int)op,
                              cur_stream()),
            "custom collective");
-}
-
-// ---- uncached device memory (in-launch hand-off workspaces) ----
-// Split-K slabs and attention partials are written by one workgroup and read by another
-// inside the same launch. In uncached memory (MTYPE UC: no L1/L2 copy of any line) a reader
-// can never see a stale copy held by its own CU or XCD, whatever the placement, so the
-// hand-off needs no L2 write-back on the producer side.
-at::Tensor empty_uncached(int64_t numel, at::ScalarType dtype, int64_t device) {
-  TORCH_CHECK(numel > 0, "empty_uncached: numel must be positive");
-  const int64_t bytes = numel * (int64_t)c10::elementSize(dtype);
-  int prev = 0;
-  TORCH_CHECK(hipGetDevice(&prev) == hipSuccess, "hipGetDevice failed");
-  TORCH_CHECK(hipSetDevice((int)device) == hipSuccess, "hipSetDevice failed");
-  void* p = nullptr;
-  const hipError_t e = hipExtMallocWithFlags(&p, (size_t)bytes, hipDeviceMallocUncached);
-  if (e == hipSuccess) (void)hipMemset(p, 0, (size_t)bytes);
-  (void)hipSetDevice(prev);
-  TORCH_CHECK(e == hipSuccess && p != nullptr, "empty_uncached: hipExtMallocWithFlags(", bytes,
-              " bytes, uncached) failed");
-  TORCH_CHECK(hipDeviceSynchronize() == hipSuccess, "empty_uncached: memset failed");
-  auto opts = at::TensorOptions().dtype(dtype).device(at::Device(at::kCUDA, (int)device));
-  return torch::from_blob(p, {numel}, [](void* q) { (void)hipFree(q); }, opts);
 }
 
 PYBIND11_MODULE(_C, m) {

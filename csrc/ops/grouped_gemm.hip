@@ -1,0 +1,294 @@
+// Grouped projections: many small weight matrices, each applied to its own rows.
+//
+//   dense   every row goes through every group, group h reading its own columns of x and writing
+//           its own columns of out (per-head up-projections of latent attention)
+//   sorted  row p belongs to one group: mixture-of-experts layers, rows sorted by expert into
+//           tiles of at most TM rows (table_route_kernel below)
+//
+// Weights are packed per group like the other projections ([N/16, K/32, 64, 8], one 16-B lane
+// vector per MFMA operand). The MFMA's A operand is W and its B operand x, so a lane's four
+// accumulators are four consecutive outputs of one row: 8-byte stores, and the gated pair
+// (tiles 2i: gate, 2i + 1: up) is lane-local.
+//
+// Epilogues: plain, or the clamped gated unit
+//   g' = min(g, limit), u' = clamp(u, -limit, limit),  out = g' * sigmoid(alpha * g') * (u' + bias).
+#include "common.h"
+
+namespace pa {
+namespace gg {
+
+struct Args {
+  const void* x;
+  const void* w;
+  void* out;
+  long long wstride;       // elements per group
+  int ldx, xg, ldo, og;    // row strides and per-group column offsets (dense)
+  int rows, N16, K32;      // dense rows; N16 = packed 16-row tiles per group
+  const int4* tiles;       // sorted: {group, first position, rows, 0}
+  const int* n_tiles;
+  const int* order;        // sorted: position -> token * top + k
+  int x_div;               // sorted: x row = order / x_div (0: x row = position)
+  int out_order;           // sorted: out row = order[position] (0: out row = position)
+  float limit, alpha, bias;
+};
+
+__device__ __forceinline__ float glu(float g, float u, const Args& A) {
+  g = fminf(g, A.limit);
+  u = fminf(fmaxf(u, -A.limit), A.limit);
+  return g / (1.f + __expf(-A.alpha * g)) * (u + A.bias);
+}
+
+template <int MT, int NT, int KU, bool GLU>
+__global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int c = lane & 15, g = lane >> 4;
+  int grp, start, n;
+  if (A.tiles) {
+    if ((int)blockIdx.y >= A.n_tiles[0]) return;
+    const int4 tl = A.tiles[blockIdx.y];
+    grp = tl.x;
+    start = tl.y;
+    n = tl.z;
+  } else {
+    grp = blockIdx.z;
+    start = blockIdx.y * (16 * MT);
+    n = min(16 * MT, A.rows - start);
+  }
+  const int nt0 = (blockIdx.x * 4 + wid) * NT;
+  if (nt0 >= A.N16) return;
+  const bf16* wp = (const bf16*)A.w + (size_t)grp * A.wstride + lane * 8;
+  const bf16* wt[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) wt[i] = wp + (size_t)min(nt0 + i, A.N16 - 1) * A.K32 * 512;
+  const bf16* xr[MT];
+  int pos[MT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    const int i = min(16 * m + c, n - 1);
+    pos[m] = start + i;
+    int row = pos[m];
+    if (A.tiles && A.x_div) row = A.order[pos[m]] / A.x_div;
+    xr[m] = (const bf16*)A.x + (size_t)row * A.ldx + (A.tiles ? 0 : (size_t)grp * A.xg) + 8 * g;
+  }
+  f32x4 acc[MT][NT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int i = 0; i < NT; ++i) acc[m][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  bf16x8 a[KU][NT], b[KU][MT];
+  auto load = [&](int s, bf16x8 (&aa)[KU][NT], bf16x8 (&bb)[KU][MT]) {
+#pragma unroll
+    for (int k = 0; k < KU; ++k) {
+#pragma unroll
+      for (int i = 0; i < NT; ++i) aa[k][i] = *reinterpret_cast<const bf16x8*>(wt[i] + (size_t)(s + k) * 512);
+#pragma unroll
+      for (int m = 0; m < MT; ++m) bb[k][m] = *reinterpret_cast<const bf16x8*>(xr[m] + (size_t)(s + k) * 32);
+    }
+  };
+  load(0, a, b);
+  for (int s = 0; s < A.K32; s += KU) {
+    bf16x8 an[KU][NT], bn[KU][MT];
+    if (s + KU < A.K32) load(s + KU, an, bn);
+#pragma unroll
+    for (int k = 0; k < KU; ++k)
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int i = 0; i < NT; ++i)
+          acc[m][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[k][i], b[k][m], acc[m][i], 0, 0, 0);
+#pragma unroll
+    for (int k = 0; k < KU; ++k) {
+#pragma unroll
+      for (int i = 0; i < NT; ++i) a[k][i] = an[k][i];
+#pragma unroll
+      for (int m = 0; m < MT; ++m) b[k][m] = bn[k][m];
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    if (16 * m + c >= n) continue;
+    const int orow = (A.tiles && A.out_order) ? A.order[pos[m]] : pos[m];
+    bf16* o = (bf16*)A.out + (size_t)orow * A.ldo + (A.tiles ? 0 : (size_t)grp * A.og) + 4 * g;
+    if constexpr (GLU) {
+#pragma unroll
+      for (int i = 0; i + 1 < NT; i += 2) {
+        if (nt0 + i >= A.N16) break;
+        bf16x4 v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = (bf16)glu(acc[m][i][j], acc[m][i + 1][j], A);
+        *reinterpret_cast<bf16x4*>(o + (nt0 + i) * 8) = v;
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        if (nt0 + i >= A.N16) break;
+        bf16x4 v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = (bf16)acc[m][i][j];
+        *reinterpret_cast<bf16x4*>(o + (nt0 + i) * 16) = v;
+      }
+    }
+  }
+}
+
+// fp32: one output (or gated pair) per thread, weights row-major [G, 16 N16, 32 K32] in the same
+// row order as the packed ones. The exact path; not tuned.
+template <bool GLU>
+__global__ __launch_bounds__(256) void gemm_f32_kernel(const Args A) {
+  constexpr int TM = 16;
+  __shared__ float xs[TM][33], w0[16][33], w1[16][33];
+  const int tn = threadIdx.x & 15, tm = threadIdx.x >> 4;
+  int grp, start, n;
+  if (A.tiles) {
+    if ((int)blockIdx.y >= A.n_tiles[0]) return;
+    const int4 tl = A.tiles[blockIdx.y];
+    grp = tl.x; start = tl.y; n = tl.z;
+  } else {
+    grp = blockIdx.z;
+    start = blockIdx.y * TM;
+    n = min(TM, A.rows - start);
+  }
+  const int K = A.K32 * 32;
+  const float* wg = (const float*)A.w + (size_t)grp * A.wstride + (size_t)blockIdx.x * (GLU ? 32 : 16) * K;
+  float a0 = 0.f, a1 = 0.f;
+  for (int k0 = 0; k0 < K; k0 += 32) {
+    __syncthreads();
+    for (int e = threadIdx.x; e < TM * 32; e += 256) {
+      const int m = e >> 5, k = e & 31, p = start + min(m, n - 1);
+      int row = p;
+      if (A.tiles && A.x_div) row = A.order[p] / A.x_div;
+      xs[m][k] = ((const float*)A.x)[(size_t)row * A.ldx + (A.tiles ? 0 : (size_t)grp * A.xg) + k0 + k];
+      w0[m][k] = wg[(size_t)m * K + k0 + k];
+      if (GLU) w1[m][k] = wg[(size_t)(16 + m) * K + k0 + k];
+    }
+    __syncthreads();
+#pragma unroll 8
+    for (int k = 0; k < 32; ++k) {
+      a0 += xs[tm][k] * w0[tn][k];
+      if (GLU) a1 += xs[tm][k] * w1[tn][k];
+    }
+  }
+  if (tm >= n) return;
+  const int p = start + tm;
+  const int orow = (A.tiles && A.out_order) ? A.order[p] : p;
+  float* o = (float*)A.out + (size_t)orow * A.ldo + (A.tiles ? 0 : (size_t)grp * A.og) + blockIdx.x * 16 + tn;
+  *o = GLU ? glu(a0, a1, A) : a0;
+}
+
+// Routing by token id, for every expert layer of the model in one launch (workgroup = layer):
+// layer l's table [vocab, top] (int32, at tables + desc[0]) names the token's experts. Rows with
+// slot < 0 (padding) are left out. Writes, at the layer's offsets,
+//   order[p] = token * top + k, positions sorted by expert;  tiles: at most tm rows of one expert each.
+constexpr int ROUTE_DESC = 8;  // {table offset, vocab, top, experts, order offset, tile offset, max tiles, 0}
+constexpr int ROUTE_EMAX = 2048;
+
+__global__ __launch_bounds__(1024) void table_route_kernel(const int* __restrict__ tables, const int* __restrict__ desc,
+                                                           const int* __restrict__ ids, const int* __restrict__ slots,
+                                                           int T, int tm, int* __restrict__ order,
+                                                           int4* __restrict__ tiles, int* __restrict__ n_tiles) {
+  __shared__ int cnt[ROUTE_EMAX], base[ROUTE_EMAX], tbase[ROUTE_EMAX], ws[2][16];
+  const int* d = desc + blockIdx.x * ROUTE_DESC;
+  const int V = d[1], top = d[2], E = d[3];
+  const int* tab = tables + d[0];
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  for (int e = threadIdx.x; e < E; e += 1024) cnt[e] = 0;
+  __syncthreads();
+  auto expert = [&](int p) {
+    const int t = p / top;
+    if (slots[t] < 0) return -1;
+    const int e = tab[(size_t)min(max(ids[t], 0), V - 1) * top + (p - t * top)];
+    return min(max(e, 0), E - 1);
+  };
+  for (int p = threadIdx.x; p < T * top; p += 1024) {
+    const int e = expert(p);
+    if (e >= 0) atomicAdd(&cnt[e], 1);
+  }
+  __syncthreads();
+  // exclusive scans of the row and tile counts, 1,024 experts at a time
+  int carry_r = 0, carry_t = 0;
+  for (int e0 = 0; e0 < E; e0 += 1024) {
+    const int e = e0 + threadIdx.x;
+    const int r = e < E ? cnt[e] : 0, q = (r + tm - 1) / tm;
+    int sr = r, sq = q;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const int a = __shfl_up(sr, o, 64), b = __shfl_up(sq, o, 64);
+      if (lane >= o) { sr += a; sq += b; }
+    }
+    if (lane == 63) { ws[0][wid] = sr; ws[1][wid] = sq; }
+    __syncthreads();
+    int or_ = carry_r, oq = carry_t, tr = 0, tq = 0;
+    for (int w = 0; w < 16; ++w) {
+      if (w < wid) { or_ += ws[0][w]; oq += ws[1][w]; }
+      tr += ws[0][w];
+      tq += ws[1][w];
+    }
+    if (e < E) { base[e] = or_ + sr - r; tbase[e] = oq + sq - q; }
+    carry_r += tr;
+    carry_t += tq;
+    __syncthreads();
+  }
+  int4* tl = tiles + d[5];
+  for (int e = threadIdx.x; e < E; e += 1024)
+    for (int i = 0, k = tbase[e]; i < cnt[e]; i += tm, ++k)
+      if (k < d[6]) tl[k] = int4{e, base[e] + i, min(tm, cnt[e] - i), 0};
+  if (threadIdx.x == 0) n_tiles[blockIdx.x] = min(carry_t, d[6]);
+  __syncthreads();
+  int* ord = order + d[4];
+  for (int p = threadIdx.x; p < T * top; p += 1024) {
+    const int e = expert(p);
+    if (e >= 0) ord[atomicAdd(&base[e], 1)] = p;
+  }
+}
+
+}  // namespace gg
+}  // namespace pa
+
+extern "C" int pa_table_route(const int* tables, const int* desc, int layers, const int* ids, const int* slots, int T,
+                              int tm, int* order, int* tiles, int* n_tiles, hipStream_t st) {
+  if (layers <= 0 || T <= 0) return 0;
+  hipLaunchKernelGGL(pa::gg::table_route_kernel, dim3(layers), dim3(1024), 0, st, tables, desc, ids, slots, T, tm,
+                     order, (int4*)tiles, n_tiles);
+  return (int)hipGetLastError();
+}
+
+// tm: rows per sorted tile (16 or 64; dense: the kernel's choice by row count)
+extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out, long long wstride, int groups,
+                               int ldx, int xg, int ldo, int og, int rows, int N16, int K32, const int* tiles,
+                               int max_tiles, const int* n_tiles, const int* order, int x_div, int out_order, int tm,
+                               int epi, float limit, float alpha, float bias, hipStream_t st) {
+  if (N16 <= 0 || K32 <= 0 || (epi == 1 && N16 % 2)) return -1;
+  if (tiles ? max_tiles <= 0 : rows <= 0) return 0;
+  const pa::gg::Args A{x, w, out, wstride, ldx, xg, ldo, og, rows, N16, K32, (const int4*)tiles, n_tiles,
+                       order, x_div, out_order, limit, alpha, bias};
+  if (fp32) {
+    if (tiles && tm != 16) return -2;
+    const dim3 grid(epi == 1 ? N16 / 2 : N16, tiles ? max_tiles : (rows + 15) / 16, tiles ? 1 : groups);
+    if (epi == 1) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<true>), grid, dim3(256), 0, st, A);
+    else hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<false>), grid, dim3(256), 0, st, A);
+    return (int)hipGetLastError();
+  }
+  if (!tiles) tm = rows <= 32 ? 16 : 64;
+  if (tm != 16 && tm != 64) return -2;
+#define PA_GG(MT, NT, KU, G)                                                                                   \
+  hipLaunchKernelGGL((pa::gg::gemm_kernel<MT, NT, KU, G>),                                                     \
+                     dim3((N16 + 4 * NT - 1) / (4 * NT), tiles ? max_tiles : (rows + 16 * MT - 1) / (16 * MT), \
+                          tiles ? 1 : groups),                                                                 \
+                     dim3(256), 0, st, A)
+#define PA_GGK(MT, NT, G)                      \
+  do {                                         \
+    if (K32 % 4 == 0) PA_GG(MT, NT, 4, G);     \
+    else if (K32 % 2 == 0) PA_GG(MT, NT, 2, G);\
+    else PA_GG(MT, NT, 1, G);                  \
+  } while (0)
+  if (tm == 16) {
+    if (epi == 1) PA_GGK(1, 2, true);
+    else PA_GGK(1, 1, false);
+  } else {
+    if (epi == 1) PA_GG(4, 4, 1, true);
+    else PA_GG(4, 4, 1, false);
+  }
+#undef PA_GGK
+#undef PA_GG
+  return (int)hipGetLastError();
+}

@@ -33,8 +33,9 @@ __device__ __forceinline__ KeyIdx better(KeyIdx a, KeyIdx b) {
   return a;
 }
 
+template <typename T8>
 __global__ __launch_bounds__(256) void sample_chunk_kernel(
-    float* __restrict__ part_k, int* __restrict__ part_i, const bf16* __restrict__ logits,
+    float* __restrict__ part_k, int* __restrict__ part_i, const T8* __restrict__ logits,
     int V, int ld, int vocab_offset, const float* __restrict__ temperature,
     const int* __restrict__ mask_class, const uint32_t* __restrict__ class_masks, int mask_words,
     const int64_t* __restrict__ seeds, const int* __restrict__ offsets, int nchunk,
@@ -47,14 +48,15 @@ __global__ __launch_bounds__(256) void sample_chunk_kernel(
   const int mc = mask_class[row];
   const uint64_t seed = (uint64_t)seeds[row];
   const uint32_t off = (uint32_t)offsets[row];
-  const bf16* lr = logits + (size_t)row * ld;
+  const T8* lr = logits + (size_t)row * ld;
   KeyIdx best{-INFINITY, 0x7fffffff};
   const int base = chunk * SMP_CHUNK + threadIdx.x * 8;
 #pragma unroll
   for (int h = 0; h < 2; ++h) {
     const int i0 = base + h * 2048;
     if (i0 >= V) break;
-    bf16x8 v = *reinterpret_cast<const bf16x8*>(lr + i0);
+    T8 v[8];
+    __builtin_memcpy(v, __builtin_assume_aligned(lr + i0, 16), sizeof(v));
     uint32_t bits = 0xffffffffu;
     if (mc >= 0) {
       const int gi = vocab_offset + i0;  // global vocab index (TP shards)
@@ -64,7 +66,7 @@ __global__ __launch_bounds__(256) void sample_chunk_kernel(
     for (int j = 0; j < 8; ++j) {
       const int i = i0 + j;
       if (i >= V || !((bits >> j) & 1u)) continue;
-      const float lv = bf2f(v[j]);
+      const float lv = (float)v[j];
       if (lv < thr) continue;
       float key = lv * invT;
       if (!greedy) {
@@ -416,19 +418,22 @@ extern "C" int pa_sample_workspace_floats(int rows, int V) {
 // workspace: float[rows * nchunk] keys followed by int[rows * nchunk] indices.
 // out_keys (optional) receives the winning perturbed key per row, used by the
 // tensor-parallel sampler to pick the global winner across vocab shards.
-extern "C" int pa_sample(int* out_tokens, float* out_keys, float* workspace, const void* logits,
+extern "C" int pa_sample(int fp32, int* out_tokens, float* out_keys, float* workspace, const void* logits,
                          int rows, int V, int ld, int vocab_offset, const float* temperature,
                          const int* mask_class, const uint32_t* class_masks, int mask_words,
                          const int64_t* seeds, const int* offsets, const int* forced,
                          const float* tau, hipStream_t st) {
   if (rows <= 0) return 0;
-  if (V % 8 != 0 || ld % 8 != 0) return -1;
+  if (ld % 8 != 0 || ld < (V + 7) / 8 * 8) return -1;  // 16-byte reads may pass V within a row
   const int nchunk = (V + pa::SMP_CHUNK - 1) / pa::SMP_CHUNK;
   float* pk = workspace;
   int* pi = reinterpret_cast<int*>(workspace + (size_t)rows * nchunk);
-  hipLaunchKernelGGL(pa::sample_chunk_kernel, dim3(nchunk, rows), dim3(256), 0, st, pk, pi,
-                     (const pa::bf16*)logits, V, ld, vocab_offset, temperature, mask_class,
-                     class_masks, mask_words, seeds, offsets, nchunk, tau);
+#define PA_SC(T)                                                                                       \
+  hipLaunchKernelGGL((pa::sample_chunk_kernel<T>), dim3(nchunk, rows), dim3(256), 0, st, pk, pi,       \
+                     (const T*)logits, V, ld, vocab_offset, temperature, mask_class, class_masks,      \
+                     mask_words, seeds, offsets, nchunk, tau)
+  if (fp32) PA_SC(float); else PA_SC(pa::bf16);
+#undef PA_SC
   hipLaunchKernelGGL(pa::sample_final_kernel, dim3(rows), dim3(64), 0, st, out_tokens, out_keys,
                      pk, pi, forced, nchunk);
   return (int)hipGetLastError();

@@ -153,6 +153,8 @@ PYBIND11_MODULE(_runtime, m) {
         if (d.contains("max_model_len")) c.max_model_len = d["max_model_len"].cast<int32_t>();
         if (d.contains("gqa_group")) c.gqa_group = d["gqa_group"].cast<int32_t>();
         if (d.contains("att_qcols")) c.att_qcols = d["att_qcols"].cast<int32_t>();
+        if (d.contains("att_narrow_qcols")) c.att_narrow_qcols = d["att_narrow_qcols"].cast<int32_t>();
+        if (d.contains("att_max_keys")) c.att_max_keys = d["att_max_keys"].cast<int32_t>();
         if (d.contains("att_wide_min_tokens")) c.att_wide_min_tokens = d["att_wide_min_tokens"].cast<int32_t>();
         if (d.contains("prefill_split_keys")) c.prefill_split_keys = d["prefill_split_keys"].cast<int32_t>();
         if (d.contains("prefix_caching")) c.prefix_caching = d["prefix_caching"].cast<bool>();
@@ -201,6 +203,11 @@ PYBIND11_MODULE(_runtime, m) {
       .def("schedule", [](Scheduler& s, uintptr_t buf) {
         py::gil_scoped_release nogil;
         return s.schedule(reinterpret_cast<int32_t*>(buf));
+      })
+      .def("schedule_fed", [](Scheduler& s, uintptr_t buf, const std::vector<std::pair<int64_t, std::vector<int32_t>>>& in) {
+        std::vector<Scheduler::FedEntry> e;
+        for (const auto& x : in) e.push_back({x.first, x.second});
+        return s.schedule_fed(reinterpret_cast<int32_t*>(buf), e);
       })
       .def("commit", [](Scheduler& s, uintptr_t sampled, int32_t n) {
         std::vector<SeqOutput> outs;

@@ -197,7 +197,7 @@ int32_t Scheduler::schedule(int32_t* buf) {
       // (and not listed by an in-flight step)
       Sequence* victim = nullptr;
       for (size_t j = running_.size(); j-- > i + 1;) {
-        if (running_[j]->running && running_[j]->inflight == 0 && !running_[j]->abort_pending) {
+        if (running_[j]->running && running_[j]->inflight == 0 && !running_[j]->abort_pending && !running_[j]->fed) {
           victim = running_[j];
           break;
         }
@@ -303,6 +303,55 @@ int32_t Scheduler::schedule(int32_t* buf) {
     }
   }
 
+  return emit(buf);
+}
+
+int32_t Scheduler::schedule_fed(int32_t* buf, const std::vector<FedEntry>& entries) {
+  if (!plans_.empty()) throw std::logic_error("scheduler: a fed step follows a committed step");
+  // check the whole step before anything is taken from the pool
+  int64_t total = 0;
+  int32_t fresh = 0, need = 0;
+  std::unordered_set<int64_t> seen;
+  for (const FedEntry& e : entries) {
+    auto it = seqs_.find(e.id);
+    const Sequence* s = it == seqs_.end() ? nullptr : it->second.get();
+    if (e.tokens.empty()) throw std::invalid_argument("scheduler: a fed entry without tokens");
+    if (!seen.insert(e.id).second) throw std::invalid_argument("scheduler: a request fed twice in one step");
+    if (s && !s->fed) throw std::invalid_argument("scheduler: the id belongs to a generating request");
+    const int64_t len = (s ? (int64_t)s->tokens.size() : 0) + (int64_t)e.tokens.size();
+    if (len > cfg_.max_model_len) throw std::invalid_argument("scheduler: a fed request exceeds max_model_len");
+    need += (int32_t)((len + cfg_.block_size - 1) / cfg_.block_size) - (s ? (int32_t)s->blocks.size() : 0);
+    total += (int64_t)e.tokens.size();
+    fresh += s == nullptr;
+  }
+  if (total > cfg_.max_num_batched_tokens) throw std::invalid_argument("scheduler: fed step exceeds max_num_batched_tokens");
+  if ((int32_t)running_.size() + fresh > cfg_.max_num_seqs) throw std::runtime_error("scheduler: more live requests than slots");
+  if (need > bm_.num_free()) throw std::runtime_error("scheduler: the cache pool is exhausted");
+  last_plan_.clear();
+  for (const FedEntry& e : entries) {
+    auto it = seqs_.find(e.id);
+    if (it == seqs_.end()) {
+      auto n = std::make_unique<Sequence>();
+      n->id = e.id;
+      n->fed = true;
+      n->running = true;
+      n->arrival = arrival_counter_++;
+      n->cached_prompt_tokens = 0;
+      running_.push_back(n.get());
+      it = seqs_.emplace(e.id, std::move(n)).first;
+    }
+    Sequence* s = it->second.get();
+    s->tokens.insert(s->tokens.end(), e.tokens.begin(), e.tokens.end());
+    s->prompt_len = (int32_t)s->tokens.size();
+    if (!ensure_blocks(s, s->prompt_len)) throw std::runtime_error("scheduler: the cache pool is exhausted");
+    last_plan_.push_back({s, (int32_t)e.tokens.size(), false});
+  }
+  return emit(buf);
+}
+
+int32_t Scheduler::emit(int32_t* buf) {
+  const StepLayout& L = lay_;
+  const int32_t B = cfg_.block_size;
   // 3) emit the step description
   int32_t* counts = buf + L.counts;
   int32_t* ids = buf + L.input_ids;
@@ -346,13 +395,18 @@ int32_t Scheduler::schedule(int32_t* buf) {
       ++prefill_seqs;
     }
   const bool wide = prefill_tokens >= cfg_.att_wide_min_tokens && prefill_seqs >= 2;
-  const int32_t qcols = wide ? std::max(32, cfg_.att_qcols) : 32;
+  const int32_t qcols = wide ? std::max(cfg_.att_narrow_qcols, cfg_.att_qcols) : cfg_.att_narrow_qcols;
   const int32_t qtile = std::max(1, qcols / std::max(1, cfg_.gqa_group));
   int32_t psz = 512;
+  // keys a decode row attends to (a model whose every layer has a window never reads more)
+  auto att_keys = [this](const Planned& p) {
+    const int32_t c = p.s->num_computed + p.n;
+    return cfg_.att_max_keys > 0 ? std::min(c, cfg_.att_max_keys + p.n - 1) : c;
+  };
   if (cfg_.split_decode) {
     int64_t parts512 = 0, parts256 = 0, nprefill = 0;
     for (const Planned& p : last_plan_) {
-      const int32_t c = p.s->num_computed + p.n;
+      const int32_t c = att_keys(p);
       if (p.n <= tpw) {
         parts512 += std::max(1, (c + 511) / 512);
         parts256 += std::max(1, (c + 255) / 256);
@@ -373,7 +427,7 @@ int32_t Scheduler::schedule(int32_t* buf) {
       for (const Planned& p : last_plan_)
         if (p.n <= tpw) {
           ++ndec;
-          const int64_t c = p.s->num_computed + p.n;
+          const int64_t c = att_keys(p);
           maxc = std::max<int64_t>(maxc, c);
           sumc += c;
         }
@@ -393,7 +447,7 @@ int32_t Scheduler::schedule(int32_t* buf) {
         }
         int64_t parts = 0;
         for (const Planned& p : last_plan_)
-          if (p.n <= tpw) parts += std::max<int64_t>(1, (p.s->num_computed + p.n + cand - 1) / cand);
+          if (p.n <= tpw) parts += std::max<int64_t>(1, (att_keys(p) + cand - 1) / cand);
         if (nprefill + parts <= L.max_items) psz = (int32_t)cand;
       }
     }
@@ -460,14 +514,15 @@ int32_t Scheduler::schedule(int32_t* buf) {
     }
     // attention work items (mirrors pilottai_amd/ops/attn_meta.py)
     if (n <= tpw) {
-      const int32_t nparts = cfg_.split_decode ? std::max(1, (ctx + psz - 1) / psz) : 1;
+      const int32_t akeys = cfg_.att_max_keys > 0 ? std::min(ctx, cfg_.att_max_keys + n - 1) : ctx;
+      const int32_t nparts = cfg_.split_decode ? std::max(1, (akeys + psz - 1) / psz) : 1;
       if (nparts > 1) {
         for (int32_t q = 0; q < nparts; ++q)
-          dec.push_back({std::min(psz, ctx - q * psz), ns, 0, n | (q << 8) | (nparts << 20), pslot + q});
+          dec.push_back({std::min(psz, akeys - q * psz), ns, 0, n | (q << 8) | (nparts << 20), pslot + q});
         ++nparted;  // merged in-kernel by the last partition (attention.hip)
         pslot += nparts;
       } else {
-        dec.push_back({ctx, ns, 0, n | (1 << 20), 0});
+        dec.push_back({akeys, ns, 0, n | (1 << 20), 0});
       }
     }
     s->num_computed = ctx;
@@ -485,7 +540,7 @@ int32_t Scheduler::schedule(int32_t* buf) {
   int32_t t_step_all = 0;
   for (const Planned& p : last_plan_) t_step_all += p.n;
   const int32_t G = std::max(1, cfg_.gqa_group);
-  if (cfg_.prefill_split_keys > 0 && qtile * G > 32 && t_step_all > cfg_.small_step_tokens) {
+  if (cfg_.prefill_split_keys > 0 && qtile * G > cfg_.att_narrow_qcols && t_step_all > cfg_.small_step_tokens) {
     std::vector<ItemCost> split;
     int64_t n_items_total = (int64_t)pre.size() + (int64_t)dec.size();
     for (const ItemCost& c : pre) {

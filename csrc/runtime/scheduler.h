@@ -34,6 +34,10 @@ struct SchedulerConfig {
   int32_t gqa_group = 4;               // query heads per KV head (attention work items)
   int32_t att_qcols = 128;             // MFMA columns (heads x tokens) per prefill attention item:
                                        // 128 = the LDS-staged 4-wave path, 32 = one wave per item
+  int32_t att_narrow_qcols = 32;       // ... of the steps that take no wide items
+  // > 0: no layer attends to more than this many keys back (every layer has a window): decode rows
+  // are cut into partitions of the keys they really read, not of the whole context
+  int32_t att_max_keys = 0;
   int32_t att_wide_min_tokens = 2048;
   // wide prefill items whose causal key range reaches this many keys are cut into
   // min(4, keys / prefill_split_keys) partitions of whole 32-key tiles, merged in-kernel by the
@@ -130,6 +134,7 @@ struct Sequence {
   int64_t arrival = 0;
   double t_first_token = -1.0;
   bool running = false;
+  bool fed = false;  // its tokens come from schedule_fed(); schedule() never plans or preempts it
   // embedding request: the whole prompt is computed (no prefix-cache reuse: every token's
   // final hidden state is summed into pooling row embed_slot), nothing is sampled
   bool embed = false;
@@ -174,6 +179,15 @@ class Scheduler {
   // speculative entry (its sample is dropped, its KV beyond the pending token is
   // recomputed) — only the sampled token's own KV is kept, and it is always right.
   int32_t schedule(int32_t* buf);
+  // A step whose tokens come from the caller (trace replay, scoring given continuations): every
+  // entry appends its tokens to a request, admitted at its first entry, and all entries run as
+  // one batch. Nothing is sampled: commit(nullptr, 0) ends the step, abort() gives back what a
+  // request holds. Throws, with nothing changed, when the step does not fit.
+  struct FedEntry {
+    int64_t id;
+    std::vector<int32_t> tokens;
+  };
+  int32_t schedule_fed(int32_t* buf, const std::vector<FedEntry>& entries);
   // Consume the sampled tokens of the oldest uncommitted step (one per sampling row).
   std::vector<SeqOutput> commit(const int32_t* sampled, int32_t n);
   int32_t inflight_steps() const { return (int32_t)plans_.size(); }
@@ -206,6 +220,7 @@ class Scheduler {
   int32_t num_free_embed_rows() const { return (int32_t)embed_free_.size(); }
 
  private:
+  int32_t emit(int32_t* buf);  // write last_plan_ into buf and queue it as an uncommitted step
   bool ensure_blocks(Sequence* s, int32_t upto_tokens);
   void preempt(Sequence* s);
   void match_prefix(Sequence* s);

@@ -1,10 +1,13 @@
 """In-tree builder for the native parts of pilottai_amd.
 
-Two shared objects are produced next to the Python sources so they travel with
+Three shared objects are produced next to the Python sources so they travel with
 the repository snapshot to the GPU box:
 
 * ``pilottai_amd/_C.so``       — CDNA4 HIP kernels (csrc/ops/*.hip, gfx950 only)
                                   + torch/pybind11 bindings (csrc/ops/bindings.cpp)
+* ``pilottai_amd/_latent.so`` — the kernels of models with latent attention and table-routed
+                                  experts, with the packed projections they share (so that
+                                  such a model needs no other kernel to run)
 * ``pilottai_amd/_runtime.so`` — C++ serving runtime: paged-KV block manager,
                                   prefix cache, continuous-batching scheduler,
                                   grammar FSM + tokenizer (csrc/runtime/*.cpp),
@@ -32,6 +35,12 @@ ARCH = os.environ.get("PILOTTAI_GPU_ARCH", "gfx950")
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # Per-file code-generation flags. gemm_mid.hip: MFMA accumulators in the VGPR form; with
 # the AGPR form hipcc shuffles them through v_accvgpr moves in the software-pipelined loop.
+# No file may use packed fp32 arithmetic (v_pk_*_f32): some forms have given wrong results.
+HIP_FLAGS = ["-ffast-math", "-fno-gpu-rdc", "-Wno-unused-result", "-Xclang", "-target-feature", "-Xclang",
+             "-packed-fp32-ops"]
+# the sources of _latent.so; the GEMM sources are in _C.so too
+LATENT_HIP = ["grouped_gemm.hip", "latent_attention.hip", "latent_cache.hip", "residual_norm.hip"]
+SHARED_HIP = ["gemm_decode.hip", "gemm_prefill.hip"]
 FILE_FLAGS = {"gemm_mid.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"],
               "gemm_stream.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"]}
 
@@ -75,40 +84,53 @@ def _compile_many(jobs, workers: int):
     return len(todo)
 
 
-def build_ops(verbose: bool = False, workers: int | None = None) -> Path:
-    """Compile csrc/ops into pilottai_amd/_C.so (gfx950 code objects)."""
+def _build_ext(name: str, hips, binding: str, verbose: bool, workers: int | None) -> Path:
+    """Compile csrc/ops sources and one binding file into pilottai_amd/<name>.so (gfx950 code objects)."""
     incs, libdirs = _torch_paths()
-    out = PKG / ("_C" + sysconfig.get_config_var("EXT_SUFFIX"))
+    out = PKG / (name + sysconfig.get_config_var("EXT_SUFFIX"))
     BUILD.mkdir(exist_ok=True)
     headers = glob.glob(str(CSRC / "ops" / "*.h"))
     jobs = []
     objs = []
-    for src in sorted(glob.glob(str(CSRC / "ops" / "*.hip"))):
+    for src in hips:
+        src = str(CSRC / "ops" / src)
         obj = str(BUILD / (Path(src).stem + ".hip.o"))
         cmd = [HIPCC, f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-c", src,
-               "-o", obj, "-ffast-math", "-fno-gpu-rdc", "-Wno-unused-result",
-               *FILE_FLAGS.get(Path(src).name, [])]
+               "-o", obj, *HIP_FLAGS, *FILE_FLAGS.get(Path(src).name, [])]
         jobs.append((src, obj, cmd, headers))
         objs.append(obj)
-    bsrc = str(CSRC / "ops" / "bindings.cpp")
-    bobj = str(BUILD / "ops_bindings.o")
-    defs = ["-D__HIP_PLATFORM_AMD__=1", "-DUSE_ROCM=1", "-DTORCH_EXTENSION_NAME=_C",
+    bsrc = str(CSRC / "ops" / binding)
+    bobj = str(BUILD / f"ops_{Path(binding).stem}.o")
+    defs = ["-D__HIP_PLATFORM_AMD__=1", "-DUSE_ROCM=1", f"-DTORCH_EXTENSION_NAME={name}",
             "-DTORCH_API_INCLUDE_EXTENSION_H", "-D_GLIBCXX_USE_CXX11_ABI=1"]
     bcmd = ["g++", "-O2", "-std=c++17", "-fPIC", "-c", bsrc, "-o", bobj, *defs,
             "-I/opt/rocm/include", f"-I{_py_include()}"] + [f"-I{i}" for i in incs]
-    jobs.append((bsrc, bobj, bcmd, []))
+    jobs.append((bsrc, bobj, bcmd, headers))
     objs.append(bobj)
     n = _compile_many(jobs, workers or min(8, os.cpu_count() or 4))
     if n or not out.exists() or out.stat().st_mtime < _newest(objs):
-        link = [HIPCC, "-shared", "-fPIC", f"--offload-arch={ARCH}", "-o", str(out), *objs]
+        part = str(out) + f".{os.getpid()}"  # several processes may build at once: rename into place
+        link = [HIPCC, "-shared", "-fPIC", f"--offload-arch={ARCH}", "-o", part, *objs]
         for d in libdirs:
             link += [f"-L{d}", f"-Wl,-rpath,{d}"]
         link += ["-lc10", "-lc10_hip", "-ltorch", "-ltorch_cpu", "-ltorch_hip",
                  "-ltorch_python", "-lamdhip64"]
         _run(link)
+        os.replace(part, out)
         if verbose:
             print(f"[pilottai_amd] linked {out}")
     return out
+
+
+def build_ops(verbose: bool = False, workers: int | None = None) -> Path:
+    """pilottai_amd/_C.so: every kernel but the latent-attention models' own."""
+    hips = sorted(Path(p).name for p in glob.glob(str(CSRC / "ops" / "*.hip")))
+    return _build_ext("_C", [h for h in hips if h not in LATENT_HIP], "bindings.cpp", verbose, workers)
+
+
+def build_latent(verbose: bool = False, workers: int | None = None) -> Path:
+    """pilottai_amd/_latent.so: what a latent-attention model runs."""
+    return _build_ext("_latent", LATENT_HIP + SHARED_HIP, "bindings_latent.cpp", verbose, workers)
 
 
 def build_runtime(verbose: bool = False, workers: int | None = None) -> Path:
@@ -133,8 +155,42 @@ def build_runtime(verbose: bool = False, workers: int | None = None) -> Path:
     return out
 
 
+def _stale(so: Path, sources) -> bool:
+    return not so.exists() or so.stat().st_mtime < _newest(sources)
+
+
+def ensure(kind: str = "latent", gpu: bool = True) -> None:
+    """Build what running a model of `kind` needs, where it is missing or older than its sources: the
+    serving runtime and, for a GPU, the kernel module ("latent": _latent, "llama": _C). One process
+    builds at a time; the others wait for it."""
+    import fcntl
+
+    ext = sysconfig.get_config_var("EXT_SUFFIX")
+    ops_dir, name = CSRC / "ops", {"latent": "_latent", "llama": "_C"}[kind]
+    srcs = [str(p) for p in ops_dir.glob("*.h")]
+    if kind == "latent":
+        srcs += [str(ops_dir / h) for h in LATENT_HIP + SHARED_HIP + ["bindings_latent.cpp"]]
+    else:
+        srcs += [str(p) for p in ops_dir.glob("*.hip") if p.name not in LATENT_HIP] + [str(ops_dir / "bindings.cpp")]
+    rt = [str(p) for p in (CSRC / "runtime").glob("*.*")]
+
+    def todo():
+        return [f for f, so, src in ((build_runtime, PKG / ("_runtime" + ext), rt),
+                                     (build_latent if kind == "latent" else build_ops, PKG / (name + ext), srcs))
+                if _stale(so, src) and (gpu or f is build_runtime)]
+
+    if not todo():
+        return
+    BUILD.mkdir(exist_ok=True)
+    with open(BUILD / ".lock", "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        for f in todo():
+            f()
+
+
 def build_all(verbose: bool = False) -> None:
     build_runtime(verbose)
+    build_latent(verbose)
     build_ops(verbose)
 
 

@@ -41,10 +41,13 @@ from typing import Any, Callable, Dict, List, Optional, Sequence, Union
 
 import numpy as np
 import torch
+import torch.nn.functional as F
 
 from pilottai_amd import ops
 from pilottai_amd.engine.tp_sampling import tp_topkp_threshold
-from pilottai_amd.models.llama import KVCache, LlamaModel, StepMeta, get_config
+from pilottai_amd.models import registry
+from pilottai_amd.models.cache import StepMeta
+from pilottai_amd.models.llama import LlamaModel, get_config
 from pilottai_amd.parallel.comm import TPGroup
 from pilottai_amd.utils.tracing import trace_range
 
@@ -63,13 +66,17 @@ DEFAULT_BUCKETS = ([8, 16, 32, 48, 64, 80] + list(range(96, 513, 16)) + list(ran
 
 @dataclass
 class EngineConfig:
-    model: str = "llama-3-8b"
+    model: Any = "llama-3-8b"  # a preset's name, a checkpoint folder or a configuration (models/registry.py)
+    # arithmetic of the model: "bfloat16" (fp32 where its design asks for it) or "float32" throughout
+    dtype: str = "bfloat16"
     max_num_seqs: int = 256
     max_num_batched_tokens: int = 2048
     max_prefill_tokens: int = 2048
     max_model_len: int = 8192
     block_size: int = 16
     num_kv_blocks: Optional[int] = None
+    # take num_kv_blocks as it is, also when one request of max_model_len would not fit
+    exact_kv_blocks: bool = False
     kv_cache_gb: Optional[float] = None
     kv_cache_fraction: float = 0.5
     kv_reserve_gb: float = 20.0  # HBM always left outside the KV pool (graphs, activations, workspaces)
@@ -214,14 +221,15 @@ class LLMEngine:
         self.device = torch.device(device)
         self.on_gpu = self.device.type == "cuda"
         if self.on_gpu:
-            ops.require_native()
             torch.cuda.set_device(self.device)
         self.tp = tp or TPGroup.single()
         self.tok = tokenizer or get_tokenizer()
         self.grammar = GrammarCompiler(self.tok, reply_tokens=cfg.reply_tokens)
         self.model_cfg = get_config(cfg.model)
         mc = self.model_cfg
-        if self.on_gpu:
+        model_cls = registry.model_class(mc)
+        if self.on_gpu and model_cls is LlamaModel:
+            ops.require_native()
             from .gemm_tuning import load_tuned_gemms
 
             self.tuned_gemms = load_tuned_gemms(mc.name, self.tp.size)
@@ -231,8 +239,19 @@ class LLMEngine:
             lim = max(LlamaModel.MID_MAX_T if cfg.mid_max_t is None else int(cfg.mid_max_t),
                       LlamaModel.PREFILL_MAX_T if cfg.prefill_max_t is None else int(cfg.prefill_max_t))
             keep_dense = True if lim < cfg.max_num_batched_tokens else None
-        self.model = LlamaModel(mc, self.device, tp=self.tp, seed=cfg.seed, weights_path=cfg.weights_path,
-                                decode_pack=cfg.decode_fused, keep_dense=keep_dense)
+        if cfg.dtype not in ("bfloat16", "float32"):
+            raise ValueError(f"dtype must be 'bfloat16' or 'float32', not {cfg.dtype!r}")
+        self.dtype = getattr(torch, cfg.dtype)
+        self.max_model_len = min(cfg.max_model_len, mc.max_position)
+        if model_cls is LlamaModel:
+            if self.dtype != torch.bfloat16:
+                raise ValueError("Llama models run in bfloat16 only")
+            self.model = LlamaModel(mc, self.device, tp=self.tp, seed=cfg.seed, weights_path=cfg.weights_path,
+                                    decode_pack=cfg.decode_fused, keep_dense=keep_dense)
+        else:
+            self.model = model_cls(mc, self.device, dtype=self.dtype, tp=self.tp, seed=cfg.seed,
+                                   weights_path=cfg.weights_path or registry.default_weights(cfg.model),
+                                   max_len=self.max_model_len)
         if cfg.decode_fused_max_t is not None:
             self.model.DECODE_FUSED_MAX_T = int(cfg.decode_fused_max_t)
         if cfg.mid_max_t is not None:
@@ -248,10 +267,8 @@ class LLMEngine:
         if cfg.pf_midrange is not None:
             self.model.PF_MIDRANGE = frozenset(cfg.pf_midrange)
         self.load_time = time.time() - t0
-        self.max_model_len = min(cfg.max_model_len, mc.max_position)
         # ---- KV cache sizing (288 GB HBM: the default leaves room for graphs/activations)
-        kv_local = self.model.kv_local
-        bpb = KVCache.bytes_per_block(mc.num_layers, kv_local, cfg.block_size)
+        bpb = self.model.cache_bytes_per_block(cfg.block_size)
         nb = cfg.num_kv_blocks
         if nb is None:
             if cfg.kv_cache_gb is not None:
@@ -264,12 +281,13 @@ class LLMEngine:
             else:
                 nb = 2048
         need_min = (self.max_model_len + cfg.block_size - 1) // cfg.block_size + 1
-        nb = max(nb, need_min)
+        if not cfg.exact_kv_blocks:
+            nb = max(nb, need_min)
         if self.tp.size > 1:  # block ids travel in the metadata: every rank needs the same pool
             t = torch.tensor([nb], dtype=torch.int64)
             torch.distributed.all_reduce(t, op=torch.distributed.ReduceOp.MIN, group=self.tp.cpu_group)
             nb = int(t.item())
-        self.kv = KVCache(mc.num_layers, nb, kv_local, self.device, block_size=cfg.block_size)
+        self.kv = self.model.make_cache(nb, cfg.block_size)
         self.num_kv_blocks = nb
         # ---- native scheduler + step buffers
         # the model runs 8-wave decode attention on the fused decode path only, keyed on the
@@ -280,11 +298,11 @@ class LLMEngine:
                               {cfg.max_num_batched_tokens})
         small = [b for b in self.buckets if b <= self.model.DECODE_FUSED_MAX_T]
         small_step = max(small) if (small and self.model.ATT_DECODE_WAVES == 8 and self.model.decode_packed) else 0
+        att = self.model.attention_items()
         self.sched = _runtime.Scheduler({
             "num_blocks": nb, "block_size": cfg.block_size, "max_num_seqs": cfg.max_num_seqs,
             "max_num_batched_tokens": cfg.max_num_batched_tokens,
             "max_prefill_tokens": cfg.max_prefill_tokens, "max_model_len": self.max_model_len,
-            "gqa_group": self.model.h_local // self.model.kv_local,
             "att_qcols": cfg.att_qcols,
             "att_wide_min_tokens": cfg.att_wide_min_tokens,
             "prefill_split_keys": cfg.prefill_split_keys,
@@ -292,12 +310,11 @@ class LLMEngine:
             "dedup_inflight_prefix": cfg.dedup_inflight_prefix,
             "embed_first": bool(cfg.embed_first),
             "token_align": cfg.token_align, "align_slack": cfg.align_slack,
-            "kv_heads": self.model.kv_local,
             "small_step_tokens": small_step,
             "small_step_part": int(cfg.small_step_part) if small_step else 0,
             "small_step_target": int(cfg.small_step_target) if small_step else 0,
             "decode_part_target": int(cfg.decode_part_target),
-            "eos_ids": list(self.tok.eos_ids)})
+            "eos_ids": list(self.tok.eos_ids), **att})
         L = self.L = self.sched.layout()
         pin = self.on_gpu
         # pipelined steps: two host-side step descriptions (one being copied / in flight,
@@ -314,8 +331,9 @@ class LLMEngine:
         # prefill_split_keys on -- one per (partial slot, KV head) for split prefill items
         # (csrc/ops/attention.hip prefill_item_wg). Without that room the kernel runs its
         # instantiation with the partition hand-off compiled out (no register spills).
-        pf_slots = L["max_items"] if cfg.prefill_split_keys > 0 else 0
-        self._att_counters = torch.zeros((L["max_seqs"] + pf_slots) * kv_local, dtype=torch.int32,
+        po, pml, tickets = self.model.attention_workspace(L["max_items"])
+        pf_slots = L["max_items"] if att.get("prefill_split_keys", cfg.prefill_split_keys) > 0 else 0
+        self._att_counters = torch.zeros((L["max_seqs"] + pf_slots) * tickets, dtype=torch.int32,
                                          device=self.device)
         self._init_views()
         V = mc.vocab_size
@@ -347,14 +365,13 @@ class LLMEngine:
         # waiting (.cpu()) for the step queued after it
         self._embed_hosts = [torch.zeros_like(self._embed_pool, device="cpu", pin_memory=self.on_gpu)
                              for _ in range(2)] if self._async else None
-        tpw = 16 // (self.model.h_local // self.model.kv_local)
+        tpw = 16 // att["gqa_group"]
         self._tpw = tpw
         self._max_parts = (self.max_model_len + ops.ATT_PART - 1) // ops.ATT_PART
-        max_items = L["max_items"]
         # attention partition partials: written and merged inside one launch -> uncached memory
-        self._part_o = ops.empty_handoff(max_items * kv_local * 16 * 128, torch.float32, self.device)
-        self._part_ml = ops.empty_handoff(max_items * kv_local * 16 * 2, torch.float32, self.device)
-        self._sample_ws = ops.sample_workspace(S, self.model.v_local, self.device) if self.on_gpu else None
+        self._part_o = ops.empty_handoff(po, torch.float32, self.device)
+        self._part_ml = ops.empty_handoff(pml, torch.float32, self.device)
+        self._sample_ws = None  # with the first sampled step (a fed step samples nothing)
         # one graph per (token bucket, top-k/top-p pass); truncating variants are
         # captured on first use, so steps without truncation pay nothing for it
         self._graphs: Dict[tuple, "torch.cuda.CUDAGraph"] = {}
@@ -404,9 +421,7 @@ class LLMEngine:
             self._health_dev.append(("custom all-reduce barrier timed out (a TP peer stalled > 5 s): "
                                      "the step's activations are partial", self._car.err))
         if self.on_gpu:
-            self._health_dev.append(("weight-streaming GEMM split-K group barrier timed out (a "
-                                     "partner workgroup never ran): the step's projections are partial",
-                                     ops.stream_workspace(self.device)[2]))
+            self._health_dev += self.model.health_words()
         self._health_host = torch.zeros(max(1, len(self._health_dev)), dtype=torch.int32, pin_memory=pin)
         self._tp_ring = None
         if self.tp.size > 1:
@@ -450,7 +465,8 @@ class LLMEngine:
         if reg.version == self._mask_version:
             return False
         packed = torch.from_numpy(reg.packed())
-        self._class_masks[: packed.shape[0]].copy_(packed.to(self.device))
+        w = min(packed.shape[1], self._mask_words)  # (a vocabulary smaller than the tokenizer's has no grammars)
+        self._class_masks[: packed.shape[0], :w].copy_(packed[:, :w].to(self.device))
         self._mask_version = reg.version
         return True
 
@@ -465,6 +481,8 @@ class LLMEngine:
                         part_size=m.part_size)
 
     def _forward_and_sample(self, bucket: int, s_b: int, ns: int, trunc: bool = False, embed: bool = False):
+        if self._sample_ws is None and self.on_gpu:  # (before graph capture: its warm-up runs come first)
+            self._sample_ws = ops.sample_workspace(self.cfg.max_num_seqs, self.model.v_local, self.device)
         meta = self._meta_for(bucket, s_b, ns)
         if self._async:  # pending tokens of rows that sampled in the previous step
             ops.patch_pending_ids(meta.input_ids[:bucket], self._sampled_dev)
@@ -472,6 +490,9 @@ class LLMEngine:
                                     embed=(self._embed_rows, self._embed_pool) if embed else None)
         tau = None
         if trunc:
+            if logits.dtype == torch.float32:  # the threshold kernel orders bf16 values
+                V = logits.shape[1]
+                logits = F.pad(logits, (0, -V % 8)).to(torch.bfloat16)[:, :V]
             # exact top-k / top-p threshold on the full vocabulary; under TP from all-reduced
             # per-shard radix histograms (engine/tp_sampling.py), not an all-gather of the logits
             if self.tp.size == 1:
@@ -590,6 +611,12 @@ class LLMEngine:
         task text across an agent's lookups is computed once)."""
         if self._err is not None:
             raise RuntimeError(f"engine failed: {self._err!r}")
+        V = self.model_cfg.vocab_size
+        if V < self.tok.vocab_size:
+            if grammar is not None:
+                raise ValueError("grammars need a model with the tokenizer's vocabulary")
+            if len(prompt_ids) and not 0 <= min(prompt_ids) <= max(prompt_ids) < V:
+                raise ValueError(f"token ids must lie in 0 .. {V - 1}")
         rid = request_id if request_id is not None else self.new_request_id()
         if seed is None:
             seed = (self.cfg.seed * 0x9E3779B1 + rid * 0x85EBCA77) & 0x7FFFFFFFFFFFFFFF
@@ -941,6 +968,53 @@ class LLMEngine:
             self._flush_deliveries()  # nothing to overlap with: deliver now
         return True
 
+    # ------------------------------------------------------------- fed steps
+    def feed_step(self, entries, residuals: Optional[list] = None) -> torch.Tensor:
+        """Run one step on tokens the caller gives and return logits instead of sampling.
+
+        entries: [(request id, tokens, wanted)]; each appends its tokens to a request (admitted at
+        its first entry), all as one batch through the scheduler, the paged cache and the model's
+        forward; `wanted` are places among the entry's tokens. Returns fp32 logits [wanted, vocab]
+        in order. release_fed() gives a request's pages back. TP = 1, beside no running engine
+        thread. `residuals`: see the model's forward."""
+        if self._async or self.tp.size > 1 or self._thread is not None:
+            raise RuntimeError("fed steps need a serial single-GPU engine without its thread")
+        V, want, at = self.model_cfg.vocab_size, [], 0
+        for _, toks, w in entries:
+            if not toks or not 0 <= min(toks) <= max(toks) < V:
+                raise ValueError(f"a fed entry needs token ids in 0 .. {V - 1}")
+            if w and not 0 <= min(w) <= max(w) < len(toks):
+                raise ValueError("a wanted place lies outside its entry")
+            want += [at + int(k) for k in w]
+            at += len(toks)
+        L = self.L
+        T = self.sched.schedule_fed(self._host_ptr, [(int(r), [int(t) for t in toks]) for r, toks, _ in entries])
+        ns = len(entries)
+        bucket = next(b for b in self.buckets if b >= T)
+        if self.on_gpu:
+            n_copy = L["block_table"] + ns * L["max_blocks"]
+            self._dev_meta[:n_copy].copy_(self._host_meta[:n_copy], non_blocking=True)
+        meta = self._meta_for(bucket, self._seq_bucket(bucket), ns)
+        meta.logit_rows = torch.tensor(want or [0], dtype=torch.int32, device=self.device)
+        kw = {} if residuals is None else {"residuals": residuals}
+        with torch.inference_mode():
+            logits = self.model.forward(meta, self.kv, bucket, max(1, len(want)), self._part_o, self._part_ml, **kw)
+            out = logits.float()[:len(want)]
+        self._health_fetch()
+        if self.on_gpu:
+            torch.cuda.current_stream().synchronize()
+        self._health_check()
+        self.sched.commit(0, 0)
+        self.stats["steps"] += 1
+        self.stats["tokens"] += T
+        return out
+
+    def release_fed(self, rid: int):
+        """End a fed request: its pages and slot are free for the next ones."""
+        if not self.sched.abort(int(rid)):
+            raise KeyError(f"no live request {rid}")
+        self.sched.drain_aborted()
+
     # ------------------------------------------------------------- pipelined steps
     def _step_pipelined(self) -> bool:
         """One turn of the pipelined loop: launch the next step if fewer than two are in
@@ -1107,7 +1181,7 @@ class LLMEngine:
             "preemptions": s.total_preemptions, "graphs": len(self._graphs), "aligned_steps": s.aligned_steps,
             "prefix_defers": s.prefix_defers,
             "spec_rows": s.spec_rows, "spec_voided": s.spec_voided,
-            "kv_cache_gb": self.kv.k.numel() * 2 * 2 / 2**30,
+            "kv_cache_gb": self.kv.nbytes() / 2**30,
             "weights_gb": self.model.weight_bytes() / 2**30,
         })
         if self.on_gpu:

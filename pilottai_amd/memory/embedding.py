@@ -107,7 +107,7 @@ class EngineEmbedder:
             # the projection on a stream of its own: on the device's default stream it would
             # queue behind the engine steps already in flight there (1-2 steps of latency)
             if self._stream is None:
-                self._stream = torch.cuda.Stream(device=self.proj.device, priority=-1)
+                self._stream = torch.cuda.Stream(device=self.proj.device)
             with torch.cuda.stream(self._stream):
                 hd = torch.from_numpy(h).to(self.proj.device)
                 return F.normalize(hd @ self.proj, dim=1).cpu().numpy()

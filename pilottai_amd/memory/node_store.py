@@ -188,7 +188,7 @@ class NodeSemanticStore:
             torch.cuda.set_device(self.index.device)
             # the round's copies and RCCL collectives are ordered behind this stream only, not
             # behind the engine's work on the default stream (a round must not wait for a step)
-            ctx = torch.cuda.stream(torch.cuda.Stream(device=self.index.device, priority=-1))
+            ctx = torch.cuda.stream(torch.cuda.Stream(device=self.index.device))
         with ctx:
             self._loop()
 

@@ -367,10 +367,9 @@ class SemanticIndex:
         if self.device.type != "cuda":
             return contextlib.nullcontext()
         if self._stream is None:
-            # high priority: a lookup pass is on an agent step's critical path, and at
-            # normal priority its workgroups wait behind the engine's (10M rows: 36 ms
-            # per pass beside a 64-worker engine vs ~4 ms alone)
-            self._stream = torch.cuda.Stream(device=self.device, priority=-1)
+            # its own stream, at the default priority (work on streams of different priorities
+            # has hung): a lookup pass shares the device with the engine's steps
+            self._stream = torch.cuda.Stream(device=self.device)
         st = contextlib.ExitStack()
         st.enter_context(torch.cuda.device(self.device))
         st.enter_context(torch.cuda.stream(self._stream))

@@ -1,0 +1,468 @@
+"""Bozupel: a decoder with windowed latent attention, token-table experts, sandwich norms and a
+looped stack, on the engine's paged cache, scheduler and packed projections.
+
+    x = E[token]
+    per layer run:   x += norm(attn(norm(x)));   x += norm(experts(norm(x)))
+    logits = head . norm(x) * logit_scale
+
+A loop runs layers start .. stop-1 `times` times with the same weights; before each repeated pass
+E[token] is added to x. Every pass has its own cache pool (models/cache.py LatentKVCache).
+
+The residual stream, norms, rotations, scores and softmax are fp32; activations and matrix products
+are the model's dtype (bf16, or fp32 throughout).
+
+One step of T tokens (decode rows and prompt portions alike):
+
+  once      table_route       every expert layer's rows sorted by expert, from the token ids
+            residual_norm     x = E[id], norm -> h
+  per run   linear            [query latent | kv latent | rotated key] = W_down h, one projection
+            latent_cache      both latent norms, key rotation, paged cache row
+            linear            q = W_uq c_q
+            head_gemm         q~ = W_uk^T q per head; latent_qrot: the rotated part beside it
+            latent_attention  windowed paged attention in the latent space
+            head_gemm, linear W_uv per head, W_o
+            residual_norm     x += norm(y), next norm -> h
+            expert_gemm x 2   clamped gated experts, rows sorted; one partial output per choice
+            residual_norm     x += norm(sum of partials / top) (+ E[id] into a repeated pass), next norm -> h
+
+Weights are stored once, packed for the kernels, with every dimension padded by zero rows and columns
+to whole MFMA tiles, so any sizes run on the same kernels.
+"""
+from __future__ import annotations
+
+import os
+from dataclasses import dataclass, field
+from typing import Dict, List, Optional, Tuple
+
+import torch
+import torch.nn.functional as F
+
+from pilottai_amd import ops
+from pilottai_amd.models.cache import LatentKVCache, StepMeta
+from pilottai_amd.ops import reference as ref
+from pilottai_amd.ops.latent import latent_pad, pad_to
+from pilottai_amd.parallel.comm import TPGroup
+
+GLU_ALPHA = 1.702  # the gated unit g * sigmoid(alpha g) * (u + bias)
+GLU_BIAS = 1.0
+
+
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    heads: int
+    dim: int          # unrotated query / key dimensions per head
+    rot_dim: int      # rotated dimensions per head (one key part shared by all heads)
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot_base: float
+    rot_dims: int     # rotated dimensions of rot_dim (rotate-half pairs)
+    window: int = 0   # keys a position sees, itself included; 0: all before it
+
+
+@dataclass(frozen=True)
+class TableExpertsSpec:
+    experts: int
+    top: int
+    ff: int
+    limit: float
+
+
+@dataclass(frozen=True)
+class BozupelLayer:
+    mixer: LatentAttentionSpec
+    mlp: Optional[TableExpertsSpec]
+
+
+@dataclass
+class BozupelConfig:
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: List[BozupelLayer]
+    eps: float = 1e-5
+    logit_scale: float = 1.0
+    loop: Optional[Tuple[int, int, int]] = None  # (start, stop, times)
+    max_position: int = 1 << 20
+    init_std: float = 0.02
+    extra: dict = field(default_factory=dict, repr=False)
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def runs(self) -> List[Tuple[int, bool]]:
+        """(layer, whether a repeated pass starts here) for every layer run of a step, in order."""
+        n = len(self.layers)
+        start, stop, times = self.loop or (0, 0, 1)
+        out = []
+        for again in range(times):
+            lo = start if again else 0
+            out += [(i, again > 0 and i == start) for i in range(lo, stop)]
+        return out + [(i, False) for i in range(stop, n)]
+
+    @classmethod
+    def from_dict(cls, d: dict, name: str = "bozupel") -> "BozupelConfig":
+        layers = []
+        for i, L in enumerate(d["layers"]):
+            if L.get("type") != "latent_attention":
+                raise ValueError(f"layer {i}: unknown mixer {L.get('type')!r}")
+            m = L["mixer"]
+            mixer = LatentAttentionSpec(
+                heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]), scale=float(m["scale"]),
+                rot_base=float(m["rot"]["base"]), rot_dims=int(m["rot"].get("dims", m["rot_dim"])),
+                window=int((m.get("mask") or {}).get("size") or 0))
+            if mixer.rot_dims > mixer.rot_dim or mixer.rot_dims % 2:
+                raise ValueError(f"layer {i}: {mixer.rot_dims} rotated of {mixer.rot_dim} dimensions")
+            p, mlp = L.get("mlp"), None
+            if p is not None:
+                if p.get("kind") != "moe":
+                    raise ValueError(f"layer {i}: unknown feed-forward {p.get('kind')!r}")
+                mlp = TableExpertsSpec(experts=int(p["router"]["experts"]), top=int(p["router"]["top"]),
+                                       ff=int(p["expert"]["ff"]), limit=float(p["expert"]["limit"]))
+            layers.append(BozupelLayer(mixer, mlp))
+        loop = d.get("loop")
+        if loop:
+            loop = (int(loop["start"]), int(loop["stop"]), int(loop["times"]))
+            if not (0 <= loop[0] < loop[1] <= len(layers) and loop[2] >= 1):
+                raise ValueError(f"loop {loop} does not fit {len(layers)} layers")
+        return cls(name=name, vocab_size=int(d["vocab"]), hidden_size=int(d["width"]), layers=layers,
+                   eps=float(d["norm"]["eps"]), logit_scale=float(d.get("logit_scale", 1.0)), loop=loop or None)
+
+    def num_params(self) -> int:
+        d, n = self.hidden_size, 2 * self.vocab_size * self.hidden_size + self.hidden_size
+        for L in self.layers:
+            m = L.mixer
+            n += d * (m.q_rank + m.kv_rank + m.rot_dim) + m.heads * (m.dim + m.rot_dim) * m.q_rank
+            n += m.heads * (m.dim + m.vdim) * m.kv_rank + m.heads * m.vdim * d
+            if L.mlp:
+                n += 3 * L.mlp.experts * L.mlp.ff * d
+        return n
+
+
+def _uniform(name: str, n_layers: int, vocab: int, width: int, mixer: LatentAttentionSpec, mlp: TableExpertsSpec,
+             loop=None, logit_scale: float = 1.0) -> BozupelConfig:
+    return BozupelConfig(name=name, vocab_size=vocab, hidden_size=width,
+                         layers=[BozupelLayer(mixer, mlp) for _ in range(n_layers)], loop=loop, logit_scale=logit_scale)
+
+
+PRESETS: Dict[str, BozupelConfig] = {
+    # a small shape for tests of the engine around the model (the tokenizer's vocabulary)
+    "bozupel-tiny": _uniform("bozupel-tiny", 2, 128256, 192,
+                             LatentAttentionSpec(heads=4, dim=48, rot_dim=32, vdim=40, q_rank=64, kv_rank=128,
+                                                 scale=0.11, rot_base=10000.0, rot_dims=32, window=200),
+                             TableExpertsSpec(experts=6, top=2, ff=80, limit=4.0), loop=(0, 1, 2)),
+    # layers of a real model's size (bench.py --bozupel), at two widths
+    "bozupel-base": _uniform("bozupel-base", 8, 128256, 2048,
+                             LatentAttentionSpec(heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512,
+                                                 scale=192 ** -0.5, rot_base=10000.0, rot_dims=64, window=4096),
+                             TableExpertsSpec(experts=64, top=6, ff=1408, limit=7.0)),
+    "bozupel-wide": _uniform("bozupel-wide", 4, 128256, 4096,
+                             LatentAttentionSpec(heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512,
+                                                 scale=192 ** -0.5, rot_base=10000.0, rot_dims=64, window=4096),
+                             TableExpertsSpec(experts=64, top=6, ff=2048, limit=7.0)),
+}
+
+
+class _Linear:
+    """y = x W^T with W [N, K] padded to [128 n, 64 k] by zeros: the packed projections in bf16
+    (decode kernel up to 64 rows, prefill kernel above), the library's fp32 GEMM in fp32."""
+
+    def __init__(self, w: torch.Tensor, dtype, device):
+        N, K = w.shape
+        full = torch.zeros(pad_to(N, 128), pad_to(K, 64), dtype=dtype, device=device)
+        full[:N, :K] = w.to(device=device, dtype=dtype)
+        self.N, self.K = full.shape
+        self.w = ops.pack_decode_weight(full) if dtype == torch.bfloat16 else full
+
+    def __call__(self, x: torch.Tensor) -> torch.Tensor:
+        if self.w.dim() == 2:
+            return F.linear(x, self.w)
+        if x.shape[0] <= 64:
+            return ops.decode_gemm(x, self.w)
+        return ops.prefill_gemm(x, self.w)
+
+
+class LatentAttention:
+    """Latent attention over the paged latent cache, queries absorbed into the latent space."""
+
+    def __init__(self, spec: LatentAttentionSpec, t: Dict[str, torch.Tensor], eps: float, dtype, device, cos_sin):
+        m = self.spec = spec
+        self.eps, self.dtype, self.device, self.cos_sin = eps, dtype, device, cos_sin
+        H, n, r, vd, R = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank
+        self.np, self.rp, self.vp = pad_to(n, 32), pad_to(r, 32), pad_to(vd, 16)
+        self.Rp = latent_pad(R)
+        self.D = self.Rp + self.rp
+        self.down = _Linear(torch.cat([t["dq"], t["dkv"]], 0), dtype, device)
+        self.w_q = t["dq.norm"].float().to(device)
+        self.w_c = t["dkv.norm"].float().to(device)
+        q = t["uq"].view(H, n + r, m.q_rank)
+        uq = torch.zeros(H, self.np + self.rp, m.q_rank, dtype=q.dtype, device=q.device)
+        uq[:, :n], uq[:, self.np:self.np + r] = q[:, :n], q[:, n:]
+        self.uq = _Linear(uq.view(-1, m.q_rank), dtype, device)
+        uk = torch.zeros(H, self.Rp, self.np, dtype=dtype, device=device)
+        uk[:, :R, :n] = t["uk"].to(device).view(H, n, R).transpose(1, 2)
+        self.uk = ops.pack_groups(uk, dtype)
+        uv = torch.zeros(H, self.vp, self.Rp, dtype=dtype, device=device)
+        uv[:, :vd, :R] = t["uv"].to(device).view(H, vd, R)
+        self.uv = ops.pack_groups(uv, dtype)
+        d = t["o"].shape[0]
+        o = torch.zeros(d, H, self.vp, dtype=t["o"].dtype, device=t["o"].device)
+        o[:, :, :vd] = t["o"].view(d, H, vd)
+        self.o = _Linear(o.view(d, -1), dtype, device)
+
+    def tensors(self):
+        return [self.down.w, self.uq.w, self.uk, self.uv, self.o.w]
+
+    def __call__(self, h, meta: StepMeta, pages, part_o, part_ml, dec_tokens: int, tile_tokens: int) -> torch.Tensor:
+        m, T, H = self.spec, h.shape[0], self.spec.heads
+        new = lambda *s: torch.empty(*s, dtype=self.dtype, device=self.device)  # noqa: E731
+        a = self.down(h)
+        cq = new(T, self.uq.K)
+        ops.latent_cache(a, m.q_rank, m.kv_rank, m.rot_dim, self.w_q, self.w_c, cq, pages, self.Rp, meta.positions,
+                         meta.slots, self.cos_sin, self.eps)
+        q = self.uq(cq)
+        qa = new(T, H, self.D)
+        ops.head_gemm(q, self.np + self.rp, self.uk, qa.view(T, -1), self.D)
+        ops.latent_qrot(q, self.np + self.rp, self.np, m.rot_dim, qa, self.Rp, meta.positions, self.cos_sin)
+        oc = new(T, H, self.Rp)
+        ops.latent_attention(oc, part_o, part_ml, qa, pages, meta.items, meta.n_items, meta.att_counters, meta.q_start,
+                             meta.q_len, meta.ctx_len, meta.block_table, m.scale, m.window, dec_tokens, tile_tokens,
+                             num_seqs=meta.num_seqs)
+        v = new(T, self.o.K)
+        if self.o.K > H * self.vp:
+            v[:, H * self.vp:] = 0
+        ops.head_gemm(oc.view(T, -1), self.Rp, self.uv, v, self.vp)
+        return self.o(v)
+
+
+class TableExperts:
+    """Experts chosen by a token-id table, each a clamped gated unit; returns one partial output
+    per (token, choice), [T * top, >= width], to be summed and divided by top."""
+
+    def __init__(self, spec: TableExpertsSpec, t: Dict[str, torch.Tensor], width: int, dtype, device):
+        self.spec, self.dtype, self.device = spec, dtype, device
+        E, f, d = spec.experts, spec.ff, width
+        fp, dk, dn = pad_to(f, 32), pad_to(d, 32), pad_to(d, 16)
+        self.fp, self.dn = fp, dn
+        w13, w2 = [], []
+        for e in range(E):
+            g = torch.zeros(2, 1, fp, dk, dtype=dtype, device=device)
+            g[0, 0, :f, :d], g[1, 0, :f, :d] = t[f"e{e}.gate"].to(device), t[f"e{e}.up"].to(device)
+            w13.append(ops.pack_groups(ops.interleave_gate_up(g[0], g[1]), dtype))
+            w = torch.zeros(1, dn, fp, dtype=dtype, device=device)
+            w[0, :d, :f] = t[f"e{e}.down"].to(device)
+            w2.append(ops.pack_groups(w, dtype))
+        self.w13, self.w2 = torch.cat(w13), torch.cat(w2)
+
+    def tensors(self):
+        return [self.w13, self.w2]
+
+    def __call__(self, h, T: int, route) -> torch.Tensor:
+        order, tiles, n_tiles, tm = route
+        s, rows = self.spec, T * self.spec.top
+        act = torch.empty(rows, self.fp, dtype=self.dtype, device=self.device)
+        ops.expert_gemm(h, self.w13, act, tiles, n_tiles, order, rows, x_div=s.top, out_order=False, tm=tm,
+                        glu=(s.limit, GLU_ALPHA, GLU_BIAS))
+        y = torch.empty(rows, self.dn, dtype=self.dtype, device=self.device)
+        return ops.expert_gemm(act, self.w2, y, tiles, n_tiles, order, rows, x_div=0, out_order=True, tm=tm)
+
+
+class BozupelModel:
+    # the engine's decode-sized steps (EngineConfig attention settings of the Llama kernels do not apply)
+    DECODE_FUSED_MAX_T = 16
+    MID_MAX_T = 256
+    PREFILL_MAX_T = 1 << 30
+    ATT_DECODE_WAVES = 4
+    PF_MIDRANGE = frozenset()
+    decode_packed = True
+
+    def __init__(self, cfg: BozupelConfig, device, dtype=torch.bfloat16, tp: Optional[TPGroup] = None, seed: int = 0,
+                 weights_path: Optional[str] = None, max_len: int = 8192, **_):
+        self.cfg, self.device, self.dtype = cfg, torch.device(device), dtype
+        self.tp = tp or TPGroup.single()
+        if self.tp.size > 1:
+            raise ValueError("Bozupel models run on one GPU: tensor parallelism is not implemented for them")
+        if dtype not in (torch.bfloat16, torch.float32):
+            raise ValueError(f"unsupported dtype {dtype}")
+        self.v_local, self.vocab_offset = cfg.vocab_size, 0
+        self.max_len = int(max_len)
+        self.runs = cfg.runs()
+        heads = max(L.mixer.heads for L in cfg.layers)
+        group = min(heads, 16)
+        self.dec_tokens, self.tile_tokens = 16 // group, 128 // group  # tokens of an attention work item
+        self._group = group
+        get = self._checkpoint(weights_path) if weights_path else self._random(seed)
+        eps, d = cfg.eps, cfg.hidden_size
+        rot: Dict[tuple, torch.Tensor] = {}
+        f32 = lambda name: get(name, (d,)).float().to(self.device)  # noqa: E731
+        self.embed = get("embed", (cfg.vocab_size, d)).to(self.device, dtype).contiguous()
+        self.layers = []
+        tables = []
+        for i, L in enumerate(cfg.layers):
+            m, p, pre = L.mixer, L.mlp, f"l{i}."
+            key = (m.rot_dims, m.rot_base)
+            if key not in rot:
+                rot[key] = ref.rope_cos_sin(self.max_len, m.rot_dims, m.rot_base).to(self.device)
+            shapes = {"dq": (m.q_rank, d), "dq.norm": (m.q_rank,), "uq": (m.heads * (m.dim + m.rot_dim), m.q_rank),
+                      "dkv": (m.kv_rank + m.rot_dim, d), "dkv.norm": (m.kv_rank,), "uk": (m.heads * m.dim, m.kv_rank),
+                      "uv": (m.heads * m.vdim, m.kv_rank), "o": (d, m.heads * m.vdim)}
+            layer = {"norm1": f32(pre + "norm1"), "norm1b": f32(pre + "norm1b"),
+                     "attn": LatentAttention(m, {k: get(f"{pre}mix.{k}", s) for k, s in shapes.items()}, eps, dtype,
+                                             self.device, rot[key]), "mlp": None}
+            if p is not None:
+                layer["norm2"], layer["norm2b"] = f32(pre + "norm2"), f32(pre + "norm2b")
+                w = {}
+                for e in range(p.experts):
+                    for k, s in (("gate", (p.ff, d)), ("up", (p.ff, d)), ("down", (d, p.ff))):
+                        w[f"e{e}.{k}"] = get(f"{pre}mlp.e{e}.{k}", s)
+                layer["mlp"] = TableExperts(p, w, d, dtype, self.device)
+                layer["route"] = len(tables)
+                tables.append(get(f"{pre}mlp.table", (cfg.vocab_size, p.top)).to(torch.int32))
+            self.layers.append(layer)
+        for i, t in enumerate(tables):
+            E = [L.mlp for L in cfg.layers if L.mlp][i].experts
+            if int(t.min()) < 0 or int(t.max()) >= E:
+                raise ValueError(f"expert table {i} names experts outside 0 .. {E - 1}")
+        self.tables = torch.cat([t.reshape(-1) for t in tables]).to(self.device) if tables else None
+        self.norm = f32("final.norm")
+        self.norm_scaled = self.norm * cfg.logit_scale  # logits = head . norm(x) * logit_scale
+        self.head = _Linear(get("head", (cfg.vocab_size, d)), dtype, self.device)
+        self._route_desc: Dict[tuple, tuple] = {}
+        if self.device.type == "cuda" and dtype == torch.bfloat16:  # before any graph capture
+            ops.decode_workspace(self.device)
+            ops.prefill_workspace(self.device)
+
+    # -- weights -----------------------------------------------------------------
+    @staticmethod
+    def _checkpoint(path: str):
+        from safetensors import safe_open
+
+        where = {}
+        for f in sorted(os.listdir(path)):
+            if f.endswith(".safetensors"):
+                fh = safe_open(os.path.join(path, f), framework="pt")
+                where.update({k: fh for k in fh.keys()})
+
+        def get(name, shape):
+            if name not in where:
+                raise ValueError(f"{path}: tensor {name!r} is missing")
+            t = where[name].get_tensor(name)
+            if tuple(t.shape) != tuple(shape):
+                raise ValueError(f"{path}: {name} has shape {tuple(t.shape)}, the configuration gives {tuple(shape)}")
+            return t
+        return get
+
+    def _random(self, seed: int):
+        cfg, dev = self.cfg, self.device
+        g = torch.Generator(device=dev).manual_seed(seed)
+        tops = {f"l{i}.mlp.table": L.mlp.experts for i, L in enumerate(cfg.layers) if L.mlp}
+
+        def get(name, shape):
+            if name in tops:  # `top` different experts for every token
+                a = torch.randint(0, tops[name], (shape[0], 1), device=dev, generator=g)
+                step = torch.arange(shape[1], device=dev)[None, :]
+                return (a + step) % tops[name]
+            if "norm" in name:
+                return torch.ones(shape, dtype=torch.bfloat16, device=dev)
+            return torch.empty(shape, dtype=torch.bfloat16, device=dev).normal_(0.0, cfg.init_std, generator=g)
+        return get
+
+    def weight_bytes(self) -> int:
+        ts = [self.embed, self.head.w]
+        for L in self.layers:
+            ts += L["attn"].tensors() + (L["mlp"].tensors() if L["mlp"] else [])
+        return sum(t.numel() * t.element_size() for t in ts)
+
+    # -- what the engine asks of every model ----------------------------------------
+    def _widths(self) -> List[int]:
+        return [self.layers[i]["attn"].D for i, _ in self.runs]
+
+    def cache_bytes_per_block(self, block_size: int) -> int:
+        return LatentKVCache.bytes_per_block(self._widths(), self.embed.element_size(), block_size)
+
+    def make_cache(self, num_blocks: int, block_size: int) -> LatentKVCache:
+        return LatentKVCache(self._widths(), num_blocks, self.device, self.dtype, block_size)
+
+    def attention_items(self) -> dict:
+        windows = [L.mixer.window for L in self.cfg.layers]
+        return {"gqa_group": self._group, "kv_heads": 1, "att_qcols": 128, "att_narrow_qcols": 128,
+                "prefill_split_keys": 0, "att_max_keys": max(windows) if all(windows) else 0}
+
+    def attention_workspace(self, max_items: int) -> tuple:
+        """(partial outputs, partial (max, sum) pairs) in floats, and tickets per sequence."""
+        nb = [(self.dec_tokens * L["attn"].spec.heads + 15) // 16 for L in self.layers]
+        o = max(b * 16 * L["attn"].Rp for b, L in zip(nb, self.layers))
+        return max_items * o, max_items * max(nb) * 32, max(nb)
+
+    def health_words(self) -> list:
+        return []
+
+    # -- forward -----------------------------------------------------------------
+    def _route(self, meta: StepMeta, T: int):
+        """Rows of every expert layer sorted by expert: [(order, tiles, n_tiles, rows per tile)]."""
+        mlps = [L.mlp for L in self.cfg.layers if L.mlp]
+        if not mlps:
+            return []
+        dev = self.device
+        if T not in self._route_desc:  # (before graph capture: the capture's warm-up runs come first)
+            big = self.dtype == torch.bfloat16 and T * max(p.top / p.experts for p in mlps) > 32
+            tm, rows, tab, o, t = 64 if big else 16, [], 0, 0, 0
+            for p in mlps:
+                n = T * p.top
+                cap = n // (64 if big else 16) + min(p.experts, n)
+                rows.append([tab, self.cfg.vocab_size, p.top, p.experts, o, t, cap, 0])
+                tab, o, t = tab + self.cfg.vocab_size * p.top, o + n, t + cap
+            host = torch.tensor(rows, dtype=torch.int32)
+            self._route_desc[T] = (host, host.to(dev), o, t, tm)
+        host, desc, no, nt, tm = self._route_desc[T]
+        order = torch.empty(no, dtype=torch.int32, device=dev)
+        tiles = torch.empty(nt, 4, dtype=torch.int32, device=dev)
+        n_tiles = torch.empty(len(mlps), dtype=torch.int32, device=dev)
+        ops.table_route(self.tables, desc, host, meta.input_ids, meta.slots, T, tm, order, tiles, n_tiles)
+        out = []
+        for i, (_, _, top, _, o, t, cap, _) in enumerate(host.tolist()):
+            out.append((order[o:o + T * top], tiles[t:t + cap], n_tiles[i:i + 1], tm))
+        return out
+
+    def forward(self, meta: StepMeta, kv: LatentKVCache, num_tokens: int, num_logit_rows: int, part_o: torch.Tensor,
+                part_ml: torch.Tensor, embed=None, residuals: Optional[list] = None) -> torch.Tensor:
+        """Logits [num_logit_rows, vocab] of rows meta.logit_rows. embed = (rows, pool): see
+        LlamaModel.forward. `residuals` (a list) collects the residual stream after every layer run."""
+        cfg, T, dev = self.cfg, num_tokens, self.device
+        eps, d = cfg.eps, cfg.hidden_size
+        ids = meta.input_ids[:T]
+        ldh = pad_to(d, 64)
+        new_h = lambda n=T: torch.empty(n, ldh, dtype=self.dtype, device=dev)  # noqa: E731
+        rows = meta.logit_rows[:num_logit_rows]
+        routes = self._route(meta, T)
+        resid = torch.empty(T, d, dtype=torch.float32, device=dev)
+        h = ops.residual_norm(resid, eps, emb=self.embed, ids=ids, w_next=self.layers[self.runs[0][0]]["norm1"], out=new_h())
+        for j, (i, _) in enumerate(self.runs):
+            L = self.layers[i]
+            y = L["attn"](h, meta, kv.pages[j], part_o, part_ml, self.dec_tokens, self.tile_tokens)
+            post, k = L["norm1b"], 1
+            if L["mlp"] is not None:
+                h = ops.residual_norm(resid, eps, y=y, w_post=post, w_next=L["norm2"], out=new_h())
+                y = L["mlp"](h, T, routes[L["route"]])
+                post, k = L["norm2b"], L["mlp"].spec.top
+            step = dict(y=y, partials=k, y_scale=1.0 / k, w_post=post)
+            if residuals is not None:
+                after = resid.clone()
+                ops.residual_norm(after, eps, **step)
+                residuals.append(after)
+            if j + 1 < len(self.runs):
+                nxt, again = self.runs[j + 1]
+                if again:
+                    step.update(emb=self.embed, ids=ids, emb_add=True)
+                h = ops.residual_norm(resid, eps, w_next=self.layers[nxt]["norm1"], out=new_h(), **step)
+        if embed is not None:
+            hn = ops.residual_norm(resid, eps, w_next=self.norm, out=new_h(), **step)
+            pool_rows, pool = embed
+            pool[-1].zero_()  # the row of tokens that no embedding request owns
+            pool.index_add_(0, pool_rows[:T].long(), hn[:, :d].float())
+            step = {}
+        hs = ops.residual_norm(resid, eps, w_next=self.norm_scaled, out=new_h(num_logit_rows), rows=rows, **step)
+        return self.head(hs)[:, :cfg.vocab_size]

@@ -1,0 +1,73 @@
+"""Paged cache pools and the per-step metadata every model's forward reads.
+
+A block id names the same 16-token page in every pool of a model, so the scheduler and its block
+manager (csrc/runtime) know nothing of what a page holds:
+
+  KVCache        per-head keys and values (Llama)
+  LatentKVCache  one latent row per token for all heads (latent attention), one pool per layer RUN:
+                 a layer that a looped stack runs several times has a pool for each pass, and
+                 layers of different widths have pools of their own widths
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+from typing import List, Optional, Sequence
+
+import torch
+
+
+@dataclass
+class StepMeta:
+    """Device views of one step's metadata (layout from the native scheduler)."""
+    input_ids: torch.Tensor
+    positions: torch.Tensor
+    slots: torch.Tensor
+    q_start: torch.Tensor
+    q_len: torch.Tensor
+    ctx_len: torch.Tensor
+    block_table: torch.Tensor
+    items: torch.Tensor
+    n_items: torch.Tensor
+    att_counters: torch.Tensor  # persistent zeroed workspace (partition tickets), not step data
+    logit_rows: torch.Tensor
+    num_seqs: int = 0  # host-side count, used only by the CPU reference path
+    part_size: Optional[torch.Tensor] = None  # device int[1]: decode partition size of the step
+
+
+class KVCache:
+    """Per-layer paged pools (bf16): K [NB, KV, 128/8, 16, 8] fragment-major,
+    V^T [NB, KV, 128, 16] (layouts: csrc/ops/rope_cache.hip)."""
+
+    def __init__(self, num_layers: int, num_blocks: int, kv_heads: int, device, dtype=torch.bfloat16,
+                 block_size: int = 16):
+        self.num_blocks = num_blocks
+        self.block_size = block_size
+        self.k = torch.zeros(num_layers, num_blocks, kv_heads, 16, block_size, 8, dtype=dtype, device=device)
+        self.v = torch.zeros(num_layers, num_blocks, kv_heads, 128, block_size, dtype=dtype, device=device)
+
+    def nbytes(self) -> int:
+        return self.k.numel() * self.k.element_size() + self.v.numel() * self.v.element_size()
+
+    @staticmethod
+    def bytes_per_block(num_layers: int, kv_heads: int, block_size: int = 16) -> int:
+        return 2 * num_layers * kv_heads * block_size * 128 * 2
+
+
+class LatentKVCache:
+    """Pools [blocks, D/8, 16, 8] of the given widths D (one per layer run): fragment-major rows
+    (csrc/ops/latent_cache.hip)."""
+
+    def __init__(self, widths: Sequence[int], num_blocks: int, device, dtype=torch.bfloat16, block_size: int = 16):
+        if block_size != 16:
+            raise ValueError("latent pages hold 16 tokens")
+        self.num_blocks = num_blocks
+        self.block_size = block_size
+        self.pages: List[torch.Tensor] = [
+            torch.zeros(num_blocks, d // 8, block_size, 8, dtype=dtype, device=device) for d in widths]
+
+    @staticmethod
+    def bytes_per_block(widths: Sequence[int], itemsize: int, block_size: int = 16) -> int:
+        return sum(widths) * block_size * itemsize
+
+    def nbytes(self) -> int:
+        return sum(p.numel() * p.element_size() for p in self.pages)

@@ -33,6 +33,7 @@ import torch
 import torch.nn.functional as F
 
 from pilottai_amd import ops
+from pilottai_amd.models.cache import KVCache, StepMeta
 from pilottai_amd.ops import reference as ref
 from pilottai_amd.parallel.comm import TPGroup
 
@@ -93,47 +94,11 @@ PRESETS: Dict[str, LlamaConfig] = {
 }
 
 
-def get_config(name_or_cfg) -> LlamaConfig:
-    if isinstance(name_or_cfg, LlamaConfig):
-        return name_or_cfg
-    key = str(name_or_cfg).lower()
-    if key not in PRESETS:
-        raise ValueError(f"unknown model {name_or_cfg!r}; known: {sorted(PRESETS)}")
-    return PRESETS[key]
+def get_config(name_or_cfg):
+    """The configuration of a preset's name, a checkpoint folder or a configuration (models/registry.py)."""
+    from pilottai_amd.models import registry
 
-
-@dataclass
-class StepMeta:
-    """Device views of one step's metadata (layout from the native scheduler)."""
-    input_ids: torch.Tensor
-    positions: torch.Tensor
-    slots: torch.Tensor
-    q_start: torch.Tensor
-    q_len: torch.Tensor
-    ctx_len: torch.Tensor
-    block_table: torch.Tensor
-    items: torch.Tensor
-    n_items: torch.Tensor
-    att_counters: torch.Tensor  # persistent zeroed workspace (partition tickets), not step data
-    logit_rows: torch.Tensor
-    num_seqs: int = 0  # host-side count, used only by the CPU reference path
-    part_size: Optional[torch.Tensor] = None  # device int[1]: decode partition size of the step
-
-
-class KVCache:
-    """Per-layer paged pools (bf16): K [NB, KV, 128/8, 16, 8] fragment-major,
-    V^T [NB, KV, 128, 16] (layouts: csrc/ops/rope_cache.hip)."""
-
-    def __init__(self, num_layers: int, num_blocks: int, kv_heads: int, device, dtype=torch.bfloat16,
-                 block_size: int = 16):
-        self.num_blocks = num_blocks
-        self.block_size = block_size
-        self.k = torch.zeros(num_layers, num_blocks, kv_heads, 16, block_size, 8, dtype=dtype, device=device)
-        self.v = torch.zeros(num_layers, num_blocks, kv_heads, 128, block_size, dtype=dtype, device=device)
-
-    @staticmethod
-    def bytes_per_block(num_layers: int, kv_heads: int, block_size: int = 16) -> int:
-        return 2 * num_layers * kv_heads * block_size * 128 * 2
+    return registry.get_config(name_or_cfg)
 
 
 DENSE_KINDS = ("wqkv", "wo", "w13", "w2")
@@ -353,6 +318,26 @@ class LlamaModel:
 
     def _dense_needed(self, T: int) -> bool:
         return not self.decode_packed or T > max(self.MID_MAX_T, self.PREFILL_MAX_T)
+
+    # -- what the engine asks of every model ----------------------------------------
+    def cache_bytes_per_block(self, block_size: int) -> int:
+        return KVCache.bytes_per_block(self.cfg.num_layers, self.kv_local, block_size)
+
+    def make_cache(self, num_blocks: int, block_size: int) -> KVCache:
+        return KVCache(self.cfg.num_layers, num_blocks, self.kv_local, self.device, block_size=block_size)
+
+    def attention_items(self) -> dict:
+        """Scheduler settings for the work items of this model's attention kernel."""
+        return {"gqa_group": self.h_local // self.kv_local, "kv_heads": self.kv_local}
+
+    def attention_workspace(self, max_items: int) -> tuple:
+        """(partial outputs, partial (max, sum) pairs) in floats, and tickets per sequence."""
+        return max_items * self.kv_local * 16 * 128, max_items * self.kv_local * 16 * 2, self.kv_local
+
+    def health_words(self) -> list:
+        """(message, device int32) pairs that the engine checks after every step."""
+        return [("weight-streaming GEMM split-K group barrier timed out (a partner workgroup never ran): "
+                 "the step's projections are partial", ops.stream_workspace(self.device)[2])]
 
     # -- weights -----------------------------------------------------------------
     def _init_random(self, seed: int):

@@ -47,6 +47,26 @@ def require_native():
     return mod
 
 
+_LATENT = None
+
+
+def require_latent():
+    """The _latent module (latent attention, expert tables, fp32 residual; csrc/ops/bindings_latent.cpp)."""
+    global _LATENT
+    if _LATENT is None:
+        try:
+            _LATENT = importlib.import_module("pilottai_amd._latent")
+        except ImportError as e:
+            raise RuntimeError(f"pilottai_amd latent kernels (_latent.so) are not available: {e!r}. Build them with "
+                               "`python -m pilottai_amd._build` (hipcc --offload-arch=gfx950).") from e
+    return _LATENT
+
+
+def _packed_module():
+    """The module with the packed-weight projections: _C, or _latent where only that one is built."""
+    return _load() or require_latent()
+
+
 def native_module_path() -> Optional[str]:
     mod = _load()
     return getattr(mod, "__file__", None) if mod is not None else None
@@ -69,7 +89,7 @@ def empty_handoff(numel: int, dtype=torch.float32, device=None) -> torch.Tensor:
     device = torch.device(device) if device is not None else torch.device("cpu")
     if device.type == "cuda":
         idx = device.index if device.index is not None else torch.cuda.current_device()
-        return require_native().empty_uncached(int(numel), dtype, int(idx))
+        return _packed_module().empty_uncached(int(numel), dtype, int(idx))
     return torch.zeros(int(numel), dtype=dtype, device=device)
 
 
@@ -383,7 +403,7 @@ def decode_gemm(x: torch.Tensor, wp: torch.Tensor, epi: str = "plain", norm: boo
         out = torch.empty(M, NO, dtype=x.dtype, device=x.device)
     if _on_gpu(x):
         ws, cnt = decode_workspace(x.device)
-        if not require_native().decode_gemm(out, x, wp, resid, code, bool(norm), float(eps), int(nt), int(waves),
+        if not _packed_module().decode_gemm(out, x, wp, resid, code, bool(norm), float(eps), int(nt), int(waves),
                                             int(splits), ws, cnt):
             raise ValueError(f"decode_gemm does not handle M={M} N={N} K={K} epi={epi} nt={nt} waves={waves}")
         return out
@@ -655,7 +675,7 @@ def prefill_gemm(x: torch.Tensor, wp: torch.Tensor, epi: str = "plain", resid: O
         ss_in = row_sumsq(x)
     if _on_gpu(x):
         ws, cnt = prefill_workspace(x.device)
-        if not require_native().prefill_gemm(out, x, wp, resid, ws, cnt, code, ss_in if norm else None, ss_out,
+        if not _packed_module().prefill_gemm(out, x, wp, resid, ws, cnt, code, ss_in if norm else None, ss_out,
                                               ss_zero, float(eps), int(full), int(splits), int(bn), int(variant)):
             raise ValueError(f"prefill_gemm does not handle M={M} N={N} K={K} epi={epi} full={full} S={splits}")
         return out

@@ -297,3 +297,115 @@ def pack_mask(allowed) -> torch.Tensor:
     if pad:
         a = np.concatenate([a, np.zeros(pad, dtype=bool)])
     return torch.from_numpy(np.packbits(a, bitorder="little").view(np.int32).copy())
+
+
+# ---------------------------------------------------------------------------
+# fp32 residual stream, latent attention, grouped projections (ops/latent.py)
+# ---------------------------------------------------------------------------
+
+
+def _norm32(x: torch.Tensor, eps: float) -> torch.Tensor:
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def residual_norm(resid, eps, y, partials, y_scale, w_post, emb, ids, emb_add, w_next, out, rows):
+    T, D = resid.shape
+    sel = torch.arange(T) if rows is None else rows.long()
+    r = resid[sel]
+    if y is not None:
+        d = y[:, :D].float().view(T, partials, D).sum(1)[sel] * y_scale
+        r = r + (_norm32(d, eps) * w_post if w_post is not None else d)
+    if emb is not None:
+        e = emb[ids[:T].long()[sel].clamp(0, emb.shape[0] - 1)].float()
+        r = r + e if emb_add else e  # (set: before any y)
+    if rows is None:
+        resid.copy_(r)
+    if out is not None:
+        out[:len(sel), :D] = (_norm32(r, eps) * w_next).to(out.dtype)
+        out[:len(sel), D:] = 0
+    return out
+
+
+def _rotate_part(x: torch.Tensor, positions: torch.Tensor, cos_sin: torch.Tensor) -> torch.Tensor:
+    """fp32 [T, ..., r]: rotate-half over the first cos_sin.shape[1] of r dimensions."""
+    rd = cos_sin.shape[1]
+    half = rd // 2
+    cs = cos_sin[positions.long()].view(x.shape[0], *([1] * (x.dim() - 2)), rd)
+    c, s = cs[..., :half], cs[..., half:]
+    u, v = x[..., :half], x[..., half:rd]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., rd:]], -1)
+
+
+def latent_cache(x, nq, R, r, w_q, w_c, cq, pages, Rp, positions, slots, cos_sin, eps):
+    T = x.shape[0]
+    xf = x.float()
+    cq.zero_()
+    cq[:, :nq] = (_norm32(xf[:, :nq], eps) * w_q).to(cq.dtype)
+    D = pages.shape[1] * 8
+    row = torch.zeros(T, D)
+    row[:, :R] = _norm32(xf[:, nq:nq + R], eps) * w_c
+    row[:, Rp:Rp + r] = _rotate_part(xf[:, nq + R:nq + R + r], positions[:T], cos_sin)
+    for t in range(T):
+        s = int(slots[t])
+        if s >= 0:
+            pages[s // 16, :, s % 16, :] = row[t].view(D // 8, 8).to(pages.dtype)
+
+
+def latent_qrot(q, head_stride, skip, r, dst, Rp, positions, cos_sin):
+    T, H = dst.shape[:2]
+    x = torch.stack([q[:, h * head_stride + skip:h * head_stride + skip + r] for h in range(H)], 1).float()
+    dst[:, :, Rp:] = 0
+    dst[:, :, Rp:Rp + r] = _rotate_part(x, positions[:T], cos_sin).to(dst.dtype)
+
+
+def latent_attention(out, q, pages, q_start, q_len, ctx_len, block_table, scale, window, num_seqs):
+    Rp = out.shape[2]
+    for s in range(num_seqs):
+        n, ctx, q0 = int(q_len[s]), int(ctx_len[s]), int(q_start[s])
+        if n <= 0:
+            continue
+        blk = block_table[s, :(ctx + 15) // 16].long()
+        rows = pages[blk].permute(0, 2, 1, 3).reshape(-1, pages.shape[1] * 8)[:ctx].float()
+        sc = torch.einsum("thd,kd->htk", q[q0:q0 + n].float(), rows) * scale
+        back = torch.arange(ctx - n, ctx)[:, None] - torch.arange(ctx)[None, :]
+        seen = (back >= 0) & (back < window) if window > 0 else back >= 0
+        p = torch.softmax(sc.masked_fill(~seen, float("-inf")), -1)
+        out[q0:q0 + n] = torch.einsum("htk,kd->thd", p, rows[:, :Rp]).to(out.dtype)
+
+
+def head_gemm(x, x_step, w, out, out_step):
+    N, K = w.shape[1:]
+    for g in range(w.shape[0]):
+        out[:, g * out_step:g * out_step + N] = (x[:, g * x_step:g * x_step + K].float() @ w[g].float().T).to(out.dtype)
+
+
+def table_route(tables, desc, ids, slots, T, tm, order, tiles, n_tiles):
+    for layer in range(desc.shape[0]):
+        off, V, top, E, o0, t0, tmax, _ = (int(v) for v in desc[layer])
+        tab = tables[off:off + V * top].view(V, top)
+        e = tab[ids[:T].long().clamp(0, V - 1)].clamp(0, E - 1).reshape(-1)
+        live = (slots[:T] >= 0).repeat_interleave(top)
+        p = torch.arange(T * top)[live]
+        p = p[torch.argsort(e[p], stable=True)]
+        order[o0:o0 + len(p)] = p.to(torch.int32)
+        k, start = 0, 0
+        for x, c in enumerate(torch.bincount(e[p].long(), minlength=E).tolist()):
+            for i in range(0, c, tm):
+                tiles[t0 + k] = torch.tensor([x, start + i, min(tm, c - i), 0], dtype=torch.int32)
+                k += 1
+            start += c
+        n_tiles[layer] = min(k, tmax)
+
+
+def expert_gemm(x, w, out, tiles, n_tiles, order, x_div, out_order, glu):
+    K = w.shape[2]
+    for e, start, n, _ in tiles[:int(n_tiles[0])].tolist():
+        p = torch.arange(start, start + n)
+        xr = order[p].long() // x_div if x_div else p
+        y = x[xr, :K].float() @ w[e].float().T
+        if glu is not None:
+            lim, alpha, bias = glu
+            y = y.view(n, -1, 2, 16)
+            g, u = y[:, :, 0].reshape(n, -1).clamp(max=lim), y[:, :, 1].reshape(n, -1).clamp(-lim, lim)
+            y = g * torch.sigmoid(alpha * g) * (u + bias)
+        out[order[p].long() if out_order else p, :y.shape[1]] = y.to(out.dtype)
