@@ -424,8 +424,6 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
         for (int r = 0; r < 4; ++r) tmax = fmaxf(tmax, sc[x][k][r]);
       tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
       tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
-      // masked scores stay near NEG_BIG in log2 units; a column with no key yet is wiped by
-      // alpha = 0 when its first key arrives
       const float m_new = fmaxf(m_run[x], fmaxf(tmax * A.scale_log2, NEG_BIG));
       if (__any(m_new > m_run[x])) {
         const float alpha = exp2f(m_run[x] - m_new);
@@ -434,7 +432,8 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
         for (int n = 0; n < 2 * RT; ++n) o[x][n] *= alpha;
         m_run[x] = m_new;
       }
-      const float nm = -m_run[x];
+      // a column that has seen no key yet (its window starts in a later tile): every weight is 0
+      const float nm = m_run[x] < 0.01f * NEG_BIG ? 0.f : -m_run[x];
 #pragma unroll
       for (int k = 0; k < 2; ++k)
 #pragma unroll

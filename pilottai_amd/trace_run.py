@@ -50,7 +50,7 @@ def main(argv=None) -> int:
     eng = LLMEngine(EngineConfig(model=a.model, dtype=a.dtype, max_num_seqs=SLOTS, max_num_batched_tokens=n,
                                  max_model_len=n, num_kv_blocks=n // 16, exact_kv_blocks=True, prefix_caching=False,
                                  use_graphs=False),
-                    device=torch.device(a.device or "cuda"))
+                    device=torch.device(a.device or "cuda:0"))
     os.makedirs(a.out, exist_ok=True)
     ids = {}
     for line in sys.stdin:
