@@ -648,8 +648,9 @@ void tp_topkp_phase(int64_t phase, at::Tensor tau, at::Tensor ws, at::Tensor log
 // all-gather [shards, rows, V/shards] (then V is the full vocabulary).
 void topkp_threshold(at::Tensor tau, at::Tensor logits, int64_t V, at::Tensor temperature,
                      at::Tensor top_k, at::Tensor top_p, at::Tensor mask_class, at::Tensor class_masks) {
-  for (auto* t : {&tau, &logits, &temperature, &top_k, &top_p, &mask_class, &class_masks})
+  for (auto* t : {&tau, &temperature, &top_k, &top_p, &mask_class, &class_masks})
     check_gpu(*t, "topkp_threshold arg");
+  TORCH_CHECK(logits.is_cuda(), "logits must be a GPU tensor");  // rows may be wider than V
   check_dtype(tau, at::kFloat, "tau"); check_dtype(logits, at::kBFloat16, "logits");
   check_dtype(temperature, at::kFloat, "temperature"); check_dtype(top_k, at::kInt, "top_k");
   check_dtype(top_p, at::kFloat, "top_p"); check_dtype(mask_class, at::kInt, "mask_class");
