@@ -120,6 +120,11 @@ def parse():
                          "the manager Serve, the control plane and all clients; ranks > 0 are CPU processes whose "
                          "agents answer with model-free schema LLMs after this many seconds per call (the measured "
                          "per-call latency of an 8-worker GPU rank). Use with PILOTTAI_DIST_BACKEND=gloo.")
+    ap.add_argument("--design", default=None, choices=["bozupel"],
+                    help="instead of the workload: step throughput of this model design beside Llama layers of equal "
+                         "size, one JSON line per case (benchmarks/model_step.py)")
+    ap.add_argument("--design-cases", default="", help="with --design: only the cases whose name contains this")
+    ap.add_argument("--design-sizes", default="", help="with --design: base, wide (default: both)")
     return ap.parse_args()
 
 
@@ -584,6 +589,11 @@ def _launch_ranks(n: int) -> int:
 
 def main():
     a = parse()
+    if a.design:
+        from benchmarks.model_step import run
+
+        run(a.design, a.steps, a.warmup, a.design_cases, a.design_sizes)
+        return
     if a.gpus > 1 and "WORLD_SIZE" not in os.environ:
         sys.exit(_launch_ranks(a.gpus))
     import torch

@@ -15,8 +15,8 @@ int pa_latent_cache(int fp32, const void* x, int ldx, int NQ, int R, int r, int 
 int pa_latent_qrot(int fp32, const void* q, int ldq, int hs, int ns, int r, int rp, int rd, void* dst, int Rp, int D,
                    int H, const int* positions, const float* cos_sin, int T, hipStream_t st);
 int pa_latent_pad(int R);
-int pa_latent_attention(int fp32, void* out, float* part_o, float* part_ml, int* counters, const void* q,
-                        const void* pages, const int* items, const int* n_items, int max_items, const int* q_start,
+int pa_latent_attention(int fp32, void* out, float* part_o, float* part_ml, const void* q, const void* pages,
+                        const int* items, const int* n_items, int max_items, const int* q_start,
                         const int* q_len, const int* ctx_len, const int* block_table, int max_blocks, int H, int Rp,
                         int rp, int dec_tokens, int tile_tokens, int window, float scale_log2, int simple,
                         hipStream_t st);
@@ -132,7 +132,7 @@ void latent_qrot(at::Tensor q, int64_t hs, int64_t ns, int64_t r, at::Tensor dst
            "latent_qrot");
 }
 
-void latent_attention(at::Tensor out, at::Tensor part_o, at::Tensor part_ml, at::Tensor counters, at::Tensor q,
+void latent_attention(at::Tensor out, at::Tensor part_o, at::Tensor part_ml, at::Tensor q,
                       at::Tensor pages, at::Tensor items, at::Tensor n_items, at::Tensor q_start, at::Tensor q_len,
                       at::Tensor ctx_len, at::Tensor block_table, int64_t dec_tokens, int64_t tile_tokens,
                       int64_t window, double scale, bool simple) {
@@ -150,9 +150,8 @@ void latent_attention(at::Tensor out, at::Tensor part_o, at::Tensor part_ml, at:
   const int64_t NB = (dec_tokens * H + 15) / 16;
   TORCH_CHECK(Rp > 0 && rp > 0 && dec_tokens >= 1 && tile_tokens >= 1, "latent_attention sizes");
   TORCH_CHECK(part_o.numel() >= mi * NB * 16 * Rp && part_ml.numel() >= mi * NB * 32, "partition workspace too small");
-  ints(counters, S * NB, "counters");
   check_rc(pa_latent_attention(f, out.data_ptr(), (float*)opt_f32(part_o, 0, "part_o"),
-                               (float*)opt_f32(part_ml, 0, "part_ml"), counters.data_ptr<int>(), q.data_ptr(),
+                               (float*)opt_f32(part_ml, 0, "part_ml"), q.data_ptr(),
                                pages.data_ptr(), ints(items, 0, "items"), ints(n_items, 1, "n_items"), mi,
                                ints(q_start, S, "q_start"), ints(q_len, S, "q_len"), ints(ctx_len, S, "ctx_len"),
                                ints(block_table, 0, "block_table"), block_table.size(1), H, Rp, rp, dec_tokens,
@@ -221,6 +220,8 @@ void expert_gemm(at::Tensor x, at::Tensor w, at::Tensor out, at::Tensor tiles, a
   TORCH_CHECK(K <= x.size(1) && (glu ? N / 2 : N) <= out.size(1) && out.size(0) >= rows &&
                   x.size(0) * (x_div ? x_div : 1) >= rows, "expert_gemm sizes");
   TORCH_CHECK(f || (x.stride(0) % 8 == 0 && out.stride(0) % 4 == 0), "expert_gemm: 16-byte aligned rows");
+  TORCH_CHECK(tm != 256 || (!f && K % 64 == 0 && K >= 128 && N % 128 == 0 && out.stride(0) % 8 == 0),
+              "expert_gemm: tiles of 256 rows need K % 64 == 0, K >= 128, N % 128 == 0");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 4, "tiles must be [n, 4]");
   check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, G, x.stride(0), 0, out.stride(0), 0, 0,
                            N / 16, K / 32, ints(tiles, 4, "tiles"), tiles.size(0), ints(n_tiles, 1, "n_tiles"),

@@ -52,7 +52,10 @@ constexpr int PP_BUF = 4 * PP_PART;
 // schedule at `body6`: N = 6,144, Llama-3-8B qkv, is 32 column tiles, so M in
 // (1,280, 2,048] fills the 256 CUs in one round instead of 144-192 256 x 256 tiles);
 // 4 -> 256 x 128 tiles (three 48-KiB buffers of parts A B0 B1, schedule at `body4`).
-template <int EPI, bool NORM, bool STAMP = false, int F = 8>
+// GR (grouped rows): A describes ONE row tile of a group (M rows, at most 256; wp the group's
+// weights), bid is the column tile, and xmap / ymap (optional) map a row of the tile to its row of
+// x (xmap[i] / xdiv) and of y.
+template <int EPI, bool NORM, bool STAMP = false, int F = 8, bool GR = false>
 __device__ __forceinline__ void pingpong_tile(const Args& A, const int bid, const int nblocks, char* smem) {
   static_assert(F == 8 || F == 6 || F == 4, "256-, 192- or 128-wide tiles");
   constexpr int NA = F / 4;                 // W parts per 64-k tile (F = 8, 4)
@@ -73,7 +76,11 @@ __device__ __forceinline__ void pingpong_tile(const Args& A, const int bid, cons
 
   const int KT = A.K >> 6;
   int tile, kt0, kt1, slice = -1;
-  if (bid < A.full) {
+  if constexpr (GR) {
+    tile = bid;
+    kt0 = 0;
+    kt1 = KT;
+  } else if (bid < A.full) {
     const int q8 = A.full >> 3, r8 = A.full & 7, xcd = bid & 7;
     tile = (xcd < r8 ? xcd * (q8 + 1) : r8 * (q8 + 1) + (xcd - r8) * q8) + (bid >> 3);
     kt0 = 0;
@@ -108,6 +115,8 @@ __device__ __forceinline__ void pingpong_tile(const Args& A, const int bid, cons
       const int lr = (2 * wid + h) * 8 + (lane >> 3);
       xrow[cc][h] = min(row0 + (lr >> 5) * 64 + cc * 32 + (lr & 31), A.M - 1);
       xunit[cc][h] = (lane & 7) ^ ((lr >> 1) & 7);
+      if constexpr (GR)
+        if (A.xmap) xrow[cc][h] = A.xmap[xrow[cc][h]] / A.xdiv;
     }
   char* const sbase = smem;
   auto buf = [&](int t) -> char* { return sbase + (NBUF == 2 ? (t & 1) : (t % 3)) * BUFB; };
@@ -430,8 +439,10 @@ __device__ __forceinline__ void pingpong_tile(const Args& A, const int bid, cons
   const float inv_k = 1.f / (float)A.K;
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
-    const int m = row0 + wc * 64 + 16 * j + c;
+    int m = row0 + wc * 64 + 16 * j + c;
     const bool ok = m < A.M;
+    if constexpr (GR)
+      if (A.ymap && ok) m = A.ymap[m];
     float sq = 0.f;
     if (ok) {
       float rs = 1.f;

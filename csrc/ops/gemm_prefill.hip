@@ -69,6 +69,11 @@ struct Args {
   const float* cos_sin;
   int H, KV;
   int acq;
+  // grouped rows (gemm_pingpong.h GR) and the clamped gated unit
+  const int* xmap = nullptr;
+  const int* ymap = nullptr;
+  int xdiv = 1;
+  float limit = 0.f, alpha = 0.f, bias = 0.f;
 };
 
 typedef __attribute__((address_space(3))) void lds_t;
@@ -717,4 +722,67 @@ extern "C" int pa_prefill_gemm(void* y, const void* x, const void* wp, const voi
   }
 #undef PA_PF
   return (int)hipGetLastError() == 0 ? 0 : -2;
+}
+
+// Rows sorted by group (mixture-of-experts layers): tiles {group, first position, rows <= 256, 0}
+// on the ping-pong kernels, group g's packed weights at wp + g * wstride. x row of position p =
+// order[p] / x_div (x_div 0: p), y row = order[p] (out_order) or p. epi 0 plain, 5 clamped gated
+// unit. K % 64 == 0, K >= 128, N % 128 == 0; y rows 16-byte aligned.
+namespace pa {
+namespace pf {
+template <int EPI, int F>
+__global__ __launch_bounds__(512) void pingpong_grouped_kernel(Args A, const int4* __restrict__ tiles,
+                                                               const int* __restrict__ n_tiles,
+                                                               const int* __restrict__ order, long long wstride,
+                                                               int x_div, int out_order) {
+  __shared__ __attribute__((aligned(1024))) char smem[(F == 8 ? 2 * 4 : 3 * 3) * PP_PART];
+  // column tiles of one row tile next to each other on one XCD: they share its rows of x
+  const int W = A.NT * n_tiles[0], per = (W + 7) >> 3;
+  const int b = blockIdx.x, w = (b & 7) * per + (b >> 3);
+  if ((b >> 3) >= per || w >= W) return;
+  const int4 tl = tiles[w / A.NT];
+  A.wp += (size_t)tl.x * wstride;
+  A.M = tl.z;
+  if (x_div) {
+    A.xmap = order + tl.y;
+    A.xdiv = x_div;
+  } else {
+    A.x += (size_t)tl.y * A.ldx;
+  }
+  if (out_order) A.ymap = order + tl.y;
+  else A.y += (size_t)tl.y * A.ldy;
+  A.MT = 1;
+  // MT = 1: pingpong_tile's tile index is the column tile
+  pingpong_tile<EPI, false, false, F, true>(A, w % A.NT, A.NT, smem);
+}
+}  // namespace pf
+}  // namespace pa
+
+extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long wstride, int N, int K, int ldx, int ldy,
+                               const int* tiles, int max_tiles, const int* n_tiles, const int* order, int x_div,
+                               int out_order, int epi, float limit, float alpha, float bias, hipStream_t st) {
+  using namespace pa::pf;
+  if (K % 64 || K < 128 || N % 128 || ldx % 8 || ldy % 8 || (epi != EP_PLAIN && epi != EP_GLU)) return -1;
+  if (max_tiles <= 0) return 0;
+  Args a{};
+  a.y = (pa::bf16*)y;
+  a.x = (const pa::bf16*)x;
+  a.wp = (const pa::bf16*)wp;
+  a.N = N;
+  a.K = K;
+  a.ldx = ldx;
+  a.ldy = ldy;
+  a.limit = limit;
+  a.alpha = alpha;
+  a.bias = bias;
+  const bool wide = N % 256 == 0;
+  a.NT = N / (wide ? 256 : 128);
+  const int grid = (a.NT * max_tiles + 7) / 8 * 8;
+#define PA_EX(E, F)                                                                                              \
+  hipLaunchKernelGGL((pingpong_grouped_kernel<E, F>), dim3(grid), dim3(512), 0, st, a, (const int4*)tiles, n_tiles, \
+                     order, wstride, x_div, out_order)
+  if (epi == EP_GLU) { if (wide) PA_EX(EP_GLU, 8); else PA_EX(EP_GLU, 4); }
+  else { if (wide) PA_EX(EP_PLAIN, 8); else PA_EX(EP_PLAIN, 4); }
+#undef PA_EX
+  return (int)hipGetLastError();
 }

@@ -8,11 +8,17 @@
 // Weights are packed per group like the other projections ([N/16, K/32, 64, 8], one 16-B lane
 // vector per MFMA operand). The MFMA's A operand is W and its B operand x, so a lane's four
 // accumulators are four consecutive outputs of one row: 8-byte stores, and the gated pair
-// (tiles 2i: gate, 2i + 1: up) is lane-local.
+// (tiles 2i: gate, 2i + 1: up) is lane-local. Tiles of 16 rows stream the weights (decode steps); 64
+// rows share them; prompts with 256 rows and more per group run the ping-pong kernels instead
+// (gemm_prefill.hip pa_expert_tiles).
 //
 // Epilogues: plain, or the clamped gated unit
 //   g' = min(g, limit), u' = clamp(u, -limit, limit),  out = g' * sigmoid(alpha * g') * (u' + bias).
-#include "common.h"
+#include "packed_epi.h"
+
+extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long wstride, int N, int K, int ldx, int ldy,
+                               const int* tiles, int max_tiles, const int* n_tiles, const int* order, int x_div,
+                               int out_order, int epi, float limit, float alpha, float bias, hipStream_t st);
 
 namespace pa {
 namespace gg {
@@ -33,9 +39,7 @@ struct Args {
 };
 
 __device__ __forceinline__ float glu(float g, float u, const Args& A) {
-  g = fminf(g, A.limit);
-  u = fminf(fmaxf(u, -A.limit), A.limit);
-  return g / (1.f + __expf(-A.alpha * g)) * (u + A.bias);
+  return pk::clamped_glu(g, u, A.limit, A.alpha, A.bias);
 }
 
 template <int MT, int NT, int KU, bool GLU>
@@ -252,7 +256,7 @@ extern "C" int pa_table_route(const int* tables, const int* desc, int layers, co
   return (int)hipGetLastError();
 }
 
-// tm: rows per sorted tile (16 or 64; dense: the kernel's choice by row count)
+// tm: rows per sorted tile (16, 64 or 256; dense: the kernel's choice by row count)
 extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out, long long wstride, int groups,
                                int ldx, int xg, int ldo, int og, int rows, int N16, int K32, const int* tiles,
                                int max_tiles, const int* n_tiles, const int* order, int x_div, int out_order, int tm,
@@ -268,6 +272,9 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
     else hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<false>), grid, dim3(256), 0, st, A);
     return (int)hipGetLastError();
   }
+  if (tiles && tm == 256)
+    return pa_expert_tiles(out, x, w, wstride, N16 * 16, K32 * 32, ldx, ldo, tiles, max_tiles, n_tiles, order, x_div,
+                           out_order, epi == 1 ? 5 : 0, limit, alpha, bias, st);
   if (!tiles) tm = rows <= 32 ? 16 : 64;
   if (tm != 16 && tm != 64) return -2;
 #define PA_GG(MT, NT, KU, G)                                                                                   \

@@ -20,8 +20,10 @@
 // Items come from the scheduler like paged_attention's (seq, q_begin, nq | part<<8 | nparts<<20,
 // partial slot):
 //   nq <= dec_tokens: split over keys. The 4 waves take every 4th page with a private LDS tile and
-//                     merge; nparts > 1 divides the item's own (windowed) key range evenly and the
-//                     last partition to arrive merges all (common.h handoff_last).
+//                     merge; nparts > 1 divides the item's own (windowed) key range evenly, the
+//                     partials go to memory and merge_kernel, a second launch, combines them: at
+//                     16 x Rp floats a partition, one last arriver would read for longer than all
+//                     partitions compute, while the launch spreads the columns over the chip.
 //   otherwise:        64 * CT columns per workgroup, 16 * CT per wave; all waves share
 //                     double-buffered 32-key tiles that arrive by direct global -> LDS loads.
 #include "common.h"
@@ -36,13 +38,11 @@ typedef short s16x4 __attribute__((ext_vector_type(4)));
 typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4;
 typedef __attribute__((address_space(3))) void lds_void;
 typedef const __attribute__((address_space(1))) void glb_void;
-typedef __attribute__((address_space(1))) unsigned long long gu64;
 
 struct Args {
   void* out;             // [T, H, Rp]
-  float* part_o;         // [slots, NB, 16, Rp] (uncached)
+  float* part_o;         // [slots, NB, 16, Rp]
   float* part_ml;        // [slots, NB, 16, 2]
-  int* counters;         // [seqs, NB], zero between launches
   const void* q;         // [T, H, D]
   const void* pages;
   const int4* items;
@@ -50,7 +50,6 @@ struct Args {
   const int *q_start, *q_len, *ctx_len, *block_table;
   int max_blocks, H, NB, Rp, D, dec_tokens, window;
   float scale_log2;
-  int acq;
 };
 
 // ---------------------------------------------------------------------------
@@ -216,7 +215,6 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
   float* mo = reinterpret_cast<float*>(smem);                                // [4][16][MERGE_LD]
   float* mm = reinterpret_cast<float*>(smem + 4 * 16 * MERGE_LD * 4);        // [4][16]
   float* ml = mm + 64;
-  int* lflag = reinterpret_cast<int*>(ml + 64);
   __syncthreads();
   if (g == 0) {
     mm[wid * 16 + c] = m_run;
@@ -254,13 +252,9 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
         acc[j] = a;
       }
       if (nparts > 1) {
-        const __amdgpu_buffer_rsrc_t ps = __builtin_amdgcn_make_buffer_rsrc(
-            A.part_o + ((size_t)pidx * A.NB + cb) * 16 * RP, 0, 16 * RP * 4, 0x00020000);
-        const int so = (ccol * RP + d0) * 4;
-        __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(u32x4, f32x4{acc[0], acc[1], acc[2], acc[3]}), ps,
-                                               so, 0, 16);
-        __builtin_amdgcn_raw_buffer_store_b128(__builtin_bit_cast(u32x4, f32x4{acc[4], acc[5], acc[6], acc[7]}), ps,
-                                               so + 16, 0, 16);
+        f32x4* ps = reinterpret_cast<f32x4*>(A.part_o + (((size_t)pidx * A.NB + cb) * 16 + ccol) * RP + d0);
+        ps[0] = f32x4{acc[0], acc[1], acc[2], acc[3]};
+        ps[1] = f32x4{acc[4], acc[5], acc[6], acc[7]};
       } else if (cvalid) {
         const float inv = 1.f / L;
         bf16x8 v;
@@ -270,57 +264,59 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
       }
     }
   }
-  if (nparts <= 1) return;
-  if ((threadIdx.x & 15) == 0) {
-    const unsigned long long v = ((unsigned long long)__float_as_uint(L) << 32) | __float_as_uint(mt);
-    __hip_atomic_store((gu64*)(A.part_ml + (((size_t)pidx * A.NB + cb) * 16 + ccol) * 2), v, __ATOMIC_RELAXED,
-                       __HIP_MEMORY_SCOPE_AGENT);
-  }
-  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-  if (!handoff_last(A.counters + (size_t)s * A.NB + cb, nparts, lflag, A.acq) || !cvalid) return;
-  const int p0 = pidx - part;
-  auto load_ml = [&](int p) {
-    return __hip_atomic_load((gu64*)(A.part_ml + (((size_t)(p0 + p) * A.NB + cb) * 16 + ccol) * 2), __ATOMIC_RELAXED,
-                             __HIP_MEMORY_SCOPE_AGENT);
-  };
-  float gm = NEG_BIG, GL = 0.f;
-  for (int p = 0; p < nparts; ++p) gm = fmaxf(gm, __uint_as_float((unsigned)load_ml(p)));
-  constexpr int NV = (RP + 127) / 128;
-  float ga[NV][8];
+  if (nparts > 1 && (threadIdx.x & 15) == 0)
+    reinterpret_cast<float2*>(A.part_ml)[((size_t)pidx * A.NB + cb) * 16 + ccol] = float2{mt, L};
+}
+
+// The partitions of split items, merged: a wave per (item, column), 8 dims per lane and step.
+template <int RT>
+__global__ __launch_bounds__(256) void merge_kernel(const Args A) {
+  constexpr int RP = 32 * RT;
+  const int col = blockIdx.x * 4 + (threadIdx.x >> 6), cb = col >> 4, cc = col & 15, lane = threadIdx.x & 63;
+  const int n = A.n_items[0];
+  for (int item = blockIdx.y; item < n; item += gridDim.y) {
+    const int4 it = A.items[item];
+    const int nq = it.z & 0xff, nparts = it.z >> 20;
+    if (nq > A.dec_tokens || nparts <= 1 || ((it.z >> 8) & 0xfff) != 0 || col >= nq * A.H) continue;
+    auto slot = [&](int p) { return ((size_t)(it.w + p) * A.NB + cb) * 16 + cc; };
+    const float2* ml = reinterpret_cast<const float2*>(A.part_ml);
+    float gm = NEG_BIG, L = 0.f;
+    for (int p = 0; p < nparts; ++p) gm = fmaxf(gm, ml[slot(p)].x);
+    float a[(RP + 511) / 512][8];
 #pragma unroll
-  for (int e = 0; e < NV; ++e)
+    for (int e = 0; e < (RP + 511) / 512; ++e)
 #pragma unroll
-    for (int j = 0; j < 8; ++j) ga[e][j] = 0.f;
-  for (int p = 0; p < nparts; ++p) {
-    const unsigned long long v = load_ml(p);
-    const float w = exp2f(__uint_as_float((unsigned)v) - gm);
-    GL += w * __uint_as_float((unsigned)(v >> 32));
-    const __amdgpu_buffer_rsrc_t rs = __builtin_amdgcn_make_buffer_rsrc(
-        A.part_o + ((size_t)(p0 + p) * A.NB + cb) * 16 * RP, 0, 16 * RP * 4, 0x00020000);
+      for (int j = 0; j < 8; ++j) a[e][j] = 0.f;
+#pragma unroll 4
+    for (int p = 0; p < nparts; ++p) {
+      const float2 v = ml[slot(p)];
+      const float w = exp2f(v.x - gm);
+      L += w * v.y;
 #pragma unroll
-    for (int e = 0; e < NV; ++e) {
-      const int d0 = e * 128 + d8;
-      if (d0 < RP) {
-        const int ro = (ccol * RP + d0) * 4;
-        const f32x4 x = __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, ro, 0, 16));
-        const f32x4 y = __builtin_bit_cast(f32x4, __builtin_amdgcn_raw_buffer_load_b128(rs, ro + 16, 0, 16));
+      for (int e = 0; e < (RP + 511) / 512; ++e) {
+        const int d = e * 512 + lane * 8;
+        if (d < RP) {
+          const f32x4* s = reinterpret_cast<const f32x4*>(A.part_o + slot(p) * RP + d);
+          const f32x4 x = s[0], y = s[1];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          ga[e][j] += w * x[j];
-          ga[e][4 + j] += w * y[j];
+          for (int j = 0; j < 4; ++j) {
+            a[e][j] += w * x[j];
+            a[e][4 + j] += w * y[j];
+          }
         }
       }
     }
-  }
-  const float ginv = 1.f / GL;
+    const float inv = 1.f / L;
+    bf16* o = (bf16*)A.out + ((size_t)(A.q_start[it.x] + it.y) * A.H + col) * RP;
 #pragma unroll
-  for (int e = 0; e < NV; ++e) {
-    const int d0 = e * 128 + d8;
-    if (d0 < RP) {
-      bf16x8 v;
+    for (int e = 0; e < (RP + 511) / 512; ++e) {
+      const int d = e * 512 + lane * 8;
+      if (d < RP) {
+        bf16x8 v;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] = (bf16)(ga[e][j] * ginv);
-      *reinterpret_cast<bf16x8*>((bf16*)A.out + (row0 + ccol) * RP + d0) = v;
+        for (int j = 0; j < 8; ++j) v[j] = (bf16)(a[e][j] * inv);
+        *reinterpret_cast<bf16x8*>(o + d) = v;
+      }
     }
   }
 }
@@ -506,16 +502,15 @@ extern "C" int pa_latent_pad(int R) {
   return need * 32;
 }
 
-extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* part_ml, int* counters, const void* q,
-                                   const void* pages, const int* items, const int* n_items, int max_items,
+extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* part_ml, const void* q, const void* pages, const int* items, const int* n_items, int max_items,
                                    const int* q_start, const int* q_len, const int* ctx_len, const int* block_table,
                                    int max_blocks, int H, int Rp, int rp, int dec_tokens, int tile_tokens, int window,
                                    float scale_log2, int simple, hipStream_t st) {
   if (max_items <= 0) return 0;
   const int D = Rp + rp, NB = (dec_tokens * H + 15) / 16;
   if (Rp % 32 || rp % 32 || H <= 0 || dec_tokens <= 0 || tile_tokens <= 0) return -1;
-  pa::la::Args A{out, part_o, part_ml, counters, q, pages, (const int4*)items, n_items, q_start, q_len, ctx_len,
-                 block_table, max_blocks, H, NB, Rp, D, dec_tokens, window, scale_log2, pa::g_handoff_attn};
+  pa::la::Args A{out, part_o, part_ml, q, pages, (const int4*)items, n_items, q_start, q_len, ctx_len,
+                 block_table, max_blocks, H, NB, Rp, D, dec_tokens, window, scale_log2};
   const int RT = Rp / 32, PT = rp / 32;
   if (!fp32 && !simple && PT >= 1 && PT <= 2) {
 #define PA_LA(R, P)                                                                                           \
@@ -531,6 +526,7 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
     const int gt = (tile_tokens * H + 64 * CT - 1) / (64 * CT), gx = NB > gt ? NB : gt;                       \
     const int gy = max_items < 4096 ? max_items : 4096;                                                       \
     hipLaunchKernelGGL((pa::la::mfma_kernel<R, P, CT>), dim3(gx, gy), dim3(256), lds, st, A);                 \
+    hipLaunchKernelGGL((pa::la::merge_kernel<R>), dim3(4 * NB, gy), dim3(256), 0, st, A);                     \
     return (int)hipGetLastError();                                                                            \
   } while (0)
     switch (RT) {

@@ -5,6 +5,7 @@
 //
 //   EP_PLAIN     y = acc
 //   EP_SILU      y = silu(gate) * up over the interleaved (gate t, up t) packed tiles
+//   EP_GLU       y = clamped gated unit over the same pairs (limit, alpha, bias; clamped_glu below)
 //   EP_RESID     y = resid + acc, returning sum(y^2) of the written bf16 values (the next
 //                RMSNorm's row statistics, accumulated by the caller)
 //   EP_ROPEPERM  y = acc in the natural QKV column order (rope-permuted packed tiles)
@@ -19,10 +20,17 @@
 namespace pa {
 namespace pk {
 
-enum { EP_PLAIN = 0, EP_SILU = 1, EP_RESID = 2, EP_ROPEPERM = 3, EP_ROPEKV = 4 };
+enum { EP_PLAIN = 0, EP_SILU = 1, EP_RESID = 2, EP_ROPEPERM = 3, EP_ROPEKV = 4, EP_GLU = 5 };
 
 template <int EPI>
-constexpr bool pair_epi() { return EPI == EP_SILU || EPI == EP_ROPEKV; }
+constexpr bool pair_epi() { return EPI == EP_SILU || EPI == EP_ROPEKV || EPI == EP_GLU; }
+
+// g' = min(g, limit), u' = clamp(u, -limit, limit): g' sigmoid(alpha g') (u' + bias)
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float bias) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + __expf(-alpha * g)) * (u + bias);
+}
 
 // packed rope-QKV tile -> first column of its original tile
 __device__ __forceinline__ int ropeperm_tile(int tile) {
@@ -34,7 +42,13 @@ __device__ __forceinline__ int ropeperm_tile(int tile) {
 // `tile` (and, for the pair epilogues, the same 4 columns of tile + 1 in v2).
 template <int EPI, class AT>
 __device__ __forceinline__ float store_quad(const AT& A, int m, int tile, int cq, f32x4 v, f32x4 v2) {
-  if constexpr (EPI == EP_SILU) {
+  if constexpr (EPI == EP_GLU) {
+    bf16x4 o;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) o[r] = (bf16)clamped_glu(v[r], v2[r], A.limit, A.alpha, A.bias);
+    *reinterpret_cast<bf16x4*>(A.y + (size_t)m * A.ldy + (tile >> 1) * 16 + cq) = o;
+    return 0.f;
+  } else if constexpr (EPI == EP_SILU) {
     bf16x4 o;
 #pragma unroll
     for (int r = 0; r < 4; ++r) o[r] = (bf16)(v[r] / (1.f + __expf(-v[r])) * v2[r]);

@@ -368,9 +368,10 @@ class LLMEngine:
         tpw = 16 // att["gqa_group"]
         self._tpw = tpw
         self._max_parts = (self.max_model_len + ops.ATT_PART - 1) // ops.ATT_PART
-        # attention partition partials: written and merged inside one launch -> uncached memory
-        self._part_o = ops.empty_handoff(po, torch.float32, self.device)
-        self._part_ml = ops.empty_handoff(pml, torch.float32, self.device)
+        # attention partition partials: uncached memory where one launch writes and merges them
+        make = ops.empty_handoff if self.model.ATT_HANDOFF else lambda n, dt, dev: torch.zeros(n, dtype=dt, device=dev)
+        self._part_o = make(po, torch.float32, self.device)
+        self._part_ml = make(pml, torch.float32, self.device)
         self._sample_ws = None  # with the first sampled step (a fed step samples nothing)
         # one graph per (token bucket, top-k/top-p pass); truncating variants are
         # captured on first use, so steps without truncation pay nothing for it

@@ -228,7 +228,7 @@ class LatentAttention:
         ops.head_gemm(q, self.np + self.rp, self.uk, qa.view(T, -1), self.D)
         ops.latent_qrot(q, self.np + self.rp, self.np, m.rot_dim, qa, self.Rp, meta.positions, self.cos_sin)
         oc = new(T, H, self.Rp)
-        ops.latent_attention(oc, part_o, part_ml, qa, pages, meta.items, meta.n_items, meta.att_counters, meta.q_start,
+        ops.latent_attention(oc, part_o, part_ml, qa, pages, meta.items, meta.n_items, meta.q_start,
                              meta.q_len, meta.ctx_len, meta.block_table, m.scale, m.window, dec_tokens, tile_tokens,
                              num_seqs=meta.num_seqs)
         v = new(T, self.o.K)
@@ -245,7 +245,7 @@ class TableExperts:
     def __init__(self, spec: TableExpertsSpec, t: Dict[str, torch.Tensor], width: int, dtype, device):
         self.spec, self.dtype, self.device = spec, dtype, device
         E, f, d = spec.experts, spec.ff, width
-        fp, dk, dn = pad_to(f, 32), pad_to(d, 32), pad_to(d, 16)
+        fp, dk, dn = pad_to(f, 64), pad_to(d, 64), pad_to(d, 128)
         self.fp, self.dn = fp, dn
         w13, w2 = [], []
         for e in range(E):
@@ -277,6 +277,9 @@ class BozupelModel:
     PREFILL_MAX_T = 1 << 30
     ATT_DECODE_WAVES = 4
     PF_MIDRANGE = frozenset()
+    # average rows per expert above which an expert's rows go in tiles of 64 / 256
+    EXPERT_ROWS_64 = 32
+    EXPERT_ROWS_256 = 96
     decode_packed = True
 
     def __init__(self, cfg: BozupelConfig, device, dtype=torch.bfloat16, tp: Optional[TPGroup] = None, seed: int = 0,
@@ -389,13 +392,15 @@ class BozupelModel:
     def attention_items(self) -> dict:
         windows = [L.mixer.window for L in self.cfg.layers]
         return {"gqa_group": self._group, "kv_heads": 1, "att_qcols": 128, "att_narrow_qcols": 128,
-                "prefill_split_keys": 0, "att_max_keys": max(windows) if all(windows) else 0}
+                "prefill_split_keys": 0, "decode_part_target": 256, "att_max_keys": max(windows) if all(windows) else 0}
+
+    ATT_HANDOFF = False  # partials are merged by a launch of their own: ordinary memory
 
     def attention_workspace(self, max_items: int) -> tuple:
-        """(partial outputs, partial (max, sum) pairs) in floats, and tickets per sequence."""
+        """(partial outputs, partial (max, sum) pairs) in floats, and tickets per sequence (none)."""
         nb = [(self.dec_tokens * L["attn"].spec.heads + 15) // 16 for L in self.layers]
         o = max(b * 16 * L["attn"].Rp for b, L in zip(nb, self.layers))
-        return max_items * o, max_items * max(nb) * 32, max(nb)
+        return max_items * o, max_items * max(nb) * 32, 1
 
     def health_words(self) -> list:
         return []
@@ -408,11 +413,14 @@ class BozupelModel:
             return []
         dev = self.device
         if T not in self._route_desc:  # (before graph capture: the capture's warm-up runs come first)
-            big = self.dtype == torch.bfloat16 and T * max(p.top / p.experts for p in mlps) > 32
-            tm, rows, tab, o, t = 64 if big else 16, [], 0, 0, 0
+            per = T * max(p.top / p.experts for p in mlps)  # rows an expert gets on average
+            tm, rows, tab, o, t = 16, [], 0, 0, 0
+            if self.dtype == torch.bfloat16 and per > self.EXPERT_ROWS_64:
+                ok = min(min(L["mlp"].fp for L in self.layers if L["mlp"]), pad_to(self.cfg.hidden_size, 64)) >= 128
+                tm = 256 if ok and per > self.EXPERT_ROWS_256 else 64
             for p in mlps:
                 n = T * p.top
-                cap = n // (64 if big else 16) + min(p.experts, n)
+                cap = n // tm + min(p.experts, n)
                 rows.append([tab, self.cfg.vocab_size, p.top, p.experts, o, t, cap, 0])
                 tab, o, t = tab + self.cfg.vocab_size * p.top, o + n, t + cap
             host = torch.tensor(rows, dtype=torch.int32)

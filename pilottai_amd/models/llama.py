@@ -330,6 +330,8 @@ class LlamaModel:
         """Scheduler settings for the work items of this model's attention kernel."""
         return {"gqa_group": self.h_local // self.kv_local, "kv_heads": self.kv_local}
 
+    ATT_HANDOFF = True  # partials are handed over inside the launch: uncached memory
+
     def attention_workspace(self, max_items: int) -> tuple:
         """(partial outputs, partial (max, sum) pairs) in floats, and tickets per sequence."""
         return max_items * self.kv_local * 16 * 128, max_items * self.kv_local * 16 * 2, self.kv_local

@@ -61,14 +61,14 @@ def latent_qrot(q, head_stride: int, skip: int, r: int, dst, Rp: int, positions,
         ref.latent_qrot(q, head_stride, skip, r, dst, Rp, positions, cos_sin)
 
 
-def latent_attention(out, part_o, part_ml, q, pages, items, n_items, counters, q_start, q_len, ctx_len, block_table,
+def latent_attention(out, part_o, part_ml, q, pages, items, n_items, q_start, q_len, ctx_len, block_table,
                      scale: float, window: int, dec_tokens: int, tile_tokens: int, num_seqs: Optional[int] = None,
                      simple: bool = False):
     """Attention of absorbed queries q [T, H, D] over latent pages -> out [T, H, Rp]; `window` 0: none.
     dec_tokens / tile_tokens: the scheduler's items hold at most dec_tokens tokens (split over keys) or
     tile_tokens (csrc/ops/latent_attention.hip). `simple`: the any-size kernel."""
     if _on_gpu(q):
-        require_latent().latent_attention(out, part_o, part_ml, counters, q, pages, items, n_items, q_start, q_len,
+        require_latent().latent_attention(out, part_o, part_ml, q, pages, items, n_items, q_start, q_len,
                                           ctx_len, block_table, int(dec_tokens), int(tile_tokens), int(window),
                                           float(scale), bool(simple))
     else:

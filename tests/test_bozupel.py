@@ -273,7 +273,7 @@ def test_latent_attention_module(folder, device):
         dec, tile = 16 // min(H, 16), 128 // min(H, 16)
         items = [[0, b, min(tile, T - b) | 1 << 20, 0] for b in range(0, T, tile)]
         meta = StepMeta(iv(0), torch.arange(T, dtype=torch.int32, device=dev), slots.to(dev), iv(0), iv(T), iv(T),
-                        table.to(dev), torch.tensor(items, dtype=torch.int32, device=dev), iv(len(items)), iv(*[0] * 64),
+                        table.to(dev), torch.tensor(items, dtype=torch.int32, device=dev), iv(len(items)), iv(0),
                         iv(0), num_seqs=1)
         z = torch.zeros(len(items) * 64 * m.Rp, device=dev)
         pages = torch.zeros(5, m.D // 8, 16, 8, device=dev)
