@@ -12,8 +12,6 @@ int pa_residual_norm(int fp32, float* resid, const void* y, int K, int ldy, floa
 int pa_latent_cache(int fp32, const void* x, int ldx, int NQ, int R, int r, int rd, const float* w_q, const float* w_c,
                     void* cq, int ldq, void* pages, int Rp, int D, const int* positions, const int* slots,
                     const float* cos_sin, float eps, int T, hipStream_t st);
-int pa_latent_qrot(int fp32, const void* q, int ldq, int hs, int ns, int r, int rp, int rd, void* dst, int Rp, int D,
-                   int H, const int* positions, const float* cos_sin, int T, hipStream_t st);
 int pa_latent_pad(int R);
 int pa_latent_attention(int fp32, void* out, float* part_o, float* part_ml, const void* q, const void* pages,
                         const int* items, const int* n_items, int max_items, const int* q_start,
@@ -25,7 +23,7 @@ int pa_table_route(const int* tables, const int* desc, int layers, const int* id
 int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out, long long wstride, int groups, int ldx, int xg,
                     int ldo, int og, int rows, int N16, int K32, const int* tiles, int max_tiles, const int* n_tiles,
                     const int* order, int x_div, int out_order, int tm, int epi, float limit, float alpha, float bias,
-                    hipStream_t st);
+                    const int* positions, const float* cos_sin, int rskip, int r, int rp, int rd, hipStream_t st);
 }
 
 namespace {
@@ -115,23 +113,6 @@ void latent_cache(at::Tensor x, int64_t NQ, int64_t R, int64_t r, at::Tensor w_q
            "latent_cache");
 }
 
-void latent_qrot(at::Tensor q, int64_t hs, int64_t ns, int64_t r, at::Tensor dst, int64_t Rp, at::Tensor positions,
-                 at::Tensor cos_sin) {
-  const int f = is_f32(q, "q");
-  check_rows(q, q.scalar_type(), "q");
-  check_gpu(dst, "dst");
-  check_dtype(dst, q.scalar_type(), "dst");
-  TORCH_CHECK(dst.dim() == 3 && dst.size(0) == q.size(0), "dst must be [T, H, D]");
-  const int64_t T = q.size(0), H = dst.size(1), D = dst.size(2);
-  check_gpu(cos_sin, "cos_sin");
-  check_dtype(cos_sin, at::kFloat, "cos_sin");
-  TORCH_CHECK(q.size(1) >= (H - 1) * hs + ns + r && r <= D - Rp && cos_sin.dim() == 2 && cos_sin.size(1) <= r &&
-                  cos_sin.size(1) % 2 == 0, "latent_qrot sizes");
-  check_rc(pa_latent_qrot(f, q.data_ptr(), q.stride(0), hs, ns, r, D - Rp, cos_sin.size(1), dst.data_ptr(), Rp, D, H,
-                          ints(positions, T, "positions"), cos_sin.data_ptr<float>(), T, cur_stream()),
-           "latent_qrot");
-}
-
 void latent_attention(at::Tensor out, at::Tensor part_o, at::Tensor part_ml, at::Tensor q,
                       at::Tensor pages, at::Tensor items, at::Tensor n_items, at::Tensor q_start, at::Tensor q_len,
                       at::Tensor ctx_len, at::Tensor block_table, int64_t dec_tokens, int64_t tile_tokens,
@@ -189,8 +170,10 @@ void dims(const at::Tensor& w, int f, int64_t* G, int64_t* N, int64_t* K) {
   }
 }
 
-// every row of x through every group: x columns g * xg .. + K -> out columns g * og .. + N
-void head_gemm(at::Tensor x, int64_t xg, at::Tensor w, at::Tensor out, int64_t og) {
+// every row of x through every group: x columns g * xg .. + K -> out columns g * og .. + N; with
+// positions / cos_sin also the rotated part: x columns g * xg + rskip .. + r -> out columns g * og + N .. + rp
+void head_gemm(at::Tensor x, int64_t xg, at::Tensor w, at::Tensor out, int64_t og, Opt positions, Opt cos_sin,
+               int64_t rskip, int64_t r, int64_t rp) {
   const int f = is_f32(x, "x");
   check_rows(x, x.scalar_type(), "x");
   check_rows(out, x.scalar_type(), "out");
@@ -199,11 +182,24 @@ void head_gemm(at::Tensor x, int64_t xg, at::Tensor w, at::Tensor out, int64_t o
   dims(w, f, &G, &N, &K);
   TORCH_CHECK(out.size(0) == x.size(0) && (G - 1) * xg + K <= x.size(1) && (G - 1) * og + N <= out.size(1),
               "head_gemm sizes");
+  const int* pos = nullptr;
+  const float* cs = nullptr;
+  int64_t rd = 0;
+  if (positions.has_value()) {
+    TORCH_CHECK(cos_sin.has_value() && cos_sin->dim() == 2 && cos_sin->size(1) % 2 == 0, "cos_sin must be [max_pos, dims]");
+    rd = cos_sin->size(1);
+    pos = ints(*positions, x.size(0), "positions");
+    cs = opt_f32(cos_sin, 0, "cos_sin");
+    TORCH_CHECK(rd <= r && r <= rp && rp > 0 && rskip >= 0 && (G - 1) * xg + rskip + r <= x.size(1) &&
+                    (G - 1) * og + N + rp <= out.size(1), "head_gemm rotation sizes");
+  } else {
+    rp = 0;
+  }
   TORCH_CHECK(f || (x.stride(0) % 8 == 0 && xg % 8 == 0 && out.stride(0) % 4 == 0 && og % 4 == 0),
               "head_gemm: 16-byte aligned operands");
   check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, G, x.stride(0), xg, out.stride(0), og,
                            x.size(0), N / 16, K / 32, nullptr, 0, nullptr, nullptr, 0, 0, 0, 0, 0.f, 0.f, 0.f,
-                           cur_stream()),
+                           pos, cs, rskip, r, rp, rd, cur_stream()),
            "head_gemm");
 }
 
@@ -226,7 +222,7 @@ void expert_gemm(at::Tensor x, at::Tensor w, at::Tensor out, at::Tensor tiles, a
   check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, G, x.stride(0), 0, out.stride(0), 0, 0,
                            N / 16, K / 32, ints(tiles, 4, "tiles"), tiles.size(0), ints(n_tiles, 1, "n_tiles"),
                            ints(order, rows, "order"), x_div, out_order ? 1 : 0, tm, glu ? 1 : 0, (float)limit,
-                           (float)alpha, (float)bias, cur_stream()),
+                           (float)alpha, (float)bias, nullptr, nullptr, 0, 0, 0, 0, cur_stream()),
            "expert_gemm");
 }
 
@@ -236,7 +232,6 @@ PYBIND11_MODULE(_latent, m) {
   m.doc() = "pilottai_amd CDNA4 (gfx950) kernels: latent attention, table-routed experts, fp32 residual";
   m.def("residual_norm", &residual_norm);
   m.def("latent_cache", &latent_cache);
-  m.def("latent_qrot", &latent_qrot);
   m.def("latent_pad", [](int R) { return pa_latent_pad(R); });
   m.def("latent_attention", &latent_attention);
   m.def("table_route", &table_route);

@@ -36,7 +36,30 @@ struct Args {
   int x_div;               // sorted: x row = order / x_div (0: x row = position)
   int out_order;           // sorted: out row = order[position] (0: out row = position)
   float limit, alpha, bias;
+  // dense, optional: after a group's N columns of out, the rotated part of the row's head (r columns of
+  // x at the group's offset + rskip, the first rd turned by the row's position), padded to rp columns
+  const int* positions;
+  const float* cos_sin;
+  int rskip, r, rp, rd;
 };
+
+// The rotated columns of `n` rows from `start` of group grp (one workgroup).
+template <typename T>
+__device__ __forceinline__ void rotate_rows(const Args& A, int grp, int start, int n) {
+  const int half = A.rd >> 1, N = A.N16 * 16;
+  for (int e = threadIdx.x; e < n * A.rp; e += 256) {
+    const int t = start + e / A.rp, j = e % A.rp;
+    const T* src = (const T*)A.x + (size_t)t * A.ldx + (size_t)grp * A.xg + A.rskip;
+    float v = 0.f;
+    if (j < A.r) {
+      v = (float)src[j];
+      const float* cs = A.cos_sin + (size_t)A.positions[t] * A.rd;
+      if (j < half) v = v * cs[j] - (float)src[j + half] * cs[half + j];
+      else if (j < A.rd) v = v * cs[j - half] + (float)src[j - half] * cs[j];
+    }
+    ((T*)A.out)[(size_t)t * A.ldo + (size_t)grp * A.og + N + j] = (T)v;
+  }
+}
 
 __device__ __forceinline__ float glu(float g, float u, const Args& A) {
   return pk::clamped_glu(g, u, A.limit, A.alpha, A.bias);
@@ -57,6 +80,10 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
     grp = blockIdx.z;
     start = blockIdx.y * (16 * MT);
     n = min(16 * MT, A.rows - start);
+  }
+  if (A.rp && blockIdx.x == gridDim.x - 1) {
+    rotate_rows<bf16>(A, grp, start, n);
+    return;
   }
   const int nt0 = (blockIdx.x * 4 + wid) * NT;
   if (nt0 >= A.N16) return;
@@ -151,6 +178,10 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const Args A) {
     grp = blockIdx.z;
     start = blockIdx.y * TM;
     n = min(TM, A.rows - start);
+  }
+  if (A.rp && blockIdx.x == gridDim.x - 1) {
+    rotate_rows<float>(A, grp, start, n);
+    return;
   }
   const int K = A.K32 * 32;
   const float* wg = (const float*)A.w + (size_t)grp * A.wstride + (size_t)blockIdx.x * (GLU ? 32 : 16) * K;
@@ -260,14 +291,16 @@ extern "C" int pa_table_route(const int* tables, const int* desc, int layers, co
 extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out, long long wstride, int groups,
                                int ldx, int xg, int ldo, int og, int rows, int N16, int K32, const int* tiles,
                                int max_tiles, const int* n_tiles, const int* order, int x_div, int out_order, int tm,
-                               int epi, float limit, float alpha, float bias, hipStream_t st) {
+                               int epi, float limit, float alpha, float bias, const int* positions,
+                               const float* cos_sin, int rskip, int r, int rp, int rd, hipStream_t st) {
   if (N16 <= 0 || K32 <= 0 || (epi == 1 && N16 % 2)) return -1;
   if (tiles ? max_tiles <= 0 : rows <= 0) return 0;
   const pa::gg::Args A{x, w, out, wstride, ldx, xg, ldo, og, rows, N16, K32, (const int4*)tiles, n_tiles,
-                       order, x_div, out_order, limit, alpha, bias};
+                       order, x_div, out_order, limit, alpha, bias, positions, cos_sin, rskip, r, rp, rd};
+  const int rot = rp > 0 ? 1 : 0;  // one more column of workgroups
   if (fp32) {
     if (tiles && tm != 16) return -2;
-    const dim3 grid(epi == 1 ? N16 / 2 : N16, tiles ? max_tiles : (rows + 15) / 16, tiles ? 1 : groups);
+    const dim3 grid((epi == 1 ? N16 / 2 : N16) + rot, tiles ? max_tiles : (rows + 15) / 16, tiles ? 1 : groups);
     if (epi == 1) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<true>), grid, dim3(256), 0, st, A);
     else hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<false>), grid, dim3(256), 0, st, A);
     return (int)hipGetLastError();
@@ -279,7 +312,7 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
   if (tm != 16 && tm != 64) return -2;
 #define PA_GG(MT, NT, KU, G)                                                                                   \
   hipLaunchKernelGGL((pa::gg::gemm_kernel<MT, NT, KU, G>),                                                     \
-                     dim3((N16 + 4 * NT - 1) / (4 * NT), tiles ? max_tiles : (rows + 16 * MT - 1) / (16 * MT), \
+                     dim3((N16 + 4 * NT - 1) / (4 * NT) + rot, tiles ? max_tiles : (rows + 16 * MT - 1) / (16 * MT), \
                           tiles ? 1 : groups),                                                                 \
                      dim3(256), 0, st, A)
 #define PA_GGK(MT, NT, G)                      \

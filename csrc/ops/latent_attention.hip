@@ -280,32 +280,40 @@ __global__ __launch_bounds__(256) void merge_kernel(const Args A) {
     if (nq > A.dec_tokens || nparts <= 1 || ((it.z >> 8) & 0xfff) != 0 || col >= nq * A.H) continue;
     auto slot = [&](int p) { return ((size_t)(it.w + p) * A.NB + cb) * 16 + cc; };
     const float2* ml = reinterpret_cast<const float2*>(A.part_ml);
+    // lane p holds partition p's weight (64 at a time): the loads of a round are independent
     float gm = NEG_BIG, L = 0.f;
-    for (int p = 0; p < nparts; ++p) gm = fmaxf(gm, ml[slot(p)].x);
+    for (int p0 = 0; p0 < nparts; p0 += 64) gm = fmaxf(gm, p0 + lane < nparts ? ml[slot(p0 + lane)].x : NEG_BIG);
+    gm = wave_max(gm);
     float a[(RP + 511) / 512][8];
 #pragma unroll
     for (int e = 0; e < (RP + 511) / 512; ++e)
 #pragma unroll
       for (int j = 0; j < 8; ++j) a[e][j] = 0.f;
-#pragma unroll 4
-    for (int p = 0; p < nparts; ++p) {
-      const float2 v = ml[slot(p)];
-      const float w = exp2f(v.x - gm);
-      L += w * v.y;
+    for (int p0 = 0; p0 < nparts; p0 += 64) {
+      float w = 0.f;
+      if (p0 + lane < nparts) {
+        const float2 v = ml[slot(p0 + lane)];
+        w = exp2f(v.x - gm);
+        L += w * v.y;
+      }
+      const int np = min(64, nparts - p0);
+#pragma unroll 8
+      for (int p = 0; p < np; ++p) {
+        const float wp = __shfl(w, p, 64);
 #pragma unroll
-      for (int e = 0; e < (RP + 511) / 512; ++e) {
-        const int d = e * 512 + lane * 8;
-        if (d < RP) {
-          const f32x4* s = reinterpret_cast<const f32x4*>(A.part_o + slot(p) * RP + d);
+        for (int e = 0; e < (RP + 511) / 512; ++e) {
+          const int d = min(e * 512 + lane * 8, RP - 8);
+          const f32x4* s = reinterpret_cast<const f32x4*>(A.part_o + slot(p0 + p) * RP + d);
           const f32x4 x = s[0], y = s[1];
 #pragma unroll
           for (int j = 0; j < 4; ++j) {
-            a[e][j] += w * x[j];
-            a[e][4 + j] += w * y[j];
+            a[e][j] += wp * x[j];
+            a[e][4 + j] += wp * y[j];
           }
         }
       }
     }
+    L = wave_sum(L);
     const float inv = 1.f / L;
     bf16* o = (bf16*)A.out + ((size_t)(A.q_start[it.x] + it.y) * A.H + col) * RP;
 #pragma unroll
@@ -524,7 +532,8 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
       attr = true;                                                                                            \
     }                                                                                                         \
     const int gt = (tile_tokens * H + 64 * CT - 1) / (64 * CT), gx = NB > gt ? NB : gt;                       \
-    const int gy = max_items < 4096 ? max_items : 4096;                                                       \
+    /* items are strided over the grid: at least one workgroup per CU */                                      \
+    const int gy = max_items < 256 ? 256 : (max_items < 4096 ? max_items : 4096);                             \
     hipLaunchKernelGGL((pa::la::mfma_kernel<R, P, CT>), dim3(gx, gy), dim3(256), lds, st, A);                 \
     hipLaunchKernelGGL((pa::la::merge_kernel<R>), dim3(4 * NB, gy), dim3(256), 0, st, A);                     \
     return (int)hipGetLastError();                                                                            \

@@ -53,28 +53,6 @@ __global__ __launch_bounds__(256) void latent_cache_kernel(
   }
 }
 
-// q [T, ldq] (per head: ns columns to skip, then the rotary part) -> dst[t, h, Rp .. Rp + rp):
-// the first rd of r columns turned by the token's position, the rest copied, padding zero.
-template <typename T>
-__global__ __launch_bounds__(256) void latent_qrot_kernel(const T* __restrict__ q, int ldq, int hs, int ns, int r,
-                                                          int rp, int rd, T* __restrict__ dst, int Rp, int D, int H,
-                                                          const int* __restrict__ positions,
-                                                          const float* __restrict__ cos_sin) {
-  const int t = blockIdx.x, half = rd >> 1;
-  const float* cs = cos_sin + (size_t)positions[t] * rd;
-  for (int e = threadIdx.x; e < H * rp; e += 256) {
-    const int h = e / rp, j = e - h * rp;
-    const T* src = q + (size_t)t * ldq + (size_t)h * hs + ns;
-    float v = 0.f;
-    if (j < r) {
-      v = (float)src[j];
-      if (j < half) v = v * cs[j] - (float)src[j + half] * cs[half + j];
-      else if (j < rd) v = v * cs[j - half] + (float)src[j - half] * cs[j];
-    }
-    dst[((size_t)t * H + h) * D + Rp + j] = (T)v;
-  }
-}
-
 }  // namespace pa
 
 extern "C" int pa_latent_cache(int fp32, const void* x, int ldx, int NQ, int R, int r, int rd, const float* w_q,
@@ -86,17 +64,5 @@ extern "C" int pa_latent_cache(int fp32, const void* x, int ldx, int NQ, int R, 
                      w_q, w_c, (TT*)cq, ldq, (TT*)pages, Rp, D, positions, slots, cos_sin, eps)
   if (fp32) PA_LC(float); else PA_LC(pa::bf16);
 #undef PA_LC
-  return (int)hipGetLastError();
-}
-
-extern "C" int pa_latent_qrot(int fp32, const void* q, int ldq, int hs, int ns, int r, int rp, int rd, void* dst,
-                              int Rp, int D, int H, const int* positions, const float* cos_sin, int T,
-                              hipStream_t st) {
-  if (T <= 0) return 0;
-#define PA_QR(TT)                                                                                               \
-  hipLaunchKernelGGL((pa::latent_qrot_kernel<TT>), dim3(T), dim3(256), 0, st, (const TT*)q, ldq, hs, ns, r, rp, \
-                     rd, (TT*)dst, Rp, D, H, positions, cos_sin)
-  if (fp32) PA_QR(float); else PA_QR(pa::bf16);
-#undef PA_QR
   return (int)hipGetLastError();
 }

@@ -18,7 +18,7 @@ One step of T tokens (decode rows and prompt portions alike):
   per run   linear            [query latent | kv latent | rotated key] = W_down h, one projection
             latent_cache      both latent norms, key rotation, paged cache row
             linear            q = W_uq c_q
-            head_gemm         q~ = W_uk^T q per head; latent_qrot: the rotated part beside it
+            head_gemm         q~ = [W_uk^T q | rotated part of q] per head
             latent_attention  windowed paged attention in the latent space
             head_gemm, linear W_uv per head, W_o
             residual_norm     x += norm(y), next norm -> h
@@ -225,8 +225,8 @@ class LatentAttention:
                          meta.slots, self.cos_sin, self.eps)
         q = self.uq(cq)
         qa = new(T, H, self.D)
-        ops.head_gemm(q, self.np + self.rp, self.uk, qa.view(T, -1), self.D)
-        ops.latent_qrot(q, self.np + self.rp, self.np, m.rot_dim, qa, self.Rp, meta.positions, self.cos_sin)
+        ops.head_gemm(q, self.np + self.rp, self.uk, qa.view(T, -1), self.D,
+                      rot=(meta.positions, self.cos_sin, self.np, m.rot_dim, self.rp))
         oc = new(T, H, self.Rp)
         ops.latent_attention(oc, part_o, part_ml, qa, pages, meta.items, meta.n_items, meta.q_start,
                              meta.q_len, meta.ctx_len, meta.block_table, m.scale, m.window, dec_tokens, tile_tokens,

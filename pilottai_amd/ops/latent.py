@@ -53,14 +53,6 @@ def latent_cache(x, nq: int, R: int, r: int, w_q, w_c, cq, pages, Rp: int, posit
         ref.latent_cache(x, nq, R, r, w_q, w_c, cq, pages, Rp, positions, slots, cos_sin, eps)
 
 
-def latent_qrot(q, head_stride: int, skip: int, r: int, dst, Rp: int, positions, cos_sin):
-    """dst[t, h, Rp:] = the rotated part of every query head of q (columns head_stride * h + skip ...)."""
-    if _on_gpu(q):
-        require_latent().latent_qrot(q, int(head_stride), int(skip), int(r), dst, int(Rp), positions, cos_sin)
-    else:
-        ref.latent_qrot(q, head_stride, skip, r, dst, Rp, positions, cos_sin)
-
-
 def latent_attention(out, part_o, part_ml, q, pages, items, n_items, q_start, q_len, ctx_len, block_table,
                      scale: float, window: int, dec_tokens: int, tile_tokens: int, num_seqs: Optional[int] = None,
                      simple: bool = False):
@@ -102,12 +94,15 @@ def interleave_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
     return torch.stack([gate.reshape(G, F // 16, 16, K), up.reshape(G, F // 16, 16, K)], 2).reshape(G, 2 * F, K)
 
 
-def head_gemm(x, x_step: int, w, out, out_step: int):
-    """out[:, g * out_step : + N] = x[:, g * x_step : + K] @ w[g].T for every group g."""
+def head_gemm(x, x_step: int, w, out, out_step: int, rot: Optional[tuple] = None):
+    """out[:, g * out_step : + N] = x[:, g * x_step : + K] @ w[g].T for every group g. rot = (positions,
+    cos_sin, skip, r, rp): beside them, out[:, g * out_step + N : + rp] = x[:, g * x_step + skip : + r] rotated
+    by the row's position and padded with zeros."""
     if _on_gpu(x):
-        require_latent().head_gemm(x, int(x_step), w, out, int(out_step))
+        pos, cs, skip, r, rp = rot or (None, None, 0, 0, 0)
+        require_latent().head_gemm(x, int(x_step), w, out, int(out_step), pos, cs, int(skip), int(r), int(rp))
     else:
-        ref.head_gemm(x, x_step, unpack_groups(w), out, out_step)
+        ref.head_gemm(x, x_step, unpack_groups(w), out, out_step, rot)
     return out
 
 

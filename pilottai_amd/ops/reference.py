@@ -351,13 +351,6 @@ def latent_cache(x, nq, R, r, w_q, w_c, cq, pages, Rp, positions, slots, cos_sin
             pages[s // 16, :, s % 16, :] = row[t].view(D // 8, 8).to(pages.dtype)
 
 
-def latent_qrot(q, head_stride, skip, r, dst, Rp, positions, cos_sin):
-    T, H = dst.shape[:2]
-    x = torch.stack([q[:, h * head_stride + skip:h * head_stride + skip + r] for h in range(H)], 1).float()
-    dst[:, :, Rp:] = 0
-    dst[:, :, Rp:Rp + r] = _rotate_part(x, positions[:T], cos_sin).to(dst.dtype)
-
-
 def latent_attention(out, q, pages, q_start, q_len, ctx_len, block_table, scale, window, num_seqs):
     Rp = out.shape[2]
     for s in range(num_seqs):
@@ -373,10 +366,16 @@ def latent_attention(out, q, pages, q_start, q_len, ctx_len, block_table, scale,
         out[q0:q0 + n] = torch.einsum("htk,kd->thd", p, rows[:, :Rp]).to(out.dtype)
 
 
-def head_gemm(x, x_step, w, out, out_step):
+def head_gemm(x, x_step, w, out, out_step, rot):
     N, K = w.shape[1:]
     for g in range(w.shape[0]):
-        out[:, g * out_step:g * out_step + N] = (x[:, g * x_step:g * x_step + K].float() @ w[g].float().T).to(out.dtype)
+        at = g * out_step
+        out[:, at:at + N] = (x[:, g * x_step:g * x_step + K].float() @ w[g].float().T).to(out.dtype)
+        if rot is not None:
+            pos, cs, skip, r, rp = rot
+            out[:, at + N:at + N + rp] = 0
+            v = x[:, g * x_step + skip:g * x_step + skip + r].float()
+            out[:, at + N:at + N + r] = _rotate_part(v, pos[:x.shape[0]], cs).to(out.dtype)
 
 
 def table_route(tables, desc, ids, slots, T, tm, order, tiles, n_tiles):

@@ -145,14 +145,17 @@ def test_latent_cache_and_query_rotation(gpu, dt, NQ, R, r, rd, H):
         assert not row[R:Rp].any() and not row[Rp + r:].any()
     free = [s for s in range(80) if s not in slots.tolist()]
     assert (rows[free] == 4.0).all()
-    hs = 32 + rp
-    q = torch.randn(T, H * hs, generator=g).to(dt)
-    dst = torch.full((T, H, Rp + rp), 6.0, dtype=dt, device=gpu)
-    ops.latent_qrot(q.to(gpu), hs, 32, r, dst, Rp, pos.to(gpu), cs.to(gpu))
+    # the queries' rotated part, beside their projection
+    hs, N = 32 + rp, 48
+    q, w = torch.randn(T, H * hs, generator=g).to(dt), (torch.randn(H, N, 32, generator=g) / 6).to(dt)
+    dst = torch.full((T, H, N + rp + 16), 6.0, dtype=dt, device=gpu)
+    ops.head_gemm(q.to(gpu), hs, ops.pack_groups(w, dt).to(gpu), dst.view(T, -1), N + rp + 16,
+                  rot=(pos.to(gpu), cs.to(gpu), 32, r, rp))
     d = dst.float().cpu()
-    assert (d[:, :, :Rp] == 6.0).all() and not d[:, :, Rp + r:].any()
+    assert (d[:, :, N + rp:] == 6.0).all() and not d[:, :, N + r:N + rp].any()
+    torch.testing.assert_close(d[:, :, :N], torch.einsum("thk,hnk->thn", q.float().view(T, H, hs)[:, :, :32], w.float()), **tol(dt))
     for t in range(T):
-        torch.testing.assert_close(d[t, :, Rp:Rp + r], rot(q[t].float().view(H, hs)[:, 32:32 + r], int(pos[t])), **tol(dt))
+        torch.testing.assert_close(d[t, :, N:N + r], rot(q[t].float().view(H, hs)[:, 32:32 + r], int(pos[t])), **tol(dt))
 
 
 def fed_meta(gpu, H, reqs, split_target=384, window=0, nblocks=600):
