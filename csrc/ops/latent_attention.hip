@@ -19,13 +19,13 @@
 //
 // Items come from the scheduler like paged_attention's (seq, q_begin, nq | part<<8 | nparts<<20,
 // partial slot):
-//   nq <= dec_tokens: split over keys. The 4 waves take every 4th page with a private LDS tile and
+//   nq <= dec_tokens: split over keys. The 8 waves take every 8th page with a private LDS tile and
 //                     merge; nparts > 1 divides the item's own (windowed) key range evenly, the
 //                     partials go to memory and merge_kernel, a second launch, combines them: at
 //                     16 x Rp floats a partition, one last arriver would read for longer than all
 //                     partitions compute, while the launch spreads the columns over the chip.
-//   otherwise:        64 * CT columns per workgroup, 16 * CT per wave; all waves share
-//                     double-buffered 32-key tiles that arrive by direct global -> LDS loads.
+//   otherwise:        128 columns per workgroup, 16 per wave; all waves share double-buffered 32-key
+//                     tiles that arrive by direct global -> LDS loads.
 #include "common.h"
 
 #include <algorithm>
@@ -127,6 +127,7 @@ __device__ __forceinline__ bf16x4 tr_read(const char* p) {
   return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)p);
 }
 
+constexpr int NW = 8;          // waves per workgroup: two a SIMD, one's softmax under the other's MFMAs
 constexpr int MERGE_LD = 132;  // floats per merge row of 128 dims
 
 template <int RT, int PT>
@@ -149,10 +150,12 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
   const int p_begin = p_lo + part * per, p_end = min(p_hi, p_begin + per);
   const int* bt = A.block_table + (size_t)s * A.max_blocks;
 
-  bf16x8 qf[NK];
-#pragma unroll
-  for (int m = 0; m < NK; ++m)
-    qf[m] = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + row * D + 32 * m + 8 * g);
+  // all waves share the 16 columns: their Q^T operands (1 KB per k-step) live in LDS
+  char* sq = smem + NW * (RP * 32);
+  for (int m = wid; m < NK; m += NW)
+    *reinterpret_cast<bf16x8*>(sq + m * 1024 + (g * 16 + c) * 16) =
+        *reinterpret_cast<const bf16x8*>((const bf16*)A.q + row * D + 32 * m + 8 * g);
+  __syncthreads();
   f32x4 o[2 * RT];
 #pragma unroll
   for (int n = 0; n < 2 * RT; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -168,14 +171,15 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
     for (int m = 0; m < NK; ++m) k[m] = *reinterpret_cast<const bf16x8*>(b + m * 512);
   };
   if (p_begin + wid < p_end) load(p_begin + wid, kf);
-  for (int p = p_begin + wid; p < p_end; p += 4) {
+  for (int p = p_begin + wid; p < p_end; p += NW) {
     f32x4 sc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int m = 0; m < NK; ++m) {
-      sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[m], qf[m], sc, 0, 0, 0);
+      const bf16x8 qf = *reinterpret_cast<const bf16x8*>(sq + m * 1024 + loff);
+      sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[m], qf, sc, 0, 0, 0);
       if (m < RT) *reinterpret_cast<bf16x8*>(my + m * 1024 + loff) = kf[m];
     }
-    if (p + 4 < p_end) load(p + 4, kf);
+    if (p + NW < p_end) load(p + NW, kf);
     float tmax = NEG_BIG;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -212,59 +216,51 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
   l_run += __shfl_xor(l_run, 32, 64);
 
   // merge the waves, 128 dims at a time
-  float* mo = reinterpret_cast<float*>(smem);                                // [4][16][MERGE_LD]
-  float* mm = reinterpret_cast<float*>(smem + 4 * 16 * MERGE_LD * 4);        // [4][16]
-  float* ml = mm + 64;
+  float* mo = reinterpret_cast<float*>(smem);                           // [NW][16][MERGE_LD]
+  float* mm = reinterpret_cast<float*>(smem + NW * 16 * MERGE_LD * 4);  // [NW][16]
+  float* ml = mm + NW * 16;
   __syncthreads();
   if (g == 0) {
     mm[wid * 16 + c] = m_run;
     ml[wid * 16 + c] = l_run;
   }
-  const int ccol = threadIdx.x >> 4, d8 = (threadIdx.x & 15) * 8;
+  const int ccol = threadIdx.x >> 5, d4 = (threadIdx.x & 31) * 4;
   const bool cvalid = cb * 16 + ccol < cols;
-  float wgt[4], L = 0.f, mt = NEG_BIG;
+  float wgt[NW], L = 0.f, mt = NEG_BIG;
 #pragma unroll
   for (int nb = 0; nb < (RT + 3) / 4; ++nb) {
     if (nb) __syncthreads();
 #pragma unroll
     for (int n = 0; n < 8; ++n)
-      if (nb * 8 + n < 2 * RT)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) mo[(wid * 16 + c) * MERGE_LD + 16 * n + 4 * g + r] = o[nb * 8 + n][r];
+      if (nb * 8 + n < 2 * RT) *reinterpret_cast<f32x4*>(mo + (wid * 16 + c) * MERGE_LD + 16 * n + 4 * g) = o[nb * 8 + n];
     __syncthreads();
     if (nb == 0) {
 #pragma unroll
-      for (int w = 0; w < 4; ++w) mt = fmaxf(mt, mm[w * 16 + ccol]);
+      for (int w = 0; w < NW; ++w) mt = fmaxf(mt, mm[w * 16 + ccol]);
 #pragma unroll
-      for (int w = 0; w < 4; ++w) {
+      for (int w = 0; w < NW; ++w) {
         wgt[w] = exp2f(mm[w * 16 + ccol] - mt);
         L += wgt[w] * ml[w * 16 + ccol];
       }
     }
-    const int d0 = nb * 128 + d8;
+    const int d0 = nb * 128 + d4;
     if (d0 < RP) {
-      float acc[8];
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        float a = 0.f;
-#pragma unroll
-        for (int w = 0; w < 4; ++w) a += wgt[w] * mo[(w * 16 + ccol) * MERGE_LD + d8 + j];
-        acc[j] = a;
-      }
+      for (int w = 0; w < NW; ++w)
+        acc += wgt[w] * *reinterpret_cast<const f32x4*>(mo + (w * 16 + ccol) * MERGE_LD + d4);
       if (nparts > 1) {
-        f32x4* ps = reinterpret_cast<f32x4*>(A.part_o + (((size_t)pidx * A.NB + cb) * 16 + ccol) * RP + d0);
-        ps[0] = f32x4{acc[0], acc[1], acc[2], acc[3]};
-        ps[1] = f32x4{acc[4], acc[5], acc[6], acc[7]};
+        *reinterpret_cast<f32x4*>(A.part_o + (((size_t)pidx * A.NB + cb) * 16 + ccol) * RP + d0) = acc;
       } else if (cvalid) {
         const float inv = 1.f / L;
-        bf16x8 v;
+        bf16x4 v;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) v[j] = (bf16)(acc[j] * inv);
-        *reinterpret_cast<bf16x8*>((bf16*)A.out + (row0 + ccol) * RP + d0) = v;
+        for (int j = 0; j < 4; ++j) v[j] = (bf16)(acc[j] * inv);
+        *reinterpret_cast<bf16x4*>((bf16*)A.out + (row0 + ccol) * RP + d0) = v;
       }
     }
   }
-  if (nparts > 1 && (threadIdx.x & 15) == 0)
+  if (nparts > 1 && (threadIdx.x & 31) == 0)
     reinterpret_cast<float2*>(A.part_ml)[((size_t)pidx * A.NB + cb) * 16 + ccol] = float2{mt, L};
 }
 
@@ -333,7 +329,7 @@ template <int RT, int PT, int CT>
 __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* smem) {
   constexpr int NK = RT + PT, D = 32 * NK, RP = 32 * RT, TILE = 32 * D * 2;
   const int s = it.x, qb = it.y, nq = it.z & 0xff;
-  const int cols = nq * A.H, cw = blockIdx.x * (64 * CT);
+  const int cols = nq * A.H, cw = blockIdx.x * (16 * NW * CT);
   if (cw >= cols) return;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
   const int ctx = A.ctx_len[s], ql = A.q_len[s];
@@ -353,7 +349,7 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
       qf[t][m] = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + (row0 + cc) * D + 32 * m + 8 * g);
   }
   // positions of the workgroup's columns -> its key tiles
-  const int f = pos0 + cw / A.H, e = pos0 + min(cw + 64 * CT - 1, cols - 1) / A.H;
+  const int f = pos0 + cw / A.H, e = pos0 + min(cw + 16 * NW * CT - 1, cols - 1) / A.H;
   const int t_lo = (A.window > 0 ? max(0, f - A.window + 1) : 0) >> 5, t_hi = (e + 32) >> 5;
   const int nblk = (ctx + 15) >> 4;
   // this wave's columns: keys below all of their windows' starts / above all positions are masked
@@ -375,16 +371,14 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
   }
   // direct loads: the tile is two whole pages, copied linearly, 1 KB per wave and instruction
   auto issue = [&](int t, char* dst) {
+    const bf16* src0 = (const bf16*)A.pages + (size_t)bt[min(2 * t, nblk - 1)] * (D * 16) + lane * 8;
+    const bf16* src1 = (const bf16*)A.pages + (size_t)bt[min(2 * t + 1, nblk - 1)] * (D * 16) + lane * 8;
 #pragma unroll
-    for (int pg = 0; pg < 2; ++pg) {
-      const bf16* src = (const bf16*)A.pages + (size_t)bt[min(2 * t + pg, nblk - 1)] * (D * 16) + lane * 8;
-#pragma unroll
-      for (int i = 0; i < (NK + 3) / 4; ++i) {
-        const int ch = i * 4 + wid;  // wave-uniform
-        if (NK % 4 == 0 || ch < NK)
-          __builtin_amdgcn_global_load_lds((glb_void*)(src + ch * 512), (lds_void*)(dst + pg * (D * 32) + ch * 1024),
-                                           16, 0, 0);
-      }
+    for (int i = 0; i < (2 * NK + NW - 1) / NW; ++i) {
+      const int ch = i * NW + wid;  // wave-uniform
+      if (2 * NK % NW == 0 || ch < 2 * NK)
+        __builtin_amdgcn_global_load_lds((glb_void*)((ch < NK ? src0 : src1 - NK * 512) + ch * 512),
+                                         (lds_void*)(dst + ch * 1024), 16, 0, 0);
     }
   };
   const int loff = (g * 16 + c) * 16;
@@ -480,11 +474,12 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
 
 template <int RT, int PT>
 constexpr int lds_bytes() {
-  return std::max({2 * 32 * 32 * (RT + PT) * 2, 4 * 16 * 32 * RT * 2, 4 * 16 * MERGE_LD * 4 + 2 * 64 * 4 + 16});
+  return std::max({2 * 32 * 32 * (RT + PT) * 2, NW * 32 * 32 * RT + 1024 * (RT + PT),
+                   NW * 16 * MERGE_LD * 4 + 2 * NW * 16 * 4});
 }
 
 template <int RT, int PT, int CT>
-__global__ __launch_bounds__(256, RT <= 8 ? 2 : 1) void mfma_kernel(const Args A) {
+__global__ __launch_bounds__(64 * NW, 2) void mfma_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int n = A.n_items[0];
   for (int item = blockIdx.y; item < n; item += gridDim.y) {
@@ -523,7 +518,7 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
   if (!fp32 && !simple && PT >= 1 && PT <= 2) {
 #define PA_LA(R, P)                                                                                           \
   do {                                                                                                        \
-    constexpr int CT = R <= 8 ? 2 : 1;                                                                        \
+    constexpr int CT = 1;                                                                                     \
     constexpr int lds = pa::la::lds_bytes<R, P>();                                                            \
     static bool attr = false;                                                                                 \
     if (!attr) {                                                                                              \
@@ -531,10 +526,10 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
                                 hipFuncAttributeMaxDynamicSharedMemorySize, lds);                             \
       attr = true;                                                                                            \
     }                                                                                                         \
-    const int gt = (tile_tokens * H + 64 * CT - 1) / (64 * CT), gx = NB > gt ? NB : gt;                       \
+    const int cw = 16 * pa::la::NW * CT, gt = (tile_tokens * H + cw - 1) / cw, gx = NB > gt ? NB : gt;                       \
     /* items are strided over the grid: at least one workgroup per CU */                                      \
     const int gy = max_items < 256 ? 256 : (max_items < 4096 ? max_items : 4096);                             \
-    hipLaunchKernelGGL((pa::la::mfma_kernel<R, P, CT>), dim3(gx, gy), dim3(256), lds, st, A);                 \
+    hipLaunchKernelGGL((pa::la::mfma_kernel<R, P, CT>), dim3(gx, gy), dim3(64 * pa::la::NW), lds, st, A);     \
     hipLaunchKernelGGL((pa::la::merge_kernel<R>), dim3(4 * NB, gy), dim3(256), 0, st, A);                     \
     return (int)hipGetLastError();                                                                            \
   } while (0)
