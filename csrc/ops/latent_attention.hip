@@ -25,7 +25,8 @@
 //                     16 x Rp floats a partition, one last arriver would read for longer than all
 //                     partitions compute, while the launch spreads the columns over the chip.
 //   otherwise:        128 columns per workgroup, 16 per wave; all waves share double-buffered 32-key
-//                     tiles that arrive by direct global -> LDS loads.
+//                     tiles that arrive by direct global -> LDS loads. A step with few such items
+//                     has them cut into partitions of their keys too (8 slots each).
 #include "common.h"
 
 #include <algorithm>
@@ -45,8 +46,9 @@ struct Args {
   float* part_ml;        // [slots, NB, 16, 2]
   const void* q;         // [T, H, D]
   const void* pages;
-  const int4* items;
+  const int4* items;  // at least max_items; more are in the buffer when n_items says so
   const int* n_items;
+  int max_items;
   const int *q_start, *q_len, *ctx_len, *block_table;
   int max_blocks, H, NB, Rp, D, dec_tokens, window;
   float scale_log2;
@@ -264,62 +266,65 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
     reinterpret_cast<float2*>(A.part_ml)[((size_t)pidx * A.NB + cb) * 16 + ccol] = float2{mt, L};
 }
 
-// The partitions of split items, merged: a wave per (item, column), 8 dims per lane and step.
+// The partitions of an item, merged: a wave per (item, column), 8 dims per lane and step.
 template <int RT>
 __global__ __launch_bounds__(256) void merge_kernel(const Args A) {
   constexpr int RP = 32 * RT;
-  const int col = blockIdx.x * 4 + (threadIdx.x >> 6), cb = col >> 4, cc = col & 15, lane = threadIdx.x & 63;
+  const int lane = threadIdx.x & 63;
   const int n = A.n_items[0];
   for (int item = blockIdx.y; item < n; item += gridDim.y) {
     const int4 it = A.items[item];
     const int nq = it.z & 0xff, nparts = it.z >> 20;
-    if (nq > A.dec_tokens || nparts <= 1 || ((it.z >> 8) & 0xfff) != 0 || col >= nq * A.H) continue;
-    auto slot = [&](int p) { return ((size_t)(it.w + p) * A.NB + cb) * 16 + cc; };
-    const float2* ml = reinterpret_cast<const float2*>(A.part_ml);
-    // lane p holds partition p's weight (64 at a time): the loads of a round are independent
-    float gm = NEG_BIG, L = 0.f;
-    for (int p0 = 0; p0 < nparts; p0 += 64) gm = fmaxf(gm, p0 + lane < nparts ? ml[slot(p0 + lane)].x : NEG_BIG);
-    gm = wave_max(gm);
-    float a[(RP + 511) / 512][8];
+    if (nparts <= 1 || ((it.z >> 8) & 0xfff) != 0) continue;
+    const int step = nq <= A.dec_tokens ? 1 : 8;  // slots of a partition
+    for (int col = blockIdx.x * 4 + (threadIdx.x >> 6); col < nq * A.H; col += gridDim.x * 4) {
+      auto slot = [&](int p) { return (size_t)(it.w + p * step) * A.NB * 16 + col; };
+      const float2* ml = reinterpret_cast<const float2*>(A.part_ml);
+      // lane p holds partition p's weight (64 at a time): the loads of a round are independent
+      float gm = NEG_BIG, L = 0.f;
+      for (int p0 = 0; p0 < nparts; p0 += 64) gm = fmaxf(gm, p0 + lane < nparts ? ml[slot(p0 + lane)].x : NEG_BIG);
+      gm = wave_max(gm);
+      float a[(RP + 511) / 512][8];
 #pragma unroll
-    for (int e = 0; e < (RP + 511) / 512; ++e)
+      for (int e = 0; e < (RP + 511) / 512; ++e)
 #pragma unroll
-      for (int j = 0; j < 8; ++j) a[e][j] = 0.f;
-    for (int p0 = 0; p0 < nparts; p0 += 64) {
-      float w = 0.f;
-      if (p0 + lane < nparts) {
-        const float2 v = ml[slot(p0 + lane)];
-        w = exp2f(v.x - gm);
-        L += w * v.y;
-      }
-      const int np = min(64, nparts - p0);
+        for (int j = 0; j < 8; ++j) a[e][j] = 0.f;
+      for (int p0 = 0; p0 < nparts; p0 += 64) {
+        float w = 0.f;
+        if (p0 + lane < nparts) {
+          const float2 v = ml[slot(p0 + lane)];
+          w = exp2f(v.x - gm);
+          L += w * v.y;
+        }
+        const int np = min(64, nparts - p0);
 #pragma unroll 8
-      for (int p = 0; p < np; ++p) {
-        const float wp = __shfl(w, p, 64);
+        for (int p = 0; p < np; ++p) {
+          const float wp = __shfl(w, p, 64);
 #pragma unroll
-        for (int e = 0; e < (RP + 511) / 512; ++e) {
-          const int d = min(e * 512 + lane * 8, RP - 8);
-          const f32x4* s = reinterpret_cast<const f32x4*>(A.part_o + slot(p0 + p) * RP + d);
-          const f32x4 x = s[0], y = s[1];
+          for (int e = 0; e < (RP + 511) / 512; ++e) {
+            const int d = min(e * 512 + lane * 8, RP - 8);
+            const f32x4* s = reinterpret_cast<const f32x4*>(A.part_o + slot(p0 + p) * RP + d);
+            const f32x4 x = s[0], y = s[1];
 #pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            a[e][j] += wp * x[j];
-            a[e][4 + j] += wp * y[j];
+            for (int j = 0; j < 4; ++j) {
+              a[e][j] += wp * x[j];
+              a[e][4 + j] += wp * y[j];
+            }
           }
         }
       }
-    }
-    L = wave_sum(L);
-    const float inv = 1.f / L;
-    bf16* o = (bf16*)A.out + ((size_t)(A.q_start[it.x] + it.y) * A.H + col) * RP;
+      L = wave_sum(L);
+      const float inv = 1.f / L;
+      bf16* o = (bf16*)A.out + ((size_t)(A.q_start[it.x] + it.y) * A.H + col) * RP;
 #pragma unroll
-    for (int e = 0; e < (RP + 511) / 512; ++e) {
-      const int d = e * 512 + lane * 8;
-      if (d < RP) {
-        bf16x8 v;
+      for (int e = 0; e < (RP + 511) / 512; ++e) {
+        const int d = e * 512 + lane * 8;
+        if (d < RP) {
+          bf16x8 v;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) v[j] = (bf16)(a[e][j] * inv);
-        *reinterpret_cast<bf16x8*>(o + d) = v;
+          for (int j = 0; j < 8; ++j) v[j] = (bf16)(a[e][j] * inv);
+          *reinterpret_cast<bf16x8*>(o + d) = v;
+        }
       }
     }
   }
@@ -328,7 +333,7 @@ __global__ __launch_bounds__(256) void merge_kernel(const Args A) {
 template <int RT, int PT, int CT>
 __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* smem) {
   constexpr int NK = RT + PT, D = 32 * NK, RP = 32 * RT, TILE = 32 * D * 2;
-  const int s = it.x, qb = it.y, nq = it.z & 0xff;
+  const int s = it.x, qb = it.y, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff, nparts = it.z >> 20;
   const int cols = nq * A.H, cw = blockIdx.x * (16 * NW * CT);
   if (cw >= cols) return;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
@@ -350,7 +355,12 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
   }
   // positions of the workgroup's columns -> its key tiles
   const int f = pos0 + cw / A.H, e = pos0 + min(cw + 16 * NW * CT - 1, cols - 1) / A.H;
-  const int t_lo = (A.window > 0 ? max(0, f - A.window + 1) : 0) >> 5, t_hi = (e + 32) >> 5;
+  int t_lo = (A.window > 0 ? max(0, f - A.window + 1) : 0) >> 5, t_hi = (e + 32) >> 5;
+  if (nparts > 1) {  // this partition's tiles (possibly none)
+    const int per = (t_hi - t_lo + nparts - 1) / nparts;
+    t_lo += part * per;
+    t_hi = min(t_hi, t_lo + per);
+  }
   const int nblk = (ctx + 15) >> 4;
   // this wave's columns: keys below all of their windows' starts / above all positions are masked
   // (t needs no mask when every column sees all its 32 keys)
@@ -383,7 +393,7 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
   };
   const int loff = (g * 16 + c) * 16;
   const int toff = ((c & 3) >> 1) * 256 + (4 * g + (c >> 2)) * 16 + (c & 1) * 8;
-  issue(t_lo, smem);
+  if (t_lo < t_hi) issue(t_lo, smem);
   for (int t = t_lo; t < t_hi; ++t) {
     char* cur = smem + ((t - t_lo) & 1) * TILE;
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
@@ -460,6 +470,14 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
     if (ci[x] >= cols) continue;
+    if (nparts > 1) {  // 8 slots hold the item's columns in a row
+      const size_t pc = (size_t)it.w * A.NB * 16 + ci[x];
+      float* po = A.part_o + pc * RP + 4 * g;
+#pragma unroll
+      for (int n = 0; n < 2 * RT; ++n) *reinterpret_cast<f32x4*>(po + 16 * n) = o[x][n];
+      if (g == 0) reinterpret_cast<float2*>(A.part_ml)[pc] = float2{m_run[x], l};
+      continue;
+    }
     const float inv = 1.f / l;
     bf16* orow = (bf16*)A.out + (row0 + ci[x]) * RP + 4 * g;
 #pragma unroll
@@ -481,9 +499,11 @@ constexpr int lds_bytes() {
 template <int RT, int PT, int CT>
 __global__ __launch_bounds__(64 * NW, 2) void mfma_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
+  // the first item is loaded beside the count, not after it
   const int n = A.n_items[0];
+  int4 it = A.items[min((int)blockIdx.y, A.max_items - 1)];
   for (int item = blockIdx.y; item < n; item += gridDim.y) {
-    const int4 it = A.items[item];
+    if (item != (int)blockIdx.y || item >= A.max_items) it = A.items[item];
     if ((it.z & 0xff) <= A.dec_tokens) split_item<RT, PT>(A, it, smem);
     else tile_item<RT, PT, CT>(A, it, smem);
     __syncthreads();
@@ -512,7 +532,7 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
   if (max_items <= 0) return 0;
   const int D = Rp + rp, NB = (dec_tokens * H + 15) / 16;
   if (Rp % 32 || rp % 32 || H <= 0 || dec_tokens <= 0 || tile_tokens <= 0) return -1;
-  pa::la::Args A{out, part_o, part_ml, q, pages, (const int4*)items, n_items, q_start, q_len, ctx_len,
+  pa::la::Args A{out, part_o, part_ml, q, pages, (const int4*)items, n_items, max_items, q_start, q_len, ctx_len,
                  block_table, max_blocks, H, NB, Rp, D, dec_tokens, window, scale_log2};
   const int RT = Rp / 32, PT = rp / 32;
   if (!fp32 && !simple && PT >= 1 && PT <= 2) {
@@ -530,7 +550,7 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
     /* items are strided over the grid: at least one workgroup per CU */                                      \
     const int gy = max_items < 256 ? 256 : (max_items < 4096 ? max_items : 4096);                             \
     hipLaunchKernelGGL((pa::la::mfma_kernel<R, P, CT>), dim3(gx, gy), dim3(64 * pa::la::NW), lds, st, A);     \
-    hipLaunchKernelGGL((pa::la::merge_kernel<R>), dim3(4 * NB, gy), dim3(256), 0, st, A);                     \
+    hipLaunchKernelGGL((pa::la::merge_kernel<R>), dim3(NB > 8 ? 4 * NB : 32, gy), dim3(256), 0, st, A);       \
     return (int)hipGetLastError();                                                                            \
   } while (0)
     switch (RT) {

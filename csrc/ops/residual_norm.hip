@@ -33,6 +33,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(
       float v[VEC];
 #pragma unroll
       for (int j = 0; j < VEC; ++j) v[j] = 0.f;
+#pragma unroll 4
       for (int k = 0; k < K; ++k) {
         T a[VEC];
         __builtin_memcpy(a, __builtin_assume_aligned(yr + (size_t)k * ldy + i, sizeof(T) * VEC), sizeof(T) * VEC);
@@ -96,7 +97,7 @@ extern "C" int pa_residual_norm(int fp32, float* resid, const void* y, int K, in
                                 hipStream_t st) {
   if (n <= 0) return 0;
   if (D <= 0 || D * 4 > 96 * 1024) return -1;  // the row in LDS
-  const bool vec = D % 4 == 0 && ldy % 4 == 0 && ldo % 4 == 0;
+  const bool vec = D % 8 == 0 && ldy % 8 == 0 && ldo % 8 == 0;
 #define PA_RN(T, V)                                                                                        \
   do {                                                                                                     \
     static bool attr = false;                                                                              \
@@ -110,9 +111,9 @@ extern "C" int pa_residual_norm(int fp32, float* resid, const void* y, int K, in
                        (T*)out, ldo, rows, D, eps);                                                        \
   } while (0)
   if (fp32) {
-    if (vec) PA_RN(float, 4); else PA_RN(float, 1);
+    if (vec) PA_RN(float, 8); else PA_RN(float, 1);
   } else {
-    if (vec) PA_RN(pa::bf16, 4); else PA_RN(pa::bf16, 1);
+    if (vec) PA_RN(pa::bf16, 8); else PA_RN(pa::bf16, 1);
   }
 #undef PA_RN
   return (int)hipGetLastError();

@@ -154,6 +154,8 @@ PYBIND11_MODULE(_runtime, m) {
         if (d.contains("gqa_group")) c.gqa_group = d["gqa_group"].cast<int32_t>();
         if (d.contains("att_qcols")) c.att_qcols = d["att_qcols"].cast<int32_t>();
         if (d.contains("att_narrow_qcols")) c.att_narrow_qcols = d["att_narrow_qcols"].cast<int32_t>();
+        if (d.contains("att_min_part")) c.att_min_part = d["att_min_part"].cast<int32_t>();
+        if (d.contains("att_tile_target")) c.att_tile_target = d["att_tile_target"].cast<int32_t>();
         if (d.contains("att_max_keys")) c.att_max_keys = d["att_max_keys"].cast<int32_t>();
         if (d.contains("att_wide_min_tokens")) c.att_wide_min_tokens = d["att_wide_min_tokens"].cast<int32_t>();
         if (d.contains("prefill_split_keys")) c.prefill_split_keys = d["prefill_split_keys"].cast<int32_t>();

@@ -440,10 +440,10 @@ int32_t Scheduler::emit(int32_t* buf) {
         const int64_t share = ((sumc * kv + tgt - 1) / tgt + 31) / 32 * 32;
         int64_t cand;
         if (ndec * kv >= tgt) {
-          cand = std::max<int64_t>(32, std::min(maxc, std::max<int64_t>(share, 128)));
+          cand = std::max<int64_t>(32, std::min(maxc, std::max<int64_t>(share, cfg_.att_min_part)));
         } else {
           const int64_t np = (tgt + ndec * kv - 1) / (ndec * kv);
-          cand = std::max<int64_t>(128, std::min(((maxc + np - 1) / np + 31) / 32 * 32, share));
+          cand = std::max<int64_t>(cfg_.att_min_part, std::min(((maxc + np - 1) / np + 31) / 32 * 32, share));
         }
         int64_t parts = 0;
         for (const Planned& p : last_plan_)
@@ -540,6 +540,25 @@ int32_t Scheduler::emit(int32_t* buf) {
   int32_t t_step_all = 0;
   for (const Planned& p : last_plan_) t_step_all += p.n;
   const int32_t G = std::max(1, cfg_.gqa_group);
+  if (cfg_.att_tile_target > 0 && !pre.empty() && (int32_t)pre.size() * 2 <= cfg_.att_tile_target) {
+    const int32_t want = std::min<int32_t>(16, cfg_.att_tile_target / (int32_t)pre.size());
+    std::vector<ItemCost> split;
+    int64_t total = (int64_t)pre.size() + (int64_t)dec.size();
+    for (const ItemCost& c : pre) {
+      const int32_t nq = c.c & 0xff;
+      const int32_t keys = cfg_.att_max_keys > 0 ? std::min(c.keys, cfg_.att_max_keys + nq - 1) : c.keys;
+      const int32_t np = std::min(want, keys / 256);
+      if (np >= 2 && pslot + 8 * np <= L.max_items && total + np - 1 <= L.max_items) {
+        for (int32_t q = 0; q < np; ++q)
+          split.push_back({keys / np, c.a, c.b, nq | (q << 8) | (np << 20), pslot + 8 * q});
+        pslot += 8 * np;
+        total += np - 1;
+      } else {
+        split.push_back(c);
+      }
+    }
+    pre.swap(split);
+  }
   if (cfg_.prefill_split_keys > 0 && qtile * G > cfg_.att_narrow_qcols && t_step_all > cfg_.small_step_tokens) {
     std::vector<ItemCost> split;
     int64_t n_items_total = (int64_t)pre.size() + (int64_t)dec.size();

@@ -38,6 +38,10 @@ struct SchedulerConfig {
   // > 0: no layer attends to more than this many keys back (every layer has a window): decode rows
   // are cut into partitions of the keys they really read, not of the whole context
   int32_t att_max_keys = 0;
+  int32_t att_min_part = 128;          // smallest decode partition (keys)
+  // > 0: a step with fewer prefill items than this cuts each over its keys, at least 256 a partition,
+  // towards this many work items (kernels whose tile path merges partitions; 8 partial slots each)
+  int32_t att_tile_target = 0;
   int32_t att_wide_min_tokens = 2048;
   // wide prefill items whose causal key range reaches this many keys are cut into
   // min(4, keys / prefill_split_keys) partitions of whole 32-key tiles, merged in-kernel by the

@@ -392,7 +392,7 @@ class BozupelModel:
     def attention_items(self) -> dict:
         windows = [L.mixer.window for L in self.cfg.layers]
         return {"gqa_group": self._group, "kv_heads": 1, "att_qcols": 128, "att_narrow_qcols": 128,
-                "prefill_split_keys": 0, "decode_part_target": 256, "att_max_keys": max(windows) if all(windows) else 0}
+                "prefill_split_keys": 0, "decode_part_target": 256, "att_min_part": 256, "att_tile_target": 256, "att_max_keys": max(windows) if all(windows) else 0}
 
     ATT_HANDOFF = False  # partials are merged by a launch of their own: ordinary memory
 

@@ -158,7 +158,7 @@ def test_latent_cache_and_query_rotation(gpu, dt, NQ, R, r, rd, H):
         torch.testing.assert_close(d[t, :, N:N + r], rot(q[t].float().view(H, hs)[:, 32:32 + r], int(pos[t])), **tol(dt))
 
 
-def fed_meta(gpu, H, reqs, split_target=384, window=0, nblocks=600):
+def fed_meta(gpu, H, reqs, split_target=384, window=0, nblocks=600, part=128, tiles=0):
     """Scheduler-built step: reqs [(cached tokens, new tokens)]; pages in scrambled order."""
     from pilottai_amd import _runtime
 
@@ -166,7 +166,7 @@ def fed_meta(gpu, H, reqs, split_target=384, window=0, nblocks=600):
     s = _runtime.Scheduler({"num_blocks": nblocks, "block_size": 16, "max_num_seqs": 16, "max_num_batched_tokens": 4096,
                             "max_model_len": 4096, "gqa_group": group, "kv_heads": 1, "att_qcols": 128,
                             "att_narrow_qcols": 128, "prefix_caching": False, "decode_part_target": split_target,
-                            "att_max_keys": window})
+                            "att_max_keys": window, "att_min_part": part, "att_tile_target": tiles})
     L = s.layout()
     buf = np.zeros(L["total"], dtype=np.int32)
     junk = [(1000 + i, [1] * (16 * (1 + i % 3))) for i in range(8)]  # fragment the pool first
@@ -190,14 +190,14 @@ def fed_meta(gpu, H, reqs, split_target=384, window=0, nblocks=600):
     return T, m, 16 // group, 128 // group
 
 
-def run_attention(gpu, dt, H, R, r, reqs, window, simple=False, split_target=384, seed=0, spike=None):
+def run_attention(gpu, dt, H, R, r, reqs, window, simple=False, split_target=384, seed=0, spike=None, **kw):
     from pilottai_amd import ops
     from pilottai_amd.ops.latent import latent_pad, pad_to
 
     g = torch.Generator().manual_seed(seed)
     Rp, rp = latent_pad(R), pad_to(r, 32)
     D = Rp + rp
-    T, m, dec, tile = fed_meta(gpu, H, reqs, split_target, window)
+    T, m, dec, tile = fed_meta(gpu, H, reqs, split_target, window, **kw)
     pages = torch.randn(600, D // 8, 16, 8, generator=g).to(dt)
     pages[:, R // 8:Rp // 8] = 0
     q = (torch.randn(T, H, D, generator=g) * 2).to(dt)
@@ -232,6 +232,13 @@ STEPS = {"prompt": [(0, 75)], "decode": [(0, 1), (15, 1), (16, 1), (700, 1), (33
 @pytest.mark.parametrize("H,R,r", SHAPES)
 def test_latent_attention_bf16(gpu, H, R, r, step, window):
     run_attention(gpu, torch.bfloat16, H, R, r, STEPS[step], window)
+
+
+@pytest.mark.parametrize("window", [0, 45, 600])
+@pytest.mark.parametrize("H,R,r", SHAPES)
+def test_latent_attention_split_tiles(gpu, H, R, r, window):
+    """Prompt portions cut over their keys: partitions of one item meet in the merge launch."""
+    run_attention(gpu, torch.bfloat16, H, R, r, [(1500, 40), (900, 1), (0, 20), (700, 3)], window, tiles=64, part=256)
 
 
 @pytest.mark.parametrize("dt", DTYPES)
