@@ -550,7 +550,7 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
     /* items are strided over the grid: at least one workgroup per CU */                                      \
     const int gy = max_items < 256 ? 256 : (max_items < 4096 ? max_items : 4096);                             \
     hipLaunchKernelGGL((pa::la::mfma_kernel<R, P, CT>), dim3(gx, gy), dim3(64 * pa::la::NW), lds, st, A);     \
-    hipLaunchKernelGGL((pa::la::merge_kernel<R>), dim3(NB > 8 ? 4 * NB : 32, gy), dim3(256), 0, st, A);       \
+    hipLaunchKernelGGL((pa::la::merge_kernel<R>), dim3(16, std::min(gy, 256)), dim3(256), 0, st, A);           \
     return (int)hipGetLastError();                                                                            \
   } while (0)
     switch (RT) {
