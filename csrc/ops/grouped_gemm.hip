@@ -47,17 +47,21 @@ struct Args {
 template <typename T>
 __device__ __forceinline__ void rotate_rows(const Args& A, int grp, int start, int n) {
   const int half = A.rd >> 1, N = A.N16 * 16;
-  for (int e = threadIdx.x; e < n * A.rp; e += 256) {
-    const int t = start + e / A.rp, j = e % A.rp;
-    const T* src = (const T*)A.x + (size_t)t * A.ldx + (size_t)grp * A.xg + A.rskip;
-    float v = 0.f;
-    if (j < A.r) {
-      v = (float)src[j];
-      const float* cs = A.cos_sin + (size_t)A.positions[t] * A.rd;
-      if (j < half) v = v * cs[j] - (float)src[j + half] * cs[half + j];
-      else if (j < A.rd) v = v * cs[j - half] + (float)src[j - half] * cs[j];
+  const int per = max(1, 256 / A.rp), i0 = threadIdx.x / A.rp;  // rows at a time
+  for (int j = threadIdx.x % A.rp; j < A.rp && i0 < per; j += 256) {
+#pragma unroll 4
+    for (int i = i0; i < n; i += per) {
+      const int t = start + i;
+      const T* src = (const T*)A.x + (size_t)t * A.ldx + (size_t)grp * A.xg + A.rskip;
+      float v = 0.f;
+      if (j < A.r) {
+        v = (float)src[j];
+        const float* cs = A.cos_sin + (size_t)A.positions[t] * A.rd;
+        if (j < half) v = v * cs[j] - (float)src[j + half] * cs[half + j];
+        else if (j < A.rd) v = v * cs[j - half] + (float)src[j - half] * cs[j];
+      }
+      ((T*)A.out)[(size_t)t * A.ldo + (size_t)grp * A.og + N + j] = (T)v;
     }
-    ((T*)A.out)[(size_t)t * A.ldo + (size_t)grp * A.og + N + j] = (T)v;
   }
 }
 
@@ -81,11 +85,11 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
     start = blockIdx.y * (16 * MT);
     n = min(16 * MT, A.rows - start);
   }
-  if (A.rp && blockIdx.x == gridDim.x - 1) {
+  if (A.rp && blockIdx.x == 0) {
     rotate_rows<bf16>(A, grp, start, n);
     return;
   }
-  const int nt0 = (blockIdx.x * 4 + wid) * NT;
+  const int nt0 = (((int)blockIdx.x - (A.rp ? 1 : 0)) * 4 + wid) * NT;
   if (nt0 >= A.N16) return;
   const bf16* wp = (const bf16*)A.w + (size_t)grp * A.wstride + lane * 8;
   const bf16* wt[NT];
@@ -179,12 +183,13 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const Args A) {
     start = blockIdx.y * TM;
     n = min(TM, A.rows - start);
   }
-  if (A.rp && blockIdx.x == gridDim.x - 1) {
+  if (A.rp && blockIdx.x == 0) {
     rotate_rows<float>(A, grp, start, n);
     return;
   }
+  const int bx = (int)blockIdx.x - (A.rp ? 1 : 0);
   const int K = A.K32 * 32;
-  const float* wg = (const float*)A.w + (size_t)grp * A.wstride + (size_t)blockIdx.x * (GLU ? 32 : 16) * K;
+  const float* wg = (const float*)A.w + (size_t)grp * A.wstride + (size_t)bx * (GLU ? 32 : 16) * K;
   float a0 = 0.f, a1 = 0.f;
   for (int k0 = 0; k0 < K; k0 += 32) {
     __syncthreads();
@@ -206,7 +211,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const Args A) {
   if (tm >= n) return;
   const int p = start + tm;
   const int orow = (A.tiles && A.out_order) ? A.order[p] : p;
-  float* o = (float*)A.out + (size_t)orow * A.ldo + (A.tiles ? 0 : (size_t)grp * A.og) + blockIdx.x * 16 + tn;
+  float* o = (float*)A.out + (size_t)orow * A.ldo + (A.tiles ? 0 : (size_t)grp * A.og) + bx * 16 + tn;
   *o = GLU ? glu(a0, a1, A) : a0;
 }
 

@@ -46,9 +46,8 @@ struct Args {
   float* part_ml;        // [slots, NB, 16, 2]
   const void* q;         // [T, H, D]
   const void* pages;
-  const int4* items;  // at least max_items; more are in the buffer when n_items says so
+  const int4* items;
   const int* n_items;
-  int max_items;
   const int *q_start, *q_len, *ctx_len, *block_table;
   int max_blocks, H, NB, Rp, D, dec_tokens, window;
   float scale_log2;
@@ -499,11 +498,9 @@ constexpr int lds_bytes() {
 template <int RT, int PT, int CT>
 __global__ __launch_bounds__(64 * NW, 2) void mfma_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  // the first item is loaded beside the count, not after it
   const int n = A.n_items[0];
-  int4 it = A.items[min((int)blockIdx.y, A.max_items - 1)];
   for (int item = blockIdx.y; item < n; item += gridDim.y) {
-    if (item != (int)blockIdx.y || item >= A.max_items) it = A.items[item];
+    const int4 it = A.items[item];
     if ((it.z & 0xff) <= A.dec_tokens) split_item<RT, PT>(A, it, smem);
     else tile_item<RT, PT, CT>(A, it, smem);
     __syncthreads();
@@ -532,7 +529,7 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
   if (max_items <= 0) return 0;
   const int D = Rp + rp, NB = (dec_tokens * H + 15) / 16;
   if (Rp % 32 || rp % 32 || H <= 0 || dec_tokens <= 0 || tile_tokens <= 0) return -1;
-  pa::la::Args A{out, part_o, part_ml, q, pages, (const int4*)items, n_items, max_items, q_start, q_len, ctx_len,
+  pa::la::Args A{out, part_o, part_ml, q, pages, (const int4*)items, n_items, q_start, q_len, ctx_len,
                  block_table, max_blocks, H, NB, Rp, D, dec_tokens, window, scale_log2};
   const int RT = Rp / 32, PT = rp / 32;
   if (!fp32 && !simple && PT >= 1 && PT <= 2) {
