@@ -171,8 +171,12 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
 #pragma unroll
     for (int m = 0; m < NK; ++m) k[m] = *reinterpret_cast<const bf16x8*>(b + m * 512);
   };
-  if (p_begin + wid < p_end) load(p_begin + wid, kf);
+  // the widest latents load a page when they need it: its next page does not fit the registers
+  // beside the outputs, and the SIMD's other wave computes meanwhile
+  constexpr bool AHEAD = RT < 16;
+  if (AHEAD && p_begin + wid < p_end) load(p_begin + wid, kf);
   for (int p = p_begin + wid; p < p_end; p += NW) {
+    if (!AHEAD) load(p, kf);
     f32x4 sc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int m = 0; m < NK; ++m) {
@@ -180,7 +184,7 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
       sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[m], qf, sc, 0, 0, 0);
       if (m < RT) *reinterpret_cast<bf16x8*>(my + m * 1024 + loff) = kf[m];
     }
-    if (p + NW < p_end) load(p + NW, kf);
+    if (AHEAD && p + NW < p_end) load(p + NW, kf);
     float tmax = NEG_BIG;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -499,10 +503,17 @@ template <int RT, int PT, int CT>
 __global__ __launch_bounds__(64 * NW, 2) void mfma_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int n = A.n_items[0];
+  // two passes over the workgroup's items, so that neither path's registers carry the other's
   for (int item = blockIdx.y; item < n; item += gridDim.y) {
     const int4 it = A.items[item];
-    if ((it.z & 0xff) <= A.dec_tokens) split_item<RT, PT>(A, it, smem);
-    else tile_item<RT, PT, CT>(A, it, smem);
+    if ((it.z & 0xff) <= A.dec_tokens) continue;
+    tile_item<RT, PT, CT>(A, it, smem);
+    __syncthreads();
+  }
+  for (int item = blockIdx.y; item < n; item += gridDim.y) {
+    const int4 it = A.items[item];
+    if ((it.z & 0xff) > A.dec_tokens) continue;
+    split_item<RT, PT>(A, it, smem);
     __syncthreads();
   }
 }
