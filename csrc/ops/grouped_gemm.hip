@@ -41,12 +41,39 @@ struct Args {
   const int* positions;
   const float* cos_sin;
   int rskip, r, rp, rd;
+  int wide;  // out rows and group offsets are multiples of 8 elements
 };
 
 // The rotated columns of `n` rows from `start` of group grp (one workgroup).
 template <typename T>
 __device__ __forceinline__ void rotate_rows(const Args& A, int grp, int start, int n) {
   const int half = A.rd >> 1, N = A.N16 * 16;
+  if (sizeof(T) == 2 && half % 8 == 0 && A.rd == A.r && A.rskip % 8 == 0 && A.xg % 8 == 0 && A.og % 8 == 0 &&
+      A.ldo % 8 == 0) {
+    // 8 pairs a thread, 16-byte accesses
+    const int hp = half >> 3;
+    for (int e = threadIdx.x; e < n * hp; e += 256) {
+      const int t = start + e / hp, j = (e % hp) * 8;
+      const bf16* src = (const bf16*)A.x + (size_t)t * A.ldx + (size_t)grp * A.xg + A.rskip + j;
+      bf16* dst = (bf16*)A.out + (size_t)t * A.ldo + (size_t)grp * A.og + N + j;
+      const float* cs = A.cos_sin + (size_t)A.positions[t] * A.rd + j;
+      const bf16x8 u = *reinterpret_cast<const bf16x8*>(src), v = *reinterpret_cast<const bf16x8*>(src + half);
+      float c[8], s[8];
+      __builtin_memcpy(c, cs, 32);
+      __builtin_memcpy(s, cs + half, 32);
+      bf16x8 a, b;
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        a[k] = (bf16)((float)u[k] * c[k] - (float)v[k] * s[k]);
+        b[k] = (bf16)((float)v[k] * c[k] + (float)u[k] * s[k]);
+      }
+      *reinterpret_cast<bf16x8*>(dst) = a;
+      *reinterpret_cast<bf16x8*>(dst + half) = b;
+    }
+    for (int e = threadIdx.x; e < n * (A.rp - A.r); e += 256)
+      ((T*)A.out)[(size_t)(start + e / (A.rp - A.r)) * A.ldo + (size_t)grp * A.og + N + A.r + e % (A.rp - A.r)] = (T)0.f;
+    return;
+  }
   const int per = max(1, 256 / A.rp), i0 = threadIdx.x / A.rp;  // rows at a time
   for (int j = threadIdx.x % A.rp; j < A.rp && i0 < per; j += 256) {
 #pragma unroll 4
@@ -152,6 +179,14 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) v[j] = (bf16)glu(acc[m][i][j], acc[m][i + 1][j], A);
         *reinterpret_cast<bf16x4*>(o + (nt0 + i) * 8) = v;
+      }
+    } else if (NT % 2 == 0 && A.N16 % 2 == 0 && A.wide) {
+      // 16-byte stores: lanes of neighbouring lane groups trade halves
+      const struct { bf16* y; int ldy; } row{o - 4 * g, 0};
+#pragma unroll
+      for (int i = 0; i + 1 < NT; i += 2) {
+        if (nt0 + i >= A.N16) break;
+        pk::store_pair_wide<pk::EP_PLAIN>(row, 0, nt0 + i, g, acc[m][i], acc[m][i + 1]);
       }
     } else {
 #pragma unroll
@@ -301,7 +336,8 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
   if (N16 <= 0 || K32 <= 0 || (epi == 1 && N16 % 2)) return -1;
   if (tiles ? max_tiles <= 0 : rows <= 0) return 0;
   const pa::gg::Args A{x, w, out, wstride, ldx, xg, ldo, og, rows, N16, K32, (const int4*)tiles, n_tiles,
-                       order, x_div, out_order, limit, alpha, bias, positions, cos_sin, rskip, r, rp, rd};
+                       order, x_div, out_order, limit, alpha, bias, positions, cos_sin, rskip, r, rp, rd,
+                       ldo % 8 == 0 && og % 8 == 0 && ((uintptr_t)out & 15) == 0};
   const int rot = rp > 0 ? 1 : 0;  // one more column of workgroups
   if (fp32) {
     if (tiles && tm != 16) return -2;
@@ -313,7 +349,8 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
   if (tiles && tm == 256)
     return pa_expert_tiles(out, x, w, wstride, N16 * 16, K32 * 32, ldx, ldo, tiles, max_tiles, n_tiles, order, x_div,
                            out_order, epi == 1 ? 5 : 0, limit, alpha, bias, st);
-  if (!tiles) tm = rows <= 32 ? 16 : 64;
+  // dense: 64-row tiles once they fill the chip
+  if (!tiles) tm = (N16 + 15) / 16 * ((rows + 63) / 64) * groups < 256 ? 16 : 64;
   if (tm != 16 && tm != 64) return -2;
 #define PA_GG(MT, NT, KU, G)                                                                                   \
   hipLaunchKernelGGL((pa::gg::gemm_kernel<MT, NT, KU, G>),                                                     \

@@ -72,9 +72,12 @@ def _run(cmd):
     return r.stdout
 
 
+_FORCE = False  # compile up-to-date objects too
+
+
 def _compile_many(jobs, workers: int):
     todo = [(src, obj, cmd) for src, obj, cmd, deps in jobs
-            if not os.path.exists(obj) or os.path.getmtime(obj) < _newest([src] + deps)]
+            if _FORCE or not os.path.exists(obj) or os.path.getmtime(obj) < _newest([src] + deps)]
     if not todo:
         return 0
     with cf.ThreadPoolExecutor(max_workers=max(1, workers)) as ex:
@@ -188,10 +191,15 @@ def ensure(kind: str = "latent", gpu: bool = True) -> None:
             f()
 
 
-def build_all(verbose: bool = False) -> None:
-    build_runtime(verbose)
-    build_latent(verbose)
-    build_ops(verbose)
+def build_all(verbose: bool = False, force: bool = False) -> None:
+    global _FORCE
+    _FORCE = force
+    try:
+        build_runtime(verbose)
+        build_latent(verbose)
+        build_ops(verbose)
+    finally:
+        _FORCE = False
 
 
 if __name__ == "__main__":

@@ -22,13 +22,15 @@ def register_engine(model: str, engine: LLMEngine):
 
 
 def get_engine(model: str = "llama-3-8b", **overrides) -> LLMEngine:
+    from pilottai_amd.models.registry import is_folder
+
     key = model.lower()
     with _LOCK:
         eng = _ENGINES.get(key)
         if eng is None:
             kw = dict(_DEFAULTS.get(key, {}))
             kw.update(overrides)
-            eng = LLMEngine(EngineConfig(model=key, **kw))
+            eng = LLMEngine(EngineConfig(model=model if is_folder(model) else key, **kw))
             _ENGINES[key] = eng
         return eng
 

@@ -191,7 +191,8 @@ def create_app(llm, model_name: Optional[str] = None, engine=None) -> FastAPI:
 
 def main():
     ap = argparse.ArgumentParser(description=__doc__.split("\n\n")[0])
-    ap.add_argument("--model", default="llama-3-8b")
+    ap.add_argument("--model", default="llama-3-8b", help="a preset's name, or a folder with config.json and weights")
+    ap.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16")
     ap.add_argument("--host", default="127.0.0.1")
     ap.add_argument("--port", type=int, default=8000)
     ap.add_argument("--schema", action="store_true", help="model-free SchemaLLM backend (no GPU)")
@@ -211,7 +212,10 @@ def main():
         from pilottai_amd.engine.engine import EngineConfig, LLMEngine
 
         dev = torch.device("cuda", 0) if torch.cuda.is_available() else torch.device("cpu")
-        eng = LLMEngine(EngineConfig(model=a.model if dev.type == "cuda" else "tiny",
+        from pilottai_amd.models.registry import is_folder
+
+        eng = LLMEngine(EngineConfig(model=a.model if dev.type == "cuda" or is_folder(a.model) else "tiny",
+                                     dtype=a.dtype,
                                      kv_cache_gb=a.kv_gb if dev.type == "cuda" else None,
                                      num_kv_blocks=None if dev.type == "cuda" else 1024,
                                      freeze_heap=True), device=dev)

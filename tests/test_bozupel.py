@@ -389,6 +389,19 @@ def test_configuration_errors(folder, tmp_path):
         engine(lambda _: str(tmp_path), "x", "cpu", "float32")
 
 
+def test_engine_registry_takes_a_folder(folder):
+    """The process-wide registry that serving and agents use (case of the path kept)."""
+    from pilottai_amd.engine import registry
+
+    eng = registry.get_engine(folder("once"), num_kv_blocks=32, max_model_len=128, max_num_batched_tokens=64, max_num_seqs=4)
+    try:
+        assert registry.get_engine(folder("once")) is eng and eng.model_cfg.vocab_size == 64
+        p = tokens("once", 9)
+        greedy_is_right(folder, "once", p, eng.generate([p], temperature=0.0, max_tokens=5, ignore_eos=True)[0].token_ids, "bfloat16")
+    finally:
+        registry.shutdown_engines()
+
+
 def test_requests_that_do_not_fit_are_refused(folder):
     eng = engine(folder, "once", "cpu", "float32", num_kv_blocks=4)
     with pytest.raises(ValueError):

@@ -19,7 +19,7 @@ HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 def test_mid_gemm_kernels_use_no_scratch(tmp_path):
     out = tmp_path / "mid.s"
     subprocess.run([HIPCC, "--offload-arch=gfx950", "-O3", "-std=c++17", "-S", "--cuda-device-only",
-                    "-ffast-math", "-mllvm", "-amdgpu-mfma-vgpr-form", os.path.join(ROOT, "csrc", "ops", "gemm_mid.hip"), "-o", str(out)],
+                    "-ffast-math", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-mllvm", "-amdgpu-mfma-vgpr-form", os.path.join(ROOT, "csrc", "ops", "gemm_mid.hip"), "-o", str(out)],
                    check=True, capture_output=True)
     text = out.read_text()
     sizes = re.findall(r"\.set (_ZN2pa3mid\w+)\.private_seg_size, (\d+)", text)
