@@ -151,6 +151,15 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
   const int p_begin = p_lo + part * per, p_end = min(p_hi, p_begin + per);
   const int* bt = A.block_table + (size_t)s * A.max_blocks;
 
+  constexpr bool AHEAD = RT < 16;
+  bf16x8 kf[NK];
+  auto load = [&](int p, bf16x8 (&k)[NK]) {
+    const bf16* b = (const bf16*)A.pages + (size_t)bt[p] * (D * 16) + (g * 16 + c) * 8;
+#pragma unroll
+    for (int m = 0; m < NK; ++m) k[m] = *reinterpret_cast<const bf16x8*>(b + m * 512);
+  };
+  // the wave's first page is under way while the queries are staged
+  if (AHEAD && p_begin + wid < p_end) load(p_begin + wid, kf);
   // all waves share the 16 columns: their Q^T operands (1 KB per k-step) live in LDS
   char* sq = smem + NW * (RP * 32);
   for (int m = wid; m < NK; m += NW)
@@ -165,16 +174,8 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
   const int loff = (g * 16 + c) * 16;  // this lane's 16 B of a k-step
   const int toff = ((c & 3) >> 1) * 256 + (4 * g + (c >> 2)) * 16 + (c & 1) * 8;
 
-  bf16x8 kf[NK];
-  auto load = [&](int p, bf16x8 (&k)[NK]) {
-    const bf16* b = (const bf16*)A.pages + (size_t)bt[p] * (D * 16) + (g * 16 + c) * 8;
-#pragma unroll
-    for (int m = 0; m < NK; ++m) k[m] = *reinterpret_cast<const bf16x8*>(b + m * 512);
-  };
-  // the widest latents load a page when they need it: its next page does not fit the registers
-  // beside the outputs, and the SIMD's other wave computes meanwhile
-  constexpr bool AHEAD = RT < 16;
-  if (AHEAD && p_begin + wid < p_end) load(p_begin + wid, kf);
+  // the widest latents load a later page when they need it: it does not fit the registers beside the
+  // outputs' update, and the SIMD's other wave computes meanwhile
   for (int p = p_begin + wid; p < p_end; p += NW) {
     if (!AHEAD) load(p, kf);
     f32x4 sc = {0.f, 0.f, 0.f, 0.f};
@@ -345,7 +346,11 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
   const size_t row0 = (size_t)(A.q_start[s] + qb) * A.H;
   const int* bt = A.block_table + (size_t)s * A.max_blocks;
   int ci[CT], cpos[CT], klo[CT];
-  bf16x8 qf[CT][NK];
+  // the widest rows keep their rotated part's queries in LDS (lane-private, above the key tiles)
+  constexpr int NQ = NK > 17 ? RT : NK;
+  const int loff = (g * 16 + c) * 16;
+  char* qs = smem + 2 * TILE + wid * (CT * (NK - NQ) * 1024) + loff;
+  bf16x8 qf[CT][NQ];
 #pragma unroll
   for (int t = 0; t < CT; ++t) {
     ci[t] = cw + (wid * CT + t) * 16 + c;
@@ -353,8 +358,11 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
     cpos[t] = pos0 + cc / A.H;
     klo[t] = A.window > 0 ? max(0, cpos[t] - A.window + 1) : 0;
 #pragma unroll
-    for (int m = 0; m < NK; ++m)
-      qf[t][m] = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + (row0 + cc) * D + 32 * m + 8 * g);
+    for (int m = 0; m < NK; ++m) {
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + (row0 + cc) * D + 32 * m + 8 * g);
+      if (m < NQ) qf[t][m] = v;
+      else *reinterpret_cast<bf16x8*>(qs + (t * (NK - NQ) + m - NQ) * 1024) = v;
+    }
   }
   // positions of the workgroup's columns -> its key tiles
   const int f = pos0 + cw / A.H, e = pos0 + min(cw + 16 * NW * CT - 1, cols - 1) / A.H;
@@ -394,7 +402,6 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
                                          (lds_void*)(dst + ch * 1024), 16, 0, 0);
     }
   };
-  const int loff = (g * 16 + c) * 16;
   const int toff = ((c & 3) >> 1) * 256 + (4 * g + (c >> 2)) * 16 + (c & 1) * 8;
   if (t_lo < t_hi) issue(t_lo, smem);
   for (int t = t_lo; t < t_hi; ++t) {
@@ -413,7 +420,11 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
       for (int k = 0; k < 2; ++k) {
         const bf16x8 kf = *reinterpret_cast<const bf16x8*>(cur + k * (D * 32) + m * 1024 + loff);
 #pragma unroll
-        for (int x = 0; x < CT; ++x) sc[x][k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[x][m], sc[x][k], 0, 0, 0);
+        for (int x = 0; x < CT; ++x) {
+          const bf16x8 q = m < NQ ? qf[x][m < NQ ? m : 0]
+                                  : *reinterpret_cast<const bf16x8*>(qs + (x * (NK - NQ) + m - NQ) * 1024);
+          sc[x][k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, q, sc[x][k], 0, 0, 0);
+        }
       }
     const bool mask = 32 * t < full_lo || 32 * t + 31 > full_hi;  // wave-uniform
     bf16x8 pf[CT];
@@ -495,7 +506,7 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
 
 template <int RT, int PT>
 constexpr int lds_bytes() {
-  return std::max({2 * 32 * 32 * (RT + PT) * 2, NW * 32 * 32 * RT + 1024 * (RT + PT),
+  return std::max({2 * 32 * 32 * (RT + PT) * 2 + (RT + PT > 17 ? NW * PT * 1024 : 0), NW * 32 * 32 * RT + 1024 * (RT + PT),
                    NW * 16 * MERGE_LD * 4 + 2 * NW * 16 * 4});
 }
 
