@@ -154,7 +154,7 @@ PRESETS: Dict[str, BozupelConfig] = {
                              LatentAttentionSpec(heads=4, dim=48, rot_dim=32, vdim=40, q_rank=64, kv_rank=128,
                                                  scale=0.11, rot_base=10000.0, rot_dims=32, window=200),
                              TableExpertsSpec(experts=6, top=2, ff=80, limit=4.0), loop=(0, 1, 2)),
-    # layers of a real model's size (bench.py --bozupel), at two widths
+    # layers of a real model's size (bench.py --design bozupel), at two widths
     "bozupel-base": _uniform("bozupel-base", 8, 128256, 2048,
                              LatentAttentionSpec(heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512,
                                                  scale=192 ** -0.5, rot_base=10000.0, rot_dims=64, window=4096),
