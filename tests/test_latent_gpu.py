@@ -109,7 +109,7 @@ def test_table_experts(gpu, dt, tm, T, E, top, ff, D):
 
 
 @pytest.mark.parametrize("dt", DTYPES)
-@pytest.mark.parametrize("NQ,R,r,rd,H", [(80, 96, 16, 16, 3), (50, 70, 24, 12, 5), (256, 512, 64, 64, 2)])
+@pytest.mark.parametrize("NQ,R,r,rd,H", [(72, 104, 48, 48, 3), (50, 70, 24, 12, 5), (256, 512, 64, 64, 2)])
 def test_latent_cache_and_query_rotation(gpu, dt, NQ, R, r, rd, H):
     from pilottai_amd import ops
     from pilottai_amd.ops import reference as ref
@@ -222,7 +222,7 @@ def run_attention(gpu, dt, H, R, r, reqs, window, simple=False, split_target=384
         torch.testing.assert_close(o[q0:q0 + n], want, **tol(dt), msg=lambda s, i=i: f"request {i} {reqs[i]}: {s}")
 
 
-SHAPES = [(1, 32, 8), (3, 96, 16), (8, 100, 40), (16, 512, 64), (20, 256, 32), (40, 192, 64)]
+SHAPES = [(1, 32, 8), (3, 96, 24), (8, 100, 40), (16, 512, 64), (20, 256, 32), (40, 192, 64)]
 STEPS = {"prompt": [(0, 75)], "decode": [(0, 1), (15, 1), (16, 1), (700, 1), (33, 1)], "two": [(130, 2), (0, 2)],
          "mixed": [(300, 1), (17, 40), (0, 3), (531, 130), (64, 1), (5, 2)]}
 
