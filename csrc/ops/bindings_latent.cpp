@@ -3,7 +3,7 @@
 // packed-weight projections it shares with the other models. Built as its own module so that such
 // a model needs no other kernel. Every entry point checks shapes on the host and launches on the
 // caller's stream.
-#include "bind_common.h"
+#include "bind_grouped.h"
 
 extern "C" {
 int pa_residual_norm(int fp32, float* resid, const void* y, int K, int ldy, float y_scale, const float* w_post,
@@ -20,41 +20,9 @@ int pa_latent_attention(int fp32, void* out, float* part_o, float* part_ml, cons
                         hipStream_t st);
 int pa_table_route(const int* tables, const int* desc, int layers, const int* ids, const int* slots, int T, int tm,
                    int* order, int* tiles, int* n_tiles, hipStream_t st);
-int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out, long long wstride, int groups, int ldx, int xg,
-                    int ldo, int og, int rows, int N16, int K32, const int* tiles, int max_tiles, const int* n_tiles,
-                    const int* order, int x_div, int out_order, int tm, int epi, float limit, float alpha, float bias,
-                    const int* positions, const float* cos_sin, int rskip, int r, int rp, int rd, hipStream_t st);
 }
 
 namespace {
-
-using Opt = c10::optional<at::Tensor>;
-
-int is_f32(const at::Tensor& t, const char* name) {
-  TORCH_CHECK(t.scalar_type() == at::kFloat || t.scalar_type() == at::kBFloat16, name, " must be bfloat16 or float32");
-  return t.scalar_type() == at::kFloat ? 1 : 0;
-}
-
-// 2-D (rows x columns, unit inner stride) operand of the model's dtype
-void check_rows(const at::Tensor& t, at::ScalarType dt, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.stride(1) == 1, name, " must be a 2-D GPU tensor, unit inner stride");
-  check_dtype(t, dt, name);
-}
-
-const float* opt_f32(const Opt& t, int64_t n, const char* name) {
-  if (!t.has_value()) return nullptr;
-  check_gpu(*t, name);
-  check_dtype(*t, at::kFloat, name);
-  TORCH_CHECK(t->numel() >= n, name, " is too short");
-  return t->data_ptr<float>();
-}
-
-const int* ints(const at::Tensor& t, int64_t n, const char* name) {
-  check_gpu(t, name);
-  check_dtype(t, at::kInt, name);
-  TORCH_CHECK(t.numel() >= n, name, " is too short");
-  return t.data_ptr<int>();
-}
 
 void residual_norm(at::Tensor resid, Opt y, int64_t K, double y_scale, Opt w_post, Opt emb, Opt ids, bool emb_add,
                    Opt w_next, Opt out, Opt rows, double eps) {
@@ -156,74 +124,6 @@ void table_route(at::Tensor tables, at::Tensor desc, at::Tensor desc_host, at::T
                           ints(slots, T, "slots"), T, tm, (int*)ints(order, 0, "order"), (int*)ints(tiles, 0, "tiles"),
                           (int*)ints(n_tiles, L, "n_tiles"), cur_stream()),
            "table_route");
-}
-
-// w: bf16 packed [G, N/16, K/32, 64, 8] or fp32 [G, N, K]; epi 1: gated pair (out has N/2 columns per group)
-void dims(const at::Tensor& w, int f, int64_t* G, int64_t* N, int64_t* K) {
-  check_gpu(w, "w");
-  if (f) {
-    TORCH_CHECK(w.dim() == 3 && w.size(1) % 16 == 0 && w.size(2) % 32 == 0, "w must be [G, 16 n, 32 k]");
-    *G = w.size(0); *N = w.size(1); *K = w.size(2);
-  } else {
-    TORCH_CHECK(w.dim() == 5 && w.size(3) == 64 && w.size(4) == 8, "w must be packed [G, N/16, K/32, 64, 8]");
-    *G = w.size(0); *N = w.size(1) * 16; *K = w.size(2) * 32;
-  }
-}
-
-// every row of x through every group: x columns g * xg .. + K -> out columns g * og .. + N; with
-// positions / cos_sin also the rotated part: x columns g * xg + rskip .. + r -> out columns g * og + N .. + rp
-void head_gemm(at::Tensor x, int64_t xg, at::Tensor w, at::Tensor out, int64_t og, Opt positions, Opt cos_sin,
-               int64_t rskip, int64_t r, int64_t rp) {
-  const int f = is_f32(x, "x");
-  check_rows(x, x.scalar_type(), "x");
-  check_rows(out, x.scalar_type(), "out");
-  check_dtype(w, x.scalar_type(), "w");
-  int64_t G, N, K;
-  dims(w, f, &G, &N, &K);
-  TORCH_CHECK(out.size(0) == x.size(0) && (G - 1) * xg + K <= x.size(1) && (G - 1) * og + N <= out.size(1),
-              "head_gemm sizes");
-  const int* pos = nullptr;
-  const float* cs = nullptr;
-  int64_t rd = 0;
-  if (positions.has_value()) {
-    TORCH_CHECK(cos_sin.has_value() && cos_sin->dim() == 2 && cos_sin->size(1) % 2 == 0, "cos_sin must be [max_pos, dims]");
-    rd = cos_sin->size(1);
-    pos = ints(*positions, x.size(0), "positions");
-    cs = opt_f32(cos_sin, 0, "cos_sin");
-    TORCH_CHECK(rd <= r && r <= rp && rp > 0 && rskip >= 0 && (G - 1) * xg + rskip + r <= x.size(1) &&
-                    (G - 1) * og + N + rp <= out.size(1), "head_gemm rotation sizes");
-  } else {
-    rp = 0;
-  }
-  TORCH_CHECK(f || (x.stride(0) % 8 == 0 && xg % 8 == 0 && out.stride(0) % 4 == 0 && og % 4 == 0),
-              "head_gemm: 16-byte aligned operands");
-  check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, G, x.stride(0), xg, out.stride(0), og,
-                           x.size(0), N / 16, K / 32, nullptr, 0, nullptr, nullptr, 0, 0, 0, 0, 0.f, 0.f, 0.f,
-                           pos, cs, rskip, r, rp, rd, cur_stream()),
-           "head_gemm");
-}
-
-// rows sorted by group: x row = order[p] / x_div (x_div 0: p), out row = out_order ? order[p] : p
-void expert_gemm(at::Tensor x, at::Tensor w, at::Tensor out, at::Tensor tiles, at::Tensor n_tiles, at::Tensor order,
-                 int64_t rows, int64_t x_div, bool out_order, int64_t tm, bool glu, double limit, double alpha,
-                 double bias) {
-  const int f = is_f32(x, "x");
-  check_rows(x, x.scalar_type(), "x");
-  check_rows(out, x.scalar_type(), "out");
-  check_dtype(w, x.scalar_type(), "w");
-  int64_t G, N, K;
-  dims(w, f, &G, &N, &K);
-  TORCH_CHECK(K <= x.size(1) && (glu ? N / 2 : N) <= out.size(1) && out.size(0) >= rows &&
-                  x.size(0) * (x_div ? x_div : 1) >= rows, "expert_gemm sizes");
-  TORCH_CHECK(f || (x.stride(0) % 8 == 0 && out.stride(0) % 4 == 0), "expert_gemm: 16-byte aligned rows");
-  TORCH_CHECK(tm != 256 || (!f && K % 64 == 0 && K >= 128 && N % 128 == 0 && out.stride(0) % 8 == 0),
-              "expert_gemm: tiles of 256 rows need K % 64 == 0, K >= 128, N % 128 == 0");
-  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 4, "tiles must be [n, 4]");
-  check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, G, x.stride(0), 0, out.stride(0), 0, 0,
-                           N / 16, K / 32, ints(tiles, 4, "tiles"), tiles.size(0), ints(n_tiles, 1, "n_tiles"),
-                           ints(order, rows, "order"), x_div, out_order ? 1 : 0, tm, glu ? 1 : 0, (float)limit,
-                           (float)alpha, (float)bias, nullptr, nullptr, 0, 0, 0, 0, cur_stream()),
-           "expert_gemm");
 }
 
 }  // namespace

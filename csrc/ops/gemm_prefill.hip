@@ -73,7 +73,7 @@ struct Args {
   const int* xmap = nullptr;
   const int* ymap = nullptr;
   int xdiv = 1;
-  float limit = 0.f, alpha = 0.f, bias = 0.f;
+  float limit = 0.f, alpha = 0.f, cubic = 0.f, bias = 0.f;
 };
 
 typedef __attribute__((address_space(3))) void lds_t;
@@ -726,7 +726,7 @@ extern "C" int pa_prefill_gemm(void* y, const void* x, const void* wp, const voi
 
 // Rows sorted by group (mixture-of-experts layers): tiles {group, first position, rows <= 256, 0}
 // on the ping-pong kernels, group g's packed weights at wp + g * wstride. x row of position p =
-// order[p] / x_div (x_div 0: p), y row = order[p] (out_order) or p. epi 0 plain, 5 clamped gated
+// order[p] / x_div (x_div 0: p), y row = order[p] (out_order) or p. epi 0 plain, 5 gated
 // unit. K % 64 == 0, K >= 128, N % 128 == 0; y rows 16-byte aligned.
 namespace pa {
 namespace pf {
@@ -760,7 +760,8 @@ __global__ __launch_bounds__(512) void pingpong_grouped_kernel(Args A, const int
 
 extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long wstride, int N, int K, int ldx, int ldy,
                                const int* tiles, int max_tiles, const int* n_tiles, const int* order, int x_div,
-                               int out_order, int epi, float limit, float alpha, float bias, hipStream_t st) {
+                               int out_order, int epi, float limit, float alpha, float cubic, float bias,
+                               hipStream_t st) {
   using namespace pa::pf;
   if (K % 64 || K < 128 || N % 128 || ldx % 8 || ldy % 8 || (epi != EP_PLAIN && epi != EP_GLU)) return -1;
   if (max_tiles <= 0) return 0;
@@ -774,6 +775,7 @@ extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long
   a.ldy = ldy;
   a.limit = limit;
   a.alpha = alpha;
+  a.cubic = cubic;
   a.bias = bias;
   const bool wide = N % 256 == 0;
   a.NT = N / (wide ? 256 : 128);

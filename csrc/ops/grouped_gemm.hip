@@ -12,13 +12,12 @@
 // rows share them; prompts with 256 rows and more per group run the ping-pong kernels instead
 // (gemm_prefill.hip pa_expert_tiles).
 //
-// Epilogues: plain, or the clamped gated unit
-//   g' = min(g, limit), u' = clamp(u, -limit, limit),  out = g' * sigmoid(alpha * g') * (u' + bias).
+// Epilogues: plain, or the gated unit of packed_epi.h (limit, alpha, cubic, bias).
 #include "packed_epi.h"
 
 extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long wstride, int N, int K, int ldx, int ldy,
                                const int* tiles, int max_tiles, const int* n_tiles, const int* order, int x_div,
-                               int out_order, int epi, float limit, float alpha, float bias, hipStream_t st);
+                               int out_order, int epi, float limit, float alpha, float cubic, float bias, hipStream_t st);
 
 namespace pa {
 namespace gg {
@@ -35,7 +34,7 @@ struct Args {
   const int* order;        // sorted: position -> token * top + k
   int x_div;               // sorted: x row = order / x_div (0: x row = position)
   int out_order;           // sorted: out row = order[position] (0: out row = position)
-  float limit, alpha, bias;
+  float limit, alpha, cubic, bias;
   // dense, optional: after a group's N columns of out, the rotated part of the row's head (r columns of
   // x at the group's offset + rskip, the first rd turned by the row's position), padded to rp columns
   const int* positions;
@@ -93,7 +92,7 @@ __device__ __forceinline__ void rotate_rows(const Args& A, int grp, int start, i
 }
 
 __device__ __forceinline__ float glu(float g, float u, const Args& A) {
-  return pk::clamped_glu(g, u, A.limit, A.alpha, A.bias);
+  return pk::gated_unit(g, u, A.limit, A.alpha, A.cubic, A.bias);
 }
 
 template <int MT, int NT, int KU, bool GLU>
@@ -331,12 +330,12 @@ extern "C" int pa_table_route(const int* tables, const int* desc, int layers, co
 extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out, long long wstride, int groups,
                                int ldx, int xg, int ldo, int og, int rows, int N16, int K32, const int* tiles,
                                int max_tiles, const int* n_tiles, const int* order, int x_div, int out_order, int tm,
-                               int epi, float limit, float alpha, float bias, const int* positions,
+                               int epi, float limit, float alpha, float cubic, float bias, const int* positions,
                                const float* cos_sin, int rskip, int r, int rp, int rd, hipStream_t st) {
   if (N16 <= 0 || K32 <= 0 || (epi == 1 && N16 % 2)) return -1;
   if (tiles ? max_tiles <= 0 : rows <= 0) return 0;
   const pa::gg::Args A{x, w, out, wstride, ldx, xg, ldo, og, rows, N16, K32, (const int4*)tiles, n_tiles,
-                       order, x_div, out_order, limit, alpha, bias, positions, cos_sin, rskip, r, rp, rd,
+                       order, x_div, out_order, limit, alpha, cubic, bias, positions, cos_sin, rskip, r, rp, rd,
                        ldo % 8 == 0 && og % 8 == 0 && ((uintptr_t)out & 15) == 0};
   const int rot = rp > 0 ? 1 : 0;  // one more column of workgroups
   if (fp32) {
@@ -348,7 +347,7 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
   }
   if (tiles && tm == 256)
     return pa_expert_tiles(out, x, w, wstride, N16 * 16, K32 * 32, ldx, ldo, tiles, max_tiles, n_tiles, order, x_div,
-                           out_order, epi == 1 ? 5 : 0, limit, alpha, bias, st);
+                           out_order, epi == 1 ? 5 : 0, limit, alpha, cubic, bias, st);
   // dense: 64-row tiles once they fill the chip
   if (!tiles) tm = (N16 + 15) / 16 * ((rows + 63) / 64) * groups < 256 ? 16 : 64;
   if (tm != 16 && tm != 64) return -2;

@@ -5,7 +5,7 @@
 //
 //   EP_PLAIN     y = acc
 //   EP_SILU      y = silu(gate) * up over the interleaved (gate t, up t) packed tiles
-//   EP_GLU       y = clamped gated unit over the same pairs (limit, alpha, bias; clamped_glu below)
+//   EP_GLU       y = gated unit over the same pairs (limit, alpha, cubic, bias; gated_unit below)
 //   EP_RESID     y = resid + acc, returning sum(y^2) of the written bf16 values (the next
 //                RMSNorm's row statistics, accumulated by the caller)
 //   EP_ROPEPERM  y = acc in the natural QKV column order (rope-permuted packed tiles)
@@ -25,11 +25,13 @@ enum { EP_PLAIN = 0, EP_SILU = 1, EP_RESID = 2, EP_ROPEPERM = 3, EP_ROPEKV = 4, 
 template <int EPI>
 constexpr bool pair_epi() { return EPI == EP_SILU || EPI == EP_ROPEKV || EPI == EP_GLU; }
 
-// g' = min(g, limit), u' = clamp(u, -limit, limit): g' sigmoid(alpha g') (u' + bias)
-__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float bias) {
+// g' = min(g, limit), u' = clamp(u, -limit, limit): g' sigmoid(alpha (g' + cubic g'^3)) (u' + bias).
+// alpha 1, cubic 0: silu; alpha 2 sqrt(2 / pi), cubic 0.044715: the tanh form of gelu, since
+// (1 + tanh z) / 2 = sigmoid(2 z).
+__device__ __forceinline__ float gated_unit(float g, float u, float limit, float alpha, float cubic, float bias) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + __expf(-alpha * g)) * (u + bias);
+  return g / (1.f + __expf(-alpha * (g + cubic * g * g * g))) * (u + bias);
 }
 
 // packed rope-QKV tile -> first column of its original tile
@@ -45,7 +47,7 @@ __device__ __forceinline__ float store_quad(const AT& A, int m, int tile, int cq
   if constexpr (EPI == EP_GLU) {
     bf16x4 o;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) o[r] = (bf16)clamped_glu(v[r], v2[r], A.limit, A.alpha, A.bias);
+    for (int r = 0; r < 4; ++r) o[r] = (bf16)gated_unit(v[r], v2[r], A.limit, A.alpha, A.cubic, A.bias);
     *reinterpret_cast<bf16x4*>(A.y + (size_t)m * A.ldy + (tile >> 1) * 16 + cq) = o;
     return 0.f;
   } else if constexpr (EPI == EP_SILU) {

@@ -1,0 +1,141 @@
+// From a [q | k | v] projection row to the attention kernel's operands (window_attention.hip), in one
+// launch: biases, the rotation of the first rd dimensions of every query and key head, queries to
+// q_out, keys and values to their pages, and, where a token ends a block of `pool` tokens, the block's
+// mean key and value.
+//
+//   x [T, ldx]    H x DK queries | G x DK keys | G x DV values, bias likewise
+//   pages         [pages, G, D/8, 16, 8]; pooled rows [pages, npb, G, D] with the page of the block's
+//                 last token, blocks that end in one page in order
+//
+// A block's mean is taken over its rows as the cache holds them (rotated, in T): rows of earlier steps
+// are read from their pages, rows of this step are computed again from the projection, so nothing
+// waits for another workgroup. Arithmetic is fp32.
+#include "common.h"
+
+namespace pa {
+namespace kv {
+
+struct Args {
+  const void* x;
+  const float* bias;  // optional
+  void *q, *kp, *vp, *pk, *pv;
+  const int *positions, *slots, *q_start, *q_len, *ctx_len, *block_table;
+  const float* cos_sin;  // [max_pos, rd]: cos | sin
+  int ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs;
+};
+
+// 8 values of head part `off` (columns off .. off + D of a row) from dimension d, rotated by cs if `rot`
+template <typename T>
+__device__ __forceinline__ void chunk(const Args& A, const T* row, int off, int d, const float* cs, bool rot, float (&v)[8]) {
+  const int half = A.rd >> 1;
+  T a[8];
+  __builtin_memcpy(a, __builtin_assume_aligned(row + off + d, sizeof(T) * 8), sizeof(T) * 8);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = (float)a[j] + (A.bias ? A.bias[off + d + j] : 0.f);
+  if (!rot || d >= A.rd) return;
+  if (half % 8 == 0) {
+    const int pd = d < half ? d + half : d - half, i = d < half ? d : d - half;
+    __builtin_memcpy(a, __builtin_assume_aligned(row + off + pd, sizeof(T) * 8), sizeof(T) * 8);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float u = (float)a[j] + (A.bias ? A.bias[off + pd + j] : 0.f);
+      const float c = cs[i + j], s = cs[half + i + j];
+      v[j] = d < half ? v[j] * c - u * s : v[j] * c + u * s;
+    }
+    return;
+  }
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const int e = d + j;
+    if (e >= A.rd) break;
+    const int pd = e < half ? e + half : e - half, i = e < half ? e : e - half;
+    const float u = (float)row[off + pd] + (A.bias ? A.bias[off + pd] : 0.f);
+    v[j] = e < half ? v[j] * cs[i] - u * cs[half + i] : v[j] * cs[i] + u * cs[half + i];
+  }
+}
+
+template <typename T>
+__device__ __forceinline__ void put(T* dst, const float (&v)[8]) {
+  T a[8];
+#pragma unroll
+  for (int j = 0; j < 8; ++j) a[j] = (T)v[j];
+  __builtin_memcpy(__builtin_assume_aligned(dst, sizeof(T) * 8), a, sizeof(T) * 8);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
+  const int t = blockIdx.x, slot = A.slots[t];
+  if (slot < 0) return;
+  const int pos = A.positions[t];
+  const T* row = (const T*)A.x + (size_t)t * A.ldx;
+  const float* cs = A.cos_sin + (size_t)pos * A.rd;
+  const int ck = A.DK >> 3, cv = A.DV >> 3, nq = A.H * ck, nk = A.G * ck, nv = A.G * cv;
+  for (int u = threadIdx.x; u < nq + nk + nv; u += 256) {
+    float v[8];
+    if (u < nq) {
+      const int h = u / ck, d = (u - h * ck) * 8;
+      chunk(A, row, h * A.DK, d, cs, true, v);
+      put((T*)A.q + ((size_t)t * A.H + h) * A.DK + d, v);
+    } else {
+      const bool key = u < nq + nk;
+      const int w = key ? u - nq : u - nq - nk, per = key ? ck : cv, D = key ? A.DK : A.DV;
+      const int h = w / per, o = w - h * per;
+      chunk(A, row, (key ? A.H * A.DK : (A.H + A.G) * A.DK) + h * D, o * 8, cs, key, v);
+      put((T*)(key ? A.kp : A.vp) + (((size_t)(slot >> 4) * A.G + h) * per + o) * 128 + (slot & 15) * 8, v);
+    }
+  }
+  const int P = A.pool;
+  if (P <= 0 || (pos + 1) % P) return;
+  // this token's sequence
+  int lo = 0, hi = A.max_seqs - 1;
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (A.q_start[mid] <= t) lo = mid; else hi = mid - 1;
+  }
+  while (lo > 0 && A.q_len[lo] == 0) --lo;  // (rows of no sequence start where the last one ends)
+  const int start = A.ctx_len[lo] - A.q_len[lo];  // the step's first position
+  const int* bt = A.block_table + (size_t)lo * A.max_blocks;
+  const int page = pos >> 4, sub = pos / P - (page << 4) / P;
+  const float inv = 1.f / (float)P;
+  for (int u = threadIdx.x; u < nk + nv; u += 256) {
+    const bool key = u < nk;
+    const int w = key ? u : u - nk, per = key ? ck : cv, D = key ? A.DK : A.DV;
+    const int h = w / per, o = w - h * per, off = (key ? A.H * A.DK : (A.H + A.G) * A.DK) + h * D;
+    float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int p = pos - P + 1; p <= pos; ++p) {
+      if (p < start) {
+        T a[8];
+        const T* src = (const T*)(key ? A.kp : A.vp) + (((size_t)bt[p >> 4] * A.G + h) * per + o) * 128 + (p & 15) * 8;
+        __builtin_memcpy(a, __builtin_assume_aligned(src, sizeof(T) * 8), sizeof(T) * 8);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) sum[j] += (float)a[j];
+      } else {
+        float v[8];
+        chunk(A, row - (size_t)(pos - p) * A.ldx, off, o * 8, A.cos_sin + (size_t)p * A.rd, key, v);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) sum[j] += (float)(T)v[j];
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) sum[j] *= inv;
+    put((T*)(key ? A.pk : A.pv) + (((size_t)(slot >> 4) * A.npb + sub) * A.G + h) * D + o * 8, sum);
+  }
+}
+
+}  // namespace kv
+}  // namespace pa
+
+extern "C" int pa_paged_kv(int fp32, const void* x, const float* bias, void* q, void* kp, void* vp, void* pk, void* pv,
+                           const int* positions, const int* slots, const int* q_start, const int* q_len,
+                           const int* ctx_len, const int* block_table, const float* cos_sin, int ldx, int H, int G,
+                           int DK, int DV, int rd, int pool, int npb, int max_blocks, int max_seqs, int T,
+                           hipStream_t st) {
+  if (T <= 0) return 0;
+  if (DK % 8 || DV % 8 || rd % 2 || rd > DK || ldx % 8) return -1;
+  const pa::kv::Args A{x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_len, block_table, cos_sin,
+                       ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs};
+  if (fp32) hipLaunchKernelGGL((pa::kv::paged_kv_kernel<float>), dim3(T), dim3(256), 0, st, A);
+  else hipLaunchKernelGGL((pa::kv::paged_kv_kernel<pa::bf16>), dim3(T), dim3(256), 0, st, A);
+  return (int)hipGetLastError();
+}

@@ -1,0 +1,587 @@
+// Paged grouped-query attention with a sliding window, pooled keys before the window and a sink in
+// the softmax's denominator, for prefill chunks, decode rows and mixed batches in one launch.
+//
+//   position i sees   keys j with 0 <= i - j < W (W 0: every j <= i), and, with P > 0,
+//                     block b (the mean key and value of positions bP .. bP + P - 1) if
+//                     bP + P - 1 <= i - W, that is b < (i - W + 1) / P
+//   out = sum p v,    p = exp(s) / (sink + sum exp(s)),  sink 0 or 1, one softmax over both kinds
+//
+// Keys and values are fragment-major pages of 16 tokens per KV head, [D/8][16][8] (paged_kv.hip); the
+// value operand of the second product comes from the same form by LDS transpose reads. A pooled
+// block's row lies with the page of its last token: [page][per page][KV head][D]. 16 of them, gathered
+// row by row, make a tile of the same form as a page, so both kinds of keys run the same code:
+//
+//   S^T[keys x cols] = K . Q^T         cols = (token, query head of the KV head's group) pairs
+//   O^T[dims x cols] += V^T . P^T      P^T = the S^T accumulator's own registers
+//
+// An item's keys are its pooled blocks (16 or 32 at a time) and then the tiles of its window. Items
+// come from the scheduler like paged_attention's (seq, q_begin, nq | part<<8 | nparts<<20, partial slot):
+//   nq <= dec_tokens: split over keys. The 8 waves take every 8th page with a private LDS tile and merge;
+//                     nparts > 1 divides the item's own key range, merge_kernel combines the partitions.
+//   otherwise:        128 columns per workgroup, 16 per wave; all waves share double-buffered 32-key tiles
+//                     that arrive by direct global -> LDS loads. Few such items are cut over keys too.
+#include "common.h"
+
+#include <algorithm>
+
+namespace pa {
+namespace wa {
+
+constexpr float NEG_BIG = -1.0e30f;
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) bf16x4 lds_bf16x4;
+typedef __attribute__((address_space(3))) void lds_void;
+typedef const __attribute__((address_space(1))) void glb_void;
+
+struct Args {
+  void* out;             // [T, H, DV]
+  float* part_o;         // [G, slots, NB, 16, DV]
+  float* part_ml;        // [G, slots, NB, 16, 2]
+  const void* q;         // [T, H, DK]
+  const void *kp, *vp;   // [pages, G, D/8, 16, 8]
+  const void *pk, *pv;   // [pages, npb, G, D]
+  const int4* items;
+  const int* n_items;
+  const int *q_start, *q_len, *ctx_len, *block_table;
+  int max_blocks, max_items, H, G, R, NB, DK, DV, dec_tokens, window, pool, npb;
+  float scale_log2, sink;
+};
+
+__device__ __forceinline__ int first_key(const Args& A, int pos) { return A.window > 0 ? max(0, pos - A.window + 1) : 0; }
+// pooled blocks that position pos sees
+__device__ __forceinline__ int blocks_of(const Args& A, int pos) {
+  return A.pool > 0 && A.window > 0 ? max(0, pos - A.window + 1) / A.pool : 0;
+}
+// row index of pooled block b of KV head h
+__device__ __forceinline__ size_t pooled_row(const Args& A, const int* bt, int b, int h) {
+  const int page = (b * A.pool + A.pool - 1) >> 4;
+  return ((size_t)bt[page] * A.npb + (b - (page << 4) / A.pool)) * A.G + h;
+}
+
+// ---------------------------------------------------------------------------
+// Any sizes, bf16 or fp32: one workgroup per (token of an item, head). The exact path.
+template <typename T>
+__global__ __launch_bounds__(256) void simple_kernel(const Args A) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  float* sq = sm;            // DK
+  float* sp = sm + A.DK;     // 256
+  float* red = sp + 256;     // 4
+  const int h = blockIdx.x, n = A.n_items[0], gk = h / A.R;
+  for (int item = blockIdx.y; item < n; item += gridDim.y) {
+    const int4 it = A.items[item];
+    const int s = it.x, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff;
+    if (part > 0) continue;  // partition 0 takes the whole range
+    const int ctx = A.ctx_len[s], ql = A.q_len[s];
+    const int* bt = A.block_table + (size_t)s * A.max_blocks;
+    for (int i = 0; i < nq; ++i) {
+      const int tok = it.y + i, pos = ctx - ql + tok;
+      const int lo = first_key(A, pos), nb = blocks_of(A, pos), total = nb + pos - lo + 1;
+      const size_t row = (size_t)(A.q_start[s] + tok) * A.H + h;
+      // element d of key (or value) kk: pooled blocks first, then the window's tokens
+      auto at = [&](const void* pages, const void* pooled, int D, int kk, int d) -> float {
+        if (kk < nb) return (float)((const T*)pooled)[pooled_row(A, bt, kk, gk) * D + d];
+        const int key = lo + kk - nb;
+        return (float)((const T*)pages)[((size_t)bt[key >> 4] * A.G + gk) * D * 16 + (size_t)(d >> 3) * 128 + (key & 15) * 8 + (d & 7)];
+      };
+      __syncthreads();
+      for (int d = threadIdx.x; d < A.DK; d += 256) sq[d] = (float)((const T*)A.q)[row * A.DK + d];
+      __syncthreads();
+      float m = A.sink > 0.f ? 0.f : NEG_BIG, l = A.sink, o[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      for (int k0 = 0; k0 < total; k0 += 256) {
+        const int kk = k0 + threadIdx.x;
+        float sc = NEG_BIG;
+        if (kk < total) {
+          float a = 0.f;
+          for (int d = 0; d < A.DK; ++d) a += sq[d] * at(A.kp, A.pk, A.DK, kk, d);
+          sc = a * A.scale_log2;
+        }
+        const float wm = wave_max(sc);
+        if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = wm;
+        __syncthreads();
+        const float mn = fmaxf(m, fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])));
+        const float alpha = exp2f(m - mn), p = kk < total ? exp2f(sc - mn) : 0.f;
+        m = mn;
+        sp[threadIdx.x] = p;
+        __syncthreads();
+        l = l * alpha + block_sum<4>(p, red);
+        const int nk = min(256, total - k0);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const int d = threadIdx.x + 256 * e;
+          if (d >= A.DV) break;
+          float a = o[e] * alpha;
+          for (int k = 0; k < nk; ++k) a += sp[k] * at(A.vp, A.pv, A.DV, k0 + k, d);
+          o[e] = a;
+        }
+        __syncthreads();
+      }
+      const float inv = 1.f / l;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int d = threadIdx.x + 256 * e;
+        if (d < A.DV) ((T*)A.out)[row * A.DV + d] = (T)(o[e] * inv);
+      }
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------
+// V^T operand: lanes 16g + i of the result hold dim i of keys 4g .. 4g + 3; each lane names the
+// 8 bytes (key 4g + i/4, dims 4 (i%4) .. + 3) of the 4 x 16 block its group transposes
+__device__ __forceinline__ bf16x4 tr_read(const char* p) {
+  return __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds_bf16x4*)p);
+}
+
+constexpr int NW = 8;          // waves per workgroup
+constexpr int MERGE_LD = 132;  // floats per merge row of 128 dims
+
+// max, sum and the factor of the unnormalised outputs once the sink has joined
+__device__ __forceinline__ float final_scale(float sink, float m, float l) {
+  if (sink <= 0.f) return 1.f / l;
+  const float t = fmaxf(m, 0.f), a = exp2f(m - t);
+  return a / (l * a + sink * exp2f(-t));
+}
+
+template <int NK, int NV>
+__device__ __forceinline__ void split_item(const Args& A, const int4 it, char* smem) {
+  constexpr int DK = 32 * NK, DV = 32 * NV;
+  const int s = it.x, qb = it.y, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff, nparts = it.z >> 20, pidx = it.w;
+  const int cb = blockIdx.x, gk = blockIdx.z, cols = nq * A.R;
+  if (cb * 16 >= cols) return;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
+  const int ctx = A.ctx_len[s], ql = A.q_len[s];
+  const int pos0 = ctx - ql + qb;
+  auto tok_of = [&](int col) { return min(col, cols - 1) / A.R; };
+  auto row_of = [&](int col) {  // q / out row of a column
+    const int cc = min(col, cols - 1), t = cc / A.R;
+    return (size_t)(A.q_start[s] + qb + t) * A.H + gk * A.R + (cc - t * A.R);
+  };
+  const int cpos = pos0 + tok_of(cb * 16 + c);  // this column's position
+  const int klo = first_key(A, cpos), cnb = blocks_of(A, cpos);
+  // the item's tiles of 16: pooled blocks, then token pages; this partition's share
+  const int last = pos0 + nq - 1, nb = blocks_of(A, last), np = (nb + 15) >> 4;
+  const int p_lo = first_key(A, pos0) >> 4, total = np + ((last + 16) >> 4) - p_lo;
+  const int per = (total + nparts - 1) / nparts;
+  const int t_begin = part * per, t_end = min(total, t_begin + per);
+  const int* bt = A.block_table + (size_t)s * A.max_blocks;
+
+  bf16x8 kf[NK], vf[NV];
+  auto load = [&](int t) {
+    if (t < np) {
+      const size_t row = pooled_row(A, bt, min(16 * t + c, nb - 1), gk);
+      const bf16 *k = (const bf16*)A.pk + row * DK + 8 * g, *v = (const bf16*)A.pv + row * DV + 8 * g;
+#pragma unroll
+      for (int m = 0; m < NK; ++m) kf[m] = *reinterpret_cast<const bf16x8*>(k + m * 32);
+#pragma unroll
+      for (int m = 0; m < NV; ++m) vf[m] = *reinterpret_cast<const bf16x8*>(v + m * 32);
+    } else {
+      const size_t page = (size_t)bt[p_lo + t - np] * A.G + gk;
+      const bf16 *k = (const bf16*)A.kp + page * (DK * 16) + lane * 8, *v = (const bf16*)A.vp + page * (DV * 16) + lane * 8;
+#pragma unroll
+      for (int m = 0; m < NK; ++m) kf[m] = *reinterpret_cast<const bf16x8*>(k + m * 512);
+#pragma unroll
+      for (int m = 0; m < NV; ++m) vf[m] = *reinterpret_cast<const bf16x8*>(v + m * 512);
+    }
+  };
+  // the wave's first tile is under way while the queries are staged
+  if (t_begin + wid < t_end) load(t_begin + wid);
+  char* sq = smem + NW * (DV * 32);
+  for (int m = wid; m < NK; m += NW)
+    *reinterpret_cast<bf16x8*>(sq + m * 1024 + lane * 16) =
+        *reinterpret_cast<const bf16x8*>((const bf16*)A.q + row_of(cb * 16 + c) * DK + 32 * m + 8 * g);
+  __syncthreads();
+  f32x4 o[2 * NV];
+#pragma unroll
+  for (int n = 0; n < 2 * NV; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m_run = NEG_BIG, l_run = 0.f;
+  char* my = smem + wid * (DV * 32);  // 16 keys x DV dims
+  const int loff = lane * 16;         // this lane's 16 B of a k-step
+  const int toff = ((c & 3) >> 1) * 256 + (4 * g + (c >> 2)) * 16 + (c & 1) * 8;
+
+  for (int t = t_begin + wid; t < t_end; t += NW) {
+    f32x4 sc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int m = 0; m < NK; ++m) {
+      const bf16x8 qf = *reinterpret_cast<const bf16x8*>(sq + m * 1024 + loff);
+      sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[m], qf, sc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int m = 0; m < NV; ++m) *reinterpret_cast<bf16x8*>(my + m * 1024 + loff) = vf[m];
+    if (t + NW < t_end) load(t + NW);
+    float tmax = NEG_BIG;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int e = 4 * g + r, key = 16 * (p_lo + t - np) + e;
+      const bool ok = t < np ? 16 * t + e < cnb : (key <= cpos && key >= klo);
+      sc[r] = ok ? sc[r] * A.scale_log2 : NEG_BIG;
+      tmax = fmaxf(tmax, sc[r]);
+    }
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
+    const float m_new = fmaxf(m_run, tmax);
+    if (__any(m_new > m_run)) {
+      const float alpha = exp2f(m_run - m_new);
+      l_run *= alpha;
+#pragma unroll
+      for (int n = 0; n < 2 * NV; ++n) o[n] *= alpha;
+      m_run = m_new;
+    }
+    bf16x4 pf;
+    const float nm = m_run < 0.01f * NEG_BIG ? 0.f : m_run;  // (a column without a key yet: weights of 0)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float e = exp2f(sc[r] - nm);
+      l_run += e;
+      pf[r] = (bf16)e;
+    }
+    // the tile is private to the wave: its LDS operations complete in order
+    const s16x4 pb = __builtin_bit_cast(s16x4, pf);
+#pragma unroll
+    for (int n = 0; n < 2 * NV; ++n) {
+      const s16x4 v = __builtin_bit_cast(s16x4, tr_read(my + n * 512 + toff));
+      o[n] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(v, pb, o[n], 0, 0, 0);
+    }
+  }
+  l_run += __shfl_xor(l_run, 16, 64);
+  l_run += __shfl_xor(l_run, 32, 64);
+
+  // merge the waves, 128 dims at a time
+  float* mo = reinterpret_cast<float*>(smem);                           // [NW][16][MERGE_LD]
+  float* mm = reinterpret_cast<float*>(smem + NW * 16 * MERGE_LD * 4);  // [NW][16]
+  float* ml = mm + NW * 16;
+  __syncthreads();
+  if (g == 0) {
+    mm[wid * 16 + c] = m_run;
+    ml[wid * 16 + c] = l_run;
+  }
+  const int ccol = threadIdx.x >> 5, d4 = (threadIdx.x & 31) * 4;
+  const bool cvalid = cb * 16 + ccol < cols;
+  const size_t orow = row_of(cb * 16 + ccol), prow = (((size_t)gk * A.max_items + pidx) * A.NB + cb) * 16 + ccol;
+  float wgt[NW], L = 0.f, mt = NEG_BIG;
+#pragma unroll
+  for (int b = 0; b < (NV + 3) / 4; ++b) {
+    if (b) __syncthreads();
+#pragma unroll
+    for (int n = 0; n < 8; ++n)
+      if (b * 8 + n < 2 * NV) *reinterpret_cast<f32x4*>(mo + (wid * 16 + c) * MERGE_LD + 16 * n + 4 * g) = o[b * 8 + n];
+    __syncthreads();
+    if (b == 0) {
+#pragma unroll
+      for (int w = 0; w < NW; ++w) mt = fmaxf(mt, mm[w * 16 + ccol]);
+#pragma unroll
+      for (int w = 0; w < NW; ++w) {
+        wgt[w] = exp2f(mm[w * 16 + ccol] - mt);
+        L += wgt[w] * ml[w * 16 + ccol];
+      }
+    }
+    const int d0 = b * 128 + d4;
+    if (d0 < DV) {
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int w = 0; w < NW; ++w)
+        acc += wgt[w] * *reinterpret_cast<const f32x4*>(mo + (w * 16 + ccol) * MERGE_LD + d4);
+      if (nparts > 1) {
+        *reinterpret_cast<f32x4*>(A.part_o + prow * DV + d0) = acc;
+      } else if (cvalid) {
+        const float f = final_scale(A.sink, mt, L);
+        bf16x4 v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = (bf16)(acc[j] * f);
+        *reinterpret_cast<bf16x4*>((bf16*)A.out + orow * DV + d0) = v;
+      }
+    }
+  }
+  if (nparts > 1 && (threadIdx.x & 31) == 0) reinterpret_cast<float2*>(A.part_ml)[prow] = float2{mt, L};
+}
+
+// The partitions of an item, merged: a wave per (item, KV head, column), 4 dims per lane and step.
+template <int NV>
+__global__ __launch_bounds__(256) void merge_kernel(const Args A) {
+  constexpr int DV = 32 * NV, NE = (DV + 255) / 256;
+  const int lane = threadIdx.x & 63, gk = blockIdx.z;
+  const int n = A.n_items[0];
+  for (int item = blockIdx.y; item < n; item += gridDim.y) {
+    const int4 it = A.items[item];
+    const int nq = it.z & 0xff, nparts = it.z >> 20;
+    if (nparts <= 1 || ((it.z >> 8) & 0xfff) != 0) continue;
+    const int step = nq <= A.dec_tokens ? 1 : 8;  // slots of a partition
+    for (int col = blockIdx.x * 4 + (threadIdx.x >> 6); col < nq * A.R; col += gridDim.x * 4) {
+      auto slot = [&](int p) { return ((size_t)gk * A.max_items + it.w + p * step) * A.NB * 16 + col; };
+      const float2* ml = reinterpret_cast<const float2*>(A.part_ml);
+      float gm = NEG_BIG, L = 0.f;
+      for (int p0 = 0; p0 < nparts; p0 += 64) gm = fmaxf(gm, p0 + lane < nparts ? ml[slot(p0 + lane)].x : NEG_BIG);
+      gm = wave_max(gm);
+      f32x4 a[NE];
+#pragma unroll
+      for (int e = 0; e < NE; ++e) a[e] = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int p0 = 0; p0 < nparts; p0 += 64) {
+        float w = 0.f;
+        if (p0 + lane < nparts) {
+          const float2 v = ml[slot(p0 + lane)];
+          w = exp2f(v.x - gm);
+          L += w * v.y;
+        }
+        const int np = min(64, nparts - p0);
+#pragma unroll 8
+        for (int p = 0; p < np; ++p) {
+          const float wp = __shfl(w, p, 64);
+#pragma unroll
+          for (int e = 0; e < NE; ++e)
+            a[e] += wp * *reinterpret_cast<const f32x4*>(A.part_o + slot(p0 + p) * DV + min(e * 256 + lane * 4, DV - 4));
+        }
+      }
+      const float f = final_scale(A.sink, gm, wave_sum(L));
+      const int t = col / A.R;
+      bf16* o = (bf16*)A.out + ((size_t)(A.q_start[it.x] + it.y + t) * A.H + gk * A.R + (col - t * A.R)) * DV;
+#pragma unroll
+      for (int e = 0; e < NE; ++e) {
+        const int d = e * 256 + lane * 4;
+        if (d < DV) {
+          bf16x4 v;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[j] = (bf16)(a[e][j] * f);
+          *reinterpret_cast<bf16x4*>(o + d) = v;
+        }
+      }
+    }
+  }
+}
+
+template <int NK, int NV>
+__device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* smem) {
+  constexpr int DK = 32 * NK, DV = 32 * NV, HALF = (NK + NV) * 1024, TILE = 2 * HALF;  // two 16-key halves: K, V
+  const int s = it.x, qb = it.y, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff, nparts = it.z >> 20;
+  const int cols = nq * A.R, cw = blockIdx.x * (16 * NW), gk = blockIdx.z;
+  if (cw >= cols) return;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
+  const int ctx = A.ctx_len[s], ql = A.q_len[s];
+  const int pos0 = ctx - ql + qb;
+  const int* bt = A.block_table + (size_t)s * A.max_blocks;
+  const int ci = cw + wid * 16 + c, cc = min(ci, cols - 1), ct = cc / A.R;
+  const int cpos = pos0 + ct, klo = first_key(A, cpos), cnb = blocks_of(A, cpos);
+  const size_t row = (size_t)(A.q_start[s] + qb + ct) * A.H + gk * A.R + (cc - ct * A.R);
+  const int loff = lane * 16;
+  bf16x8 qf[NK];
+#pragma unroll
+  for (int m = 0; m < NK; ++m) qf[m] = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + row * DK + 32 * m + 8 * g);
+  // positions of the workgroup's columns -> its tiles of 32: pooled blocks, then tokens
+  const int f = pos0 + cw / A.R, e = pos0 + min(cw + 16 * NW - 1, cols - 1) / A.R;
+  const int nb = blocks_of(A, e), np = (nb + 31) >> 5;
+  const int k_lo = first_key(A, f) >> 5;
+  int t_lo = 0, t_hi = np + ((e + 32) >> 5) - k_lo;
+  if (nparts > 1) {  // this partition's tiles (possibly none)
+    const int per = (t_hi + nparts - 1) / nparts;
+    t_lo = part * per;
+    t_hi = min(t_hi, t_lo + per);
+  }
+  const int nblk = (ctx + 15) >> 4;
+  // this wave's columns: a tile whose keys all of them see needs no mask
+  const int wf = pos0 + min(cw + wid * 16, cols - 1) / A.R;
+  const int we = pos0 + min(cw + wid * 16 + 15, cols - 1) / A.R;
+  const int full_lo = A.window > 0 ? we - A.window + 1 : 0, full_hi = wf, full_nb = blocks_of(A, wf);
+
+  f32x4 o[2 * NV];
+#pragma unroll
+  for (int n = 0; n < 2 * NV; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m_run = NEG_BIG, l_run = 0.f;
+  // direct loads, 1 KB per wave and instruction; a token page is copied linearly, pooled rows by lane
+  auto issue = [&](int t, char* dst) {
+    const bf16 *k[2], *v[2];
+    int sk, sv;
+    if (t < np) {
+#pragma unroll
+      for (int x = 0; x < 2; ++x) {
+        const size_t r = pooled_row(A, bt, min(32 * t + 16 * x + c, nb - 1), gk);
+        k[x] = (const bf16*)A.pk + r * DK + 8 * g;
+        v[x] = (const bf16*)A.pv + r * DV + 8 * g;
+      }
+      sk = sv = 32;
+    } else {
+#pragma unroll
+      for (int x = 0; x < 2; ++x) {
+        const size_t r = (size_t)bt[min(2 * (k_lo + t - np) + x, nblk - 1)] * A.G + gk;
+        k[x] = (const bf16*)A.kp + r * (DK * 16) + lane * 8;
+        v[x] = (const bf16*)A.vp + r * (DV * 16) + lane * 8;
+      }
+      sk = sv = 512;
+    }
+#pragma unroll
+    for (int i = 0; i < (2 * (NK + NV) + NW - 1) / NW; ++i) {
+      const int ch = i * NW + wid;  // wave-uniform
+      if (2 * (NK + NV) % NW == 0 || ch < 2 * (NK + NV)) {
+        const int x = ch >= NK + NV, m = ch - x * (NK + NV);
+        const bf16* src = m < NK ? (x ? k[1] : k[0]) + m * sk : (x ? v[1] : v[0]) + (m - NK) * sv;
+        __builtin_amdgcn_global_load_lds((glb_void*)src, (lds_void*)(dst + ch * 1024), 16, 0, 0);
+      }
+    }
+  };
+  const int toff = ((c & 3) >> 1) * 256 + (4 * g + (c >> 2)) * 16 + (c & 1) * 8;
+  if (t_lo < t_hi) issue(t_lo, smem);
+  for (int t = t_lo; t < t_hi; ++t) {
+    char* cur = smem + ((t - t_lo) & 1) * TILE;
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();  // tile t is whole, and nobody reads the other buffer any more
+    if (t + 1 < t_hi) issue(t + 1, smem + ((t + 1 - t_lo) & 1) * TILE);
+    f32x4 sc[2];
+#pragma unroll
+    for (int k = 0; k < 2; ++k) sc[k] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int m = 0; m < NK; ++m)
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(cur + k * HALF + m * 1024 + loff);
+        sc[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[m], sc[k], 0, 0, 0);
+      }
+    const int key0 = 32 * (k_lo + t - np);  // wave-uniform
+    if (t < np ? 32 * t + 32 > full_nb : (key0 < full_lo || key0 + 31 > full_hi)) {
+#pragma unroll
+      for (int k = 0; k < 2; ++k)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int x = 16 * k + 4 * g + r, key = key0 + x;
+          if (t < np ? 32 * t + x >= cnb : (key > cpos || key < klo)) sc[k][r] = NEG_BIG;
+        }
+    }
+    float tmax = NEG_BIG;
+#pragma unroll
+    for (int k = 0; k < 2; ++k)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) tmax = fmaxf(tmax, sc[k][r]);
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
+    const float m_new = fmaxf(m_run, fmaxf(tmax * A.scale_log2, NEG_BIG));
+    if (__any(m_new > m_run)) {
+      const float alpha = exp2f(m_run - m_new);
+      l_run *= alpha;
+#pragma unroll
+      for (int n = 0; n < 2 * NV; ++n) o[n] *= alpha;
+      m_run = m_new;
+    }
+    // a column that has seen no key yet (its window starts in a later tile): every weight is 0
+    const float nm = m_run < 0.01f * NEG_BIG ? 0.f : -m_run;
+    bf16x8 pf;
+#pragma unroll
+    for (int k = 0; k < 2; ++k)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float p = __builtin_amdgcn_exp2f(fmaf(sc[k][r], A.scale_log2, nm));
+        l_run += p;
+        pf[4 * k + r] = (bf16)p;
+      }
+#pragma unroll
+    for (int n = 0; n < 2 * NV; ++n) {
+      const bf16x4 v0 = tr_read(cur + NK * 1024 + n * 512 + toff), v1 = tr_read(cur + HALF + NK * 1024 + n * 512 + toff);
+      bf16x8 v;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        v[j] = v0[j];
+        v[4 + j] = v1[j];
+      }
+      o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pf, o[n], 0, 0, 0);
+    }
+  }
+  l_run += __shfl_xor(l_run, 16, 64);
+  l_run += __shfl_xor(l_run, 32, 64);
+  if (ci >= cols) return;
+  if (nparts > 1) {  // 8 slots hold the item's columns in a row
+    const size_t pc = ((size_t)gk * A.max_items + it.w) * A.NB * 16 + ci;
+    float* po = A.part_o + pc * DV + 4 * g;
+#pragma unroll
+    for (int n = 0; n < 2 * NV; ++n) *reinterpret_cast<f32x4*>(po + 16 * n) = o[n];
+    if (g == 0) reinterpret_cast<float2*>(A.part_ml)[pc] = float2{m_run, l_run};
+    return;
+  }
+  const float fs = final_scale(A.sink, m_run, l_run);
+  bf16* orow = (bf16*)A.out + row * DV + 4 * g;
+#pragma unroll
+  for (int n = 0; n < 2 * NV; ++n) {
+    bf16x4 v;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = (bf16)(o[n][r] * fs);
+    *reinterpret_cast<bf16x4*>(orow + 16 * n) = v;
+  }
+}
+
+template <int NK, int NV>
+constexpr int lds_bytes() {
+  return std::max({2 * 2 * 1024 * (NK + NV), NW * 32 * 32 * NV + 1024 * NK, NW * 16 * MERGE_LD * 4 + 2 * NW * 16 * 4});
+}
+
+template <int NK, int NV>
+__global__ __launch_bounds__(64 * NW, 2) void mfma_kernel(const Args A) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  const int n = A.n_items[0];
+  // two passes over the workgroup's items, so that neither path's registers carry the other's
+  for (int item = blockIdx.y; item < n; item += gridDim.y) {
+    const int4 it = A.items[item];
+    if ((it.z & 0xff) <= A.dec_tokens) continue;
+    tile_item<NK, NV>(A, it, smem);
+    __syncthreads();
+  }
+  for (int item = blockIdx.y; item < n; item += gridDim.y) {
+    const int4 it = A.items[item];
+    if ((it.z & 0xff) > A.dec_tokens) continue;
+    split_item<NK, NV>(A, it, smem);
+    __syncthreads();
+  }
+}
+
+}  // namespace wa
+}  // namespace pa
+
+// (key width, value width) in 32s with MFMA kernels, smallest first
+#define PA_WA_DIMS(X) X(1, 1) X(2, 1) X(2, 2) X(3, 3) X(4, 2) X(4, 4) X(6, 4) X(6, 6) X(8, 8)
+
+// The padded widths for key size k and value size v: the first built pair that holds both, else whole
+// 32s (the simple kernel then runs).
+extern "C" void pa_window_pad(int k, int v, int* dk, int* dv) {
+  const int a = (k + 31) / 32, b = (v + 31) / 32;
+#define PA_X(K, V)         \
+  if (a <= K && b <= V) {  \
+    *dk = 32 * K;          \
+    *dv = 32 * V;          \
+    return;                \
+  }
+  PA_WA_DIMS(PA_X)
+#undef PA_X
+  *dk = 32 * a;
+  *dv = 32 * b;
+}
+
+extern "C" int pa_window_attention(int fp32, void* out, float* part_o, float* part_ml, const void* q, const void* kp,
+                                   const void* vp, const void* pk, const void* pv, const int* items,
+                                   const int* n_items, int max_items, const int* q_start, const int* q_len,
+                                   const int* ctx_len, const int* block_table, int max_blocks, int H, int G, int DK,
+                                   int DV, int dec_tokens, int tile_tokens, int window, int pool, int npb,
+                                   int max_slots, float scale_log2, float sink, int simple, hipStream_t st) {
+  if (max_items <= 0) return 0;
+  if (DK % 32 || DV % 32 || H <= 0 || G <= 0 || H % G || dec_tokens <= 0 || tile_tokens <= 0) return -1;
+  const int R = H / G, NB = (dec_tokens * R + 15) / 16;
+  pa::wa::Args A{out, part_o, part_ml, q, kp, vp, pk, pv, (const int4*)items, n_items, q_start, q_len, ctx_len,
+                 block_table, max_blocks, max_slots, H, G, R, NB, DK, DV, dec_tokens, window, pool, npb, scale_log2, sink};
+  if (!fp32 && !simple) {
+    const int cw = 16 * pa::wa::NW, gt = (tile_tokens * R + cw - 1) / cw, gx = NB > gt ? NB : gt;
+    const int gy = max_items < 256 ? 256 : (max_items < 4096 ? max_items : 4096);
+#define PA_X(K, V)                                                                                            \
+  if (DK == 32 * K && DV == 32 * V) {                                                                         \
+    constexpr int lds = pa::wa::lds_bytes<K, V>();                                                            \
+    static bool attr = false;                                                                                 \
+    if (!attr) {                                                                                              \
+      (void)hipFuncSetAttribute((const void*)pa::wa::mfma_kernel<K, V>,                                       \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, lds);                             \
+      attr = true;                                                                                            \
+    }                                                                                                         \
+    hipLaunchKernelGGL((pa::wa::mfma_kernel<K, V>), dim3(gx, gy, G), dim3(64 * pa::wa::NW), lds, st, A);      \
+    hipLaunchKernelGGL((pa::wa::merge_kernel<V>), dim3(4, std::min(gy, 256), G), dim3(256), 0, st, A);        \
+    return (int)hipGetLastError();                                                                            \
+  }
+    PA_WA_DIMS(PA_X)
+#undef PA_X
+  }
+  if (DV > 2048 || DK > 8192) return -2;
+  const dim3 grid(H, max_items < 4096 ? max_items : 4096);
+  const int lds = (DK + 256 + 4) * 4;
+  if (fp32) hipLaunchKernelGGL((pa::wa::simple_kernel<float>), grid, dim3(256), lds, st, A);
+  else hipLaunchKernelGGL((pa::wa::simple_kernel<pa::bf16>), grid, dim3(256), lds, st, A);
+  return (int)hipGetLastError();
+}

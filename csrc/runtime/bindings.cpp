@@ -156,6 +156,9 @@ PYBIND11_MODULE(_runtime, m) {
         if (d.contains("att_narrow_qcols")) c.att_narrow_qcols = d["att_narrow_qcols"].cast<int32_t>();
         if (d.contains("att_min_part")) c.att_min_part = d["att_min_part"].cast<int32_t>();
         if (d.contains("att_tile_target")) c.att_tile_target = d["att_tile_target"].cast<int32_t>();
+        if (d.contains("att_pool")) c.att_pool = d["att_pool"].cast<int32_t>();
+        if (d.contains("scan_chunk")) c.scan_chunk = d["scan_chunk"].cast<int32_t>();
+        if (d.contains("scan_min")) c.scan_min = d["scan_min"].cast<int32_t>();
         if (d.contains("att_max_keys")) c.att_max_keys = d["att_max_keys"].cast<int32_t>();
         if (d.contains("att_wide_min_tokens")) c.att_wide_min_tokens = d["att_wide_min_tokens"].cast<int32_t>();
         if (d.contains("prefill_split_keys")) c.prefill_split_keys = d["prefill_split_keys"].cast<int32_t>();
@@ -187,6 +190,8 @@ PYBIND11_MODULE(_runtime, m) {
         d["top_k"] = L.top_k; d["top_p"] = L.top_p;
         d["items"] = L.items; d["n_items"] = L.n_items; d["part_size"] = L.part_size;
         d["counts"] = L.counts; d["block_table"] = L.block_table; d["embed_rows"] = L.embed_rows;
+        d["max_scan"] = L.max_scan; d["state_slot"] = L.state_slot; d["scan_first"] = L.scan_first;
+        d["scan_items"] = L.scan_items; d["n_scan"] = L.n_scan;
         d["total"] = L.total;
         return d;
       })
@@ -238,6 +243,7 @@ PYBIND11_MODULE(_runtime, m) {
       .def("reset_prefix_cache", &Scheduler::reset_prefix_cache)
       .def_property_readonly("num_running", &Scheduler::num_running)
       .def_property_readonly("num_waiting", &Scheduler::num_waiting)
+      .def_property_readonly("num_free_states", &Scheduler::num_free_states)
       .def_property_readonly("num_free_blocks", &Scheduler::num_free_blocks)
       .def_property_readonly("num_cached_blocks", &Scheduler::num_cached_blocks)
       .def_property_readonly("total_prompt_tokens", &Scheduler::total_prompt_tokens)

@@ -47,11 +47,21 @@ Scheduler::Scheduler(const SchedulerConfig& cfg)
   L.top_k = take(L.max_seqs);
   L.top_p = take(L.max_seqs);
   L.seeds = take(2 * L.max_seqs);
+  if (cfg_.scan_chunk > 0 && cfg_.prefix_caching)
+    throw std::invalid_argument("scheduler: recurrent states are not cached with prefixes");
+  L.max_scan = cfg.scan_chunk > 0
+                   ? L.max_tokens / cfg.scan_chunk + std::min(L.max_seqs, L.max_tokens / (cfg.scan_min + 1)) + 1 : 0;
+  L.state_slot = take(L.max_seqs);
+  L.scan_first = take(L.max_seqs);
+  L.n_scan = take(1);
+  L.scan_items = take(4 * L.max_scan);
   L.items = take(4 * L.max_items);
   L.block_table = take(L.max_seqs * L.max_blocks);
   L.embed_rows = take(L.max_tokens);
   L.total = o;
   for (int32_t r = L.max_seqs; r-- > 0;) embed_free_.push_back(r);
+  if (cfg.scan_chunk > 0)
+    for (int32_t r = L.max_seqs; r-- > 0;) state_free_.push_back(r);
 }
 
 void Scheduler::add_request(int64_t id, std::vector<int32_t> prompt, float temperature,
@@ -101,9 +111,20 @@ void Scheduler::free_seq(Sequence* s, bool keep_embed_slot) {
     embed_free_.push_back(s->embed_slot);
     s->embed_slot = -1;
   }
+  if (s->state_slot >= 0) {
+    state_free_.push_back(s->state_slot);
+    s->state_slot = -1;
+  }
   for (int32_t b : s->blocks) bm_.release(b);
   s->blocks.clear();
   s->block_hashes.clear();
+}
+
+void Scheduler::take_state(Sequence* s) {
+  if (cfg_.scan_chunk <= 0 || s->state_slot >= 0) return;
+  if (state_free_.empty()) throw std::logic_error("scheduler: more admitted sequences than state slots");
+  s->state_slot = state_free_.back();
+  state_free_.pop_back();
 }
 
 void Scheduler::preempt(Sequence* s) {
@@ -271,6 +292,7 @@ int32_t Scheduler::schedule(int32_t* buf) {
     waiting_.pop_front();
     s->running = true;
     s->preempted = false;
+    take_state(s);
     running_.push_back(s);
     if (key && s->num_computed < 2 * B) inflight.insert(key);  // its leading blocks are computed now
     last_plan_.push_back({s, n, !s->embed && s->num_computed + n == (int32_t)s->tokens.size()});
@@ -344,6 +366,7 @@ int32_t Scheduler::schedule_fed(int32_t* buf, const std::vector<FedEntry>& entri
     s->tokens.insert(s->tokens.end(), e.tokens.begin(), e.tokens.end());
     s->prompt_len = (int32_t)s->tokens.size();
     if (!ensure_blocks(s, s->prompt_len)) throw std::runtime_error("scheduler: the cache pool is exhausted");
+    take_state(s);
     last_plan_.push_back({s, (int32_t)e.tokens.size(), false});
   }
   return emit(buf);
@@ -375,7 +398,7 @@ int32_t Scheduler::emit(int32_t* buf) {
   int32_t nembed = 0;
   const int32_t tpw = 16 / std::max(1, cfg_.gqa_group);
 
-  int32_t T = 0, ns = 0, nsamp = 0, nit = 0, nparted = 0, pslot = 0;
+  int32_t T = 0, ns = 0, nsamp = 0, nit = 0, nparted = 0, pslot = 0, nscan = 0;
   // decode partition size: with few decode rows, 256-key flash-decoding partitions
   // give the attention launch more workgroups. 128-key partitions lose more to the
   // extra partial merges than they gain (profiles/r1_attention_small_batch.jsonl:
@@ -398,11 +421,14 @@ int32_t Scheduler::emit(int32_t* buf) {
   const int32_t qcols = wide ? std::max(cfg_.att_narrow_qcols, cfg_.att_qcols) : cfg_.att_narrow_qcols;
   const int32_t qtile = std::max(1, qcols / std::max(1, cfg_.gqa_group));
   int32_t psz = 512;
-  // keys a decode row attends to (a model whose every layer has a window never reads more)
-  auto att_keys = [this](const Planned& p) {
-    const int32_t c = p.s->num_computed + p.n;
-    return cfg_.att_max_keys > 0 ? std::min(c, cfg_.att_max_keys + p.n - 1) : c;
+  // keys that the last n of c positions attend to (a model whose every layer has a window never
+  // reads more than it holds, and the pooled keys before it)
+  auto keys_of = [this](int32_t c, int32_t n) {
+    const int32_t w = cfg_.att_max_keys;
+    if (w <= 0 || c <= w + n - 1) return c;
+    return w + n - 1 + (cfg_.att_pool > 0 ? (c - w) / cfg_.att_pool : 0);
   };
+  auto att_keys = [&](const Planned& p) { return keys_of(p.s->num_computed + p.n, p.n); };
   if (cfg_.split_decode) {
     int64_t parts512 = 0, parts256 = 0, nprefill = 0;
     for (const Planned& p : last_plan_) {
@@ -491,6 +517,15 @@ int32_t Scheduler::emit(int32_t* buf) {
       er[T + j] = (s->embed_last && ppos + 1 != (int32_t)s->tokens.size()) ? L.max_seqs : erow;
     }
     if (s->embed_slot >= 0) nembed += n;
+    buf[L.state_slot + ns] = s->state_slot;
+    buf[L.scan_first + ns] = -1;
+    if (cfg_.scan_chunk > 0 && n > cfg_.scan_min) {
+      buf[L.scan_first + ns] = nscan;
+      for (int32_t a = 0; a < n; a += cfg_.scan_chunk) {
+        int32_t* it = buf + L.scan_items + 4 * nscan++;
+        it[0] = ns; it[1] = a; it[2] = std::min(cfg_.scan_chunk, n - a); it[3] = 0;
+      }
+    }
     const int32_t nb = (ctx + B - 1) / B;
     std::memcpy(bt + (size_t)ns * L.max_blocks, s->blocks.data(), sizeof(int32_t) * nb);
     if (p.sample) {
@@ -514,7 +549,7 @@ int32_t Scheduler::emit(int32_t* buf) {
     }
     // attention work items (mirrors pilottai_amd/ops/attn_meta.py)
     if (n <= tpw) {
-      const int32_t akeys = cfg_.att_max_keys > 0 ? std::min(ctx, cfg_.att_max_keys + n - 1) : ctx;
+      const int32_t akeys = keys_of(ctx, n);
       const int32_t nparts = cfg_.split_decode ? std::max(1, (akeys + psz - 1) / psz) : 1;
       if (nparts > 1) {
         for (int32_t q = 0; q < nparts; ++q)
@@ -546,7 +581,7 @@ int32_t Scheduler::emit(int32_t* buf) {
     int64_t total = (int64_t)pre.size() + (int64_t)dec.size();
     for (const ItemCost& c : pre) {
       const int32_t nq = c.c & 0xff;
-      const int32_t keys = cfg_.att_max_keys > 0 ? std::min(c.keys, cfg_.att_max_keys + nq - 1) : c.keys;
+      const int32_t keys = keys_of(c.keys, nq);
       const int32_t np = std::min(want, keys / 256);
       if (np >= 2 && pslot + 8 * np <= L.max_items && total + np - 1 <= L.max_items) {
         for (int32_t q = 0; q < np; ++q)
@@ -609,7 +644,10 @@ int32_t Scheduler::emit(int32_t* buf) {
     qs[r] = T;
     ql[r] = 0;
     cl[r] = 0;
+    buf[L.state_slot + r] = -1;
+    buf[L.scan_first + r] = -1;
   }
+  buf[L.n_scan] = nscan;
   counts[0] = T;
   counts[1] = ns;
   counts[2] = nsamp;
@@ -638,6 +676,7 @@ bool Scheduler::predict(Sequence* s, Planned& e) const {
   if (ng >= s->max_tokens || ntok >= cfg_.max_model_len) return false;
   e.run.clear();
   if (!s->grammar) return true;
+  if (cfg_.scan_chunk > 0) return false;
   const Grammar& g = *s->grammar;
   Grammar::Cursor c = g.cursor();
   int32_t cls, forced;

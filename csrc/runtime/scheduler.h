@@ -38,6 +38,8 @@ struct SchedulerConfig {
   // > 0: no layer attends to more than this many keys back (every layer has a window): decode rows
   // are cut into partitions of the keys they really read, not of the whole context
   int32_t att_max_keys = 0;
+  // > 0 (with att_max_keys): every att_pool keys before the window are one pooled key
+  int32_t att_pool = 0;
   int32_t att_min_part = 128;          // smallest decode partition (keys)
   // > 0: a step with fewer prefill items than this cuts each over its keys, at least 256 a partition,
   // towards this many work items (kernels whose tile path merges partitions; 8 partial slots each)
@@ -85,6 +87,11 @@ struct SchedulerConfig {
   int32_t token_align = 0;
   int32_t kv_heads = 8;                // KV heads per rank (sizes the decode partitioning)
   int32_t align_slack = 96;
+  // recurrent layers: every admitted sequence holds one of max_num_seqs state slots, and portions of
+  // more than scan_min tokens are cut into scan items of scan_chunk tokens (0: no recurrent layers).
+  // A state cannot be taken back, so grammar rows, whose speculation can fail, are not speculated.
+  int32_t scan_chunk = 0;
+  int32_t scan_min = 8;
   std::vector<int32_t> eos_ids;
 };
 
@@ -92,6 +99,11 @@ struct StepLayout {
   int32_t max_tokens, max_seqs, max_blocks, max_items;
   int32_t input_ids, positions, slots, q_start, q_len, ctx_len, logit_rows, mask_class, forced,
       offsets, temperature, top_k, top_p, seeds, items, n_items, part_size, counts, block_table, total;
+  int32_t max_scan;    // scan items (recurrent layers)
+  int32_t state_slot;  // [max_seqs]: state slot of each sequence, -1 = none
+  int32_t scan_first;  // [max_seqs]: first scan item of each sequence, -1 = its portion has none
+  int32_t scan_items;  // [max_scan, 4]: sequence, first token of the portion, tokens, 0
+  int32_t n_scan;
   int32_t embed_rows;  // [max_tokens]: pooling row of each token (embedding requests), max_seqs = none
 };
 
@@ -125,6 +137,7 @@ struct Sequence {
   int32_t num_sampled = 0;
   int32_t num_forced = 0;
   int32_t cached_prompt_tokens = -1;
+  int32_t state_slot = -1;      // recurrent layers: held while admitted
   std::vector<int32_t> blocks;
   std::vector<uint64_t> block_hashes;  // hash chain of registered leading blocks
   std::unique_ptr<Grammar> grammar;
@@ -221,11 +234,13 @@ class Scheduler {
     int32_t embed_slot, num_computed, num_tokens, num_blocks;
   };
   std::vector<SeqState> debug_state() const;  // every live sequence (diagnostics)
+  int32_t num_free_states() const { return (int32_t)state_free_.size(); }
   int32_t num_free_embed_rows() const { return (int32_t)embed_free_.size(); }
 
  private:
   int32_t emit(int32_t* buf);  // write last_plan_ into buf and queue it as an uncommitted step
   bool ensure_blocks(Sequence* s, int32_t upto_tokens);
+  void take_state(Sequence* s);
   void preempt(Sequence* s);
   void match_prefix(Sequence* s);
   void register_full_blocks(Sequence* s);
@@ -261,6 +276,7 @@ class Scheduler {
   std::vector<Sequence*> abort_wait_;               // aborted while listed by an in-flight step  // finished, still listed by an in-flight plan
   int64_t stat_spec_rows_ = 0, stat_spec_voided_ = 0;
   std::vector<SeqOutput> aborted_;
+  std::vector<int32_t> state_free_;    // free state slots (0 .. max_seqs - 1)
   std::vector<int32_t> embed_free_;    // free pooling rows (0 .. max_seqs - 1)
   std::vector<int32_t> embed_resets_;  // rows of preempted embedding requests, to be cleared
   int64_t arrival_counter_ = 0;

@@ -1,6 +1,6 @@
 """In-tree builder for the native parts of pilottai_amd.
 
-Three shared objects are produced next to the Python sources so they travel with
+Four shared objects are produced next to the Python sources so they travel with
 the repository snapshot to the GPU box:
 
 * ``pilottai_amd/_C.so``       — CDNA4 HIP kernels (csrc/ops/*.hip, gfx950 only)
@@ -8,6 +8,8 @@ the repository snapshot to the GPU box:
 * ``pilottai_amd/_latent.so`` — the kernels of models with latent attention and table-routed
                                   experts, with the packed projections they share (so that
                                   such a model needs no other kernel to run)
+* ``pilottai_amd/_hybrid.so`` — likewise for models with windowed pooled attention, state-space layers,
+                                  score-routed experts and hyper-connected residuals
 * ``pilottai_amd/_runtime.so`` — C++ serving runtime: paged-KV block manager,
                                   prefix cache, continuous-batching scheduler,
                                   grammar FSM + tokenizer (csrc/runtime/*.cpp),
@@ -38,9 +40,14 @@ HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # No file may use packed fp32 arithmetic (v_pk_*_f32): some forms have given wrong results.
 HIP_FLAGS = ["-ffast-math", "-fno-gpu-rdc", "-Wno-unused-result", "-Xclang", "-target-feature", "-Xclang",
              "-packed-fp32-ops"]
-# the sources of _latent.so; the GEMM sources are in _C.so too
-LATENT_HIP = ["grouped_gemm.hip", "latent_attention.hip", "latent_cache.hip", "residual_norm.hip"]
+# kernel modules of the families beside Llama: sources and bindings; the GEMM sources are in _C.so too
 SHARED_HIP = ["gemm_decode.hip", "gemm_prefill.hip"]
+MODULES = {
+    "latent": (["grouped_gemm.hip", "latent_attention.hip", "latent_cache.hip", "residual_norm.hip"], "bindings_latent.cpp"),
+    "hybrid": (["grouped_gemm.hip", "hyper_norm.hip", "paged_kv.hip", "score_route.hip", "state_scan.hip",
+                "window_attention.hip"], "bindings_hybrid.cpp"),
+}
+FAMILY_HIP = {h for hips, _ in MODULES.values() for h in hips}
 FILE_FLAGS = {"gemm_mid.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"],
               "gemm_stream.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"]}
 
@@ -126,14 +133,15 @@ def _build_ext(name: str, hips, binding: str, verbose: bool, workers: int | None
 
 
 def build_ops(verbose: bool = False, workers: int | None = None) -> Path:
-    """pilottai_amd/_C.so: every kernel but the latent-attention models' own."""
+    """pilottai_amd/_C.so: every kernel but the other families' own."""
     hips = sorted(Path(p).name for p in glob.glob(str(CSRC / "ops" / "*.hip")))
-    return _build_ext("_C", [h for h in hips if h not in LATENT_HIP], "bindings.cpp", verbose, workers)
+    return _build_ext("_C", [h for h in hips if h not in FAMILY_HIP], "bindings.cpp", verbose, workers)
 
 
-def build_latent(verbose: bool = False, workers: int | None = None) -> Path:
-    """pilottai_amd/_latent.so: what a latent-attention model runs."""
-    return _build_ext("_latent", LATENT_HIP + SHARED_HIP, "bindings_latent.cpp", verbose, workers)
+def build_family(kind: str, verbose: bool = False, workers: int | None = None) -> Path:
+    """pilottai_amd/_<kind>.so: what a model of that family runs."""
+    hips, binding = MODULES[kind]
+    return _build_ext("_" + kind, hips + SHARED_HIP, binding, verbose, workers)
 
 
 def build_runtime(verbose: bool = False, workers: int | None = None) -> Path:
@@ -162,24 +170,26 @@ def _stale(so: Path, sources) -> bool:
     return not so.exists() or so.stat().st_mtime < _newest(sources)
 
 
-def ensure(kind: str = "latent", gpu: bool = True) -> None:
+def ensure(kind: str, gpu: bool = True) -> None:
     """Build what running a model of `kind` needs, where it is missing or older than its sources: the
-    serving runtime and, for a GPU, the kernel module ("latent": _latent, "llama": _C). One process
+    serving runtime and, for a GPU, the kernel module (_latent, _hybrid, or _C for "llama"). One process
     builds at a time; the others wait for it."""
     import fcntl
 
     ext = sysconfig.get_config_var("EXT_SUFFIX")
-    ops_dir, name = CSRC / "ops", {"latent": "_latent", "llama": "_C"}[kind]
+    ops_dir = CSRC / "ops"
     srcs = [str(p) for p in ops_dir.glob("*.h")]
-    if kind == "latent":
-        srcs += [str(ops_dir / h) for h in LATENT_HIP + SHARED_HIP + ["bindings_latent.cpp"]]
+    if kind in MODULES:
+        hips, binding = MODULES[kind]
+        name, srcs = "_" + kind, srcs + [str(ops_dir / h) for h in hips + SHARED_HIP + [binding]]
     else:
-        srcs += [str(p) for p in ops_dir.glob("*.hip") if p.name not in LATENT_HIP] + [str(ops_dir / "bindings.cpp")]
+        name = "_C"
+        srcs += [str(p) for p in ops_dir.glob("*.hip") if p.name not in FAMILY_HIP] + [str(ops_dir / "bindings.cpp")]
     rt = [str(p) for p in (CSRC / "runtime").glob("*.*")]
+    build_kernels = (lambda: build_family(kind)) if kind in MODULES else build_ops
 
     def todo():
-        return [f for f, so, src in ((build_runtime, PKG / ("_runtime" + ext), rt),
-                                     (build_latent if kind == "latent" else build_ops, PKG / (name + ext), srcs))
+        return [f for f, so, src in ((build_runtime, PKG / ("_runtime" + ext), rt), (build_kernels, PKG / (name + ext), srcs))
                 if _stale(so, src) and (gpu or f is build_runtime)]
 
     if not todo():
@@ -196,7 +206,8 @@ def build_all(verbose: bool = False, force: bool = False) -> None:
     _FORCE = force
     try:
         build_runtime(verbose)
-        build_latent(verbose)
+        for kind in MODULES:
+            build_family(kind, verbose)
         build_ops(verbose)
     finally:
         _FORCE = False

@@ -268,13 +268,14 @@ class LLMEngine:
             self.model.PF_MIDRANGE = frozenset(cfg.pf_midrange)
         self.load_time = time.time() - t0
         # ---- KV cache sizing (288 GB HBM: the default leaves room for graphs/activations)
-        bpb = self.model.cache_bytes_per_block(cfg.block_size)
+        bpb = max(1, self.model.cache_bytes_per_block(cfg.block_size))
+        state = cfg.max_num_seqs * self.model.state_bytes_per_slot()  # recurrent layers: one slot per sequence
         nb = cfg.num_kv_blocks
         if nb is None:
             if cfg.kv_cache_gb is not None:
                 nb = int(cfg.kv_cache_gb * (1 << 30)) // bpb
             elif self.on_gpu:
-                free, _total = torch.cuda.mem_get_info(self.device)
+                free = torch.cuda.mem_get_info(self.device)[0] - state
                 # a fraction of what is free, but never into the reserve: beside a 205 GB
                 # memory index (config 4) 15 % of the rest is too little for the graphs
                 nb = int(max(0.0, min(free * cfg.kv_cache_fraction, free - cfg.kv_reserve_gb * (1 << 30)))) // bpb
@@ -287,7 +288,7 @@ class LLMEngine:
             t = torch.tensor([nb], dtype=torch.int64)
             torch.distributed.all_reduce(t, op=torch.distributed.ReduceOp.MIN, group=self.tp.cpu_group)
             nb = int(t.item())
-        self.kv = self.model.make_cache(nb, cfg.block_size)
+        self.kv = self.model.make_cache(nb, cfg.block_size, cfg.max_num_seqs)
         self.num_kv_blocks = nb
         # ---- native scheduler + step buffers
         # the model runs 8-wave decode attention on the fused decode path only, keyed on the
@@ -452,7 +453,9 @@ class LLMEngine:
             n_items=sl("n_items", 1),
             att_counters=self._att_counters,
             part_size=sl("part_size", 1),
-            logit_rows=sl("logit_rows", ms))
+            logit_rows=sl("logit_rows", ms),
+            state_slot=sl("state_slot", ms), scan_first=sl("scan_first", ms),
+            scan_items=sl("scan_items", 4 * L["max_scan"]).view(L["max_scan"], 4), n_scan=sl("n_scan", 1))
         self._temp = sl("temperature", ms).view(torch.float32)
         self._top_k = sl("top_k", ms)
         self._top_p = sl("top_p", ms).view(torch.float32)
@@ -479,7 +482,8 @@ class LLMEngine:
         n_it = self._items_for_bucket(bucket, s_b)
         return StepMeta(m.input_ids, m.positions, m.slots, m.q_start, m.q_len, m.ctx_len,
                         m.block_table, m.items[:n_it], m.n_items, m.att_counters, m.logit_rows, num_seqs=ns,
-                        part_size=m.part_size)
+                        part_size=m.part_size, state_slot=m.state_slot, scan_first=m.scan_first,
+                        scan_items=m.scan_items, n_scan=m.n_scan)
 
     def _forward_and_sample(self, bucket: int, s_b: int, ns: int, trunc: bool = False, embed: bool = False):
         if self._sample_ws is None and self.on_gpu:  # (before graph capture: its warm-up runs come first)

@@ -30,15 +30,14 @@ to whole MFMA tiles, so any sizes run on the same kernels.
 """
 from __future__ import annotations
 
-import os
 from dataclasses import dataclass, field
 from typing import Dict, List, Optional, Tuple
 
 import torch
-import torch.nn.functional as F
 
 from pilottai_amd import ops
 from pilottai_amd.models.cache import LatentKVCache, StepMeta
+from pilottai_amd.models.common import PackedLinear, checkpoint_reader, expert_tile_rows, layer_runs, parse_loop
 from pilottai_amd.ops import reference as ref
 from pilottai_amd.ops.latent import latent_pad, pad_to
 from pilottai_amd.parallel.comm import TPGroup
@@ -94,13 +93,7 @@ class BozupelConfig:
 
     def runs(self) -> List[Tuple[int, bool]]:
         """(layer, whether a repeated pass starts here) for every layer run of a step, in order."""
-        n = len(self.layers)
-        start, stop, times = self.loop or (0, 0, 1)
-        out = []
-        for again in range(times):
-            lo = start if again else 0
-            out += [(i, again > 0 and i == start) for i in range(lo, stop)]
-        return out + [(i, False) for i in range(stop, n)]
+        return layer_runs(self.num_layers, self.loop)
 
     @classmethod
     def from_dict(cls, d: dict, name: str = "bozupel") -> "BozupelConfig":
@@ -123,13 +116,9 @@ class BozupelConfig:
                 mlp = TableExpertsSpec(experts=int(p["router"]["experts"]), top=int(p["router"]["top"]),
                                        ff=int(p["expert"]["ff"]), limit=float(p["expert"]["limit"]))
             layers.append(BozupelLayer(mixer, mlp))
-        loop = d.get("loop")
-        if loop:
-            loop = (int(loop["start"]), int(loop["stop"]), int(loop["times"]))
-            if not (0 <= loop[0] < loop[1] <= len(layers) and loop[2] >= 1):
-                raise ValueError(f"loop {loop} does not fit {len(layers)} layers")
         return cls(name=name, vocab_size=int(d["vocab"]), hidden_size=int(d["width"]), layers=layers,
-                   eps=float(d["norm"]["eps"]), logit_scale=float(d.get("logit_scale", 1.0)), loop=loop or None)
+                   eps=float(d["norm"]["eps"]), logit_scale=float(d.get("logit_scale", 1.0)),
+                   loop=parse_loop(d.get("loop"), len(layers)))
 
     def num_params(self) -> int:
         d, n = self.hidden_size, 2 * self.vocab_size * self.hidden_size + self.hidden_size
@@ -166,25 +155,6 @@ PRESETS: Dict[str, BozupelConfig] = {
 }
 
 
-class _Linear:
-    """y = x W^T with W [N, K] padded to [128 n, 64 k] by zeros: the packed projections in bf16
-    (decode kernel up to 64 rows, prefill kernel above), the library's fp32 GEMM in fp32."""
-
-    def __init__(self, w: torch.Tensor, dtype, device):
-        N, K = w.shape
-        full = torch.zeros(pad_to(N, 128), pad_to(K, 64), dtype=dtype, device=device)
-        full[:N, :K] = w.to(device=device, dtype=dtype)
-        self.N, self.K = full.shape
-        self.w = ops.pack_decode_weight(full) if dtype == torch.bfloat16 else full
-
-    def __call__(self, x: torch.Tensor) -> torch.Tensor:
-        if self.w.dim() == 2:
-            return F.linear(x, self.w)
-        if x.shape[0] <= 64:
-            return ops.decode_gemm(x, self.w)
-        return ops.prefill_gemm(x, self.w)
-
-
 class LatentAttention:
     """Latent attention over the paged latent cache, queries absorbed into the latent space."""
 
@@ -195,13 +165,13 @@ class LatentAttention:
         self.np, self.rp, self.vp = pad_to(n, 32), pad_to(r, 32), pad_to(vd, 16)
         self.Rp = latent_pad(R)
         self.D = self.Rp + self.rp
-        self.down = _Linear(torch.cat([t["dq"], t["dkv"]], 0), dtype, device)
+        self.down = PackedLinear(torch.cat([t["dq"], t["dkv"]], 0), dtype, device)
         self.w_q = t["dq.norm"].float().to(device)
         self.w_c = t["dkv.norm"].float().to(device)
         q = t["uq"].view(H, n + r, m.q_rank)
         uq = torch.zeros(H, self.np + self.rp, m.q_rank, dtype=q.dtype, device=q.device)
         uq[:, :n], uq[:, self.np:self.np + r] = q[:, :n], q[:, n:]
-        self.uq = _Linear(uq.view(-1, m.q_rank), dtype, device)
+        self.uq = PackedLinear(uq.view(-1, m.q_rank), dtype, device)
         uk = torch.zeros(H, self.Rp, self.np, dtype=dtype, device=device)
         uk[:, :R, :n] = t["uk"].to(device).view(H, n, R).transpose(1, 2)
         self.uk = ops.pack_groups(uk, dtype)
@@ -211,7 +181,7 @@ class LatentAttention:
         d = t["o"].shape[0]
         o = torch.zeros(d, H, self.vp, dtype=t["o"].dtype, device=t["o"].device)
         o[:, :, :vd] = t["o"].view(d, H, vd)
-        self.o = _Linear(o.view(d, -1), dtype, device)
+        self.o = PackedLinear(o.view(d, -1), dtype, device)
 
     def tensors(self):
         return [self.down.w, self.uq.w, self.uk, self.uv, self.o.w]
@@ -281,6 +251,7 @@ class BozupelModel:
     EXPERT_ROWS_64 = 32
     EXPERT_ROWS_256 = 96
     decode_packed = True
+    KERNELS = "latent"  # the module of its kernels (_build.py)
 
     def __init__(self, cfg: BozupelConfig, device, dtype=torch.bfloat16, tp: Optional[TPGroup] = None, seed: int = 0,
                  weights_path: Optional[str] = None, max_len: int = 8192, **_):
@@ -297,7 +268,7 @@ class BozupelModel:
         group = min(heads, 16)
         self.dec_tokens, self.tile_tokens = 16 // group, 128 // group  # tokens of an attention work item
         self._group = group
-        get = self._checkpoint(weights_path) if weights_path else self._random(seed)
+        get = checkpoint_reader(weights_path) if weights_path else self._random(seed)
         eps, d = cfg.eps, cfg.hidden_size
         rot: Dict[tuple, torch.Tensor] = {}
         f32 = lambda name: get(name, (d,)).float().to(self.device)  # noqa: E731
@@ -332,32 +303,13 @@ class BozupelModel:
         self.tables = torch.cat([t.reshape(-1) for t in tables]).to(self.device) if tables else None
         self.norm = f32("final.norm")
         self.norm_scaled = self.norm * cfg.logit_scale  # logits = head . norm(x) * logit_scale
-        self.head = _Linear(get("head", (cfg.vocab_size, d)), dtype, self.device)
+        self.head = PackedLinear(get("head", (cfg.vocab_size, d)), dtype, self.device)
         self._route_desc: Dict[tuple, tuple] = {}
         if self.device.type == "cuda" and dtype == torch.bfloat16:  # before any graph capture
             ops.decode_workspace(self.device)
             ops.prefill_workspace(self.device)
 
     # -- weights -----------------------------------------------------------------
-    @staticmethod
-    def _checkpoint(path: str):
-        from safetensors import safe_open
-
-        where = {}
-        for f in sorted(os.listdir(path)):
-            if f.endswith(".safetensors"):
-                fh = safe_open(os.path.join(path, f), framework="pt")
-                where.update({k: fh for k in fh.keys()})
-
-        def get(name, shape):
-            if name not in where:
-                raise ValueError(f"{path}: tensor {name!r} is missing")
-            t = where[name].get_tensor(name)
-            if tuple(t.shape) != tuple(shape):
-                raise ValueError(f"{path}: {name} has shape {tuple(t.shape)}, the configuration gives {tuple(shape)}")
-            return t
-        return get
-
     def _random(self, seed: int):
         cfg, dev = self.cfg, self.device
         g = torch.Generator(device=dev).manual_seed(seed)
@@ -386,7 +338,10 @@ class BozupelModel:
     def cache_bytes_per_block(self, block_size: int) -> int:
         return LatentKVCache.bytes_per_block(self._widths(), self.embed.element_size(), block_size)
 
-    def make_cache(self, num_blocks: int, block_size: int) -> LatentKVCache:
+    def state_bytes_per_slot(self) -> int:
+        return 0  # no recurrent layers
+
+    def make_cache(self, num_blocks: int, block_size: int, slots: int = 0) -> LatentKVCache:
         return LatentKVCache(self._widths(), num_blocks, self.device, self.dtype, block_size)
 
     def attention_items(self) -> dict:
@@ -414,10 +369,9 @@ class BozupelModel:
         dev = self.device
         if T not in self._route_desc:  # (before graph capture: the capture's warm-up runs come first)
             per = T * max(p.top / p.experts for p in mlps)  # rows an expert gets on average
-            tm, rows, tab, o, t = 16, [], 0, 0, 0
-            if self.dtype == torch.bfloat16 and per > self.EXPERT_ROWS_64:
-                ok = min(min(L["mlp"].fp for L in self.layers if L["mlp"]), pad_to(self.cfg.hidden_size, 64)) >= 128
-                tm = 256 if ok and per > self.EXPERT_ROWS_256 else 64
+            rows, tab, o, t = [], 0, 0, 0
+            min_k = min([L["mlp"].fp for L in self.layers if L["mlp"]] + [pad_to(self.cfg.hidden_size, 64)])
+            tm = expert_tile_rows(per, self.dtype, min_k, self.EXPERT_ROWS_64, self.EXPERT_ROWS_256)
             for p in mlps:
                 n = T * p.top
                 cap = n // tm + min(p.experts, n)

@@ -7,6 +7,9 @@ manager (csrc/runtime) know nothing of what a page holds:
   LatentKVCache  one latent row per token for all heads (latent attention), one pool per layer RUN:
                  a layer that a looped stack runs several times has a pool for each pass, and
                  layers of different widths have pools of their own widths
+  HybridCache    per layer run, per-head keys and values with their pooled blocks, or the state slots
+                 of a recurrent layer, which belong to sequences (the scheduler hands them out) and
+                 not to pages
 """
 from __future__ import annotations
 
@@ -32,6 +35,11 @@ class StepMeta:
     logit_rows: torch.Tensor
     num_seqs: int = 0  # host-side count, used only by the CPU reference path
     part_size: Optional[torch.Tensor] = None  # device int[1]: decode partition size of the step
+    # recurrent layers: each sequence's state slot and first scan item, the step's scan items
+    state_slot: Optional[torch.Tensor] = None
+    scan_first: Optional[torch.Tensor] = None
+    scan_items: Optional[torch.Tensor] = None
+    n_scan: Optional[torch.Tensor] = None
 
 
 class KVCache:
@@ -71,3 +79,38 @@ class LatentKVCache:
 
     def nbytes(self) -> int:
         return sum(p.numel() * p.element_size() for p in self.pages)
+
+
+class HybridCache:
+    """One entry of `layers` per layer run. An attention run has (keys [blocks, G, DK/8, 16, 8], values alike,
+    pooled keys [blocks, per page, G, DK], pooled values): a pooled block lies with the page of its last
+    token (csrc/ops/paged_kv.hip). A recurrent run has (state fp32 [slots, H, V, N], ring of the
+    convolution's inputs [slots, rows, channels]); a sequence that starts overwrites what its slot held."""
+
+    def __init__(self, kinds: Sequence[tuple], num_blocks: int, slots: int, device, dtype=torch.bfloat16,
+                 block_size: int = 16):
+        if block_size != 16:
+            raise ValueError("pages hold 16 tokens")
+        self.num_blocks, self.slots, self.block_size = num_blocks, slots, block_size
+        zeros = lambda dt, *s: torch.zeros(*s, dtype=dt, device=device)  # noqa: E731
+        self.layers: List[tuple] = []
+        for kind, *n in kinds:
+            if kind == "attention":
+                G, dk, dv, per = n
+                self.layers.append((zeros(dtype, num_blocks, G, dk // 8, 16, 8), zeros(dtype, num_blocks, G, dv // 8, 16, 8),
+                                    zeros(dtype, num_blocks if per else 0, per, G, dk),
+                                    zeros(dtype, num_blocks if per else 0, per, G, dv)))
+            else:
+                H, V, N, rows, channels = n
+                self.layers.append((zeros(torch.float32, slots, H, V, N), zeros(dtype, slots, rows, channels)))
+
+    @staticmethod
+    def bytes_per_block(kinds: Sequence[tuple], itemsize: int, block_size: int = 16) -> int:
+        return sum(n[0] * (n[1] + n[2]) * (block_size + n[3]) * itemsize for kind, *n in kinds if kind == "attention")
+
+    @staticmethod
+    def bytes_per_slot(kinds: Sequence[tuple], itemsize: int) -> int:
+        return sum(4 * n[0] * n[1] * n[2] + n[3] * n[4] * itemsize for kind, *n in kinds if kind == "state")
+
+    def nbytes(self) -> int:
+        return sum(t.numel() * t.element_size() for ts in self.layers for t in ts)

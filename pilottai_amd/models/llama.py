@@ -105,6 +105,7 @@ DENSE_KINDS = ("wqkv", "wo", "w13", "w2")
 
 
 class LlamaModel:
+    KERNELS = "llama"  # the module of its kernels (_build.py)
     # decode steps of at most this many tokens run the fused packed-weight path
     # (csrc/ops/gemm_decode.hip; tools/decode_gemm_bench.py, profiles/r1_decode_gemm.md)
     DECODE_FUSED_MAX_T = 16
@@ -323,7 +324,10 @@ class LlamaModel:
     def cache_bytes_per_block(self, block_size: int) -> int:
         return KVCache.bytes_per_block(self.cfg.num_layers, self.kv_local, block_size)
 
-    def make_cache(self, num_blocks: int, block_size: int) -> KVCache:
+    def state_bytes_per_slot(self) -> int:
+        return 0  # no recurrent layers
+
+    def make_cache(self, num_blocks: int, block_size: int, slots: int = 0) -> KVCache:
         return KVCache(self.cfg.num_layers, num_blocks, self.kv_local, self.device, block_size=block_size)
 
     def attention_items(self) -> dict:

@@ -1,10 +1,10 @@
 """The model families the engine serves: configuration lookup and model construction.
 
-A model is named by a preset ("llama-3-8b", "bozupel-base", ...), by a folder with a config.json
+A model is named by a preset ("llama-3-8b", "mudepel-base", ...), by a folder with a config.json
 (its "architecture" entry selects the family; the folder's weights are loaded) or by a
 configuration object. A family is a configuration class with `from_dict`, its presets, and a model
-class with the interface LlamaModel and BozupelModel share: forward, make_cache,
-cache_bytes_per_block, attention_items, attention_workspace, health_words, weight_bytes.
+class with the interface the models share: forward, make_cache, cache_bytes_per_block,
+state_bytes_per_slot, attention_items, attention_workspace, health_words, weight_bytes.
 """
 from __future__ import annotations
 
@@ -12,11 +12,12 @@ import json
 import os
 from typing import Dict, Optional
 
-from pilottai_amd.models import bozupel, llama
+from pilottai_amd.models import bozupel, llama, mudepel
 
-CONFIG_CLASSES: Dict[str, type] = {"Bozupel": bozupel.BozupelConfig}
-MODEL_CLASSES: Dict[type, type] = {llama.LlamaConfig: llama.LlamaModel, bozupel.BozupelConfig: bozupel.BozupelModel}
-PRESETS = {**llama.PRESETS, **bozupel.PRESETS}
+CONFIG_CLASSES: Dict[str, type] = {"Bozupel": bozupel.BozupelConfig, "Mudepel": mudepel.MudepelConfig}
+MODEL_CLASSES: Dict[type, type] = {llama.LlamaConfig: llama.LlamaModel, bozupel.BozupelConfig: bozupel.BozupelModel,
+                                   mudepel.MudepelConfig: mudepel.MudepelModel}
+PRESETS = {**llama.PRESETS, **bozupel.PRESETS, **mudepel.PRESETS}
 
 
 def is_folder(name) -> bool:

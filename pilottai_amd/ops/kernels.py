@@ -47,24 +47,43 @@ def require_native():
     return mod
 
 
-_LATENT = None
+_FAMILY = {}
+
+
+def _require_family(name: str):
+    if name not in _FAMILY:
+        try:
+            _FAMILY[name] = importlib.import_module("pilottai_amd._" + name)
+        except ImportError as e:
+            raise RuntimeError(f"pilottai_amd {name} kernels (_{name}.so) are not available: {e!r}. Build them with "
+                               "`python -m pilottai_amd._build` (hipcc --offload-arch=gfx950).") from e
+    return _FAMILY[name]
 
 
 def require_latent():
     """The _latent module (latent attention, expert tables, fp32 residual; csrc/ops/bindings_latent.cpp)."""
-    global _LATENT
-    if _LATENT is None:
-        try:
-            _LATENT = importlib.import_module("pilottai_amd._latent")
-        except ImportError as e:
-            raise RuntimeError(f"pilottai_amd latent kernels (_latent.so) are not available: {e!r}. Build them with "
-                               "`python -m pilottai_amd._build` (hipcc --offload-arch=gfx950).") from e
-    return _LATENT
+    return _require_family("latent")
+
+
+def require_hybrid():
+    """The _hybrid module (windowed pooled attention, state-space layers, score-routed experts;
+    csrc/ops/bindings_hybrid.cpp)."""
+    return _require_family("hybrid")
+
+
+def require_grouped():
+    """A module with the grouped projections: the one that is loaded, else the one that is built."""
+    for name in _FAMILY:
+        return _FAMILY[name]
+    try:
+        return require_latent()
+    except RuntimeError:
+        return require_hybrid()
 
 
 def _packed_module():
-    """The module with the packed-weight projections: _C, or _latent where only that one is built."""
-    return _load() or require_latent()
+    """The module with the packed-weight projections: _C, or a family's where only that one is built."""
+    return _load() or require_grouped()
 
 
 def native_module_path() -> Optional[str]:

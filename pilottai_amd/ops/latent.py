@@ -11,7 +11,7 @@ from typing import Optional
 import torch
 
 from . import reference as ref
-from .kernels import _on_gpu, require_latent
+from .kernels import _on_gpu, require_grouped, require_latent
 
 LATENT_TILES = (1, 2, 3, 4, 6, 8, 12, 16)  # latent widths (in 32s) with MFMA kernels (latent_attention.hip)
 ROT_TILES = (1, 2)
@@ -100,7 +100,7 @@ def head_gemm(x, x_step: int, w, out, out_step: int, rot: Optional[tuple] = None
     by the row's position and padded with zeros."""
     if _on_gpu(x):
         pos, cs, skip, r, rp = rot or (None, None, 0, 0, 0)
-        require_latent().head_gemm(x, int(x_step), w, out, int(out_step), pos, cs, int(skip), int(r), int(rp))
+        require_grouped().head_gemm(x, int(x_step), w, out, int(out_step), pos, cs, int(skip), int(r), int(rp))
     else:
         ref.head_gemm(x, x_step, unpack_groups(w), out, out_step, rot)
     return out
@@ -117,12 +117,13 @@ def table_route(tables, desc, desc_host, ids, slots, T: int, tm: int, order, til
 
 def expert_gemm(x, w, out, tiles, n_tiles, order, rows: int, *, x_div: int, out_order: bool, tm: int,
                 glu: Optional[tuple] = None):
-    """Rows sorted by expert: out row = x row @ w[expert].T; glu = (limit, alpha, bias): the clamped gated
-    pair of interleave_gate_up weights. x row = order[p] // x_div (0: p), out row = order[p] if out_order."""
-    lim, alpha, bias = glu or (0.0, 0.0, 0.0)
+    """Rows sorted by expert: out row = x row @ w[expert].T; glu = (limit, alpha, bias[, cubic]): the gated
+    pair of interleave_gate_up weights, min(g, limit) sigmoid(alpha (g + cubic g^3)) (clamp(u) + bias). x row =
+    order[p] // x_div (0: p), out row = order[p] if out_order."""
+    lim, alpha, bias, cubic = (tuple(glu) + (0.0,))[:4] if glu else (0.0, 0.0, 0.0, 0.0)
     if _on_gpu(x):
-        require_latent().expert_gemm(x, w, out, tiles, n_tiles, order, int(rows), int(x_div), bool(out_order), int(tm),
-                                     glu is not None, float(lim), float(alpha), float(bias))
+        require_grouped().expert_gemm(x, w, out, tiles, n_tiles, order, int(rows), int(x_div), bool(out_order), int(tm),
+                                      glu is not None, float(lim), float(alpha), float(bias), float(cubic))
     else:
         ref.expert_gemm(x, unpack_groups(w), out, tiles, n_tiles, order, x_div, out_order, glu)
     return out

@@ -403,8 +403,180 @@ def expert_gemm(x, w, out, tiles, n_tiles, order, x_div, out_order, glu):
         xr = order[p].long() // x_div if x_div else p
         y = x[xr, :K].float() @ w[e].float().T
         if glu is not None:
-            lim, alpha, bias = glu
+            lim, alpha, bias, cubic = (tuple(glu) + (0.0,))[:4]
             y = y.view(n, -1, 2, 16)
             g, u = y[:, :, 0].reshape(n, -1).clamp(max=lim), y[:, :, 1].reshape(n, -1).clamp(-lim, lim)
-            y = g * torch.sigmoid(alpha * g) * (u + bias)
+            y = g * torch.sigmoid(alpha * (g + cubic * g ** 3)) * (u + bias)
         out[order[p].long() if out_order else p, :y.shape[1]] = y.to(out.dtype)
+
+
+# ---------------------------------------------------------------------------
+# residual of several streams, windowed pooled attention, state-space layers, score routing (ops/hybrid.py)
+# ---------------------------------------------------------------------------
+
+
+def yarn_frequencies(dims: int, base: float, factor: float, original: float, fast: float, slow: float):
+    """Angles per position of dims / 2 pairs: pairs that turn often within `original` positions keep theirs,
+    slow ones are divided by `factor`, a linear ramp lies between; and the factor of cos and sin."""
+    f = base ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims)
+    at = lambda turns: dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(base))  # noqa: E731
+    lo, hi = max(math.floor(at(fast)), 0), min(math.ceil(at(slow)), dims - 1)
+    ramp = ((torch.arange(dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+    return f * (1 - ramp) + f / factor * ramp, 0.1 * math.log(factor) + 1
+
+
+def angle_table(max_pos: int, dims: int, base: float, yarn: Optional[dict] = None) -> torch.Tensor:
+    """fp32 [max_pos, dims]: cos | sin of the rotate-half pairs, YaRN-scaled if `yarn` (factor, original,
+    fast, slow) is given."""
+    f, m = yarn_frequencies(dims, base, **yarn) if yarn else \
+        (base ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims), 1.0)
+    a = torch.arange(max_pos, dtype=torch.float64)[:, None] * f[None, :]
+    return torch.cat([a.cos() * m, a.sin() * m], 1).float()
+
+
+def hyper_norm(x, eps, y, partials, y_weights, bias, mix, post, pre, emb, ids, w_next, out, rows):
+    T, S, D = x.shape
+    sel = torch.arange(T) if rows is None else rows.long()
+    r = x[sel]
+    if emb is not None:
+        r = emb[ids[:T].long()[sel].clamp(0, emb.shape[0] - 1)].float()[:, None].expand(-1, S, -1)
+    if y is not None:
+        v = y[:, :D].float().view(T, partials, D)[sel]
+        v = (v * y_weights.view(T, partials)[sel][:, :, None]).sum(1) if y_weights is not None else v.sum(1)
+        if bias is not None:
+            v = v + bias
+        r = torch.einsum("st,nsd->ntd", mix, r) + post[None, :, None] * v[:, None]
+    if rows is None:
+        x.copy_(r)
+    if out is not None:
+        u = (pre[None, :, None] * r).sum(1)
+        out[:len(sel), :D] = (_norm32(u, eps) * w_next).to(out.dtype)
+        out[:len(sel), D:] = 0
+    return out
+
+
+def _page_rows(pages, blocks, n):
+    """[n, G, D] fp32: a sequence's first n cached rows."""
+    NB, G, d8 = pages.shape[:3]
+    return pages[blocks.long()].permute(0, 3, 1, 2, 4).reshape(-1, G, d8 * 8)[:n].float()
+
+
+def paged_kv(x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_len, block_table, cos_sin, pool, num_seqs):
+    T, H, DK = q.shape
+    G, DV = kp.shape[1], vp.shape[2] * 8
+    r = x[:, :(H + G) * DK + G * DV].float()
+    if bias is not None:
+        r = r + bias
+    heads = _rotate_part(r[:, :(H + G) * DK].view(T, H + G, DK), positions[:T], cos_sin)
+    q.copy_(heads[:, :H].to(q.dtype))
+    k, v = heads[:, H:], r[:, (H + G) * DK:].view(T, G, DV)
+    for t in range(T):
+        s = int(slots[t])
+        if s >= 0:
+            kp[s // 16, :, :, s % 16] = k[t].view(G, -1, 8).to(kp.dtype)
+            vp[s // 16, :, :, s % 16] = v[t].view(G, -1, 8).to(vp.dtype)
+    if pool <= 0:
+        return
+    for s in range(num_seqs):
+        ctx, n = int(ctx_len[s]), int(q_len[s])
+        if n <= 0:
+            continue
+        blocks = block_table[s, :(ctx + 15) // 16]
+        kr, vr = _page_rows(kp, blocks, ctx), _page_rows(vp, blocks, ctx)
+        for b in range((ctx - n) // pool, ctx // pool):
+            page = (b * pool + pool - 1) // 16
+            sub = b - page * 16 // pool
+            pk[int(blocks[page]), sub] = kr[b * pool:(b + 1) * pool].mean(0).to(pk.dtype)
+            pv[int(blocks[page]), sub] = vr[b * pool:(b + 1) * pool].mean(0).to(pv.dtype)
+
+
+def window_attention(out, q, kp, vp, pk, pv, q_start, q_len, ctx_len, block_table, scale, window, pool, sink, num_seqs):
+    H, G = q.shape[1], kp.shape[1]
+    for s in range(num_seqs):
+        n, ctx, q0 = int(q_len[s]), int(ctx_len[s]), int(q_start[s])
+        if n <= 0:
+            continue
+        blocks = block_table[s, :(ctx + 15) // 16]
+        k, v = _page_rows(kp, blocks, ctx), _page_rows(vp, blocks, ctx)
+        pos = torch.arange(ctx - n, ctx)[:, None]
+        back = pos - torch.arange(ctx)[None, :]
+        seen = (back >= 0) & (back < window) if window > 0 else back >= 0
+        if pool > 0 and window > 0 and ctx // pool:
+            ends = torch.arange(ctx // pool) * pool + pool - 1
+            page = blocks[ends // 16].long()
+            sub = torch.arange(ctx // pool) - ends // 16 * 16 // pool
+            k, v = torch.cat([k, pk[page, sub].float()]), torch.cat([v, pv[page, sub].float()])
+            seen = torch.cat([seen, ends[None, :] <= pos - window], 1)
+        k, v = k.repeat_interleave(H // G, 1), v.repeat_interleave(H // G, 1)
+        sc = torch.einsum("thd,khd->htk", q[q0:q0 + n].float(), k) * scale
+        sc = sc.masked_fill(~seen, float("-inf"))
+        m = sc.amax(-1, keepdim=True)
+        if sink > 0:
+            m = m.clamp(min=0)
+        p = torch.exp(sc - m)
+        p = p / (p.sum(-1, keepdim=True) + (sink * torch.exp(-m) if sink > 0 else 0))
+        out[q0:q0 + n] = torch.einsum("htk,khd->thd", p, v).to(out.dtype)
+
+
+def state_scan(proj, y, state, ring, conv_w, conv_b, dt_bias, a, d, q_start, q_len, ctx_len, state_slot, groups, num_seqs):
+    H, V, N = state.shape[1:]
+    taps, C = conv_w.shape
+    R, inner = ring.shape[1], H * V
+    for s in range(num_seqs):
+        n, q0, slot = int(q_len[s]), int(q_start[s]), int(state_slot[s])
+        if n <= 0:
+            continue
+        p0 = int(ctx_len[s]) - n
+        rows = proj[q0:q0 + n]
+        xin = rows[:, inner:inner + C].float()
+        before = [ring[slot, p % R].float() if p >= 0 else torch.zeros(C) for p in range(p0 - taps + 1, p0)]
+        full = torch.cat([torch.stack(before), xin]) if before else xin
+        u = conv_b + sum(full[k:k + n] * conv_w[k] for k in range(taps))
+        u = (u * torch.sigmoid(u)).to(proj.dtype).float()
+        for p in range(max(p0, p0 + n - taps + 1), p0 + n):
+            ring[slot, p % R] = rows[p - p0, inner:inner + C]
+        x, B, Cm = u[:, :inner].view(n, H, V), u[:, inner:inner + groups * N], u[:, inner + groups * N:]
+        B = B.view(n, groups, N).repeat_interleave(H // groups, 1)
+        Cm = Cm.view(n, groups, N).repeat_interleave(H // groups, 1)
+        dt = rows[:, inner + C:inner + C + H].float() + dt_bias
+        dt = dt.clamp(min=0) + torch.log1p(torch.exp(-dt.abs()))
+        S = state[slot].clone() if p0 > 0 else torch.zeros(H, V, N)
+        for t in range(n):
+            S = S * torch.exp(-a * dt[t])[:, None, None] + (dt[t][:, None] * x[t])[:, :, None] * B[t][:, None, :]
+            o = (S * Cm[t][:, None, :]).sum(-1) + d[:, None] * x[t]
+            y[q0 + t, :inner] = o.reshape(-1).to(y.dtype)
+        state[slot] = S
+
+
+def gated_norm(y, z, w, heads, vdim, vpad, parts, eps):
+    T = y.shape[0]
+    g, zf = (t[:, :heads * vpad].float().view(T, heads, vpad)[:, :, :vdim].reshape(T, -1) for t in (y, z))
+    g = (g * (zf * torch.sigmoid(zf))).view(T, parts, -1)
+    g = (_norm32(g, eps).view(T, -1) * w).view(T, heads, vdim)
+    y.zero_()
+    y[:, :heads * vpad].view(T, heads, vpad)[:, :, :vdim] = g.to(y.dtype)
+
+
+def score_route(h, w, slots, weights, choice, order, tiles, n_tiles, E, top, groups, keep, always, tm):
+    T = h.shape[0]
+    s = torch.sigmoid(h[:, :w.shape[1]].float() @ w[:E].float().T)
+    per = s.view(T, groups, E // groups)
+    best = per.topk(min(2, E // groups), -1).values.sum(-1).topk(keep, -1).indices
+    ok = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True).repeat_interleave(E // groups, 1)
+    val, idx = s.masked_fill(~ok, -1).topk(top, -1)
+    live = slots[:T] >= 0
+    weights[:, :top], weights[:, top:] = val, 1.0
+    weights[~live] = 0
+    e = torch.cat([idx, torch.arange(E, E + always).expand(T, -1)], 1)
+    choice.view(T, top + always).copy_(torch.where(live[:, None], e, -1))
+    p = torch.arange(T * (top + always))[live.repeat_interleave(top + always)]
+    ep = e.reshape(-1)[p]
+    p = p[torch.argsort(ep, stable=True)]
+    order[:len(p)] = p.to(torch.int32)
+    k, start = 0, 0
+    for x, c in enumerate(torch.bincount(ep, minlength=E + always).tolist()):
+        for i in range(0, c, tm):
+            tiles[k] = torch.tensor([x, start + i, min(tm, c - i), 0], dtype=torch.int32)
+            k += 1
+        start += c
+    n_tiles[0] = k

@@ -37,7 +37,9 @@ def main(argv=None) -> int:
 
     from pilottai_amd import _build
 
-    _build.ensure("latent", gpu=a.device != "cpu")
+    from pilottai_amd.models import registry
+
+    _build.ensure(registry.model_class(registry.get_config(a.model)).KERNELS, gpu=a.device != "cpu")
     import torch
 
     from pilottai_amd.engine.engine import EngineConfig, LLMEngine
