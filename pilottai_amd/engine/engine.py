@@ -268,11 +268,14 @@ class LLMEngine:
             self.model.PF_MIDRANGE = frozenset(cfg.pf_midrange)
         self.load_time = time.time() - t0
         # ---- KV cache sizing (288 GB HBM: the default leaves room for graphs/activations)
-        bpb = max(1, self.model.cache_bytes_per_block(cfg.block_size))
+        need_min = (self.max_model_len + cfg.block_size - 1) // cfg.block_size + 1
+        bpb = self.model.cache_bytes_per_block(cfg.block_size)
         state = cfg.max_num_seqs * self.model.state_bytes_per_slot()  # recurrent layers: one slot per sequence
         nb = cfg.num_kv_blocks
         if nb is None:
-            if cfg.kv_cache_gb is not None:
+            if not bpb:  # recurrent layers only: pages are counted, but hold nothing
+                nb = cfg.max_num_seqs * need_min
+            elif cfg.kv_cache_gb is not None:
                 nb = int(cfg.kv_cache_gb * (1 << 30)) // bpb
             elif self.on_gpu:
                 free = torch.cuda.mem_get_info(self.device)[0] - state
@@ -281,7 +284,6 @@ class LLMEngine:
                 nb = int(max(0.0, min(free * cfg.kv_cache_fraction, free - cfg.kv_reserve_gb * (1 << 30)))) // bpb
             else:
                 nb = 2048
-        need_min = (self.max_model_len + cfg.block_size - 1) // cfg.block_size + 1
         if not cfg.exact_kv_blocks:
             nb = max(nb, need_min)
         if self.tp.size > 1:  # block ids travel in the metadata: every rank needs the same pool
