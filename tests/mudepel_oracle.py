@@ -52,9 +52,9 @@ def rotate(x, rot):
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half:]], -1)
 
 
-def pooled_attention(q, k, v, scale, window, pool):
+def pooled_attention(q, k, v, scale, window, pool, sink=1.0):
     """One head. q [T, n], k [T, n], v [T, m]: query i sees keys j with 0 <= i - j < window and the mean of
-    every whole block of `pool` keys that ends at or before i - window; exp(s) / (1 + sum exp(s))."""
+    every whole block of `pool` keys that ends at or before i - window; exp(s) / (sink + sum exp(s))."""
     T = q.shape[0]
     back = torch.arange(T)[:, None] - torch.arange(T)[None, :]
     seen = (back >= 0) & (back < window) if window else back >= 0
@@ -66,9 +66,11 @@ def pooled_attention(q, k, v, scale, window, pool):
         last = torch.arange(n) * pool + pool - 1
         seen = torch.cat([seen, last[None, :] <= torch.arange(T)[:, None] - window], 1)
     s = (q @ keys.T * scale).masked_fill(~seen, -math.inf)
-    top = s.max(1, keepdim=True).values.clamp(min=0)
+    top = s.max(1, keepdim=True).values
+    if sink:
+        top = top.clamp(min=0)
     e = torch.exp(s - top)
-    return e / (torch.exp(-top) + e.sum(1, keepdim=True)) @ vals
+    return e / ((sink * torch.exp(-top) if sink else 0) + e.sum(1, keepdim=True)) @ vals
 
 
 def attention(h, m, w):
