@@ -1,6 +1,6 @@
 """Step throughput of a served model design beside Llama layers of equal size (random weights).
 
-    python bench.py --design bozupel [--steps K --warmup W]
+    python bench.py --design bozupel|mudepel [--steps K --warmup W]
 
 For each size the two engines hold the same width, layer count, heads and active feed-forward width.
 A case is one scheduler-built step (prompt portions or decode rows at a context), captured as the
@@ -26,21 +26,29 @@ CASES: List[Tuple[str, List[Tuple[int, int]]]] = [
     ("decode 256 at 1024", [(1024, 1)] * 256),
 ]
 
+DESIGNS = ("bozupel", "mudepel")
+
 
 def pair(design: str):
     """[(size, design config, equal-size Llama config)]"""
-    from pilottai_amd.models import bozupel
+    from pilottai_amd.models import bozupel, mudepel
     from pilottai_amd.models.llama import LlamaConfig
 
-    if design != "bozupel":
-        raise ValueError(f"unknown design {design!r}")
+    if design not in DESIGNS:
+        raise ValueError(f"unknown design {design!r}; known: {DESIGNS}")
     out = []
     for size in ("base", "wide"):
-        c = bozupel.PRESETS[f"bozupel-{size}"]
-        m, p = c.layers[0].mixer, c.layers[0].mlp
+        if design == "bozupel":
+            c = bozupel.PRESETS[f"bozupel-{size}"]
+            m, p = c.layers[0].mixer, c.layers[0].mlp
+            heads, kv, ff = m.heads, m.heads // 4, p.top * p.ff
+        else:  # dense and expert layers in turn: the mean of their active widths
+            c = mudepel.PRESETS[f"mudepel-{size}"]
+            m, p = c.layers[0].mixer, c.layers[1].mlp
+            heads, kv, ff = m.heads, m.kv_heads, (c.layers[0].mlp.ff + p.top * p.ff + p.shared_ff) // 2 // 256 * 256
         out.append((size, c, LlamaConfig(name=f"llama-{size}", vocab_size=c.vocab_size, hidden_size=c.hidden_size,
-                                         intermediate_size=p.top * p.ff, num_layers=len(c.runs()), num_heads=m.heads,
-                                         num_kv_heads=m.heads // 4, head_dim=128)))
+                                         intermediate_size=ff, num_layers=len(c.runs()), num_heads=heads,
+                                         num_kv_heads=kv, head_dim=128)))
     return out
 
 
