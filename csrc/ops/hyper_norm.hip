@@ -118,10 +118,17 @@ __global__ __launch_bounds__(256) void hyper_norm_kernel(const Args A) {
   for (int i = D + threadIdx.x; i < A.ldo; i += 256) o[i] = (T)0.f;
 }
 
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void softcap_kernel(T* __restrict__ x, int ld, int cols, float cap) {
   T* r = x + (size_t)blockIdx.y * ld;
-  for (int i = blockIdx.x * 256 + threadIdx.x; i < cols; i += gridDim.x * 256) r[i] = (T)(cap * tanhf((float)r[i] / cap));
+  for (int i = (blockIdx.x * 256 + threadIdx.x) * VEC; i < cols; i += gridDim.x * 256 * VEC) {
+    T a[VEC];  // (columns behind cols, up to a whole vector of the row, are padding)
+    __builtin_memcpy(a, __builtin_assume_aligned(r + i, sizeof(T) * VEC), sizeof(T) * VEC);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j)
+      if (VEC == 1 || i + j < cols) a[j] = (T)(cap * tanhf((float)a[j] / cap));
+    __builtin_memcpy(__builtin_assume_aligned(r + i, sizeof(T) * VEC), a, sizeof(T) * VEC);
+  }
 }
 
 }  // namespace hn
@@ -161,8 +168,14 @@ extern "C" int pa_hyper_norm(int fp32, float* x, int S, const void* y, int K, in
 
 extern "C" int pa_softcap(int fp32, void* x, int ld, int rows, int cols, float cap, hipStream_t st) {
   if (rows <= 0 || cols <= 0) return 0;
-  const dim3 grid((cols + 1023) / 1024, rows);
-  if (fp32) hipLaunchKernelGGL(pa::hn::softcap_kernel<float>, grid, dim3(256), 0, st, (float*)x, ld, cols, cap);
-  else hipLaunchKernelGGL(pa::hn::softcap_kernel<pa::bf16>, grid, dim3(256), 0, st, (pa::bf16*)x, ld, cols, cap);
+  const bool vec = ld % 8 == 0;  // (a whole vector then never leaves the row)
+  const dim3 grid((cols + 2047) / 2048, rows);
+  if (fp32) {
+    if (vec) hipLaunchKernelGGL((pa::hn::softcap_kernel<float, 8>), grid, dim3(256), 0, st, (float*)x, ld, cols, cap);
+    else hipLaunchKernelGGL((pa::hn::softcap_kernel<float, 1>), grid, dim3(256), 0, st, (float*)x, ld, cols, cap);
+  } else {
+    if (vec) hipLaunchKernelGGL((pa::hn::softcap_kernel<pa::bf16, 8>), grid, dim3(256), 0, st, (pa::bf16*)x, ld, cols, cap);
+    else hipLaunchKernelGGL((pa::hn::softcap_kernel<pa::bf16, 1>), grid, dim3(256), 0, st, (pa::bf16*)x, ld, cols, cap);
+  }
   return (int)hipGetLastError();
 }

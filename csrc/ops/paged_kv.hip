@@ -7,9 +7,11 @@
 //   pages         [pages, G, D/8, 16, 8]; pooled rows [pages, npb, G, D] with the page of the block's
 //                 last token, blocks that end in one page in order
 //
-// A block's mean is taken over its rows as the cache holds them (rotated, in T): rows of earlier steps
-// are read from their pages, rows of this step are computed again from the projection, so nothing
-// waits for another workgroup. Arithmetic is fp32.
+// A block's mean is taken over its rows as the cache holds them (rotated, in T). Small steps do it in the
+// same launch: rows of earlier steps are read from their pages, rows of this step are computed again from
+// the projection, so nothing waits for another workgroup. Larger steps have a second launch that reads
+// all of them from their pages. Workgroups are dealt so that neighbouring tokens, which share the cache lines
+// of a page, run on one XCD. Arithmetic is fp32.
 #include "common.h"
 
 namespace pa {
@@ -21,8 +23,29 @@ struct Args {
   void *q, *kp, *vp, *pk, *pv;
   const int *positions, *slots, *q_start, *q_len, *ctx_len, *block_table;
   const float* cos_sin;  // [max_pos, rd]: cos | sin
-  int ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs;
+  int ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs, T;
 };
+
+__device__ __forceinline__ void load8(const float* p, float (&v)[8]) {
+  __builtin_memcpy(v, __builtin_assume_aligned(p, 16), 32);
+}
+
+// token of a workgroup: each of the 8 XCDs (workgroups go round) gets a contiguous eighth; -1: none
+__device__ __forceinline__ int token_of(int b, int T) {
+  const int per = (T + 7) >> 3, t = (b & 7) * per + (b >> 3);
+  return (b >> 3) < per && t < T ? t : -1;
+}
+
+// the step's sequence that token t belongs to
+__device__ __forceinline__ int seq_of(const Args& A, int t) {
+  int lo = 0, hi = A.max_seqs - 1;
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (A.q_start[mid] <= t) lo = mid; else hi = mid - 1;
+  }
+  while (lo > 0 && A.q_len[lo] == 0) --lo;  // (rows of no sequence start where the last one ends)
+  return lo;
+}
 
 // 8 values of head part `off` (columns off .. off + D of a row) from dimension d, rotated by cs if `rot`
 template <typename T>
@@ -31,17 +54,30 @@ __device__ __forceinline__ void chunk(const Args& A, const T* row, int off, int 
   T a[8];
   __builtin_memcpy(a, __builtin_assume_aligned(row + off + d, sizeof(T) * 8), sizeof(T) * 8);
 #pragma unroll
-  for (int j = 0; j < 8; ++j) v[j] = (float)a[j] + (A.bias ? A.bias[off + d + j] : 0.f);
+  for (int j = 0; j < 8; ++j) v[j] = (float)a[j];
+  float b[8];
+  if (A.bias) {
+    load8(A.bias + off + d, b);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] += b[j];
+  }
   if (!rot || d >= A.rd) return;
   if (half % 8 == 0) {
     const int pd = d < half ? d + half : d - half, i = d < half ? d : d - half;
     __builtin_memcpy(a, __builtin_assume_aligned(row + off + pd, sizeof(T) * 8), sizeof(T) * 8);
+    float c[8], s[8], u[8];
+    load8(cs + i, c);
+    load8(cs + half + i, s);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const float u = (float)a[j] + (A.bias ? A.bias[off + pd + j] : 0.f);
-      const float c = cs[i + j], s = cs[half + i + j];
-      v[j] = d < half ? v[j] * c - u * s : v[j] * c + u * s;
+    for (int j = 0; j < 8; ++j) u[j] = (float)a[j];
+    if (A.bias) {
+      load8(A.bias + off + pd, b);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) u[j] += b[j];
     }
+    const float sign = d < half ? -1.f : 1.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = v[j] * c[j] + sign * u[j] * s[j];
     return;
   }
 #pragma unroll
@@ -62,9 +98,12 @@ __device__ __forceinline__ void put(T* dst, const float (&v)[8]) {
   __builtin_memcpy(__builtin_assume_aligned(dst, sizeof(T) * 8), a, sizeof(T) * 8);
 }
 
-template <typename T>
+// POOL: blocks that end here are pooled in this launch
+template <typename T, bool POOL>
 __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
-  const int t = blockIdx.x, slot = A.slots[t];
+  const int t = token_of(blockIdx.x, A.T);
+  if (t < 0) return;
+  const int slot = A.slots[t];
   if (slot < 0) return;
   const int pos = A.positions[t];
   const T* row = (const T*)A.x + (size_t)t * A.ldx;
@@ -84,15 +123,10 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
       put((T*)(key ? A.kp : A.vp) + (((size_t)(slot >> 4) * A.G + h) * per + o) * 128 + (slot & 15) * 8, v);
     }
   }
+  if constexpr (!POOL) return;
   const int P = A.pool;
-  if (P <= 0 || (pos + 1) % P) return;
-  // this token's sequence
-  int lo = 0, hi = A.max_seqs - 1;
-  while (lo < hi) {
-    const int mid = (lo + hi + 1) >> 1;
-    if (A.q_start[mid] <= t) lo = mid; else hi = mid - 1;
-  }
-  while (lo > 0 && A.q_len[lo] == 0) --lo;  // (rows of no sequence start where the last one ends)
+  if ((pos + 1) % P) return;
+  const int lo = seq_of(A, t);
   const int start = A.ctx_len[lo] - A.q_len[lo];  // the step's first position
   const int* bt = A.block_table + (size_t)lo * A.max_blocks;
   const int page = pos >> 4, sub = pos / P - (page << 4) / P;
@@ -123,6 +157,36 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
   }
 }
 
+// The blocks that end in this step, from their pages: a workgroup per token that ends one.
+template <typename T>
+__global__ __launch_bounds__(256) void pool_kernel(const Args A) {
+  const int t = token_of(blockIdx.x, A.T), P = A.pool;
+  if (t < 0) return;
+  const int slot = A.slots[t], pos = A.positions[t];
+  if (slot < 0 || (pos + 1) % P) return;
+  const int* bt = A.block_table + (size_t)seq_of(A, t) * A.max_blocks;
+  const int ck = A.DK >> 3, cv = A.DV >> 3, nk = A.G * ck, nv = A.G * cv;
+  const int page = pos >> 4, sub = pos / P - (page << 4) / P;
+  const float inv = 1.f / (float)P;
+  for (int u = threadIdx.x; u < nk + nv; u += 256) {
+    const bool key = u < nk;
+    const int w = key ? u : u - nk, per = key ? ck : cv, D = key ? A.DK : A.DV;
+    const int h = w / per, o = w - h * per;
+    float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+    for (int p = pos - P + 1; p <= pos; ++p) {
+      T a[8];
+      const T* src = (const T*)(key ? A.kp : A.vp) + (((size_t)bt[p >> 4] * A.G + h) * per + o) * 128 + (p & 15) * 8;
+      __builtin_memcpy(a, __builtin_assume_aligned(src, sizeof(T) * 8), sizeof(T) * 8);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) sum[j] += (float)a[j];
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) sum[j] *= inv;
+    put((T*)(key ? A.pk : A.pv) + (((size_t)(slot >> 4) * A.npb + sub) * A.G + h) * D + o * 8, sum);
+  }
+}
+
 }  // namespace kv
 }  // namespace pa
 
@@ -134,8 +198,16 @@ extern "C" int pa_paged_kv(int fp32, const void* x, const float* bias, void* q, 
   if (T <= 0) return 0;
   if (DK % 8 || DV % 8 || rd % 2 || rd > DK || ldx % 8) return -1;
   const pa::kv::Args A{x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_len, block_table, cos_sin,
-                       ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs};
-  if (fp32) hipLaunchKernelGGL((pa::kv::paged_kv_kernel<float>), dim3(T), dim3(256), 0, st, A);
-  else hipLaunchKernelGGL((pa::kv::paged_kv_kernel<pa::bf16>), dim3(T), dim3(256), 0, st, A);
+                       ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs, T};
+  const dim3 grid((T + 7) / 8 * 8);
+  const bool later = pool > 0 && T > 64, now = pool > 0 && !later;
+#define PA_KV(TYPE)                                                                                              \
+  do {                                                                                                           \
+    if (now) hipLaunchKernelGGL((pa::kv::paged_kv_kernel<TYPE, true>), grid, dim3(256), 0, st, A);               \
+    else hipLaunchKernelGGL((pa::kv::paged_kv_kernel<TYPE, false>), grid, dim3(256), 0, st, A);                  \
+    if (later) hipLaunchKernelGGL(pa::kv::pool_kernel<TYPE>, grid, dim3(256), 0, st, A);                         \
+  } while (0)
+  if (fp32) PA_KV(float); else PA_KV(pa::bf16);
+#undef PA_KV
   return (int)hipGetLastError();
 }

@@ -13,6 +13,7 @@
 #include "common.h"
 
 #include <algorithm>
+#include <climits>
 
 namespace pa {
 namespace sr {
@@ -69,16 +70,6 @@ __device__ __forceinline__ void write_tiles(const Args& A, const int* cnt, const
   if (threadIdx.x == 0) A.n_tiles[0] = min(n, A.max_tiles);
 }
 
-// best (value, lowest index) over the 32 lanes of a token
-__device__ __forceinline__ void best32(float& v, int& i) {
-#pragma unroll
-  for (int o = 16; o > 0; o >>= 1) {
-    const float w = __shfl_xor(v, o, 32);
-    const int k = __shfl_xor(i, o, 32);
-    if (w > v || (w == v && k < i)) { v = w; i = k; }
-  }
-}
-
 template <typename T>
 __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
@@ -133,53 +124,53 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
     }
   }
   __syncthreads();
-  // 32 lanes per token
+  // 32 lanes per token. Nothing is chosen one after the other: a group, or an expert, is in when fewer than
+  // `keep`, or `top`, others come before it (larger, or equal and lower), and that number is its place.
+  // The scores are compared as integers: non-negative floats in the same order, and no two alike in rank
+  // whatever the bits are.
   const int tk = threadIdx.x >> 5, l = threadIdx.x & 31, t = t0 + tk, KA = A.top + A.always;
   const bool live = t < A.T && A.slots[min(t, A.T - 1)] >= 0;
   float *s = sc + tk * Ep, *gr = gs + tk * A.groups;
-  const int per = A.E / A.groups;
+  int *si = (int*)s, *gi = (int*)gr;
+  constexpr int OUT = -1, PAD = INT_MIN;
   if (A.keep < A.groups) {
+    const int per = A.E / A.groups;
     for (int i = l; i < A.groups; i += 32) {
       float a = -1.f, b = -1.f;
       for (int e = i * per; e < (i + 1) * per; ++e) {
         const float v = s[e];
-        if (v > a) { b = a; a = v; } else if (v > b) { b = v; }
+        b = fmaxf(b, fminf(a, v));
+        a = fmaxf(a, v);
       }
       gr[i] = a + (per > 1 ? b : 0.f);
     }
     __syncthreads();
-    for (int k = 0; k < A.keep; ++k) {  // (a kept group's score becomes -2)
-      float v = -1.f;
-      int at = A.groups;
-      for (int i = l; i < A.groups; i += 32)
-        if (gr[i] > v) { v = gr[i]; at = i; }
-      best32(v, at);
-      __syncthreads();
-      if (l == 0 && at < A.groups) gr[at] = -2.f;
-      __syncthreads();
+    for (int i = l; i < A.groups; i += 32) {
+      int before = 0;
+      const int v = gi[i];
+      for (int k = 0; k < A.groups; ++k) before += gi[k] > v || (gi[k] == v && k < i);
+      if (before >= A.keep)
+        for (int e = i * per; e < (i + 1) * per; ++e) si[e] = OUT;
     }
-    for (int e = l; e < A.E; e += 32)
-      if (gr[e / per] > -2.f) s[e] = -1.f;
     __syncthreads();
   }
-  for (int k = 0; k < A.top; ++k) {
-    float v = -2.f;
-    int at = A.E;
-    for (int e = l; e < A.E; e += 32)
-      if (s[e] > v) { v = s[e]; at = e; }
-    best32(v, at);
-    at = min(at, A.E - 1);
-    __syncthreads();
-    if (l == 0) {
-      s[at] = -2.f;
-      if (t < A.T) {
-        const size_t p = (size_t)t * KA + k;
-        A.choice[p] = live ? at : -1;
-        A.weights[p] = live ? v : 0.f;
-        if (live) A.rank[p] = atomicAdd(&cnt[at], 1);
-      }
+  for (int e = A.E + l; e < Ep; e += 32) si[e] = PAD;
+  __syncthreads();
+  for (int e = l; e < A.E; e += 32) {
+    int before = 0;
+    const int v = si[e];
+    for (int k = 0; k < Ep; k += 4) {
+      const int4 q = *reinterpret_cast<const int4*>(si + k);
+      const int w[4] = {q.x, q.y, q.z, q.w};
+#pragma unroll
+      for (int j = 0; j < 4; ++j) before += w[j] > v || (w[j] == v && k + j < e);
     }
-    __syncthreads();
+    if (before < A.top && t < A.T) {
+      const size_t p = (size_t)t * KA + before;
+      A.choice[p] = live ? e : -1;
+      A.weights[p] = live ? s[e] : 0.f;
+      if (live) A.rank[p] = atomicAdd(&cnt[e], 1);
+    }
   }
   if (l < A.always && t < A.T) {
     const size_t p = (size_t)t * KA + A.top + l;

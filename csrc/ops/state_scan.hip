@@ -131,26 +131,40 @@ __device__ __forceinline__ void store_ring(const Args& A, int s, int c0, int c1)
 }
 
 // ---- token by token: a workgroup per (sequence, head, part of V) -------------------------------------
-template <typename T>
-__global__ __launch_bounds__(256) void step_kernel(const Args A) {
+constexpr int REGS = 8;  // state vectors of a thread that stay in registers over the portion
+
+// TN: N / 4 as a constant (8 .. 64) where the state fits the registers of the workgroup; 0: any sizes.
+template <typename T, int TAPS, int TN>
+__global__ __launch_bounds__(256, 4) void step_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const int h = blockIdx.x / A.vsplit, vpart = blockIdx.x % A.vsplit, s = blockIdx.y;
   const int n = A.q_len[s];
   if (n <= 0 || A.state_slot[s] < 0) return;
   const bool conv = n <= A.scan_min;  // short: the convolution is done here
   if (!conv && !A.long_too) return;
-  const int V = A.V, N = A.N, g = h / (A.H / A.G), inner = A.H * V;
+  const int V = A.V, N = TN ? 4 * TN : A.N, g = h / (A.H / A.G), inner = A.H * V;
   float *sB = sm, *sC = sm + N, *sx = sm + 2 * N, *sdt = sm + 2 * N + V;  // one token
   const int q0 = A.q_start[s], p0 = A.ctx_len[s] - n;
   float* S = A.state + ((size_t)A.state_slot[s] * A.H + h) * V * N;
   T* ring = (T*)A.ring + (size_t)A.state_slot[s] * A.RING * A.Cc;
   const float* W = (const float*)A.conv_w;
   // lanes along N, 4 values each (a power of two of them, whole groups inside a wave), the rest along V
-  int tn = 1;
-  while (tn < 64 && (N >> 2) % (2 * tn) == 0) tn *= 2;
+  int tn = TN ? TN : 1;
+  if constexpr (TN == 0)
+    while (tn < 64 && (N >> 2) % (2 * tn) == 0) tn *= 2;
   const int ln = threadIdx.x % tn, lv = threadIdx.x / tn, nv = 256 / tn;
   const int v0 = vpart * (V / A.vsplit), v1 = v0 + V / A.vsplit;
   const float a = A.a[h], dd = A.d[h], bias = A.dt_bias[h];
+  // the state in registers over the portion: a lane's vectors are of rows v0 + lv + k nv
+  f32x4 st[TN ? REGS : 1];
+  float* mine = S + (size_t)(v0 + lv) * N + 4 * ln;
+  if constexpr (TN > 0) {
+#pragma unroll
+    for (int k = 0; k < REGS; ++k) {
+      st[k] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (p0 > 0 && v0 + lv + k * nv < v1) st[k] = *reinterpret_cast<const f32x4*>(mine + (size_t)k * nv * N);
+    }
+  }
   for (int t = 0; t < n; ++t) {
     const T* row = (const T*)A.proj + (size_t)(q0 + t) * A.ldp;
     __syncthreads();
@@ -159,13 +173,16 @@ __global__ __launch_bounds__(256) void step_kernel(const Args A) {
       float v;
       if (conv) {
         v = A.conv_b[c];
-        for (int k = 0; k < A.taps; ++k) {
-          const int i = t - (A.taps - 1) + k;
-          float x = 0.f;
-          if (i >= 0) x = (float)((const T*)A.proj)[(size_t)(q0 + i) * A.ldp + inner + c];
-          else if (p0 + i >= 0) x = (float)ring[(size_t)((p0 + i) % A.RING) * A.Cc + c];
-          v = fmaf(W[(size_t)k * A.Cc + c], x, v);
+        float x[TAPS];
+#pragma unroll
+        for (int k = 0; k < TAPS; ++k) {
+          const int i = t - (TAPS - 1) + k;
+          x[k] = 0.f;
+          if (i >= 0) x[k] = (float)((const T*)A.proj)[(size_t)(q0 + i) * A.ldp + inner + c];
+          else if (p0 + i >= 0) x[k] = (float)ring[(size_t)((p0 + i) % A.RING) * A.Cc + c];
         }
+#pragma unroll
+        for (int k = 0; k < TAPS; ++k) v = fmaf(W[(size_t)k * A.Cc + c], x[k], v);
         v = (float)(T)silu(v);
         // the owner of a channel keeps its input (rows that no token of this portion reads)
         if (e >= 2 * N || (h % (A.H / A.G) == 0 && vpart == 0)) ring[(size_t)((p0 + t) % A.RING) * A.Cc + c] = row[inner + c];
@@ -175,32 +192,58 @@ __global__ __launch_bounds__(256) void step_kernel(const Args A) {
       if (e < 2 * N) sm[e] = v;
       else sx[v0 + e - 2 * N] = v;
     }
-    if (threadIdx.x == 0) {
+    if (threadIdx.x == 255) {  // (a thread of the last wave, which has the fewest channels)
       const float dt = softplus((float)row[inner + A.Cc + h] + bias);
       sdt[0] = dt;
       sdt[1] = expf(-a * dt);
     }
     __syncthreads();
     const float dt = sdt[0], decay = sdt[1];
-    const bool fresh = p0 + t == 0;
-#pragma unroll 4
-    for (int v = v0 + lv; v < v1; v += nv) {
-      const float x = sx[v], w = dt * x;
+    // one vector's step; returns its part of S^T C
+    auto step = [&](f32x4& w, int i, float u) {
+      const f32x4 b = *reinterpret_cast<const f32x4*>(sB + i), c = *reinterpret_cast<const f32x4*>(sC + i);
       float acc = 0.f;
-      for (int i = ln * 4; i < N; i += tn * 4) {
-        f32x4* p = reinterpret_cast<f32x4*>(S + (size_t)v * N + i);
-        f32x4 st = fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *p;
-        const f32x4 b = *reinterpret_cast<const f32x4*>(sB + i), c = *reinterpret_cast<const f32x4*>(sC + i);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          st[j] = st[j] * decay + w * b[j];
-          acc = fmaf(st[j], c[j], acc);
-        }
-        *p = st;
+      for (int j = 0; j < 4; ++j) {
+        w[j] = w[j] * decay + u * b[j];
+        acc = fmaf(w[j], c[j], acc);
       }
-      for (int o = tn >> 1; o > 0; o >>= 1) acc += __shfl_xor(acc, o, 64);
+      return acc;
+    };
+    auto finish = [&](float acc, int v, float x) {
+#pragma unroll
+      for (int o = 32; o > 0; o >>= 1)
+        if (tn > o) acc += __shfl_xor(acc, o, 64);
       if (ln == 0) ((T*)A.y)[(size_t)(q0 + t) * A.ldy + h * V + v] = (T)(acc + dd * x);
+    };
+    if constexpr (TN > 0) {
+#pragma unroll
+      for (int k = 0; k < REGS; ++k) {
+        const int v = v0 + lv + k * nv;
+        if (v < v1) {
+          const float x = sx[v];
+          finish(step(st[k], 4 * ln, dt * x), v, x);
+        }
+      }
+    } else {
+      const bool fresh = p0 + t == 0;
+      for (int v = v0 + lv; v < v1; v += nv) {
+        const float x = sx[v];
+        float acc = 0.f;
+        for (int i = ln * 4; i < N; i += tn * 4) {
+          f32x4* p = reinterpret_cast<f32x4*>(S + (size_t)v * N + i);
+          f32x4 w = fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *p;
+          acc += step(w, i, dt * x);
+          *p = w;
+        }
+        finish(acc, v, x);
+      }
     }
+  }
+  if constexpr (TN > 0) {
+#pragma unroll
+    for (int k = 0; k < REGS; ++k)
+      if (v0 + lv + k * nv < v1) *reinterpret_cast<f32x4*>(mine + (size_t)k * nv * N) = st[k];
   }
   if (!conv && vpart == 0) {
     const int per = (A.Cc + A.H - 1) / A.H;
@@ -289,45 +332,58 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const Args A) {
   }
 }
 
+// 4 state values a thread, chunk after chunk; the next 8 chunks are on their way while 8 are written
 __global__ __launch_bounds__(256) void state_pass_kernel(const Args A) {
-  const int s = blockIdx.y, h = blockIdx.z, first = A.scan_first[s], VN = A.V * A.N;
-  const int n = A.q_len[s];
-  if (first < 0 || n <= 0 || A.state_slot[s] < 0) return;
-  const int e = (blockIdx.x * 256 + threadIdx.x) * 4, chunks = (n + LC - 1) / LC;
+  const int h = blockIdx.z, VN = A.V * A.N, e = (blockIdx.x * 256 + threadIdx.x) * 4, n_items = A.n_items[0];
   if (e >= VN) return;
-  float* S = A.state + ((size_t)A.state_slot[s] * A.H + h) * VN + e;
-  f32x4 st = {0.f, 0.f, 0.f, 0.f};
-  if (A.ctx_len[s] > n) st = *reinterpret_cast<const f32x4*>(S);
-  float* w = A.work + ((size_t)first * A.H + h) * VN + e;
-  const float* tot = A.total + (size_t)first * A.H + h;
   const size_t step = (size_t)A.H * VN;
-  for (int c0 = 0; c0 < chunks; c0 += 8) {
-    f32x4 u[8];
-    float d[8];
+  for (int item = blockIdx.y; item < n_items; item += gridDim.y) {
+    const int4 it = A.items[item];
+    if (it.y != 0) continue;  // a portion's first item takes all of them
+    const int s = it.x, n = A.q_len[s], chunks = (n + LC - 1) / LC;
+    float* S = A.state + ((size_t)A.state_slot[s] * A.H + h) * VN + e;
+    f32x4 st = {0.f, 0.f, 0.f, 0.f};
+    if (A.ctx_len[s] > n) st = *reinterpret_cast<const f32x4*>(S);
+    float* w = A.work + ((size_t)item * A.H + h) * VN + e;
+    const float* tot = A.total + (size_t)item * A.H + h;
+    f32x4 u[8], un[8];
+    float d[8], dn[8];
+    auto load = [&](int c0, f32x4 (&uu)[8], float (&ddd)[8]) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const int k = min(c0 + i, chunks - 1);
-      u[i] = *reinterpret_cast<const f32x4*>(w + k * step);
-      d[i] = tot[(size_t)k * A.H];
-    }
-#pragma unroll
-    for (int i = 0; i < 8; ++i)
-      if (c0 + i < chunks) {
-        *reinterpret_cast<f32x4*>(w + (c0 + i) * step) = st;
-        const float f = expf(d[i]);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) st[j] = st[j] * f + u[i][j];
+      for (int i = 0; i < 8; ++i) {
+        const int k = min(c0 + i, chunks - 1);
+        uu[i] = *reinterpret_cast<const f32x4*>(w + k * step);
+        ddd[i] = tot[(size_t)k * A.H];
       }
+    };
+    load(0, u, d);
+    for (int c0 = 0; c0 < chunks; c0 += 8) {
+      if (c0 + 8 < chunks) load(c0 + 8, un, dn);
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+        if (c0 + i < chunks) {
+          *reinterpret_cast<f32x4*>(w + (c0 + i) * step) = st;
+          const float f = expf(d[i]);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) st[j] = st[j] * f + u[i][j];
+        }
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        u[i] = un[i];
+        d[i] = dn[i];
+      }
+    }
+    *reinterpret_cast<f32x4*>(S) = st;
   }
-  *reinterpret_cast<f32x4*>(S) = st;
 }
 
-// STAGED: the incoming state is split into LDS once; otherwise every wave reads it from memory
-template <bool STAGED>
+// STAGED: the incoming state is split into LDS once; otherwise every wave reads it from memory.
+// NK: N / 32 as a constant, for which C stays in registers and B's loads go out together; 0: any N.
+template <bool STAGED, int NK>
 __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int h = blockIdx.x, n_items = A.n_items[0];
-  const int V = A.V, N = A.N, g = h / (A.H / A.G), inner = A.H * V, NL = N + 8;
+  const int V = A.V, N = NK ? 32 * NK : A.N, g = h / (A.H / A.G), inner = A.H * V, NL = N + 8;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, lg = lane >> 4, c = lane & 15;
   float *dt = (float*)smem, *l = dt + LC;
   bf16 *mh = (bf16*)(smem + 2 * LC * 4), *ml = mh + LC * LD;  // [i][LD], value and remainder
@@ -338,6 +394,27 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
     const int n = it.z, row0 = A.q_start[it.x] + it.y;
     const bf16* u = (const bf16*)A.u + (size_t)row0 * A.Cc;
     const float* S = A.work + ((size_t)item * A.H + h) * V * N;
+    // (rows past the end repeat the last one; their results are dropped)
+    const int i = 16 * wid + c, ri = min(i, n - 1);
+    const bf16* cr = u + (size_t)ri * A.Cc + inner + A.G * N + g * N + 8 * lg;
+    bf16x8 cf[NK ? NK : 1];
+    f32x4 cb[4];  // C_i . B_j
+    if constexpr (NK > 0) {
+#pragma unroll
+      for (int k = 0; k < NK; ++k) cf[k] = *reinterpret_cast<const bf16x8*>(cr + 32 * k);
+#pragma unroll
+      for (int jt = 0; jt < 4; ++jt) {
+        cb[jt] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (jt <= wid) {
+          const bf16* br = u + (size_t)min(16 * jt + c, n - 1) * A.Cc + inner + g * N + 8 * lg;
+          bf16x8 bf[NK ? NK : 1];
+#pragma unroll
+          for (int k = 0; k < NK; ++k) bf[k] = *reinterpret_cast<const bf16x8*>(br + 32 * k);
+#pragma unroll
+          for (int k = 0; k < NK; ++k) cb[jt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf[k], cf[k], cb[jt], 0, 0, 0);
+        }
+      }
+    }
     __syncthreads();
     chunk_steps(A, h, row0, n, dt, l);
     for (int e = threadIdx.x; e < (V >> 3) * LC; e += 256) {
@@ -366,20 +443,21 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
         *reinterpret_cast<bf16x4*>(sl + r * NL + k0) = lo;
       }
     __syncthreads();
-    // (rows past the end repeat the last one; their results are dropped)
-    const int i = 16 * wid + c, ri = min(i, n - 1);
-    const bf16* cr = u + (size_t)ri * A.Cc + inner + A.G * N + g * N + 8 * lg;
-    const float li = l[i];
     // M[i][j] = exp(l_i - l_j) dt_j (C_i . B_j), a lane's row i, its columns j = 16 jt + 4 lg ..
+    const float li = l[i];
 #pragma unroll
     for (int jt = 0; jt < 4; ++jt) {
       bf16x4 hi = {(bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f}, lo = hi;
       if (jt <= wid) {
-        const bf16* br = u + (size_t)min(16 * jt + c, n - 1) * A.Cc + inner + g * N + 8 * lg;
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-        for (int k = 0; k < N; k += 32)
-          acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(br + k),
-                                                        *reinterpret_cast<const bf16x8*>(cr + k), acc, 0, 0, 0);
+        if constexpr (NK > 0) {
+          acc = cb[jt];
+        } else {
+          const bf16* br = u + (size_t)min(16 * jt + c, n - 1) * A.Cc + inner + g * N + 8 * lg;
+          for (int k = 0; k < N; k += 32)
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(br + k),
+                                                          *reinterpret_cast<const bf16x8*>(cr + k), acc, 0, 0, 0);
+        }
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int j = 16 * jt + 4 * lg + r;
@@ -402,8 +480,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
     const float ei = expf(li), dd = A.d[h];
     for (int v0 = 0; v0 < V; v0 += 16) {
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-      for (int k = 0; k < N; k += 32) {
+      auto from_state = [&](int k) {
         bf16x8 s0, s1;
         if (STAGED) {
           s0 = *reinterpret_cast<const bf16x8*>(sh + (v0 + c) * NL + k + 8 * lg);
@@ -418,9 +495,15 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
             s1[q] = b;
           }
         }
-        const bf16x8 cf = *reinterpret_cast<const bf16x8*>(cr + k);
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(s0, cf, acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(s1, cf, acc, 0, 0, 0);
+        const bf16x8 cv = NK ? cf[NK ? k / 32 : 0] : *reinterpret_cast<const bf16x8*>(cr + k);
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(s0, cv, acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(s1, cv, acc, 0, 0, 0);
+      };
+      if constexpr (NK > 0) {
+#pragma unroll
+        for (int k = 0; k < NK; ++k) from_state(32 * k);
+      } else {
+        for (int k = 0; k < N; k += 32) from_state(k);
       }
       acc *= ei;
 #pragma unroll
@@ -516,7 +599,7 @@ extern "C" int pa_state_scan(int fp32, const void* proj, int ldp, void* u, void*
                              int scan_min, hipStream_t st) {
   using namespace pa::ss;
   if (seqs <= 0) return 0;
-  if (V % 16 || N % 32 || H % G || scan_min > MAX_SHORT || ring_rows < taps - 1 + scan_min || taps < 1 || taps > 8) return -1;
+  if (V % 16 || N % 32 || H % G || scan_min > MAX_SHORT || ring_rows < taps - 1 + scan_min || (taps != 4 && taps != 8)) return -1;  // (shorter ones are padded)
   Args A{proj, u, y, state, ring, work, total, conv_w, conv_b, dt_bias, a, d, q_start, q_len, ctx_len, state_slot,
          scan_first, (const int4*)items, n_items, ldp, ldy, H, G, V, N, H * V + 2 * G * N, taps, ring_rows, scan_min,
          seqs, fp32, 1};
@@ -528,7 +611,6 @@ extern "C" int pa_state_scan(int fp32, const void* proj, int ldp, void* u, void*
     if (taps == 4) hipLaunchKernelGGL((conv_kernel<T, 4>), grid, dim3(256), 0, st, A);                    \
     else hipLaunchKernelGGL((conv_kernel<T, 8>), grid, dim3(256), 0, st, A);                              \
   } while (0)
-    if (taps != 4 && taps != 8) return -1;  // (shorter ones are padded with zeros in front)
     if (fp32) PA_CONV(float); else PA_CONV(pa::bf16);
 #undef PA_CONV
   }
@@ -536,8 +618,24 @@ extern "C" int pa_state_scan(int fp32, const void* proj, int ldp, void* u, void*
   while (A.vsplit < 8 && H * seqs * A.vsplit < 512 && V % (A.vsplit * 2) == 0) A.vsplit *= 2;
   const int step_lds = (2 * N + V + 2) * 4;
   if (step_lds > 64 * 1024) return -2;
-  if (fp32) hipLaunchKernelGGL(step_kernel<float>, dim3(H * A.vsplit, seqs), dim3(256), step_lds, st, A);
-  else hipLaunchKernelGGL(step_kernel<pa::bf16>, dim3(H * A.vsplit, seqs), dim3(256), step_lds, st, A);
+  const dim3 sgrid(H * A.vsplit, seqs);
+  const int tn = V / A.vsplit <= REGS * 1024 / N ? N / 4 : 0;
+#define PA_STEP_N(T, K)                                                                                   \
+  do {                                                                                                    \
+    if (taps == 4) hipLaunchKernelGGL((step_kernel<T, 4, K>), sgrid, dim3(256), step_lds, st, A);         \
+    else hipLaunchKernelGGL((step_kernel<T, 8, K>), sgrid, dim3(256), step_lds, st, A);                   \
+  } while (0)
+#define PA_STEP(T)                                                                                        \
+  do {                                                                                                    \
+    if (tn == 8) PA_STEP_N(T, 8);                                                                         \
+    else if (tn == 16) PA_STEP_N(T, 16);                                                                  \
+    else if (tn == 32) PA_STEP_N(T, 32);                                                                  \
+    else if (tn == 64) PA_STEP_N(T, 64);                                                                  \
+    else PA_STEP_N(T, 0);                                                                                 \
+  } while (0)
+  if (fp32) PA_STEP(float); else PA_STEP(pa::bf16);
+#undef PA_STEP
+#undef PA_STEP_N
   if (fp32 || max_items <= 0) return (int)hipGetLastError();
   const int lds_s = 2 * LC * 4 + (N + 2 * V) * LD * 2;
   const int lds_o = 2 * LC * 4 + (2 * LC + V) * LD * 2, staged = lds_o + 2 * V * (N + 8) * 2;
@@ -546,15 +644,28 @@ extern "C" int pa_state_scan(int fp32, const void* proj, int ldp, void* u, void*
   static bool attr = false;
   if (!attr) {
     (void)hipFuncSetAttribute((const void*)chunk_state_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, MAX_LDS);
-    (void)hipFuncSetAttribute((const void*)chunk_out_kernel<true>, hipFuncAttributeMaxDynamicSharedMemorySize, MAX_LDS);
-    (void)hipFuncSetAttribute((const void*)chunk_out_kernel<false>, hipFuncAttributeMaxDynamicSharedMemorySize, MAX_LDS);
     attr = true;
   }
   const dim3 grid(H, std::min(max_items, 4096));
   hipLaunchKernelGGL(chunk_state_kernel, grid, dim3(256), lds_s, st, A);
-  hipLaunchKernelGGL(state_pass_kernel, dim3((V * N / 4 + 255) / 256, seqs, H), dim3(256), 0, st, A);
-  if (staged <= 80 * 1024) hipLaunchKernelGGL(chunk_out_kernel<true>, grid, dim3(256), staged, st, A);
-  else hipLaunchKernelGGL(chunk_out_kernel<false>, grid, dim3(256), lds_o, st, A);
+  hipLaunchKernelGGL(state_pass_kernel, dim3((V * N / 4 + 255) / 256, std::min(max_items, 16), H), dim3(256), 0, st, A);
+  const bool in_lds = staged <= 80 * 1024;
+  const int lds = in_lds ? staged : lds_o;
+#define PA_OUT(S, K)                                                                                                       \
+  do {                                                                                                                     \
+    static bool set = false;                                                                                               \
+    if (!set) {                                                                                                            \
+      (void)hipFuncSetAttribute((const void*)chunk_out_kernel<S, K>, hipFuncAttributeMaxDynamicSharedMemorySize, MAX_LDS); \
+      set = true;                                                                                                          \
+    }                                                                                                                      \
+    hipLaunchKernelGGL((chunk_out_kernel<S, K>), grid, dim3(256), lds, st, A);                                             \
+  } while (0)
+  if (!in_lds) PA_OUT(false, 0);
+  else if (N == 32) PA_OUT(true, 1);
+  else if (N == 64) PA_OUT(true, 2);
+  else if (N == 128) PA_OUT(true, 4);
+  else PA_OUT(true, 0);
+#undef PA_OUT
   return (int)hipGetLastError();
 }
 

@@ -572,7 +572,7 @@ extern "C" int pa_window_attention(int fp32, void* out, float* part_o, float* pa
       attr = true;                                                                                            \
     }                                                                                                         \
     hipLaunchKernelGGL((pa::wa::mfma_kernel<K, V>), dim3(gx, gy, G), dim3(64 * pa::wa::NW), lds, st, A);      \
-    hipLaunchKernelGGL((pa::wa::merge_kernel<V>), dim3(4, std::min(gy, 256), G), dim3(256), 0, st, A);        \
+    hipLaunchKernelGGL((pa::wa::merge_kernel<V>), dim3(8, std::min(gy, 256), G), dim3(256), 0, st, A);        \
     return (int)hipGetLastError();                                                                            \
   }
     PA_WA_DIMS(PA_X)

@@ -289,7 +289,7 @@ class MudepelModel:
         windows = [m.window for m in att]
         pools = [m.pool for m in att if m.pool]
         out = {"gqa_group": self._group, "kv_heads": self._kv_heads, "att_qcols": 128, "att_narrow_qcols": 128,
-               "prefill_split_keys": 0, "decode_part_target": 256, "att_min_part": 256, "att_tile_target": 256,
+               "prefill_split_keys": 0, "decode_part_target": 256, "att_min_part": 256, "att_tile_target": max(16, 256 // self._kv_heads),
                "att_max_keys": max(windows) if windows and all(windows) else 0, "att_pool": min(pools, default=0)}
         if self.recurrent:  # a page's worth of state is not kept, so a prefix cannot be taken from the cache
             out.update(scan_chunk=ops.SCAN_CHUNK, scan_min=ops.SCAN_MIN, prefix_caching=False)
