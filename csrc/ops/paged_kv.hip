@@ -24,7 +24,11 @@ struct Args {
   const int *positions, *slots, *q_start, *q_len, *ctx_len, *block_table;
   const float* cos_sin;  // [max_pos, rd]: cos | sin
   int ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs, T;
+  float ick, icv;  // 8 / DK, 8 / DV
 };
+
+// u / n for the small numbers of here, with inv = 1 / n
+__device__ __forceinline__ int quot(int u, float inv) { return (int)(((float)u + 0.5f) * inv); }
 
 __device__ __forceinline__ void load8(const float* p, float (&v)[8]) {
   __builtin_memcpy(v, __builtin_assume_aligned(p, 16), 32);
@@ -36,15 +40,14 @@ __device__ __forceinline__ int token_of(int b, int T) {
   return (b >> 3) < per && t < T ? t : -1;
 }
 
-// the step's sequence that token t belongs to
-__device__ __forceinline__ int seq_of(const Args& A, int t) {
-  int lo = 0, hi = A.max_seqs - 1;
-  while (lo < hi) {
-    const int mid = (lo + hi + 1) >> 1;
-    if (A.q_start[mid] <= t) lo = mid; else hi = mid - 1;
+// the step's sequence that token t belongs to; every thread of the workgroup calls it
+__device__ __forceinline__ int seq_of(const Args& A, int t, int* shared) {
+  for (int i = threadIdx.x; i < A.max_seqs; i += 256) {
+    const int q0 = A.q_start[i];
+    if (q0 <= t && t < q0 + A.q_len[i]) *shared = i;
   }
-  while (lo > 0 && A.q_len[lo] == 0) --lo;  // (rows of no sequence start where the last one ends)
-  return lo;
+  __syncthreads();
+  return *shared;
 }
 
 // 8 values of head part `off` (columns off .. off + D of a row) from dimension d, rotated by cs if `rot`
@@ -103,22 +106,21 @@ template <typename T, bool POOL>
 __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
   const int t = token_of(blockIdx.x, A.T);
   if (t < 0) return;
-  const int slot = A.slots[t];
+  const int slot = A.slots[t], pos = A.positions[t];
   if (slot < 0) return;
-  const int pos = A.positions[t];
   const T* row = (const T*)A.x + (size_t)t * A.ldx;
   const float* cs = A.cos_sin + (size_t)pos * A.rd;
   const int ck = A.DK >> 3, cv = A.DV >> 3, nq = A.H * ck, nk = A.G * ck, nv = A.G * cv;
   for (int u = threadIdx.x; u < nq + nk + nv; u += 256) {
     float v[8];
     if (u < nq) {
-      const int h = u / ck, d = (u - h * ck) * 8;
+      const int h = quot(u, A.ick), d = (u - h * ck) * 8;
       chunk(A, row, h * A.DK, d, cs, true, v);
       put((T*)A.q + ((size_t)t * A.H + h) * A.DK + d, v);
     } else {
       const bool key = u < nq + nk;
       const int w = key ? u - nq : u - nq - nk, per = key ? ck : cv, D = key ? A.DK : A.DV;
-      const int h = w / per, o = w - h * per;
+      const int h = quot(w, key ? A.ick : A.icv), o = w - h * per;
       chunk(A, row, (key ? A.H * A.DK : (A.H + A.G) * A.DK) + h * D, o * 8, cs, key, v);
       put((T*)(key ? A.kp : A.vp) + (((size_t)(slot >> 4) * A.G + h) * per + o) * 128 + (slot & 15) * 8, v);
     }
@@ -126,7 +128,8 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
   if constexpr (!POOL) return;
   const int P = A.pool;
   if ((pos + 1) % P) return;
-  const int lo = seq_of(A, t);
+  __shared__ int seq;
+  const int lo = seq_of(A, t, &seq);
   const int start = A.ctx_len[lo] - A.q_len[lo];  // the step's first position
   const int* bt = A.block_table + (size_t)lo * A.max_blocks;
   const int page = pos >> 4, sub = pos / P - (page << 4) / P;
@@ -157,33 +160,36 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
   }
 }
 
-// The blocks that end in this step, from their pages: a workgroup per token that ends one.
+// The blocks that end in this step, from their pages: a workgroup per `rows` tokens.
 template <typename T>
-__global__ __launch_bounds__(256) void pool_kernel(const Args A) {
-  const int t = token_of(blockIdx.x, A.T), P = A.pool;
-  if (t < 0) return;
-  const int slot = A.slots[t], pos = A.positions[t];
-  if (slot < 0 || (pos + 1) % P) return;
-  const int* bt = A.block_table + (size_t)seq_of(A, t) * A.max_blocks;
-  const int ck = A.DK >> 3, cv = A.DV >> 3, nk = A.G * ck, nv = A.G * cv;
-  const int page = pos >> 4, sub = pos / P - (page << 4) / P;
+__global__ __launch_bounds__(256) void pool_kernel(const Args A, int rows) {
+  __shared__ int seq;
+  const int P = A.pool, ck = A.DK >> 3, cv = A.DV >> 3, nk = A.G * ck, nv = A.G * cv;
   const float inv = 1.f / (float)P;
-  for (int u = threadIdx.x; u < nk + nv; u += 256) {
-    const bool key = u < nk;
-    const int w = key ? u : u - nk, per = key ? ck : cv, D = key ? A.DK : A.DV;
-    const int h = w / per, o = w - h * per;
-    float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  const int end = min(A.T, ((int)blockIdx.x + 1) * rows);
+  for (int t = blockIdx.x * rows; t < end; ++t) {
+    const int slot = A.slots[t], pos = A.positions[t];
+    if (slot < 0 || (pos + 1) % P) continue;
+    __syncthreads();
+    const int* bt = A.block_table + (size_t)seq_of(A, t, &seq) * A.max_blocks;
+    const int page = pos >> 4, sub = pos / P - (page << 4) / P;
+    for (int u = threadIdx.x; u < nk + nv; u += 256) {
+      const bool key = u < nk;
+      const int w = key ? u : u - nk, per = key ? ck : cv, D = key ? A.DK : A.DV;
+      const int h = quot(w, key ? A.ick : A.icv), o = w - h * per;
+      float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 #pragma unroll 8
-    for (int p = pos - P + 1; p <= pos; ++p) {
-      T a[8];
-      const T* src = (const T*)(key ? A.kp : A.vp) + (((size_t)bt[p >> 4] * A.G + h) * per + o) * 128 + (p & 15) * 8;
-      __builtin_memcpy(a, __builtin_assume_aligned(src, sizeof(T) * 8), sizeof(T) * 8);
+      for (int p = pos - P + 1; p <= pos; ++p) {
+        T a[8];
+        const T* src = (const T*)(key ? A.kp : A.vp) + (((size_t)bt[p >> 4] * A.G + h) * per + o) * 128 + (p & 15) * 8;
+        __builtin_memcpy(a, __builtin_assume_aligned(src, sizeof(T) * 8), sizeof(T) * 8);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) sum[j] += (float)a[j];
+        for (int j = 0; j < 8; ++j) sum[j] += (float)a[j];
+      }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) sum[j] *= inv;
+      put((T*)(key ? A.pk : A.pv) + (((size_t)(slot >> 4) * A.npb + sub) * A.G + h) * D + o * 8, sum);
     }
-#pragma unroll
-    for (int j = 0; j < 8; ++j) sum[j] *= inv;
-    put((T*)(key ? A.pk : A.pv) + (((size_t)(slot >> 4) * A.npb + sub) * A.G + h) * D + o * 8, sum);
   }
 }
 
@@ -198,14 +204,15 @@ extern "C" int pa_paged_kv(int fp32, const void* x, const float* bias, void* q, 
   if (T <= 0) return 0;
   if (DK % 8 || DV % 8 || rd % 2 || rd > DK || ldx % 8) return -1;
   const pa::kv::Args A{x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_len, block_table, cos_sin,
-                       ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs, T};
+                       ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs, T, 8.f / DK, 8.f / DV};
   const dim3 grid((T + 7) / 8 * 8);
   const bool later = pool > 0 && T > 64, now = pool > 0 && !later;
+  const int rows = pool < 8 ? pool : 8;  // of a workgroup of the second launch
 #define PA_KV(TYPE)                                                                                              \
   do {                                                                                                           \
     if (now) hipLaunchKernelGGL((pa::kv::paged_kv_kernel<TYPE, true>), grid, dim3(256), 0, st, A);               \
     else hipLaunchKernelGGL((pa::kv::paged_kv_kernel<TYPE, false>), grid, dim3(256), 0, st, A);                  \
-    if (later) hipLaunchKernelGGL(pa::kv::pool_kernel<TYPE>, grid, dim3(256), 0, st, A);                         \
+    if (later) hipLaunchKernelGGL(pa::kv::pool_kernel<TYPE>, dim3((T + rows - 1) / rows), dim3(256), 0, st, A, rows); \
   } while (0)
   if (fp32) PA_KV(float); else PA_KV(pa::bf16);
 #undef PA_KV

@@ -93,7 +93,7 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
       const bf16* wt[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) wt[i] = (const bf16*)A.w + (size_t)min(e0 + i, tiles - 1) * K32 * 512 + lane * 8;
-#pragma unroll 4
+#pragma unroll 8
       for (int k = wid; k < K32; k += 8) {
         const bf16x8 b = *reinterpret_cast<const bf16x8*>(hr + 32 * k);
 #pragma unroll

@@ -252,13 +252,17 @@ __global__ __launch_bounds__(256, 4) void step_kernel(const Args A) {
 }
 
 // ---- chunks -------------------------------------------------------------------------------------------
+// Loads come first and together: a chunk's work is short against their latency.
+// A token's raw step size (wave 0), rows past the end whatever the last one has
+__device__ __forceinline__ float load_dt(const Args& A, int h, int row0, int n) {
+  if (threadIdx.x >= 64) return 0.f;
+  return (float)((const bf16*)A.proj)[(size_t)(row0 + min((int)threadIdx.x, n - 1)) * A.ldp + A.H * A.V + A.Cc + h] + A.dt_bias[h];
+}
 // dt and the running log decay of a chunk's tokens (wave 0), rows past the end neutral
-__device__ __forceinline__ void chunk_steps(const Args& A, int h, int row0, int n, float* dt, float* l) {
+__device__ __forceinline__ void chunk_steps(const Args& A, int h, float raw, int n, float* dt, float* l) {
   if (threadIdx.x < 64) {
     const int j = threadIdx.x;
-    float d = 0.f;
-    if (j < n)
-      d = softplus((float)((const bf16*)A.proj)[(size_t)(row0 + j) * A.ldp + A.H * A.V + A.Cc + h] + A.dt_bias[h]);
+    const float d = j < n ? softplus(raw) : 0.f;
     float x = -A.a[h] * d;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
@@ -269,6 +273,12 @@ __device__ __forceinline__ void chunk_steps(const Args& A, int h, int row0, int 
     l[j] = x;
   }
 }
+// 8 columns of one of a chunk's rows (unit e of D / 8 columns x 64 rows); rows past the end repeat the
+// last one, and meet weights of 0
+__device__ __forceinline__ bf16x8 load_cols(const bf16* u, int ld, int e, int D, int n) {
+  return *reinterpret_cast<const bf16x8*>(u + (size_t)min(e & (LC - 1), n - 1) * ld + min((e >> 6) * 8, D - 8));
+}
+constexpr int XB = 2, BB = 4, SB = 8;  // units of x, B and the state that a thread loads ahead
 
 __global__ __launch_bounds__(256) void chunk_state_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -281,29 +291,30 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const Args A) {
   for (int item = blockIdx.y; item < n_items; item += gridDim.y) {
     const int4 it = A.items[item];
     const int n = it.z, row0 = A.q_start[it.x] + it.y;
-    __syncthreads();
-    chunk_steps(A, h, row0, n, dt, l);
-    const bf16* u = (const bf16*)A.u + (size_t)row0 * A.Cc;
-    for (int e = threadIdx.x; e < (N >> 3) * LC; e += 256) {
-      const int j = e & (LC - 1), i = (e >> 6) * 8;
-      bf16x8 b;
-      if (j < n) b = *reinterpret_cast<const bf16x8*>(u + (size_t)j * A.Cc + inner + g * N + i);
-      else
+    const bf16 *ux = (const bf16*)A.u + (size_t)row0 * A.Cc + h * V, *ub = (const bf16*)A.u + (size_t)row0 * A.Cc + inner + g * N;
+    const float raw = load_dt(A, h, row0, n);
+    bf16x8 xv[XB], bv[BB];
 #pragma unroll
-        for (int k = 0; k < 8; ++k) b[k] = (bf16)0.f;
+    for (int i = 0; i < BB; ++i) bv[i] = load_cols(ub, A.Cc, threadIdx.x + 256 * i, N, n);
+#pragma unroll
+    for (int i = 0; i < XB; ++i) xv[i] = load_cols(ux, A.Cc, threadIdx.x + 256 * i, V, n);
+    __syncthreads();
+    chunk_steps(A, h, raw, n, dt, l);
+    auto put_b = [&](int e, const bf16x8& b) {
+      const int j = e & (LC - 1), i = (e >> 6) * 8;
+      if (i >= N) return;
 #pragma unroll
       for (int k = 0; k < 8; ++k) bt[(i + k) * LD + j] = b[k];
-    }
+    };
+#pragma unroll
+    for (int i = 0; i < BB; ++i) put_b(threadIdx.x + 256 * i, bv[i]);
+    for (int e = threadIdx.x + 256 * BB; e < (N >> 3) * LC; e += 256) put_b(e, load_cols(ub, A.Cc, e, N, n));
     __syncthreads();
     const float end = l[LC - 1];
-    for (int e = threadIdx.x; e < (V >> 3) * LC; e += 256) {
+    auto put_x = [&](int e, const bf16x8& x) {
       const int j = e & (LC - 1), i = (e >> 6) * 8;
+      if (i >= V) return;
       const float w = j < n ? dt[j] * expf(end - l[j]) : 0.f;
-      bf16x8 x;
-      if (j < n) x = *reinterpret_cast<const bf16x8*>(u + (size_t)j * A.Cc + h * V + i);
-      else
-#pragma unroll
-        for (int k = 0; k < 8; ++k) x[k] = (bf16)0.f;
 #pragma unroll
       for (int k = 0; k < 8; ++k) {
         bf16 hi, lo;
@@ -311,7 +322,10 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(const Args A) {
         xh[(i + k) * LD + j] = hi;
         xl[(i + k) * LD + j] = lo;
       }
-    }
+    };
+#pragma unroll
+    for (int i = 0; i < XB; ++i) put_x(threadIdx.x + 256 * i, xv[i]);
+    for (int e = threadIdx.x + 256 * XB; e < (V >> 3) * LC; e += 256) put_x(e, load_cols(ux, A.Cc, e, V, n));
     __syncthreads();
     float* out = A.work + ((size_t)item * A.H + h) * V * N;
     const int tn = N >> 4, tv = V >> 4;
@@ -397,8 +411,18 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
     // (rows past the end repeat the last one; their results are dropped)
     const int i = 16 * wid + c, ri = min(i, n - 1);
     const bf16* cr = u + (size_t)ri * A.Cc + inner + A.G * N + g * N + 8 * lg;
-    bf16x8 cf[NK ? NK : 1];
+    const bf16* ux = u + h * V;
+    const float raw = load_dt(A, h, row0, n);
+    bf16x8 cf[NK ? NK : 1], xv[XB];
     f32x4 cb[4];  // C_i . B_j
+    f32x4 sv[STAGED ? SB : 1];
+#pragma unroll
+    for (int k = 0; k < XB; ++k) xv[k] = load_cols(ux, A.Cc, threadIdx.x + 256 * k, V, n);
+    auto load_state = [&](int e) { return *reinterpret_cast<const f32x4*>(S + min(e, V * N - 4)); };
+    if constexpr (STAGED) {
+#pragma unroll
+      for (int k = 0; k < SB; ++k) sv[k] = load_state(1024 * k + threadIdx.x * 4);
+    }
     if constexpr (NK > 0) {
 #pragma unroll
       for (int k = 0; k < NK; ++k) cf[k] = *reinterpret_cast<const bf16x8*>(cr + 32 * k);
@@ -416,20 +440,19 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
       }
     }
     __syncthreads();
-    chunk_steps(A, h, row0, n, dt, l);
-    for (int e = threadIdx.x; e < (V >> 3) * LC; e += 256) {
+    chunk_steps(A, h, raw, n, dt, l);
+    auto put_x = [&](int e, const bf16x8& x) {
       const int j = e & (LC - 1), i = (e >> 6) * 8;
-      bf16x8 x;
-      if (j < n) x = *reinterpret_cast<const bf16x8*>(u + (size_t)j * A.Cc + h * V + i);
-      else
-#pragma unroll
-        for (int k = 0; k < 8; ++k) x[k] = (bf16)0.f;
+      if (i >= V) return;
 #pragma unroll
       for (int k = 0; k < 8; ++k) xt[(i + k) * LD + j] = x[k];
-    }
-    if (STAGED)
-      for (int e = threadIdx.x * 4; e < V * N; e += 1024) {
-        const f32x4 v = *reinterpret_cast<const f32x4*>(S + e);
+    };
+#pragma unroll
+    for (int k = 0; k < XB; ++k) put_x(threadIdx.x + 256 * k, xv[k]);
+    for (int e = threadIdx.x + 256 * XB; e < (V >> 3) * LC; e += 256) put_x(e, load_cols(ux, A.Cc, e, V, n));
+    if constexpr (STAGED) {
+      auto put_state = [&](int e, const f32x4& v) {
+        if (e >= V * N) return;
         const int r = e / N, k0 = e - r * N;
         bf16x4 hi, lo;
 #pragma unroll
@@ -441,7 +464,11 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
         }
         *reinterpret_cast<bf16x4*>(sh + r * NL + k0) = hi;
         *reinterpret_cast<bf16x4*>(sl + r * NL + k0) = lo;
-      }
+      };
+#pragma unroll
+      for (int k = 0; k < SB; ++k) put_state(1024 * k + threadIdx.x * 4, sv[k]);
+      for (int e = 1024 * SB + threadIdx.x * 4; e < V * N; e += 1024) put_state(e, load_state(e));
+    }
     __syncthreads();
     // M[i][j] = exp(l_i - l_j) dt_j (C_i . B_j), a lane's row i, its columns j = 16 jt + 4 lg ..
     const float li = l[i];
@@ -513,10 +540,9 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
         acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, m1[k], acc, 0, 0, 0);
       }
       if (i < n) {
-        const bf16x4 x = *reinterpret_cast<const bf16x4*>(u + (size_t)i * A.Cc + h * V + v0 + 4 * lg);
         bf16x4 o;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) o[r] = (bf16)(acc[r] + dd * (float)x[r]);
+        for (int r = 0; r < 4; ++r) o[r] = (bf16)(acc[r] + dd * (float)xt[(v0 + 4 * lg + r) * LD + i]);
         *reinterpret_cast<bf16x4*>((bf16*)A.y + (size_t)(row0 + i) * A.ldy + h * V + v0 + 4 * lg) = o;
       }
     }

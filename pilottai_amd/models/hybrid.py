@@ -210,7 +210,8 @@ def _pack_gate_up(gate, up, fp: int, dk: int, dtype, device):
 class GatedMLP:
     """down(act(gate h) * up h): the gate and up rows interleaved in one grouped projection of one group."""
 
-    ROWS_64, ROWS_256 = 32, 96
+    # 16-row tiles (each streams the weights) up to this many rows, by weights that passes find in the caches again
+    ROWS_16, ROWS_16_LARGE, LARGE = 80, 40, 1 << 26
 
     def __init__(self, spec: DenseSpec, t: Dict[str, torch.Tensor], width: int, dtype, device):
         self.spec, self.dtype, self.device = spec, dtype, device
@@ -226,7 +227,8 @@ class GatedMLP:
     def __call__(self, h, meta: StepMeta):
         T = h.shape[0]
         if T not in self._tiles:  # (before graph capture: the capture's warm-up runs come first)
-            tm = expert_tile_rows(T, self.dtype, self.dk, self.ROWS_64, self.ROWS_256)
+            few = self.ROWS_16 if self.w13.numel() <= self.LARGE else self.ROWS_16_LARGE
+            tm = expert_tile_rows(T, self.dtype, self.dk, few, few)
             tiles = torch.tensor([[0, i, min(tm, T - i), 0] for i in range(0, T, tm)], dtype=torch.int32)
             self._tiles[T] = (tiles.to(self.device), torch.tensor([len(tiles)], dtype=torch.int32, device=self.device),
                               torch.arange(T, dtype=torch.int32, device=self.device), tm)
