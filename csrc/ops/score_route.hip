@@ -137,6 +137,7 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
     const int per = A.E / A.groups;
     for (int i = l; i < A.groups; i += 32) {
       float a = -1.f, b = -1.f;
+#pragma unroll 4
       for (int e = i * per; e < (i + 1) * per; ++e) {
         const float v = s[e];
         b = fmaxf(b, fminf(a, v));
@@ -148,6 +149,7 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
     for (int i = l; i < A.groups; i += 32) {
       int before = 0;
       const int v = gi[i];
+#pragma unroll 4
       for (int k = 0; k < A.groups; ++k) before += gi[k] > v || (gi[k] == v && k < i);
       if (before >= A.keep)
         for (int e = i * per; e < (i + 1) * per; ++e) si[e] = OUT;
@@ -156,20 +158,28 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
   }
   for (int e = A.E + l; e < Ep; e += 32) si[e] = PAD;
   __syncthreads();
-  for (int e = l; e < A.E; e += 32) {
-    int before = 0;
-    const int v = si[e];
+  for (int e0 = l; e0 < A.E; e0 += 64) {  // two experts a lane
+    const int ea = e0, eb = min(e0 + 32, Ep - 1), va = si[ea], vb = si[eb];
+    int na = 0, nb = 0;
+#pragma unroll 4
     for (int k = 0; k < Ep; k += 4) {
       const int4 q = *reinterpret_cast<const int4*>(si + k);
       const int w[4] = {q.x, q.y, q.z, q.w};
 #pragma unroll
-      for (int j = 0; j < 4; ++j) before += w[j] > v || (w[j] == v && k + j < e);
+      for (int j = 0; j < 4; ++j) {  // (v - 1: an equal score with a lower number comes first; v > INT_MIN)
+        na += w[j] > (k + j < ea ? va - 1 : va);
+        nb += w[j] > (k + j < eb ? vb - 1 : vb);
+      }
     }
-    if (before < A.top && t < A.T) {
-      const size_t p = (size_t)t * KA + before;
-      A.choice[p] = live ? e : -1;
-      A.weights[p] = live ? s[e] : 0.f;
-      if (live) A.rank[p] = atomicAdd(&cnt[e], 1);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int e = i ? e0 + 32 : e0, before = i ? nb : na;
+      if (e < A.E && before < A.top && t < A.T) {
+        const size_t p = (size_t)t * KA + before;
+        A.choice[p] = live ? e : -1;
+        A.weights[p] = live ? s[e] : 0.f;
+        if (live) A.rank[p] = atomicAdd(&cnt[e], 1);
+      }
     }
   }
   if (l < A.always && t < A.T) {
