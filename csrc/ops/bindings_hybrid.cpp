@@ -18,7 +18,7 @@ void pa_window_pad(int k, int v, int* dk, int* dv);
 int pa_window_attention(int fp32, void* out, float* part_o, float* part_ml, const void* q, const void* kp,
                         const void* vp, const void* pk, const void* pv, const int* items, const int* n_items,
                         int max_items, const int* q_start, const int* q_len, const int* ctx_len,
-                        const int* block_table, int max_blocks, int H, int G, int DK, int DV, int dec_tokens,
+                        const int* block_table, int max_blocks, int T, int H, int G, int DK, int DV, int dec_tokens,
                         int tile_tokens, int window, int pool, int npb, int max_slots, float scale_log2, float sink,
                         int simple, hipStream_t st);
 int pa_state_scan(int fp32, const void* proj, int ldp, void* u, void* y, int ldy, float* state, void* ring, float* work,
@@ -150,7 +150,7 @@ void window_attention(at::Tensor out, at::Tensor part_o, at::Tensor part_ml, at:
                                q.data_ptr(), kp.data_ptr(), vp.data_ptr(), pk.data_ptr(), pv.data_ptr(),
                                ints(items, 0, "items"), ints(n_items, 1, "n_items"), mi, ints(q_start, S, "q_start"),
                                ints(q_len, S, "q_len"), ints(ctx_len, S, "ctx_len"), ints(block_table, 0, "block_table"),
-                               block_table.size(1), H, p.G, p.DK, p.DV, dec_tokens, tile_tokens, window, pool, p.npb,
+                               block_table.size(1), q.size(0), H, p.G, p.DK, p.DV, dec_tokens, tile_tokens, window, pool, p.npb,
                                max_slots, (float)(scale * 1.4426950408889634), (float)sink, simple ? 1 : 0, cur_stream()),
            "window_attention");
 }

@@ -14,12 +14,13 @@
 //   S^T[keys x cols] = K . Q^T         cols = (token, query head of the KV head's group) pairs
 //   O^T[dims x cols] += V^T . P^T      P^T = the S^T accumulator's own registers
 //
-// An item's keys are its pooled blocks (16 or 32 at a time) and then the tiles of its window. Items
+// An item's keys are its pooled blocks (a tile at a time) and then the tiles of its window. Items
 // come from the scheduler like paged_attention's (seq, q_begin, nq | part<<8 | nparts<<20, partial slot):
 //   nq <= dec_tokens: split over keys. The 8 waves take every 8th page with a private LDS tile and merge;
 //                     nparts > 1 divides the item's own key range, merge_kernel combines the partitions.
-//   otherwise:        128 columns per workgroup, 16 per wave; all waves share double-buffered 32-key tiles
-//                     that arrive by direct global -> LDS loads. Few such items are cut over keys too.
+//   otherwise:        128 columns per workgroup, 16 per wave; all waves share double-buffered tiles of 64 keys
+//                     (32 for the widest heads) that arrive by direct global -> LDS loads. Few such items are
+//                     cut over keys too.
 #include "common.h"
 
 #include <algorithm>
@@ -348,12 +349,16 @@ __global__ __launch_bounds__(256) void merge_kernel(const Args A) {
 }
 
 template <int NK, int NV>
+constexpr int tile_parts() { return NK + NV <= 8 ? 4 : 2; }  // 16-key parts of a tile
+
+template <int NK, int NV>
 __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* smem) {
-  constexpr int DK = 32 * NK, DV = 32 * NV, HALF = (NK + NV) * 1024, TILE = 2 * HALF;  // two 16-key halves: K, V
+  constexpr int DK = 32 * NK, DV = 32 * NV, KT = tile_parts<NK, NV>(), KEYS = 16 * KT;
+  constexpr int PART = (NK + NV) * 1024, TILE = KT * PART;  // a 16-key part: K, then V
   const int s = it.x, qb = it.y, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff, nparts = it.z >> 20;
   const int cols = nq * A.R, cw = blockIdx.x * (16 * NW), gk = blockIdx.z;
   if (cw >= cols) return;
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
+  const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, c = lane & 15;
   const int ctx = A.ctx_len[s], ql = A.q_len[s];
   const int pos0 = ctx - ql + qb;
   const int* bt = A.block_table + (size_t)s * A.max_blocks;
@@ -364,11 +369,11 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
   bf16x8 qf[NK];
 #pragma unroll
   for (int m = 0; m < NK; ++m) qf[m] = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + row * DK + 32 * m + 8 * g);
-  // positions of the workgroup's columns -> its tiles of 32: pooled blocks, then tokens
+  // positions of the workgroup's columns -> its tiles: pooled blocks, then tokens
   const int f = pos0 + cw / A.R, e = pos0 + min(cw + 16 * NW - 1, cols - 1) / A.R;
-  const int nb = blocks_of(A, e), np = (nb + 31) >> 5;
-  const int k_lo = first_key(A, f) >> 5;
-  int t_lo = 0, t_hi = np + ((e + 32) >> 5) - k_lo;
+  const int nb = blocks_of(A, e), np = (nb + KEYS - 1) / KEYS;
+  const int k_lo = first_key(A, f) / KEYS;
+  int t_lo = 0, t_hi = np + (e + KEYS) / KEYS - k_lo;
   if (nparts > 1) {  // this partition's tiles (possibly none)
     const int per = (t_hi + nparts - 1) / nparts;
     t_lo = part * per;
@@ -384,67 +389,72 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
 #pragma unroll
   for (int n = 0; n < 2 * NV; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m_run = NEG_BIG, l_run = 0.f;
-  // direct loads, 1 KB per wave and instruction; a token page is copied linearly, pooled rows by lane
-  auto issue = [&](int t, char* dst) {
-    const bf16 *k[2], *v[2];
-    int sk, sv;
-    if (t < np) {
+  // direct loads, 1 KB per wave and instruction; a token page is copied linearly, pooled rows by lane. The
+  // page ids of a wave's next chunks are read a tile ahead.
+  constexpr int CHUNKS = KT * (NK + NV), PER = (CHUNKS + NW - 1) / NW;
+  int pg[PER];
+  auto pages = [&](int t) {
 #pragma unroll
-      for (int x = 0; x < 2; ++x) {
-        const size_t r = pooled_row(A, bt, min(32 * t + 16 * x + c, nb - 1), gk);
-        k[x] = (const bf16*)A.pk + r * DK + 8 * g;
-        v[x] = (const bf16*)A.pv + r * DV + 8 * g;
-      }
-      sk = sv = 32;
-    } else {
-#pragma unroll
-      for (int x = 0; x < 2; ++x) {
-        const size_t r = (size_t)bt[min(2 * (k_lo + t - np) + x, nblk - 1)] * A.G + gk;
-        k[x] = (const bf16*)A.kp + r * (DK * 16) + lane * 8;
-        v[x] = (const bf16*)A.vp + r * (DV * 16) + lane * 8;
-      }
-      sk = sv = 512;
+    for (int i = 0; i < PER; ++i) {
+      const int x = min((i * NW + wid) / (NK + NV), KT - 1);
+      pg[i] = bt[min(max(KT * (k_lo + t - np) + x, 0), nblk - 1)];
     }
+  };
+  auto issue = [&](int t, char* dst) {
 #pragma unroll
-    for (int i = 0; i < (2 * (NK + NV) + NW - 1) / NW; ++i) {
+    for (int i = 0; i < PER; ++i) {
       const int ch = i * NW + wid;  // wave-uniform
-      if (2 * (NK + NV) % NW == 0 || ch < 2 * (NK + NV)) {
-        const int x = ch >= NK + NV, m = ch - x * (NK + NV);
-        const bf16* src = m < NK ? (x ? k[1] : k[0]) + m * sk : (x ? v[1] : v[0]) + (m - NK) * sv;
+      if (CHUNKS % NW == 0 || ch < CHUNKS) {
+        const int x = ch / (NK + NV), m = ch - x * (NK + NV);
+        const bf16* src;
+        if (t < np) {
+          const size_t r = pooled_row(A, bt, min(KEYS * t + 16 * x + c, nb - 1), gk);
+          src = m < NK ? (const bf16*)A.pk + r * DK + 32 * m + 8 * g : (const bf16*)A.pv + r * DV + 32 * (m - NK) + 8 * g;
+        } else {
+          const size_t r = (size_t)pg[i] * A.G + gk;
+          src = (m < NK ? (const bf16*)A.kp + r * (DK * 16) + m * 512 : (const bf16*)A.vp + r * (DV * 16) + (m - NK) * 512) + lane * 8;
+        }
         __builtin_amdgcn_global_load_lds((glb_void*)src, (lds_void*)(dst + ch * 1024), 16, 0, 0);
       }
     }
   };
   const int toff = ((c & 3) >> 1) * 256 + (4 * g + (c >> 2)) * 16 + (c & 1) * 8;
-  if (t_lo < t_hi) issue(t_lo, smem);
+  if (t_lo < t_hi) {
+    pages(t_lo);
+    issue(t_lo, smem);
+    pages(t_lo + 1);
+  }
   for (int t = t_lo; t < t_hi; ++t) {
     char* cur = smem + ((t - t_lo) & 1) * TILE;
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();  // tile t is whole, and nobody reads the other buffer any more
-    if (t + 1 < t_hi) issue(t + 1, smem + ((t + 1 - t_lo) & 1) * TILE);
-    f32x4 sc[2];
+    if (t + 1 < t_hi) {
+      issue(t + 1, smem + ((t + 1 - t_lo) & 1) * TILE);
+      pages(t + 2);
+    }
+    f32x4 sc[KT];
 #pragma unroll
-    for (int k = 0; k < 2; ++k) sc[k] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < KT; ++k) sc[k] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int m = 0; m < NK; ++m)
 #pragma unroll
-      for (int k = 0; k < 2; ++k) {
-        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(cur + k * HALF + m * 1024 + loff);
+      for (int k = 0; k < KT; ++k) {
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(cur + k * PART + m * 1024 + loff);
         sc[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[m], sc[k], 0, 0, 0);
       }
-    const int key0 = 32 * (k_lo + t - np);  // wave-uniform
-    if (t < np ? 32 * t + 32 > full_nb : (key0 < full_lo || key0 + 31 > full_hi)) {
+    const int key0 = KEYS * (k_lo + t - np);  // wave-uniform
+    if (t < np ? KEYS * (t + 1) > full_nb : (key0 < full_lo || key0 + KEYS - 1 > full_hi)) {
 #pragma unroll
-      for (int k = 0; k < 2; ++k)
+      for (int k = 0; k < KT; ++k)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int x = 16 * k + 4 * g + r, key = key0 + x;
-          if (t < np ? 32 * t + x >= cnb : (key > cpos || key < klo)) sc[k][r] = NEG_BIG;
+          if (t < np ? KEYS * t + x >= cnb : (key > cpos || key < klo)) sc[k][r] = NEG_BIG;
         }
     }
     float tmax = NEG_BIG;
 #pragma unroll
-    for (int k = 0; k < 2; ++k)
+    for (int k = 0; k < KT; ++k)
 #pragma unroll
       for (int r = 0; r < 4; ++r) tmax = fmaxf(tmax, sc[k][r]);
     tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
@@ -459,26 +469,29 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
     }
     // a column that has seen no key yet (its window starts in a later tile): every weight is 0
     const float nm = m_run < 0.01f * NEG_BIG ? 0.f : -m_run;
-    bf16x8 pf;
+    bf16x8 pf[KT / 2];
 #pragma unroll
-    for (int k = 0; k < 2; ++k)
+    for (int k = 0; k < KT; ++k)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const float p = __builtin_amdgcn_exp2f(fmaf(sc[k][r], A.scale_log2, nm));
         l_run += p;
-        pf[4 * k + r] = (bf16)p;
+        pf[k / 2][4 * (k % 2) + r] = (bf16)p;
       }
 #pragma unroll
-    for (int n = 0; n < 2 * NV; ++n) {
-      const bf16x4 v0 = tr_read(cur + NK * 1024 + n * 512 + toff), v1 = tr_read(cur + HALF + NK * 1024 + n * 512 + toff);
-      bf16x8 v;
+    for (int k = 0; k < KT / 2; ++k)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        v[j] = v0[j];
-        v[4 + j] = v1[j];
+      for (int n = 0; n < 2 * NV; ++n) {
+        const char* vt = cur + 2 * k * PART + NK * 1024 + n * 512 + toff;
+        const bf16x4 v0 = tr_read(vt), v1 = tr_read(vt + PART);
+        bf16x8 v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          v[j] = v0[j];
+          v[4 + j] = v1[j];
+        }
+        o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pf[k], o[n], 0, 0, 0);
       }
-      o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pf, o[n], 0, 0, 0);
-    }
   }
   l_run += __shfl_xor(l_run, 16, 64);
   l_run += __shfl_xor(l_run, 32, 64);
@@ -504,26 +517,32 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
 
 template <int NK, int NV>
 constexpr int lds_bytes() {
-  return std::max({2 * 2 * 1024 * (NK + NV), NW * 32 * 32 * NV + 1024 * NK, NW * 16 * MERGE_LD * 4 + 2 * NW * 16 * 4});
+  return std::max({2 * tile_parts<NK, NV>() * 1024 * (NK + NV), NW * 32 * 32 * NV + 1024 * NK, NW * 16 * MERGE_LD * 4 + 2 * NW * 16 * 4});
 }
 
-template <int NK, int NV>
-__global__ __launch_bounds__(64 * NW, 2) void mfma_kernel(const Args A) {
+// The two paths want different registers: tiles four waves a SIMD, split items all they can hold. Small steps
+// run both in one launch, larger ones each in its own.
+enum { TILES = 1, SPLITS = 2 };
+
+template <int NK, int NV, int PATHS>
+__global__ __launch_bounds__(64 * NW, PATHS == TILES && NK + NV <= 8 ? 4 : 2) void mfma_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int n = A.n_items[0];
   // two passes over the workgroup's items, so that neither path's registers carry the other's
-  for (int item = blockIdx.y; item < n; item += gridDim.y) {
-    const int4 it = A.items[item];
-    if ((it.z & 0xff) <= A.dec_tokens) continue;
-    tile_item<NK, NV>(A, it, smem);
-    __syncthreads();
-  }
-  for (int item = blockIdx.y; item < n; item += gridDim.y) {
-    const int4 it = A.items[item];
-    if ((it.z & 0xff) > A.dec_tokens) continue;
-    split_item<NK, NV>(A, it, smem);
-    __syncthreads();
-  }
+  if constexpr ((PATHS & TILES) != 0)
+    for (int item = blockIdx.y; item < n; item += gridDim.y) {
+      const int4 it = A.items[item];
+      if ((it.z & 0xff) <= A.dec_tokens) continue;
+      tile_item<NK, NV>(A, it, smem);
+      __syncthreads();
+    }
+  if constexpr ((PATHS & SPLITS) != 0)
+    for (int item = blockIdx.y; item < n; item += gridDim.y) {
+      const int4 it = A.items[item];
+      if ((it.z & 0xff) > A.dec_tokens) continue;
+      split_item<NK, NV>(A, it, smem);
+      __syncthreads();
+    }
 }
 
 }  // namespace wa
@@ -551,7 +570,7 @@ extern "C" void pa_window_pad(int k, int v, int* dk, int* dv) {
 extern "C" int pa_window_attention(int fp32, void* out, float* part_o, float* part_ml, const void* q, const void* kp,
                                    const void* vp, const void* pk, const void* pv, const int* items,
                                    const int* n_items, int max_items, const int* q_start, const int* q_len,
-                                   const int* ctx_len, const int* block_table, int max_blocks, int H, int G, int DK,
+                                   const int* ctx_len, const int* block_table, int max_blocks, int T, int H, int G, int DK,
                                    int DV, int dec_tokens, int tile_tokens, int window, int pool, int npb,
                                    int max_slots, float scale_log2, float sink, int simple, hipStream_t st) {
   if (max_items <= 0) return 0;
@@ -561,18 +580,26 @@ extern "C" int pa_window_attention(int fp32, void* out, float* part_o, float* pa
                  block_table, max_blocks, max_slots, H, G, R, NB, DK, DV, dec_tokens, window, pool, npb, scale_log2, sink};
   if (!fp32 && !simple) {
     const int cw = 16 * pa::wa::NW, gt = (tile_tokens * R + cw - 1) / cw, gx = NB > gt ? NB : gt;
-    const int gy = max_items < 256 ? 256 : (max_items < 4096 ? max_items : 4096);
+    const int gy = std::min(max_items, std::max(256, 2048 / G));  // (workgroups loop over the rest)
 #define PA_X(K, V)                                                                                            \
   if (DK == 32 * K && DV == 32 * V) {                                                                         \
-    constexpr int lds = pa::wa::lds_bytes<K, V>();                                                            \
+    using namespace pa::wa;                                                                                   \
+    constexpr int lds = lds_bytes<K, V>();                                                                    \
     static bool attr = false;                                                                                 \
     if (!attr) {                                                                                              \
-      (void)hipFuncSetAttribute((const void*)pa::wa::mfma_kernel<K, V>,                                       \
-                                hipFuncAttributeMaxDynamicSharedMemorySize, lds);                             \
+      for (const void* f : {(const void*)mfma_kernel<K, V, TILES>, (const void*)mfma_kernel<K, V, SPLITS>,    \
+                            (const void*)mfma_kernel<K, V, TILES | SPLITS>})                                  \
+        (void)hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, lds);                        \
       attr = true;                                                                                            \
     }                                                                                                         \
-    hipLaunchKernelGGL((pa::wa::mfma_kernel<K, V>), dim3(gx, gy, G), dim3(64 * pa::wa::NW), lds, st, A);      \
-    hipLaunchKernelGGL((pa::wa::merge_kernel<V>), dim3(8, std::min(gy, 256), G), dim3(256), 0, st, A);        \
+    const dim3 wg(64 * NW);                                                                                   \
+    if (T <= 64) {                                                                                            \
+      hipLaunchKernelGGL((mfma_kernel<K, V, TILES | SPLITS>), dim3(gx, gy, G), wg, lds, st, A);               \
+    } else {                                                                                                  \
+      hipLaunchKernelGGL((mfma_kernel<K, V, TILES>), dim3(gt, gy, G), wg, lds, st, A);                        \
+      hipLaunchKernelGGL((mfma_kernel<K, V, SPLITS>), dim3(NB, gy, G), wg, lds, st, A);                       \
+    }                                                                                                         \
+    hipLaunchKernelGGL((pa::wa::merge_kernel<V>), dim3(16, std::min(gy, 64), G), dim3(256), 0, st, A);        \
     return (int)hipGetLastError();                                                                            \
   }
     PA_WA_DIMS(PA_X)
