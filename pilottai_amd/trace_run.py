@@ -9,7 +9,7 @@ Steps come from standard input, one JSON object a line:
 All entries of a step run as one batch (LLMEngine.feed_step: the scheduler, paged cache and forward
 that generation uses). The logits at the wanted places go to OUT/<step>.f32 as little-endian fp32
 [wanted, vocab], in order; then "done <step>" is printed. Requests named in "end" give back their
-pages. The cache pool holds N tokens and four requests may be live, so pages and slots are used
+pages and state slots. The cache pool holds N tokens and four requests may be live, so pages and slots are used
 again. Kernels that are not built yet are compiled first, only those the model needs.
 """
 from __future__ import annotations

@@ -23,7 +23,7 @@ def gen(seed):
 
 # ---- residual ----------------------------------------------------------------------------------------
 @kinds
-@pytest.mark.parametrize("S,D,K,weighted", [(1, 72, 1, False), (2, 50, 3, True), (3, 192, 1, True), (4, 2048, 7, True), (5, 100, 2, False), (8, 4096, 1, False)])
+@pytest.mark.parametrize("S,D,K,weighted", [(1, 72, 1, False), (2, 50, 3, True), (3, 160, 1, True), (4, 2048, 7, True), (5, 100, 2, False), (8, 4096, 1, False)])
 def test_hyper_norm(device, dt, S, D, K, weighted):
     from pilottai_amd import ops
 
@@ -72,7 +72,7 @@ def test_softcap(device, dt):
 
 # ---- rotation ----------------------------------------------------------------------------------------
 @pytest.mark.parametrize("scaling", [None, (2.5, 60.0, 4.0, 1.0), (8.0, 4096.0, 32.0, 1.0), (1.0, 100.0, 4.0, 2.0), (4.0, 16.0, 64.0, 32.0)])
-@pytest.mark.parametrize("dims,base", [(4, 10.0), (32, 300.0), (96, 20000.0), (128, 500000.0)])
+@pytest.mark.parametrize("dims,base", [(4, 10.0), (32, 300.0), (80, 30000.0), (128, 500000.0)])
 def test_angles(dims, base, scaling):
     from pilottai_amd import ops
 
@@ -220,7 +220,7 @@ def run_attention(device, dt, H, G, dk, dv, reqs, W, P, sink=1.0, simple=False, 
             torch.testing.assert_close(out[q0:q0 + n, h].double().cpu(), want, **tol(dt), msg=lambda s, i=i: f"request {i} {reqs[i]}: {s}")
 
 
-SHAPES = [(1, 1, 32, 32), (6, 2, 64, 32), (4, 4, 96, 96), (8, 1, 128, 64), (20, 1, 64, 64)]
+SHAPES = [(1, 1, 32, 32), (6, 2, 64, 32), (3, 3, 96, 96), (8, 1, 128, 64), (20, 1, 64, 64)]
 MASKS = [(0, 0), (1, 0), (45, 0), (45, 12), (128, 16), (16, 5), (33, 50), (7, 1)]
 
 
@@ -229,7 +229,7 @@ MASKS = [(0, 0), (1, 0), (45, 0), (45, 12), (128, 16), (16, 5), (33, 50), (7, 1)
 @pytest.mark.parametrize("step", list(STEPS))
 @pytest.mark.parametrize("H,G,dk,dv", SHAPES)
 def test_window_attention(device, dt, H, G, dk, dv, step, W, P):
-    if device == "cpu" and (H, W) not in ((6, 45), (6, 0), (4, 16)):
+    if device == "cpu" and (H, W) not in ((6, 45), (6, 0), (3, 16)):
         pytest.skip("a selection on the CPU")
     run_attention(device, dt, H, G, dk, dv, STEPS[step], W, P)
 
@@ -289,7 +289,7 @@ def test_window_attention_edges(device, dt, W, P, reqs):
 
 # ---- state-space layers ---------------------------------------------------------------------------------
 @kinds
-@pytest.mark.parametrize("H,V,N,G,taps", [(4, 16, 32, 2, 4), (3, 32, 64, 1, 2), (6, 48, 96, 3, 6), (2, 64, 128, 2, 4), (1, 128, 256, 1, 8)])
+@pytest.mark.parametrize("H,V,N,G,taps", [(4, 16, 32, 2, 4), (3, 32, 64, 1, 2), (6, 80, 96, 3, 6), (2, 64, 128, 2, 4), (1, 128, 256, 1, 8)])
 def test_state_scan(device, dt, H, V, N, G, taps):
     """Requests in portions of all sizes, batched and reordered, against one pass over each whole sequence."""
     from pilottai_amd import ops
