@@ -85,9 +85,10 @@ void head_gemm(at::Tensor x, int64_t xg, at::Tensor w, at::Tensor out, int64_t o
            "head_gemm");
 }
 
-// rows sorted by group: x row = order[p] / x_div (x_div 0: p), out row = out_order ? order[p] : p
+// rows sorted by group: x row = order[p] / x_div (x_div 0: p), out row = out_order ? order[p] : p; epi 1: the gated
+// unit, 2: the square of relu
 void expert_gemm(at::Tensor x, at::Tensor w, at::Tensor out, at::Tensor tiles, at::Tensor n_tiles, at::Tensor order,
-                 int64_t rows, int64_t x_div, bool out_order, int64_t tm, bool glu, double limit, double alpha,
+                 int64_t rows, int64_t x_div, bool out_order, int64_t tm, int64_t epi, double limit, double alpha,
                  double bias, double cubic) {
   const int f = is_f32(x, "x");
   check_rows(x, x.scalar_type(), "x");
@@ -95,15 +96,17 @@ void expert_gemm(at::Tensor x, at::Tensor w, at::Tensor out, at::Tensor tiles, a
   check_dtype(w, x.scalar_type(), "w");
   int64_t G, N, K;
   dims(w, f, &G, &N, &K);
-  TORCH_CHECK(K <= x.size(1) && (glu ? N / 2 : N) <= out.size(1) && out.size(0) >= rows &&
+  TORCH_CHECK(K <= x.size(1) && epi >= 0 && epi <= 2 && (epi == 1 ? N / 2 : N) <= out.size(1) && out.size(0) >= rows &&
                   x.size(0) * (x_div ? x_div : 1) >= rows, "expert_gemm sizes");
-  TORCH_CHECK(f || (x.stride(0) % 8 == 0 && out.stride(0) % 4 == 0), "expert_gemm: 16-byte aligned rows");
-  TORCH_CHECK(tm != 256 || (!f && K % 64 == 0 && K >= 128 && N % 128 == 0 && out.stride(0) % 8 == 0),
+  TORCH_CHECK(f || (x.stride(0) % 8 == 0 && out.stride(0) % 4 == 0 && ((uintptr_t)out.data_ptr() & 7) == 0),
+              "expert_gemm: 16-byte aligned rows");
+  TORCH_CHECK(tm != 256 || (!f && K % 64 == 0 && K >= 128 && N % 128 == 0 && out.stride(0) % 8 == 0 &&
+                               ((uintptr_t)out.data_ptr() & 15) == 0),
               "expert_gemm: tiles of 256 rows need K % 64 == 0, K >= 128, N % 128 == 0");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 4, "tiles must be [n, 4]");
   check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, G, x.stride(0), 0, out.stride(0), 0, 0,
                            N / 16, K / 32, ints(tiles, 4, "tiles"), tiles.size(0), ints(n_tiles, 1, "n_tiles"),
-                           ints(order, rows, "order"), x_div, out_order ? 1 : 0, tm, glu ? 1 : 0, (float)limit,
+                           ints(order, rows, "order"), x_div, out_order ? 1 : 0, tm, (int)epi, (float)limit,
                            (float)alpha, (float)cubic, (float)bias, nullptr, nullptr, 0, 0, 0, 0, cur_stream()),
            "expert_gemm");
 }

@@ -763,7 +763,7 @@ extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long
                                int out_order, int epi, float limit, float alpha, float cubic, float bias,
                                hipStream_t st) {
   using namespace pa::pf;
-  if (K % 64 || K < 128 || N % 128 || ldx % 8 || ldy % 8 || (epi != EP_PLAIN && epi != EP_GLU)) return -1;
+  if (K % 64 || K < 128 || N % 128 || ldx % 8 || ldy % 8 || (epi != EP_PLAIN && epi != EP_GLU && epi != EP_RELU2)) return -1;
   if (max_tiles <= 0) return 0;
   Args a{};
   a.y = (pa::bf16*)y;
@@ -784,6 +784,7 @@ extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long
   hipLaunchKernelGGL((pingpong_grouped_kernel<E, F>), dim3(grid), dim3(512), 0, st, a, (const int4*)tiles, n_tiles, \
                      order, wstride, x_div, out_order)
   if (epi == EP_GLU) { if (wide) PA_EX(EP_GLU, 8); else PA_EX(EP_GLU, 4); }
+  else if (epi == EP_RELU2) { if (wide) PA_EX(EP_RELU2, 8); else PA_EX(EP_RELU2, 4); }
   else { if (wide) PA_EX(EP_PLAIN, 8); else PA_EX(EP_PLAIN, 4); }
 #undef PA_EX
   return (int)hipGetLastError();

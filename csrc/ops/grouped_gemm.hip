@@ -12,7 +12,7 @@
 // rows share them; prompts with 256 rows and more per group run the ping-pong kernels instead
 // (gemm_prefill.hip pa_expert_tiles).
 //
-// Epilogues: plain, or the gated unit of packed_epi.h (limit, alpha, cubic, bias).
+// Epilogues: plain, the gated unit of packed_epi.h (limit, alpha, cubic, bias), or the square of relu.
 #include "packed_epi.h"
 
 extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long wstride, int N, int K, int ldx, int ldy,
@@ -95,7 +95,9 @@ __device__ __forceinline__ float glu(float g, float u, const Args& A) {
   return pk::gated_unit(g, u, A.limit, A.alpha, A.cubic, A.bias);
 }
 
-template <int MT, int NT, int KU, bool GLU>
+enum { PLAIN = 0, GLU = 1, RELU2 = 2 };
+
+template <int MT, int NT, int KU, int EPI>
 __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int c = lane & 15, g = lane >> 4;
@@ -170,7 +172,7 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
     if (16 * m + c >= n) continue;
     const int orow = (A.tiles && A.out_order) ? A.order[pos[m]] : pos[m];
     bf16* o = (bf16*)A.out + (size_t)orow * A.ldo + (A.tiles ? 0 : (size_t)grp * A.og) + 4 * g;
-    if constexpr (GLU) {
+    if constexpr (EPI == GLU) {
 #pragma unroll
       for (int i = 0; i + 1 < NT; i += 2) {
         if (nt0 + i >= A.N16) break;
@@ -185,7 +187,7 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
 #pragma unroll
       for (int i = 0; i + 1 < NT; i += 2) {
         if (nt0 + i >= A.N16) break;
-        pk::store_pair_wide<pk::EP_PLAIN>(row, 0, nt0 + i, g, acc[m][i], acc[m][i + 1]);
+        pk::store_pair_wide<EPI == RELU2 ? pk::EP_RELU2 : pk::EP_PLAIN>(row, 0, nt0 + i, g, acc[m][i], acc[m][i + 1]);
       }
     } else {
 #pragma unroll
@@ -193,7 +195,7 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
         if (nt0 + i >= A.N16) break;
         bf16x4 v;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = (bf16)acc[m][i][j];
+        for (int j = 0; j < 4; ++j) v[j] = (bf16)(EPI == RELU2 ? pk::relu2(acc[m][i][j]) : acc[m][i][j]);
         *reinterpret_cast<bf16x4*>(o + (nt0 + i) * 16) = v;
       }
     }
@@ -202,8 +204,9 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
 
 // fp32: one output (or gated pair) per thread, weights row-major [G, 16 N16, 32 K32] in the same
 // row order as the packed ones. The exact path; not tuned.
-template <bool GLU>
+template <int EPI>
 __global__ __launch_bounds__(256) void gemm_f32_kernel(const Args A) {
+  constexpr bool PAIR = EPI == GLU;
   constexpr int TM = 16;
   __shared__ float xs[TM][33], w0[16][33], w1[16][33];
   const int tn = threadIdx.x & 15, tm = threadIdx.x >> 4;
@@ -223,7 +226,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const Args A) {
   }
   const int bx = (int)blockIdx.x - (A.rp ? 1 : 0);
   const int K = A.K32 * 32;
-  const float* wg = (const float*)A.w + (size_t)grp * A.wstride + (size_t)bx * (GLU ? 32 : 16) * K;
+  const float* wg = (const float*)A.w + (size_t)grp * A.wstride + (size_t)bx * (PAIR ? 32 : 16) * K;
   float a0 = 0.f, a1 = 0.f;
   for (int k0 = 0; k0 < K; k0 += 32) {
     __syncthreads();
@@ -233,20 +236,20 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const Args A) {
       if (A.tiles && A.x_div) row = A.order[p] / A.x_div;
       xs[m][k] = ((const float*)A.x)[(size_t)row * A.ldx + (A.tiles ? 0 : (size_t)grp * A.xg) + k0 + k];
       w0[m][k] = wg[(size_t)m * K + k0 + k];
-      if (GLU) w1[m][k] = wg[(size_t)(16 + m) * K + k0 + k];
+      if (PAIR) w1[m][k] = wg[(size_t)(16 + m) * K + k0 + k];
     }
     __syncthreads();
 #pragma unroll 8
     for (int k = 0; k < 32; ++k) {
       a0 += xs[tm][k] * w0[tn][k];
-      if (GLU) a1 += xs[tm][k] * w1[tn][k];
+      if (PAIR) a1 += xs[tm][k] * w1[tn][k];
     }
   }
   if (tm >= n) return;
   const int p = start + tm;
   const int orow = (A.tiles && A.out_order) ? A.order[p] : p;
   float* o = (float*)A.out + (size_t)orow * A.ldo + (A.tiles ? 0 : (size_t)grp * A.og) + bx * 16 + tn;
-  *o = GLU ? glu(a0, a1, A) : a0;
+  *o = PAIR ? glu(a0, a1, A) : EPI == RELU2 ? pk::relu2(a0) : a0;
 }
 
 // Routing by token id, for every expert layer of the model in one launch (workgroup = layer):
@@ -341,13 +344,14 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
   if (fp32) {
     if (tiles && tm != 16) return -2;
     const dim3 grid((epi == 1 ? N16 / 2 : N16) + rot, tiles ? max_tiles : (rows + 15) / 16, tiles ? 1 : groups);
-    if (epi == 1) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<true>), grid, dim3(256), 0, st, A);
-    else hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<false>), grid, dim3(256), 0, st, A);
+    if (epi == 1) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<pa::gg::GLU>), grid, dim3(256), 0, st, A);
+    else if (epi == 2) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<pa::gg::RELU2>), grid, dim3(256), 0, st, A);
+    else hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<pa::gg::PLAIN>), grid, dim3(256), 0, st, A);
     return (int)hipGetLastError();
   }
   if (tiles && tm == 256)
     return pa_expert_tiles(out, x, w, wstride, N16 * 16, K32 * 32, ldx, ldo, tiles, max_tiles, n_tiles, order, x_div,
-                           out_order, epi == 1 ? 5 : 0, limit, alpha, cubic, bias, st);
+                           out_order, epi == 1 ? pa::pk::EP_GLU : epi == 2 ? pa::pk::EP_RELU2 : pa::pk::EP_PLAIN, limit, alpha, cubic, bias, st);
   // dense: 64-row tiles once they fill the chip
   if (!tiles) tm = (N16 + 15) / 16 * ((rows + 63) / 64) * groups < 256 ? 16 : 64;
   if (tm != 16 && tm != 64) return -2;
@@ -363,11 +367,13 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
     else PA_GG(MT, NT, 1, G);                  \
   } while (0)
   if (tm == 16) {
-    if (epi == 1) PA_GGK(1, 2, true);
-    else PA_GGK(1, 1, false);
+    if (epi == 1) PA_GGK(1, 2, pa::gg::GLU);
+    else if (epi == 2) PA_GGK(1, 1, pa::gg::RELU2);
+    else PA_GGK(1, 1, pa::gg::PLAIN);
   } else {
-    if (epi == 1) PA_GG(4, 4, 1, true);
-    else PA_GG(4, 4, 1, false);
+    if (epi == 1) PA_GG(4, 4, 1, pa::gg::GLU);
+    else if (epi == 2) PA_GG(4, 4, 1, pa::gg::RELU2);
+    else PA_GG(4, 4, 1, pa::gg::PLAIN);
   }
 #undef PA_GGK
 #undef PA_GG

@@ -1,7 +1,7 @@
 // The step between two sublayers of a decoder whose fp32 residual has several streams x_1 .. x_S
 // (hyper-connections; S = 1 with unit weights is the plain residual sum):
 //
-//   y   <- sum_k w_k y_k + bias                        (K partial outputs per token, weights optional)
+//   y   <- sum_k w_k y_k + y2 + bias                   (K partial outputs per token, weights optional)
 //   x_t <- sum_s mix[s][t] x_s + post[t] y              or, at the start, x_t <- E[id]
 //   out <- norm(sum_s pre[s] x_s) * w_next              (the next sublayer's input)
 //
@@ -22,6 +22,7 @@ struct Args {
   float* x;             // [T, S, D]
   const void* y;        // [T, K, ldy]
   const float* y_w;     // [T, K] or null
+  const void* y2;       // [T, ldy2] or null
   const float* bias;    // [D] or null
   const float *mix, *post, *pre;  // [S, S] from x to, [S], [S]
   const void* emb;
@@ -29,7 +30,7 @@ struct Args {
   const float* w_next;
   void* out;
   const int* rows;
-  int K, ldy, vocab, ldo, D;
+  int K, ldy, ldy2, vocab, ldo, D;
   float eps;
 };
 
@@ -71,6 +72,11 @@ __global__ __launch_bounds__(256) void hyper_norm_kernel(const Args A) {
       float y[VEC];
 #pragma unroll
       for (int j = 0; j < VEC; ++j) y[j] = A.bias ? A.bias[i + j] : 0.f;
+      if (A.y2) {
+        __builtin_memcpy(a, __builtin_assume_aligned((const T*)A.y2 + (size_t)t * A.ldy2 + i, sizeof(T) * VEC), sizeof(T) * VEC);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) y[j] += (float)a[j];
+      }
 #pragma unroll 4
       for (int k = 0; k < A.K; ++k) {
         __builtin_memcpy(a, __builtin_assume_aligned(yr + (size_t)k * A.ldy + i, sizeof(T) * VEC), sizeof(T) * VEC);
@@ -135,14 +141,14 @@ __global__ __launch_bounds__(256) void softcap_kernel(T* __restrict__ x, int ld,
 }  // namespace pa
 
 extern "C" int pa_hyper_norm(int fp32, float* x, int S, const void* y, int K, int ldy, const float* y_w,
-                             const float* bias, const float* mix, const float* post, const float* pre, const void* emb,
+                             const void* y2, int ldy2, const float* bias, const float* mix, const float* post, const float* pre, const void* emb,
                              const int* ids, int vocab, const float* w_next, void* out, int ldo, const int* rows, int n,
                              int D, float eps, hipStream_t st) {
   using namespace pa::hn;
   if (n <= 0) return 0;
   if (D <= 0 || D * 4 > 96 * 1024 || S < 1 || S > MAX_S) return -1;
-  const Args A{x, y, y_w, bias, mix, post, pre, emb, ids, w_next, out, rows, K, ldy, vocab, ldo, D, eps};
-  const bool vec = D % 4 == 0 && (!y || ldy % 4 == 0) && (!out || ldo % 4 == 0);
+  const Args A{x, y, y_w, y2, bias, mix, post, pre, emb, ids, w_next, out, rows, K, ldy, ldy2, vocab, ldo, D, eps};
+  const bool vec = D % 4 == 0 && (!y || ldy % 4 == 0) && (!y2 || ldy2 % 4 == 0) && (!out || ldo % 4 == 0);
 #define PA_HN(T, V, N)                                                                                          \
   do {                                                                                                          \
     static bool attr = false;                                                                                   \

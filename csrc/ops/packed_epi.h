@@ -6,6 +6,7 @@
 //   EP_PLAIN     y = acc
 //   EP_SILU      y = silu(gate) * up over the interleaved (gate t, up t) packed tiles
 //   EP_GLU       y = gated unit over the same pairs (limit, alpha, cubic, bias; gated_unit below)
+//   EP_RELU2     y = max(acc, 0)^2
 //   EP_RESID     y = resid + acc, returning sum(y^2) of the written bf16 values (the next
 //                RMSNorm's row statistics, accumulated by the caller)
 //   EP_ROPEPERM  y = acc in the natural QKV column order (rope-permuted packed tiles)
@@ -20,7 +21,7 @@
 namespace pa {
 namespace pk {
 
-enum { EP_PLAIN = 0, EP_SILU = 1, EP_RESID = 2, EP_ROPEPERM = 3, EP_ROPEKV = 4, EP_GLU = 5 };
+enum { EP_PLAIN = 0, EP_SILU = 1, EP_RESID = 2, EP_ROPEPERM = 3, EP_ROPEKV = 4, EP_GLU = 5, EP_RELU2 = 6 };
 
 template <int EPI>
 constexpr bool pair_epi() { return EPI == EP_SILU || EPI == EP_ROPEKV || EPI == EP_GLU; }
@@ -32,6 +33,11 @@ __device__ __forceinline__ float gated_unit(float g, float u, float limit, float
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
   return g / (1.f + __expf(-alpha * (g + cubic * g * g * g))) * (u + bias);
+}
+
+__device__ __forceinline__ float relu2(float x) {
+  x = fmaxf(x, 0.f);
+  return x * x;
 }
 
 // packed rope-QKV tile -> first column of its original tile
@@ -101,6 +107,10 @@ __device__ __forceinline__ float store_quad(const AT& A, int m, int tile, int cq
 #pragma unroll
       for (int r = 0; r < 4; ++r) v[r] += (float)rv[r];
     }
+    if constexpr (EPI == EP_RELU2) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) v[r] = relu2(v[r]);
+    }
     bf16x4 o;
     float sq = 0.f;
 #pragma unroll
@@ -136,6 +146,10 @@ __device__ __forceinline__ float store_pair_wide(const AT& A, int m, int tile, i
     const bf16x8 rv = *reinterpret_cast<const bf16x8*>(A.resid + (size_t)m * A.ldr + col);
 #pragma unroll
     for (int r = 0; r < 8; ++r) v[r] += (float)rv[r];
+  }
+  if constexpr (EPI == EP_RELU2) {
+#pragma unroll
+    for (int r = 0; r < 8; ++r) v[r] = relu2(v[r]);
   }
   bf16x8 o;
   float sq = 0.f;

@@ -1,9 +1,11 @@
 // From a [q | k | v] projection row to the attention kernel's operands (window_attention.hip), in one
-// launch: biases, the rotation of the first rd dimensions of every query and key head, queries to
-// q_out, keys and values to their pages, and, where a token ends a block of `pool` tokens, the block's
-// mean key and value.
+// launch: biases, RMS norms of heads, the rotation of the first rd dimensions of every query and key head (rd 0:
+// none), queries to q_out, keys and values to their pages, and, where a token ends a block of `pool` tokens, the
+// block's mean key and value.
 //
-//   x [T, ldx]    H x DK queries | G x DK keys | G x DV values, bias likewise
+//   x [T, ldx]    H x DK queries | G x DK keys | GV x DV values, bias likewise; the values may lie elsewhere in the
+//                 row (at vcol), for instance on the keys: a value head is then a key head as projected
+//   norms         per query and key head with a weight, per value head without one, over the real dimensions
 //   pages         [pages, G, D/8, 16, 8]; pooled rows [pages, npb, G, D] with the page of the block's
 //                 last token, blocks that end in one page in order
 //
@@ -23,8 +25,11 @@ struct Args {
   void *q, *kp, *vp, *pk, *pv;
   const int *positions, *slots, *q_start, *q_len, *ctx_len, *block_table;
   const float* cos_sin;  // [max_pos, rd]: cos | sin
-  int ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs, T;
+  const float *qn, *kn;  // norm weights [DK]; null: no norm of queries and keys
+  int ldx, H, G, GV, DK, DV, rd, pool, npb, max_blocks, max_seqs, T;
+  int vcol, norm_v;
   float ick, icv;  // 8 / DK, 8 / DV
+  float idim, ivdim, eps;  // 1 / real dimensions
 };
 
 // u / n for the small numbers of here, with inv = 1 / n
@@ -50,9 +55,11 @@ __device__ __forceinline__ int seq_of(const Args& A, int t, int* shared) {
   return *shared;
 }
 
-// 8 values of head part `off` (columns off .. off + D of a row) from dimension d, rotated by cs if `rot`
-template <typename T>
-__device__ __forceinline__ void chunk(const Args& A, const T* row, int off, int d, const float* cs, bool rot, float (&v)[8]) {
+// 8 values of head part `off` (columns off .. off + D of a row) from dimension d: biased, times inv * w (NORM), rotated
+// by cs if `rot`
+template <typename T, bool NORM>
+__device__ __forceinline__ void chunk(const Args& A, const T* row, int off, int d, const float* cs, bool rot, float (&v)[8],
+                                      float inv = 1.f, const float* w = nullptr) {
   const int half = A.rd >> 1;
   T a[8];
   __builtin_memcpy(a, __builtin_assume_aligned(row + off + d, sizeof(T) * 8), sizeof(T) * 8);
@@ -63,6 +70,11 @@ __device__ __forceinline__ void chunk(const Args& A, const T* row, int off, int 
     load8(A.bias + off + d, b);
 #pragma unroll
     for (int j = 0; j < 8; ++j) v[j] += b[j];
+  }
+  if constexpr (NORM) {
+    if (w) load8(w + d, b);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] *= w ? inv * b[j] : inv;
   }
   if (!rot || d >= A.rd) return;
   if (half % 8 == 0) {
@@ -78,6 +90,11 @@ __device__ __forceinline__ void chunk(const Args& A, const T* row, int off, int 
 #pragma unroll
       for (int j = 0; j < 8; ++j) u[j] += b[j];
     }
+    if constexpr (NORM) {
+      if (w) load8(w + pd, b);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) u[j] *= w ? inv * b[j] : inv;
+    }
     const float sign = d < half ? -1.f : 1.f;
 #pragma unroll
     for (int j = 0; j < 8; ++j) v[j] = v[j] * c[j] + sign * u[j] * s[j];
@@ -88,7 +105,8 @@ __device__ __forceinline__ void chunk(const Args& A, const T* row, int off, int 
     const int e = d + j;
     if (e >= A.rd) break;
     const int pd = e < half ? e + half : e - half, i = e < half ? e : e - half;
-    const float u = (float)row[off + pd] + (A.bias ? A.bias[off + pd] : 0.f);
+    float u = (float)row[off + pd] + (A.bias ? A.bias[off + pd] : 0.f);
+    if constexpr (NORM) u *= w ? inv * w[pd] : inv;
     v[j] = e < half ? v[j] * cs[i] - u * cs[half + i] : v[j] * cs[i] + u * cs[half + i];
   }
 }
@@ -110,19 +128,19 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
   if (slot < 0) return;
   const T* row = (const T*)A.x + (size_t)t * A.ldx;
   const float* cs = A.cos_sin + (size_t)pos * A.rd;
-  const int ck = A.DK >> 3, cv = A.DV >> 3, nq = A.H * ck, nk = A.G * ck, nv = A.G * cv;
+  const int ck = A.DK >> 3, cv = A.DV >> 3, nq = A.H * ck, nk = A.G * ck, nv = A.GV * cv;
   for (int u = threadIdx.x; u < nq + nk + nv; u += 256) {
     float v[8];
     if (u < nq) {
       const int h = quot(u, A.ick), d = (u - h * ck) * 8;
-      chunk(A, row, h * A.DK, d, cs, true, v);
+      chunk<T, false>(A, row, h * A.DK, d, cs, true, v);
       put((T*)A.q + ((size_t)t * A.H + h) * A.DK + d, v);
     } else {
       const bool key = u < nq + nk;
       const int w = key ? u - nq : u - nq - nk, per = key ? ck : cv, D = key ? A.DK : A.DV;
       const int h = quot(w, key ? A.ick : A.icv), o = w - h * per;
-      chunk(A, row, (key ? A.H * A.DK : (A.H + A.G) * A.DK) + h * D, o * 8, cs, key, v);
-      put((T*)(key ? A.kp : A.vp) + (((size_t)(slot >> 4) * A.G + h) * per + o) * 128 + (slot & 15) * 8, v);
+      chunk<T, false>(A, row, (key ? A.H * A.DK : A.vcol) + h * D, o * 8, cs, key, v);
+      put((T*)(key ? A.kp : A.vp) + (((size_t)(slot >> 4) * (key ? A.G : A.GV) + h) * per + o) * 128 + (slot & 15) * 8, v);
     }
   }
   if constexpr (!POOL) return;
@@ -137,7 +155,7 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
   for (int u = threadIdx.x; u < nk + nv; u += 256) {
     const bool key = u < nk;
     const int w = key ? u : u - nk, per = key ? ck : cv, D = key ? A.DK : A.DV;
-    const int h = w / per, o = w - h * per, off = (key ? A.H * A.DK : (A.H + A.G) * A.DK) + h * D;
+    const int h = w / per, o = w - h * per, off = (key ? A.H * A.DK : A.vcol) + h * D;
     float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
     for (int p = pos - P + 1; p <= pos; ++p) {
@@ -149,7 +167,7 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
         for (int j = 0; j < 8; ++j) sum[j] += (float)a[j];
       } else {
         float v[8];
-        chunk(A, row - (size_t)(pos - p) * A.ldx, off, o * 8, A.cos_sin + (size_t)p * A.rd, key, v);
+        chunk<T, false>(A, row - (size_t)(pos - p) * A.ldx, off, o * 8, A.cos_sin + (size_t)p * A.rd, key, v);
 #pragma unroll
         for (int j = 0; j < 8; ++j) sum[j] += (float)(T)v[j];
       }
@@ -157,6 +175,49 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
 #pragma unroll
     for (int j = 0; j < 8; ++j) sum[j] *= inv;
     put((T*)(key ? A.pk : A.pv) + (((size_t)(slot >> 4) * A.npb + sub) * A.G + h) * D + o * 8, sum);
+  }
+}
+
+// With norms: a power of two of lanes per head, which sum its squares. Sections (queries and keys, then values) begin
+// at whole waves.
+template <typename T>
+__global__ __launch_bounds__(256) void normed_kv_kernel(const Args A) {
+  const int t = token_of(blockIdx.x, A.T);
+  if (t < 0) return;
+  const int slot = A.slots[t], pos = A.positions[t];
+  if (slot < 0) return;
+  const T* row = (const T*)A.x + (size_t)t * A.ldx;
+  const float* cs = A.cos_sin + (size_t)pos * A.rd;
+  const int ck = A.DK >> 3, cv = A.DV >> 3;
+  const int bk = 32 - __clz(ck - 1), bv = 32 - __clz(cv - 1);  // log2 of the lanes of a head (clz(0) is 32)
+  const int nqk = (((A.H + A.G) << bk) + 63) & ~63, total = nqk + (A.GV << bv);
+  for (int u0 = 0; u0 < total; u0 += 256) {
+    const int u = u0 + threadIdx.x;
+    const bool value = u >= nqk;
+    const int w = value ? u - nqk : u, bits = value ? bv : bk, per = value ? cv : ck;
+    const int h = w >> bits, o = w & ((1 << bits) - 1);  // (query heads, then key heads)
+    const bool in = o < per && h < (value ? A.GV : A.H + A.G), query = !value && h < A.H;
+    const int off = value ? A.vcol + h * A.DV : h * A.DK;
+    const float* nw = value ? nullptr : query ? A.qn : A.kn;
+    float inv = 1.f, v[8];
+    if (value ? A.norm_v != 0 : nw != nullptr) {
+      float ss = 0.f;
+      if (in) {
+        chunk<T, false>(A, row, off, o * 8, cs, false, v);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ss = fmaf(v[j], v[j], ss);
+      }
+      for (int m = (1 << bits) >> 1; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+      inv = 1.f / sqrtf(ss * (value ? A.ivdim : A.idim) + A.eps);
+    }
+    if (!in) continue;
+    chunk<T, true>(A, row, off, o * 8, cs, !value, v, inv, nw);
+    if (query) {
+      put((T*)A.q + ((size_t)t * A.H + h) * A.DK + o * 8, v);
+    } else {
+      const int g = value ? h : h - A.H;
+      put((T*)(value ? A.vp : A.kp) + (((size_t)(slot >> 4) * (value ? A.GV : A.G) + g) * per + o) * 128 + (slot & 15) * 8, v);
+    }
   }
 }
 
@@ -198,14 +259,22 @@ __global__ __launch_bounds__(256) void pool_kernel(const Args A, int rows) {
 
 extern "C" int pa_paged_kv(int fp32, const void* x, const float* bias, void* q, void* kp, void* vp, void* pk, void* pv,
                            const int* positions, const int* slots, const int* q_start, const int* q_len,
-                           const int* ctx_len, const int* block_table, const float* cos_sin, int ldx, int H, int G,
-                           int DK, int DV, int rd, int pool, int npb, int max_blocks, int max_seqs, int T,
-                           hipStream_t st) {
+                           const int* ctx_len, const int* block_table, const float* cos_sin, int ldx, int H, int G, int GV,
+                           int DK, int DV, int rd, int pool, int npb, int max_blocks, int max_seqs, int T, int vcol,
+                           const float* qn, const float* kn, int norm_v, int dim, int vdim, float eps, hipStream_t st) {
   if (T <= 0) return 0;
-  if (DK % 8 || DV % 8 || rd % 2 || rd > DK || ldx % 8) return -1;
-  const pa::kv::Args A{x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_len, block_table, cos_sin,
-                       ldx, H, G, DK, DV, rd, pool, npb, max_blocks, max_seqs, T, 8.f / DK, 8.f / DV};
+  const bool normed = qn || kn || norm_v;
+  if (DK % 8 || DV % 8 || rd % 2 || rd > DK || ldx % 8 || vcol % 8 || (pool > 0 && (normed || G != GV))) return -1;
+  if (normed && (DK > 512 || DV > 512 || dim <= 0 || vdim <= 0)) return -2;  // a head in a wave
+  const pa::kv::Args A{x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_len, block_table, cos_sin, qn, kn,
+                       ldx, H, G, GV, DK, DV, rd, pool, npb, max_blocks, max_seqs, T, vcol, norm_v, 8.f / DK, 8.f / DV,
+                       normed ? 1.f / dim : 0.f, normed ? 1.f / vdim : 0.f, eps};
   const dim3 grid((T + 7) / 8 * 8);
+  if (normed) {
+    if (fp32) hipLaunchKernelGGL(pa::kv::normed_kv_kernel<float>, grid, dim3(256), 0, st, A);
+    else hipLaunchKernelGGL(pa::kv::normed_kv_kernel<pa::bf16>, grid, dim3(256), 0, st, A);
+    return (int)hipGetLastError();
+  }
   const bool later = pool > 0 && T > 64, now = pool > 0 && !later;
   const int rows = pool < 8 ? pool : 8;  // of a workgroup of the second launch
 #define PA_KV(TYPE)                                                                                              \

@@ -1,9 +1,11 @@
 // Routing by score: which experts a token uses, with what weights, and the rows of all tokens sorted
 // by expert for the grouped projections (grouped_gemm.hip).
 //
-//   z = W_router h (fp32 sums; h and W in T),  s = sigmoid(z)
-//   group's score = the sum of its two largest s; the `keep` best of `groups` equal groups of neighbours stay
-//   the `top` experts with the largest s among them are chosen, with weights s
+//   z = W_router h (fp32 sums; h and W in T),  s = sigmoid(z), or softmax(z) over all experts
+//   c = s + correction (if there is one)
+//   group's score = the sum of its two largest c; the `keep` best of `groups` equal groups of neighbours stay
+//   the `top` experts with the largest c among them are chosen, with weights scale * s, or with `share`
+//   scale * s / (sum of the chosen s + 1e-20)
 //   `always` more experts (numbers E .. E + always - 1) follow for every token, with weight 1
 //
 // Ties go to the lower number. One workgroup scores 16 tokens. Steps of at most 16 tokens sort in the
@@ -30,8 +32,17 @@ struct Args {
   int* order;         // position -> token * (top + always) + k
   int4* tiles;        // {expert, first position, rows, 0}
   int* n_tiles;
+  const float* correction;  // [E] or null
   int T, ldh, K, E, top, groups, keep, always, tm, max_tiles;
+  int softmax, share;
+  float scale;
 };
+
+// floats and integers in the same order, with room at both ends whatever the bits are
+__device__ __forceinline__ int ordered(float v) {
+  const int i = __float_as_int(v);
+  return min(max(i ^ ((i >> 31) & 0x7fffffff), INT_MIN + 2), INT_MAX - 1);
+}
 
 // Exclusive sums of cnt over experts into base (rows) and tbase (tiles of tm rows); returns the tiles.
 // All NT threads call it; cnt, base, tbase are in LDS.
@@ -76,8 +87,9 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
   const int Ep = (A.E + 15) / 16 * 16, EA = A.E + A.always;
   float* sc = sm;                       // [TOK][Ep] scores
   float* gs = sc + TOK * Ep;            // [TOK][groups]
-  float* red = gs + TOK * A.groups;     // bf16: [8][16][64 + 4]
-  int* cnt = (int*)(red + 8 * 16 * 68); // [EA], then base, tbase
+  float* sel = gs + TOK * A.groups;     // [TOK][top] scores of the chosen
+  float* red = sel + TOK * A.top;       // bf16: [8][16][64 + 4]; then [TOK][Ep], what the choice goes by
+  int* cnt = (int*)(red + max(8 * 16 * 68, TOK * Ep)); // [EA], then base, tbase
   int *base = cnt + EA, *tbase = base + EA;
   __shared__ int ws[2][NT / 64];
   const int t0 = blockIdx.x * TOK, lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
@@ -109,7 +121,7 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
         float z = 0.f;
 #pragma unroll
         for (int w = 0; w < 8; ++w) z += red[(w * 16 + t) * 68 + e];
-        if (e0 * 16 + e < Ep) sc[t * Ep + e0 * 16 + e] = 1.f / (1.f + expf(-z));
+        if (e0 * 16 + e < Ep) sc[t * Ep + e0 * 16 + e] = A.softmax ? z : 1.f / (1.f + expf(-z));
       }
     }
   } else {
@@ -120,32 +132,55 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
       for (int k = 0; k < A.K; k += 4)
 #pragma unroll
         for (int j = 0; j < 4; ++j) z[j] = fmaf(x[k + j], w[k + j], z[j]);
-      sc[t * Ep + e] = 1.f / (1.f + expf(-((z[0] + z[1]) + (z[2] + z[3]))));
+      const float v = (z[0] + z[1]) + (z[2] + z[3]);
+      sc[t * Ep + e] = A.softmax ? v : 1.f / (1.f + expf(-v));
     }
   }
   __syncthreads();
   // 32 lanes per token. Nothing is chosen one after the other: a group, or an expert, is in when fewer than
   // `keep`, or `top`, others come before it (larger, or equal and lower), and that number is its place.
-  // The scores are compared as integers: non-negative floats in the same order, and no two alike in rank
-  // whatever the bits are.
+  // Scores are compared as integers in the floats' order, and no two are alike in rank whatever the bits are.
   const int tk = threadIdx.x >> 5, l = threadIdx.x & 31, t = t0 + tk, KA = A.top + A.always;
   const bool live = t < A.T && A.slots[min(t, A.T - 1)] >= 0;
-  float *s = sc + tk * Ep, *gr = gs + tk * A.groups;
-  int *si = (int*)s, *gi = (int*)gr;
-  constexpr int OUT = -1, PAD = INT_MIN;
+  float *s = sc + tk * Ep, *gr = gs + tk * A.groups, *se = sel + tk * A.top;
+  float* cf = red + tk * Ep;
+  int *si = (int*)cf, *gi = (int*)gr;
+  constexpr int OUT = INT_MIN + 1, PAD = INT_MIN;
+  if (A.softmax) {
+    float m = -INFINITY, sum = 0.f;
+    for (int e = l; e < A.E; e += 32) m = fmaxf(m, s[e]);
+#pragma unroll
+    for (int o = 16; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o, 64));
+    for (int e = l; e < A.E; e += 32) {
+      const float p = expf(s[e] - m);
+      s[e] = p;
+      sum += p;
+    }
+#pragma unroll
+    for (int o = 16; o > 0; o >>= 1) sum += __shfl_xor(sum, o, 64);
+    const float inv = 1.f / sum;
+    for (int e = l; e < A.E; e += 32) s[e] *= inv;
+  }
+  for (int e = l; e < A.E; e += 32) cf[e] = A.correction ? s[e] + A.correction[e] : s[e];
+  __syncthreads();
   if (A.keep < A.groups) {
     const int per = A.E / A.groups;
     for (int i = l; i < A.groups; i += 32) {
-      float a = -1.f, b = -1.f;
+      float a = -INFINITY, b = -INFINITY;
 #pragma unroll 4
       for (int e = i * per; e < (i + 1) * per; ++e) {
-        const float v = s[e];
+        const float v = cf[e];
         b = fmaxf(b, fminf(a, v));
         a = fmaxf(a, v);
       }
-      gr[i] = a + (per > 1 ? b : 0.f);
+      gi[i] = ordered(a + (per > 1 ? b : 0.f));
     }
     __syncthreads();
+  }
+  for (int e = l; e < Ep; e += 32) si[e] = e < A.E ? ordered(cf[e]) : PAD;
+  __syncthreads();
+  if (A.keep < A.groups) {
+    const int per = A.E / A.groups;
     for (int i = l; i < A.groups; i += 32) {
       int before = 0;
       const int v = gi[i];
@@ -156,8 +191,7 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
     }
     __syncthreads();
   }
-  for (int e = A.E + l; e < Ep; e += 32) si[e] = PAD;
-  __syncthreads();
+  float chosen = 0.f;
   for (int e0 = l; e0 < A.E; e0 += 64) {  // two experts a lane
     const int ea = e0, eb = min(e0 + 32, Ep - 1), va = si[ea], vb = si[eb];
     int na = 0, nb = 0;
@@ -166,22 +200,30 @@ __global__ __launch_bounds__(NT) void score_kernel(const Args A) {
       const int4 q = *reinterpret_cast<const int4*>(si + k);
       const int w[4] = {q.x, q.y, q.z, q.w};
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {  // (v - 1: an equal score with a lower number comes first; v > INT_MIN)
-        na += w[j] > (k + j < ea ? va - 1 : va);
-        nb += w[j] > (k + j < eb ? vb - 1 : vb);
+      for (int j = 0; j < 4; ++j) {  // an equal score with a lower number comes first
+        na += w[j] >= va + (k + j >= ea);
+        nb += w[j] >= vb + (k + j >= eb);
       }
     }
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
       const int e = i ? e0 + 32 : e0, before = i ? nb : na;
-      if (e < A.E && before < A.top && t < A.T) {
-        const size_t p = (size_t)t * KA + before;
-        A.choice[p] = live ? e : -1;
-        A.weights[p] = live ? s[e] : 0.f;
-        if (live) A.rank[p] = atomicAdd(&cnt[e], 1);
+      if (e < A.E && before < A.top && live) {
+        A.choice[(size_t)t * KA + before] = e;
+        se[before] = s[e];
+        chosen += s[e];
+        A.rank[(size_t)t * KA + before] = atomicAdd(&cnt[e], 1);
       }
     }
   }
+  if (t < A.T && !live)  // (a row of padding holds anything)
+    for (int i = l; i < A.top; i += 32) A.choice[(size_t)t * KA + i] = -1;
+#pragma unroll
+  for (int o = 16; o > 0; o >>= 1) chosen += __shfl_xor(chosen, o, 64);
+  const float f = A.share ? A.scale / (chosen + 1e-20f) : A.scale;
+  __syncthreads();
+  if (t < A.T)
+    for (int i = l; i < A.top; i += 32) A.weights[(size_t)t * KA + i] = live ? se[i] * f : 0.f;
   if (l < A.always && t < A.T) {
     const size_t p = (size_t)t * KA + A.top + l;
     A.choice[p] = live ? A.E + l : -1;
@@ -227,14 +269,15 @@ __global__ __launch_bounds__(NT) void place_kernel(const Args A) {
 
 extern "C" int pa_score_route(int fp32, const void* h, int ldh, const void* w, int K, const int* slots, float* weights,
                               int* choice, int* rank, int* counts, int* order, int* tiles, int* n_tiles, int T, int E,
-                              int top, int groups, int keep, int always, int tm, int max_tiles, hipStream_t st) {
+                              int top, int groups, int keep, int always, int tm, int max_tiles, int softmax,
+                              const float* correction, int share, float scale, hipStream_t st) {
   using namespace pa::sr;
   if (T <= 0) return 0;
   if (E < 1 || E + always > MAX_E || always > 32 || groups < 1 || E % groups || keep < 1 || keep > groups || top < 1 ||
       top > keep * (E / groups) || K % 32 || ldh % 8) return -1;
-  const Args A{h, w, slots, weights, choice, rank, counts, order, (int4*)tiles, n_tiles, T, ldh, K, E, top, groups, keep,
-               always, tm, max_tiles};
-  const int Ep = (E + 15) / 16 * 16, lds = (TOK * (Ep + groups) + 3 * (E + always) + 8 * 16 * 68 + 64) * 4;
+  const Args A{h, w, slots, weights, choice, rank, counts, order, (int4*)tiles, n_tiles, correction, T, ldh, K, E, top, groups,
+               keep, always, tm, max_tiles, softmax, share, scale};
+  const int Ep = (E + 15) / 16 * 16, lds = (TOK * (Ep + groups + top) + 3 * (E + always) + std::max(8 * 16 * 68, TOK * Ep) + 64) * 4;
   static bool attr = false;
   if (!attr) {
     (void)hipFuncSetAttribute((const void*)score_kernel<float>, hipFuncAttributeMaxDynamicSharedMemorySize, 159 * 1024);

@@ -554,11 +554,13 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(const Args A) {
 }
 
 // ---- y * silu(z), normed in equal parts of the unpadded columns, times w ------------------------------
-// in place: y's columns h * Vp + v (v < V); one workgroup per token
+// in place: y's columns h * Vp + v (v < V) of `cols`; one workgroup per token. With div [T, H] a head is divided by it
+// first; with `after` the gate is sigmoid(z) behind the norm and its weight.
 template <typename T>
-__global__ __launch_bounds__(256) void gated_norm_kernel(T* __restrict__ y, int ldy, const T* __restrict__ z, int ldz,
+__global__ __launch_bounds__(256) void gated_norm_kernel(T* __restrict__ y, int ldy, int cols, const T* __restrict__ z, int ldz,
                                                          const float* __restrict__ w, const int* __restrict__ slots,
-                                                         int H, int V, int Vp, int parts, float eps) {
+                                                         const float* __restrict__ div, int after, int H, int V, int Vp,
+                                                         int parts, float eps) {
   extern __shared__ __attribute__((aligned(16))) float row[];
   __shared__ float red[4];
   const int t = blockIdx.x, inner = H * V, len = inner / parts;
@@ -567,16 +569,22 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(T* __restrict__ y, int 
   const T* zr = z + (size_t)t * ldz;
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
   auto col = [&](int i) { return V == Vp ? i : i / V * Vp + i % V; };
+  // what the norm is taken of: the gate ahead of it and the division
+  auto lead = [&](int i, float v, float g) {
+    if (!after) v *= silu(g);
+    return div ? v / div[(size_t)t * H + i / V] : v;
+  };
+  auto gate = [&](float g) { return after ? 1.f / (1.f + __expf(-g)) : 1.f; };
   if (V == Vp) {
     for (int i = threadIdx.x * 8; i < inner; i += 2048) {
       T a[8], b[8];
       __builtin_memcpy(a, __builtin_assume_aligned(yr + i, sizeof(T) * 8), sizeof(T) * 8);
       __builtin_memcpy(b, __builtin_assume_aligned(zr + i, sizeof(T) * 8), sizeof(T) * 8);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) row[i + j] = (float)a[j] * silu((float)b[j]);
+      for (int j = 0; j < 8; ++j) row[i + j] = lead(i + j, (float)a[j], (float)b[j]);
     }
   } else {
-    for (int i = threadIdx.x; i < inner; i += 256) row[i] = (float)yr[col(i)] * silu((float)zr[col(i)]);
+    for (int i = threadIdx.x; i < inner; i += 256) row[i] = lead(i, (float)yr[col(i)], (float)zr[col(i)]);
   }
   __syncthreads();
   float* inv = row + inner;  // [parts]
@@ -599,18 +607,19 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(T* __restrict__ y, int 
   if (V == Vp && len % 8 == 0) {
     for (int i = threadIdx.x * 8; i < inner; i += 2048) {
       const float f = inv[i / len];
-      T a[8];
+      T a[8], b[8];
+      if (after) __builtin_memcpy(b, __builtin_assume_aligned(zr + i, sizeof(T) * 8), sizeof(T) * 8);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) a[j] = (T)(row[i + j] * f * w[i + j]);
+      for (int j = 0; j < 8; ++j) a[j] = (T)(row[i + j] * f * w[i + j] * gate(after ? (float)b[j] : 0.f));
       __builtin_memcpy(__builtin_assume_aligned(yr + i, sizeof(T) * 8), a, sizeof(T) * 8);
     }
   } else {
-    for (int i = threadIdx.x; i < inner; i += 256) yr[col(i)] = (T)(row[i] * inv[i / len] * w[i]);
+    for (int i = threadIdx.x; i < inner; i += 256) yr[col(i)] = (T)(row[i] * inv[i / len] * w[i] * gate(after ? (float)zr[col(i)] : 0.f));
     // padded columns meet zero weights, but must be finite
     if (V != Vp)
       for (int i = threadIdx.x; i < H * (Vp - V); i += 256) yr[i / (Vp - V) * Vp + V + i % (Vp - V)] = (T)0.f;
   }
-  for (int i = H * Vp + threadIdx.x; i < ldy; i += 256) yr[i] = (T)0.f;
+  for (int i = H * Vp + threadIdx.x; i < cols; i += 256) yr[i] = (T)0.f;
 }
 
 }  // namespace ss
@@ -695,8 +704,9 @@ extern "C" int pa_state_scan(int fp32, const void* proj, int ldp, void* u, void*
   return (int)hipGetLastError();
 }
 
-extern "C" int pa_gated_norm(int fp32, void* y, int ldy, const void* z, int ldz, const float* w, const int* slots, int T,
-                             int H, int V, int Vp, int parts, float eps, hipStream_t st) {
+extern "C" int pa_gated_norm(int fp32, void* y, int ldy, int cols, const void* z, int ldz, const float* w, const int* slots,
+                             const float* div, int after, int T, int H, int V, int Vp, int parts, float eps,
+                             hipStream_t st) {
   if (T <= 0) return 0;
   if (H * V % parts || Vp % 8 || ldy % 8 || ldz % 8) return -1;
   const int lds = (H * V + parts) * 4;
@@ -707,7 +717,7 @@ extern "C" int pa_gated_norm(int fp32, void* y, int ldy, const void* z, int ldz,
     (void)hipFuncSetAttribute((const void*)pa::ss::gated_norm_kernel<pa::bf16>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 64);
     attr = true;
   }
-  if (fp32) hipLaunchKernelGGL(pa::ss::gated_norm_kernel<float>, dim3(T), dim3(256), lds, st, (float*)y, ldy, (const float*)z, ldz, w, slots, H, V, Vp, parts, eps);
-  else hipLaunchKernelGGL(pa::ss::gated_norm_kernel<pa::bf16>, dim3(T), dim3(256), lds, st, (pa::bf16*)y, ldy, (const pa::bf16*)z, ldz, w, slots, H, V, Vp, parts, eps);
+  if (fp32) hipLaunchKernelGGL(pa::ss::gated_norm_kernel<float>, dim3(T), dim3(256), lds, st, (float*)y, ldy, cols, (const float*)z, ldz, w, slots, div, after, H, V, Vp, parts, eps);
+  else hipLaunchKernelGGL(pa::ss::gated_norm_kernel<pa::bf16>, dim3(T), dim3(256), lds, st, (pa::bf16*)y, ldy, cols, (const pa::bf16*)z, ldz, w, slots, div, after, H, V, Vp, parts, eps);
   return (int)hipGetLastError();
 }

@@ -1,12 +1,15 @@
-// Paged grouped-query attention with a sliding window, pooled keys before the window and a sink in
-// the softmax's denominator, for prefill chunks, decode rows and mixed batches in one launch.
+// Paged grouped-query attention with a sliding window or chunks, kept first tokens, pooled keys before the window,
+// capped scores, a bias by distance, a sink in the softmax's denominator and an output gate, for prefill chunks,
+// decode rows and mixed batches in one launch.
 //
-//   position i sees   keys j with 0 <= i - j < W (W 0: every j <= i), and, with P > 0,
+//   position i sees   keys j <= i with i - j < W or j < keep (W 0: every j <= i), or those of its chunk of C
+//                     positions (C > 0: j >= i - i % C), and, with P > 0,
 //                     block b (the mean key and value of positions bP .. bP + P - 1) if
 //                     bP + P - 1 <= i - W, that is b < (i - W + 1) / P
-//   out = sum p v,    p = exp(s) / (sink + sum exp(s)),  sink 0 or 1, one softmax over both kinds
+//   s = cap tanh(q . k scale / cap) - slope_h (i - j)         (cap 0: no cap; no slopes: no bias)
+//   out = gain sigmoid(gate) sum p v,   p = exp(s) / (exp(sink_h) + sum exp(s)), one softmax over all kinds
 //
-// Keys and values are fragment-major pages of 16 tokens per KV head, [D/8][16][8] (paged_kv.hip); the
+// R = H / G query heads share a key head, G / GV key heads a value head (differential attention: 2). Keys and values are fragment-major pages of 16 tokens per KV head, [D/8][16][8] (paged_kv.hip); the
 // value operand of the second product comes from the same form by LDS transpose reads. A pooled
 // block's row lies with the page of its last token: [page][per page][KV head][D]. 16 of them, gathered
 // row by row, make a tile of the same form as a page, so both kinds of keys run the same code:
@@ -14,7 +17,8 @@
 //   S^T[keys x cols] = K . Q^T         cols = (token, query head of the KV head's group) pairs
 //   O^T[dims x cols] += V^T . P^T      P^T = the S^T accumulator's own registers
 //
-// An item's keys are its pooled blocks (a tile at a time) and then the tiles of its window. Items
+// An item's keys are its pooled blocks (a tile at a time), the tiles of the kept tokens that lie before its window's,
+// and then the tiles of its window or chunk. Items
 // come from the scheduler like paged_attention's (seq, q_begin, nq | part<<8 | nparts<<20, partial slot):
 //   nq <= dec_tokens: split over keys. The 8 waves take every 8th page with a private LDS tile and merge;
 //                     nparts > 1 divides the item's own key range, merge_kernel combines the partitions.
@@ -35,7 +39,7 @@ typedef __attribute__((address_space(3))) void lds_void;
 typedef const __attribute__((address_space(1))) void glb_void;
 
 struct Args {
-  void* out;             // [T, H, DV]
+  void* out;             // [T, ldo]: H x DV
   float* part_o;         // [G, slots, NB, 16, DV]
   float* part_ml;        // [G, slots, NB, 16, 2]
   const void* q;         // [T, H, DK]
@@ -45,10 +49,20 @@ struct Args {
   const int* n_items;
   const int *q_start, *q_len, *ctx_len, *block_table;
   int max_blocks, max_items, H, G, R, NB, DK, DV, dec_tokens, window, pool, npb;
-  float scale_log2, sink;
+  float scale_log2;
+  const float *sink, *slopes;  // [H] or null: log of the sink, bias per token of distance
+  const void* gate;            // [T, ldg]: H x DV, or null
+  float scale, cap, gain;
+  int GV, keep, chunk, ldo, ldg, out_f32;
 };
 
-__device__ __forceinline__ int first_key(const Args& A, int pos) { return A.window > 0 ? max(0, pos - A.window + 1) : 0; }
+constexpr float LOG2E = 1.4426950408889634f;
+
+__device__ __forceinline__ int first_key(const Args& A, int pos) {
+  return A.window > 0 ? max(0, pos - A.window + 1) : A.chunk > 0 ? pos - pos % A.chunk : 0;
+}
+// tiles of `keys` kept tokens that lie before tile k_lo
+__device__ __forceinline__ int kept_tiles(const Args& A, int keys, int k_lo) { return min((A.keep + keys - 1) / keys, k_lo); }
 // pooled blocks that position pos sees
 __device__ __forceinline__ int blocks_of(const Args& A, int pos) {
   return A.pool > 0 && A.window > 0 ? max(0, pos - A.window + 1) / A.pool : 0;
@@ -59,6 +73,42 @@ __device__ __forceinline__ size_t pooled_row(const Args& A, const int* bt, int b
   return ((size_t)bt[page] * A.npb + (b - (page << 4) / A.pool)) * A.G + h;
 }
 
+// a score's cap and bias, in units of q . k, which the softmax's scale still multiplies
+struct Mods {
+  float to_tanh, from_tanh, slope;
+  __device__ __forceinline__ Mods(const Args& A, int head) {
+    to_tanh = A.cap > 0.f ? 2.f * LOG2E * A.scale / A.cap : 0.f;
+    from_tanh = A.cap / A.scale;
+    slope = A.slopes ? A.slopes[head] / A.scale : 0.f;
+  }
+  __device__ __forceinline__ float operator()(float s, int back) const {
+    if (to_tanh != 0.f) s = from_tanh * (1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s * to_tanh)));
+    return s - slope * (float)back;
+  }
+};
+
+// four outputs of head h at dimension d of a token's row, with gain and gate
+template <typename T, int N>
+__device__ __forceinline__ void put_out(const Args& A, size_t tok, int h, int d, float (&v)[N]) {
+#pragma unroll
+  for (int j = 0; j < N; ++j) v[j] *= A.gain;
+  if (A.gate) {
+    T g[N];
+    __builtin_memcpy(g, __builtin_assume_aligned((const T*)A.gate + tok * A.ldg + (size_t)h * A.DV + d, sizeof(T) * N), sizeof(T) * N);
+#pragma unroll
+    for (int j = 0; j < N; ++j) v[j] /= 1.f + __expf(-(float)g[j]);
+  }
+  const size_t at = tok * A.ldo + (size_t)h * A.DV + d;
+  if (A.out_f32) {
+    __builtin_memcpy(__builtin_assume_aligned((float*)A.out + at, 4 * N), v, 4 * N);
+  } else {
+    T o[N];
+#pragma unroll
+    for (int j = 0; j < N; ++j) o[j] = (T)v[j];
+    __builtin_memcpy(__builtin_assume_aligned((T*)A.out + at, sizeof(T) * N), o, sizeof(T) * N);
+  }
+}
+
 // ---------------------------------------------------------------------------
 // Any sizes, bf16 or fp32: one workgroup per (token of an item, head). The exact path.
 template <typename T>
@@ -67,7 +117,8 @@ __global__ __launch_bounds__(256) void simple_kernel(const Args A) {
   float* sq = sm;            // DK
   float* sp = sm + A.DK;     // 256
   float* red = sp + 256;     // 4
-  const int h = blockIdx.x, n = A.n_items[0], gk = h / A.R;
+  const int h = blockIdx.x, n = A.n_items[0], gk = h / A.R, gv = gk / (A.G / A.GV);
+  const float slope = A.slopes ? A.slopes[h] * LOG2E : 0.f, sink = A.sink ? A.sink[h] * LOG2E : NEG_BIG;
   for (int item = blockIdx.y; item < n; item += gridDim.y) {
     const int4 it = A.items[item];
     const int s = it.x, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff;
@@ -76,25 +127,28 @@ __global__ __launch_bounds__(256) void simple_kernel(const Args A) {
     const int* bt = A.block_table + (size_t)s * A.max_blocks;
     for (int i = 0; i < nq; ++i) {
       const int tok = it.y + i, pos = ctx - ql + tok;
-      const int lo = first_key(A, pos), nb = blocks_of(A, pos), total = nb + pos - lo + 1;
+      const int lo = first_key(A, pos), nb = blocks_of(A, pos), kept = min(A.keep, lo), front = nb + kept, total = front + pos - lo + 1;
       const size_t row = (size_t)(A.q_start[s] + tok) * A.H + h;
-      // element d of key (or value) kk: pooled blocks first, then the window's tokens
-      auto at = [&](const void* pages, const void* pooled, int D, int kk, int d) -> float {
-        if (kk < nb) return (float)((const T*)pooled)[pooled_row(A, bt, kk, gk) * D + d];
-        const int key = lo + kk - nb;
-        return (float)((const T*)pages)[((size_t)bt[key >> 4] * A.G + gk) * D * 16 + (size_t)(d >> 3) * 128 + (key & 15) * 8 + (d & 7)];
+      // element d of key (or value) kk: pooled blocks first, then the kept and the window's tokens
+      auto key_of = [&](int kk) { return kk < front ? kk - nb : lo + kk - front; };
+      auto at = [&](const void* pages, const void* pooled, int heads, int g, int D, int kk, int d) -> float {
+        if (kk < nb) return (float)((const T*)pooled)[pooled_row(A, bt, kk, g) * D + d];
+        const int key = key_of(kk);
+        return (float)((const T*)pages)[((size_t)bt[key >> 4] * heads + g) * D * 16 + (size_t)(d >> 3) * 128 + (key & 15) * 8 + (d & 7)];
       };
       __syncthreads();
       for (int d = threadIdx.x; d < A.DK; d += 256) sq[d] = (float)((const T*)A.q)[row * A.DK + d];
       __syncthreads();
-      float m = A.sink > 0.f ? 0.f : NEG_BIG, l = A.sink, o[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      float m = sink, l = A.sink ? 1.f : 0.f, o[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
       for (int k0 = 0; k0 < total; k0 += 256) {
         const int kk = k0 + threadIdx.x;
         float sc = NEG_BIG;
         if (kk < total) {
           float a = 0.f;
-          for (int d = 0; d < A.DK; ++d) a += sq[d] * at(A.kp, A.pk, A.DK, kk, d);
+          for (int d = 0; d < A.DK; ++d) a += sq[d] * at(A.kp, A.pk, A.G, gk, A.DK, kk, d);
           sc = a * A.scale_log2;
+          if (A.cap > 0.f) sc = A.cap * LOG2E * tanhf(a * A.scale / A.cap);
+          if (kk >= nb) sc -= slope * (float)(pos - key_of(kk));
         }
         const float wm = wave_max(sc);
         if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = wm;
@@ -111,7 +165,7 @@ __global__ __launch_bounds__(256) void simple_kernel(const Args A) {
           const int d = threadIdx.x + 256 * e;
           if (d >= A.DV) break;
           float a = o[e] * alpha;
-          for (int k = 0; k < nk; ++k) a += sp[k] * at(A.vp, A.pv, A.DV, k0 + k, d);
+          for (int k = 0; k < nk; ++k) a += sp[k] * at(A.vp, A.pv, A.GV, gv, A.DV, k0 + k, d);
           o[e] = a;
         }
         __syncthreads();
@@ -120,7 +174,8 @@ __global__ __launch_bounds__(256) void simple_kernel(const Args A) {
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const int d = threadIdx.x + 256 * e;
-        if (d < A.DV) ((T*)A.out)[row * A.DV + d] = (T)(o[e] * inv);
+        float v[1] = {o[e] * inv};
+        if (d < A.DV) put_out<T>(A, (size_t)(A.q_start[s] + tok), h, d, v);
       }
     }
   }
@@ -136,32 +191,35 @@ __device__ __forceinline__ bf16x4 tr_read(const char* p) {
 constexpr int NW = 8;          // waves per workgroup
 constexpr int MERGE_LD = 132;  // floats per merge row of 128 dims
 
-// max, sum and the factor of the unnormalised outputs once the sink has joined
-__device__ __forceinline__ float final_scale(float sink, float m, float l) {
-  if (sink <= 0.f) return 1.f / l;
-  const float t = fmaxf(m, 0.f), a = exp2f(m - t);
-  return a / (l * a + sink * exp2f(-t));
+// the factor of the unnormalised outputs once the head's sink has joined
+__device__ __forceinline__ float final_scale(const Args& A, int head, float m, float l) {
+  if (!A.sink) return 1.f / l;
+  const float s = A.sink[head] * LOG2E, t = fmaxf(m, s), a = exp2f(m - t);
+  return a / (l * a + exp2f(s - t));
 }
 
-template <int NK, int NV>
+template <int NK, int NV, bool MODS>
 __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* smem) {
   constexpr int DK = 32 * NK, DV = 32 * NV;
   const int s = it.x, qb = it.y, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff, nparts = it.z >> 20, pidx = it.w;
-  const int cb = blockIdx.x, gk = blockIdx.z, cols = nq * A.R;
+  const int cb = blockIdx.x, gk = blockIdx.z, gv = gk / (A.G / A.GV), cols = nq * A.R;
   if (cb * 16 >= cols) return;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
   const int ctx = A.ctx_len[s], ql = A.q_len[s];
   const int pos0 = ctx - ql + qb;
   auto tok_of = [&](int col) { return min(col, cols - 1) / A.R; };
-  auto row_of = [&](int col) {  // q / out row of a column
-    const int cc = min(col, cols - 1), t = cc / A.R;
-    return (size_t)(A.q_start[s] + qb + t) * A.H + gk * A.R + (cc - t * A.R);
+  auto head_of = [&](int col) {
+    const int cc = min(col, cols - 1);
+    return gk * A.R + cc - cc / A.R * A.R;
   };
+  auto row_of = [&](int col) { return (size_t)(A.q_start[s] + qb + tok_of(col)) * A.H + head_of(col); };  // q row of a column
   const int cpos = pos0 + tok_of(cb * 16 + c);  // this column's position
   const int klo = first_key(A, cpos), cnb = blocks_of(A, cpos);
-  // the item's tiles of 16: pooled blocks, then token pages; this partition's share
+  const Mods mods(A, head_of(cb * 16 + c));
+  // the item's tiles of 16: pooled blocks, then token pages (the kept ones before the window's); this partition's share
   const int last = pos0 + nq - 1, nb = blocks_of(A, last), np = (nb + 15) >> 4;
-  const int p_lo = first_key(A, pos0) >> 4, total = np + ((last + 16) >> 4) - p_lo;
+  const int p_lo = first_key(A, pos0) >> 4, nkeep = kept_tiles(A, 16, p_lo), total = np + nkeep + ((last + 16) >> 4) - p_lo;
+  auto page_of = [&](int t) { return t - np < nkeep ? t - np : p_lo + t - np - nkeep; };
   const int per = (total + nparts - 1) / nparts;
   const int t_begin = part * per, t_end = min(total, t_begin + per);
   const int* bt = A.block_table + (size_t)s * A.max_blocks;
@@ -176,8 +234,9 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
 #pragma unroll
       for (int m = 0; m < NV; ++m) vf[m] = *reinterpret_cast<const bf16x8*>(v + m * 32);
     } else {
-      const size_t page = (size_t)bt[p_lo + t - np] * A.G + gk;
-      const bf16 *k = (const bf16*)A.kp + page * (DK * 16) + lane * 8, *v = (const bf16*)A.vp + page * (DV * 16) + lane * 8;
+      const size_t page = bt[page_of(t)];
+      const bf16 *k = (const bf16*)A.kp + (page * A.G + gk) * (DK * 16) + lane * 8;
+      const bf16* v = (const bf16*)A.vp + (page * A.GV + gv) * (DV * 16) + lane * 8;
 #pragma unroll
       for (int m = 0; m < NK; ++m) kf[m] = *reinterpret_cast<const bf16x8*>(k + m * 512);
 #pragma unroll
@@ -212,8 +271,9 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
     float tmax = NEG_BIG;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int e = 4 * g + r, key = 16 * (p_lo + t - np) + e;
-      const bool ok = t < np ? 16 * t + e < cnb : (key <= cpos && key >= klo);
+      const int e = 4 * g + r, key = 16 * page_of(t) + e;
+      const bool ok = t < np ? 16 * t + e < cnb : (key <= cpos && (key >= klo || key < A.keep));
+      if (MODS) sc[r] = mods(sc[r], t < np ? 0 : cpos - key);
       sc[r] = ok ? sc[r] * A.scale_log2 : NEG_BIG;
       tmax = fmaxf(tmax, sc[r]);
     }
@@ -257,7 +317,7 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
   }
   const int ccol = threadIdx.x >> 5, d4 = (threadIdx.x & 31) * 4;
   const bool cvalid = cb * 16 + ccol < cols;
-  const size_t orow = row_of(cb * 16 + ccol), prow = (((size_t)gk * A.max_items + pidx) * A.NB + cb) * 16 + ccol;
+  const size_t prow = (((size_t)gk * A.max_items + pidx) * A.NB + cb) * 16 + ccol;
   float wgt[NW], L = 0.f, mt = NEG_BIG;
 #pragma unroll
   for (int b = 0; b < (NV + 3) / 4; ++b) {
@@ -284,11 +344,10 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
       if (nparts > 1) {
         *reinterpret_cast<f32x4*>(A.part_o + prow * DV + d0) = acc;
       } else if (cvalid) {
-        const float f = final_scale(A.sink, mt, L);
-        bf16x4 v;
-#pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = (bf16)(acc[j] * f);
-        *reinterpret_cast<bf16x4*>((bf16*)A.out + orow * DV + d0) = v;
+        const int head = head_of(cb * 16 + ccol);
+        const float f = final_scale(A, head, mt, L);
+        float v[4] = {acc[0] * f, acc[1] * f, acc[2] * f, acc[3] * f};
+        put_out<bf16>(A, (size_t)(A.q_start[s] + qb + tok_of(cb * 16 + ccol)), head, d0, v);
       }
     }
   }
@@ -331,18 +390,13 @@ __global__ __launch_bounds__(256) void merge_kernel(const Args A) {
             a[e] += wp * *reinterpret_cast<const f32x4*>(A.part_o + slot(p0 + p) * DV + min(e * 256 + lane * 4, DV - 4));
         }
       }
-      const float f = final_scale(A.sink, gm, wave_sum(L));
-      const int t = col / A.R;
-      bf16* o = (bf16*)A.out + ((size_t)(A.q_start[it.x] + it.y + t) * A.H + gk * A.R + (col - t * A.R)) * DV;
+      const int t = col / A.R, head = gk * A.R + col - t * A.R;
+      const float f = final_scale(A, head, gm, wave_sum(L));
 #pragma unroll
       for (int e = 0; e < NE; ++e) {
         const int d = e * 256 + lane * 4;
-        if (d < DV) {
-          bf16x4 v;
-#pragma unroll
-          for (int j = 0; j < 4; ++j) v[j] = (bf16)(a[e][j] * f);
-          *reinterpret_cast<bf16x4*>(o + d) = v;
-        }
+        float v[4] = {a[e][0] * f, a[e][1] * f, a[e][2] * f, a[e][3] * f};
+        if (d < DV) put_out<bf16>(A, (size_t)(A.q_start[it.x] + it.y + t), head, d, v);
       }
     }
   }
@@ -351,12 +405,12 @@ __global__ __launch_bounds__(256) void merge_kernel(const Args A) {
 template <int NK, int NV>
 constexpr int tile_parts() { return NK + NV <= 8 ? 4 : 2; }  // 16-key parts of a tile
 
-template <int NK, int NV>
+template <int NK, int NV, bool MODS>
 __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* smem) {
   constexpr int DK = 32 * NK, DV = 32 * NV, KT = tile_parts<NK, NV>(), KEYS = 16 * KT;
   constexpr int PART = (NK + NV) * 1024, TILE = KT * PART;  // a 16-key part: K, then V
   const int s = it.x, qb = it.y, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff, nparts = it.z >> 20;
-  const int cols = nq * A.R, cw = blockIdx.x * (16 * NW), gk = blockIdx.z;
+  const int cols = nq * A.R, cw = blockIdx.x * (16 * NW), gk = blockIdx.z, gv = gk / (A.G / A.GV);
   if (cw >= cols) return;
   const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, c = lane & 15;
   const int ctx = A.ctx_len[s], ql = A.q_len[s];
@@ -364,16 +418,19 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
   const int* bt = A.block_table + (size_t)s * A.max_blocks;
   const int ci = cw + wid * 16 + c, cc = min(ci, cols - 1), ct = cc / A.R;
   const int cpos = pos0 + ct, klo = first_key(A, cpos), cnb = blocks_of(A, cpos);
-  const size_t row = (size_t)(A.q_start[s] + qb + ct) * A.H + gk * A.R + (cc - ct * A.R);
+  const int head = gk * A.R + cc - ct * A.R;
+  const size_t tok = (size_t)(A.q_start[s] + qb + ct), row = tok * A.H + head;
+  const Mods mods(A, head);
   const int loff = lane * 16;
   bf16x8 qf[NK];
 #pragma unroll
   for (int m = 0; m < NK; ++m) qf[m] = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + row * DK + 32 * m + 8 * g);
-  // positions of the workgroup's columns -> its tiles: pooled blocks, then tokens
+  // positions of the workgroup's columns -> its tiles: pooled blocks, then tokens (the kept before the window's)
   const int f = pos0 + cw / A.R, e = pos0 + min(cw + 16 * NW - 1, cols - 1) / A.R;
   const int nb = blocks_of(A, e), np = (nb + KEYS - 1) / KEYS;
-  const int k_lo = first_key(A, f) / KEYS;
-  int t_lo = 0, t_hi = np + (e + KEYS) / KEYS - k_lo;
+  const int k_lo = first_key(A, f) / KEYS, nkeep = kept_tiles(A, KEYS, k_lo);
+  int t_lo = 0, t_hi = np + nkeep + (e + KEYS) / KEYS - k_lo;
+  auto tile_of = [&](int t) { return t - np < nkeep ? t - np : k_lo + t - np - nkeep; };
   if (nparts > 1) {  // this partition's tiles (possibly none)
     const int per = (t_hi + nparts - 1) / nparts;
     t_lo = part * per;
@@ -383,7 +440,7 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
   // this wave's columns: a tile whose keys all of them see needs no mask
   const int wf = pos0 + min(cw + wid * 16, cols - 1) / A.R;
   const int we = pos0 + min(cw + wid * 16 + 15, cols - 1) / A.R;
-  const int full_lo = A.window > 0 ? we - A.window + 1 : 0, full_hi = wf, full_nb = blocks_of(A, wf);
+  const int full_lo = first_key(A, we), full_hi = wf, full_nb = blocks_of(A, wf);
 
   f32x4 o[2 * NV];
 #pragma unroll
@@ -397,7 +454,7 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
       const int x = min((i * NW + wid) / (NK + NV), KT - 1);
-      pg[i] = bt[min(max(KT * (k_lo + t - np) + x, 0), nblk - 1)];
+      pg[i] = bt[min(max(KT * tile_of(t) + x, 0), nblk - 1)];
     }
   };
   auto issue = [&](int t, char* dst) {
@@ -411,8 +468,9 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
           const size_t r = pooled_row(A, bt, min(KEYS * t + 16 * x + c, nb - 1), gk);
           src = m < NK ? (const bf16*)A.pk + r * DK + 32 * m + 8 * g : (const bf16*)A.pv + r * DV + 32 * (m - NK) + 8 * g;
         } else {
-          const size_t r = (size_t)pg[i] * A.G + gk;
-          src = (m < NK ? (const bf16*)A.kp + r * (DK * 16) + m * 512 : (const bf16*)A.vp + r * (DV * 16) + (m - NK) * 512) + lane * 8;
+          const size_t r = pg[i];
+          src = (m < NK ? (const bf16*)A.kp + (r * A.G + gk) * (DK * 16) + m * 512
+                        : (const bf16*)A.vp + (r * A.GV + gv) * (DV * 16) + (m - NK) * 512) + lane * 8;
         }
         __builtin_amdgcn_global_load_lds((glb_void*)src, (lds_void*)(dst + ch * 1024), 16, 0, 0);
       }
@@ -442,14 +500,21 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
         const bf16x8 kf = *reinterpret_cast<const bf16x8*>(cur + k * PART + m * 1024 + loff);
         sc[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[m], sc[k], 0, 0, 0);
       }
-    const int key0 = KEYS * (k_lo + t - np);  // wave-uniform
-    if (t < np ? KEYS * (t + 1) > full_nb : (key0 < full_lo || key0 + KEYS - 1 > full_hi)) {
+    const int key0 = KEYS * tile_of(t);  // wave-uniform
+    if (MODS) {
+#pragma unroll
+      for (int k = 0; k < KT; ++k)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sc[k][r] = mods(sc[k][r], t < np ? 0 : cpos - (key0 + 16 * k + 4 * g + r));
+    }
+    if (t < np ? KEYS * (t + 1) > full_nb
+               : ((key0 < full_lo && key0 + KEYS > A.keep) || key0 + KEYS - 1 > full_hi)) {
 #pragma unroll
       for (int k = 0; k < KT; ++k)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int x = 16 * k + 4 * g + r, key = key0 + x;
-          if (t < np ? KEYS * t + x >= cnb : (key > cpos || key < klo)) sc[k][r] = NEG_BIG;
+          if (t < np ? KEYS * t + x >= cnb : (key > cpos || (key < klo && key >= A.keep))) sc[k][r] = NEG_BIG;
         }
     }
     float tmax = NEG_BIG;
@@ -504,14 +569,11 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
     if (g == 0) reinterpret_cast<float2*>(A.part_ml)[pc] = float2{m_run, l_run};
     return;
   }
-  const float fs = final_scale(A.sink, m_run, l_run);
-  bf16* orow = (bf16*)A.out + row * DV + 4 * g;
+  const float fs = final_scale(A, head, m_run, l_run);
 #pragma unroll
   for (int n = 0; n < 2 * NV; ++n) {
-    bf16x4 v;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = (bf16)(o[n][r] * fs);
-    *reinterpret_cast<bf16x4*>(orow + 16 * n) = v;
+    float v[4] = {o[n][0] * fs, o[n][1] * fs, o[n][2] * fs, o[n][3] * fs};
+    put_out<bf16>(A, tok, head, 16 * n + 4 * g, v);
   }
 }
 
@@ -524,7 +586,7 @@ constexpr int lds_bytes() {
 // run both in one launch, larger ones each in its own.
 enum { TILES = 1, SPLITS = 2 };
 
-template <int NK, int NV, int PATHS>
+template <int NK, int NV, int PATHS, bool MODS>
 __global__ __launch_bounds__(64 * NW, PATHS == TILES && NK + NV <= 8 ? 4 : 2) void mfma_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int n = A.n_items[0];
@@ -533,14 +595,14 @@ __global__ __launch_bounds__(64 * NW, PATHS == TILES && NK + NV <= 8 ? 4 : 2) vo
     for (int item = blockIdx.y; item < n; item += gridDim.y) {
       const int4 it = A.items[item];
       if ((it.z & 0xff) <= A.dec_tokens) continue;
-      tile_item<NK, NV>(A, it, smem);
+      tile_item<NK, NV, MODS>(A, it, smem);
       __syncthreads();
     }
   if constexpr ((PATHS & SPLITS) != 0)
     for (int item = blockIdx.y; item < n; item += gridDim.y) {
       const int4 it = A.items[item];
       if ((it.z & 0xff) > A.dec_tokens) continue;
-      split_item<NK, NV>(A, it, smem);
+      split_item<NK, NV, MODS>(A, it, smem);
       __syncthreads();
     }
 }
@@ -567,43 +629,53 @@ extern "C" void pa_window_pad(int k, int v, int* dk, int* dv) {
   *dv = 32 * b;
 }
 
-extern "C" int pa_window_attention(int fp32, void* out, float* part_o, float* part_ml, const void* q, const void* kp,
-                                   const void* vp, const void* pk, const void* pv, const int* items,
+extern "C" int pa_window_attention(int fp32, void* out, int out_f32, int ldo, float* part_o, float* part_ml, const void* q,
+                                   const void* kp, const void* vp, const void* pk, const void* pv, const int* items,
                                    const int* n_items, int max_items, const int* q_start, const int* q_len,
-                                   const int* ctx_len, const int* block_table, int max_blocks, int T, int H, int G, int DK,
-                                   int DV, int dec_tokens, int tile_tokens, int window, int pool, int npb,
-                                   int max_slots, float scale_log2, float sink, int simple, hipStream_t st) {
+                                   const int* ctx_len, const int* block_table, int max_blocks, int T, int H, int G, int GV,
+                                   int DK, int DV, int dec_tokens, int tile_tokens, int window, int pool, int npb, int keep,
+                                   int chunk, int max_slots, float scale, const float* slopes, float cap, const float* sink,
+                                   const void* gate, int ldg, float gain, int simple, hipStream_t st) {
   if (max_items <= 0) return 0;
-  if (DK % 32 || DV % 32 || H <= 0 || G <= 0 || H % G || dec_tokens <= 0 || tile_tokens <= 0) return -1;
+  if (DK % 32 || DV % 32 || H <= 0 || G <= 0 || GV <= 0 || H % G || G % GV || dec_tokens <= 0 || tile_tokens <= 0) return -1;
+  if (scale <= 0.f || keep < 0 || (keep > 0 && window <= 0) || (chunk > 0 && window > 0) || ldo % 4 || (gate && ldg % 4) ||
+      (pool > 0 && (keep > 0 || chunk > 0 || G != GV))) return -1;
   const int R = H / G, NB = (dec_tokens * R + 15) / 16;
   pa::wa::Args A{out, part_o, part_ml, q, kp, vp, pk, pv, (const int4*)items, n_items, q_start, q_len, ctx_len,
-                 block_table, max_blocks, max_slots, H, G, R, NB, DK, DV, dec_tokens, window, pool, npb, scale_log2, sink};
+                 block_table, max_blocks, max_slots, H, G, R, NB, DK, DV, dec_tokens, window, pool, npb,
+                 scale * pa::wa::LOG2E, sink, slopes, gate, scale, cap, gain, GV, keep, chunk, ldo, ldg, out_f32};
   if (!fp32 && !simple) {
     const int cw = 16 * pa::wa::NW, gt = (tile_tokens * R + cw - 1) / cw, gx = NB > gt ? NB : gt;
     const int gy = std::min(max_items, std::max(256, 2048 / G));  // (workgroups loop over the rest)
-#define PA_X(K, V)                                                                                            \
-  if (DK == 32 * K && DV == 32 * V) {                                                                         \
-    using namespace pa::wa;                                                                                   \
+    const bool mods = cap > 0.f || slopes;
+#define PA_KERNELS(K, V, M)                                                                                   \
+  do {                                                                                                        \
     constexpr int lds = lds_bytes<K, V>();                                                                    \
     static bool attr = false;                                                                                 \
     if (!attr) {                                                                                              \
-      for (const void* f : {(const void*)mfma_kernel<K, V, TILES>, (const void*)mfma_kernel<K, V, SPLITS>,    \
-                            (const void*)mfma_kernel<K, V, TILES | SPLITS>})                                  \
+      for (const void* f : {(const void*)mfma_kernel<K, V, TILES, M>, (const void*)mfma_kernel<K, V, SPLITS, M>, \
+                            (const void*)mfma_kernel<K, V, TILES | SPLITS, M>})                               \
         (void)hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, lds);                        \
       attr = true;                                                                                            \
     }                                                                                                         \
     const dim3 wg(64 * NW);                                                                                   \
     if (T <= 64) {                                                                                            \
-      hipLaunchKernelGGL((mfma_kernel<K, V, TILES | SPLITS>), dim3(gx, gy, G), wg, lds, st, A);               \
+      hipLaunchKernelGGL((mfma_kernel<K, V, TILES | SPLITS, M>), dim3(gx, gy, G), wg, lds, st, A);            \
     } else {                                                                                                  \
-      hipLaunchKernelGGL((mfma_kernel<K, V, TILES>), dim3(gt, gy, G), wg, lds, st, A);                        \
-      hipLaunchKernelGGL((mfma_kernel<K, V, SPLITS>), dim3(NB, gy, G), wg, lds, st, A);                       \
+      hipLaunchKernelGGL((mfma_kernel<K, V, TILES, M>), dim3(gt, gy, G), wg, lds, st, A);                     \
+      hipLaunchKernelGGL((mfma_kernel<K, V, SPLITS, M>), dim3(NB, gy, G), wg, lds, st, A);                    \
     }                                                                                                         \
+  } while (0)
+#define PA_X(K, V)                                                                                            \
+  if (DK == 32 * K && DV == 32 * V) {                                                                         \
+    using namespace pa::wa;                                                                                   \
+    if (mods) PA_KERNELS(K, V, true); else PA_KERNELS(K, V, false);                                           \
     hipLaunchKernelGGL((pa::wa::merge_kernel<V>), dim3(16, std::min(gy, 64), G), dim3(256), 0, st, A);        \
     return (int)hipGetLastError();                                                                            \
   }
     PA_WA_DIMS(PA_X)
 #undef PA_X
+#undef PA_KERNELS
   }
   if (DV > 2048 || DK > 8192) return -2;
   const dim3 grid(H, max_items < 4096 ? max_items : 4096);

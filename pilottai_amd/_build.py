@@ -8,8 +8,8 @@ the repository snapshot to the GPU box:
 * ``pilottai_amd/_latent.so`` — the kernels of models with latent attention and table-routed
                                   experts, with the packed projections they share (so that
                                   such a model needs no other kernel to run)
-* ``pilottai_amd/_hybrid.so`` — likewise for models with windowed pooled attention, state-space layers,
-                                  score-routed experts and hyper-connected residuals
+* ``pilottai_amd/_hybrid.so`` — likewise for models with paged attention of many kinds, recurrent layers,
+                                  score-routed experts and fp32 residuals
 * ``pilottai_amd/_runtime.so`` — C++ serving runtime: paged-KV block manager,
                                   prefix cache, continuous-batching scheduler,
                                   grammar FSM + tokenizer (csrc/runtime/*.cpp),
@@ -44,8 +44,8 @@ HIP_FLAGS = ["-ffast-math", "-fno-gpu-rdc", "-Wno-unused-result", "-Xclang", "-t
 SHARED_HIP = ["gemm_decode.hip", "gemm_prefill.hip"]
 MODULES = {
     "latent": (["grouped_gemm.hip", "latent_attention.hip", "latent_cache.hip", "residual_norm.hip"], "bindings_latent.cpp"),
-    "hybrid": (["grouped_gemm.hip", "hyper_norm.hip", "paged_kv.hip", "score_route.hip", "state_scan.hip",
-                "window_attention.hip"], "bindings_hybrid.cpp"),
+    "hybrid": (["grouped_gemm.hip", "head_difference.hip", "hyper_norm.hip", "matrix_memory.hip", "paged_kv.hip",
+                "score_route.hip", "state_scan.hip", "window_attention.hip"], "bindings_hybrid.cpp"),
 }
 FAMILY_HIP = {h for hips, _ in MODULES.values() for h in hips}
 FILE_FLAGS = {"gemm_mid.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"],

@@ -82,35 +82,40 @@ class LatentKVCache:
 
 
 class HybridCache:
-    """One entry of `layers` per layer run. An attention run has (keys [blocks, G, DK/8, 16, 8], values alike,
-    pooled keys [blocks, per page, G, DK], pooled values): a pooled block lies with the page of its last
-    token (csrc/ops/paged_kv.hip). A recurrent run has (state fp32 [slots, H, V, N], ring of the
-    convolution's inputs [slots, rows, channels]); a sequence that starts overwrites what its slot held."""
+    """`layers` has a list per layer run, an entry for each of its mixers. Attention has (keys [blocks, G, DK/8, 16,
+    8], values alike, pooled keys [blocks, per page, G, DK], pooled values): a pooled block lies with the page of
+    its last token (csrc/ops/paged_kv.hip); several key heads may share a value head. A state space has (state
+    fp32 [slots, H, V, N], ring of the convolution's inputs [slots, rows, channels]), a matrix memory (state fp32
+    [slots, H, V, N], its running maximum at every row [slots, H, V]); a sequence that starts overwrites what its
+    slot held."""
 
-    def __init__(self, kinds: Sequence[tuple], num_blocks: int, slots: int, device, dtype=torch.bfloat16,
+    def __init__(self, kinds: Sequence[Sequence[tuple]], num_blocks: int, slots: int, device, dtype=torch.bfloat16,
                  block_size: int = 16):
         if block_size != 16:
             raise ValueError("pages hold 16 tokens")
         self.num_blocks, self.slots, self.block_size = num_blocks, slots, block_size
         zeros = lambda dt, *s: torch.zeros(*s, dtype=dt, device=device)  # noqa: E731
-        self.layers: List[tuple] = []
-        for kind, *n in kinds:
+
+        def pools(kind, *n):
             if kind == "attention":
-                G, dk, dv, per = n
-                self.layers.append((zeros(dtype, num_blocks, G, dk // 8, 16, 8), zeros(dtype, num_blocks, G, dv // 8, 16, 8),
-                                    zeros(dtype, num_blocks if per else 0, per, G, dk),
-                                    zeros(dtype, num_blocks if per else 0, per, G, dv)))
-            else:
-                H, V, N, rows, channels = n
-                self.layers.append((zeros(torch.float32, slots, H, V, N), zeros(dtype, slots, rows, channels)))
+                G, dk, dv, per, gv = n
+                return (zeros(dtype, num_blocks, G, dk // 8, 16, 8), zeros(dtype, num_blocks, gv, dv // 8, 16, 8),
+                        zeros(dtype, num_blocks if per else 0, per, G, dk), zeros(dtype, num_blocks if per else 0, per, gv, dv))
+            H, V, N = n[:3]
+            state = zeros(torch.float32, slots, H, V, N)
+            return state, zeros(torch.float32, slots, H, V) if kind == "memory" else zeros(dtype, slots, *n[3:])
+        self.layers: List[List[tuple]] = [[pools(*k) for k in run] for run in kinds]
 
     @staticmethod
-    def bytes_per_block(kinds: Sequence[tuple], itemsize: int, block_size: int = 16) -> int:
-        return sum(n[0] * (n[1] + n[2]) * (block_size + n[3]) * itemsize for kind, *n in kinds if kind == "attention")
+    def bytes_per_block(kinds: Sequence[Sequence[tuple]], itemsize: int, block_size: int = 16) -> int:
+        return sum((n[0] * n[1] + n[4] * n[2]) * (block_size + n[3]) * itemsize
+                   for run in kinds for kind, *n in run if kind == "attention")
 
     @staticmethod
-    def bytes_per_slot(kinds: Sequence[tuple], itemsize: int) -> int:
-        return sum(4 * n[0] * n[1] * n[2] + n[3] * n[4] * itemsize for kind, *n in kinds if kind == "state")
+    def bytes_per_slot(kinds: Sequence[Sequence[tuple]], itemsize: int) -> int:
+        each = {"attention": lambda *n: 0, "state": lambda H, V, N, rows, ch: 4 * H * V * N + rows * ch * itemsize,
+                "memory": lambda H, V, N: 4 * H * V * (N + 1)}
+        return sum(each[kind](*n) for run in kinds for kind, *n in run)
 
     def nbytes(self) -> int:
-        return sum(t.numel() * t.element_size() for ts in self.layers for t in ts)
+        return sum(t.numel() * t.element_size() for run in self.layers for ts in run for t in ts)

@@ -12,12 +12,14 @@ import json
 import os
 from typing import Dict, Optional
 
-from pilottai_amd.models import bozupel, llama, mudepel
+from pilottai_amd.models import bozupel, llama, mudepel, salipel
 
-CONFIG_CLASSES: Dict[str, type] = {"Bozupel": bozupel.BozupelConfig, "Mudepel": mudepel.MudepelConfig}
+CONFIG_CLASSES: Dict[str, type] = {"Bozupel": bozupel.BozupelConfig, "Mudepel": mudepel.MudepelConfig,
+                                  "Salipel": salipel.SalipelConfig}
 MODEL_CLASSES: Dict[type, type] = {llama.LlamaConfig: llama.LlamaModel, bozupel.BozupelConfig: bozupel.BozupelModel,
-                                   mudepel.MudepelConfig: mudepel.MudepelModel}
-PRESETS = {**llama.PRESETS, **bozupel.PRESETS, **mudepel.PRESETS}
+                                   mudepel.MudepelConfig: mudepel.MudepelModel,
+                                   salipel.SalipelConfig: salipel.SalipelModel}
+PRESETS = {**llama.PRESETS, **bozupel.PRESETS, **mudepel.PRESETS, **salipel.PRESETS}
 
 
 def is_folder(name) -> bool:

@@ -66,7 +66,7 @@ def require_latent():
 
 
 def require_hybrid():
-    """The _hybrid module (windowed pooled attention, state-space layers, score-routed experts;
+    """The _hybrid module (paged attention, recurrent layers, score-routed experts, fp32 residuals;
     csrc/ops/bindings_hybrid.cpp)."""
     return _require_family("hybrid")
 

@@ -116,14 +116,14 @@ def table_route(tables, desc, desc_host, ids, slots, T: int, tm: int, order, til
 
 
 def expert_gemm(x, w, out, tiles, n_tiles, order, rows: int, *, x_div: int, out_order: bool, tm: int,
-                glu: Optional[tuple] = None):
+                glu: Optional[tuple] = None, relu2: bool = False):
     """Rows sorted by expert: out row = x row @ w[expert].T; glu = (limit, alpha, bias[, cubic]): the gated
-    pair of interleave_gate_up weights, min(g, limit) sigmoid(alpha (g + cubic g^3)) (clamp(u) + bias). x row =
-    order[p] // x_div (0: p), out row = order[p] if out_order."""
+    pair of interleave_gate_up weights, min(g, limit) sigmoid(alpha (g + cubic g^3)) (clamp(u) + bias); relu2: the
+    square of what is positive. x row = order[p] // x_div (0: p), out row = order[p] if out_order."""
     lim, alpha, bias, cubic = (tuple(glu) + (0.0,))[:4] if glu else (0.0, 0.0, 0.0, 0.0)
     if _on_gpu(x):
         require_grouped().expert_gemm(x, w, out, tiles, n_tiles, order, int(rows), int(x_div), bool(out_order), int(tm),
-                                      glu is not None, float(lim), float(alpha), float(bias), float(cubic))
+                                      1 if glu is not None else 2 if relu2 else 0, float(lim), float(alpha), float(bias), float(cubic))
     else:
-        ref.expert_gemm(x, unpack_groups(w), out, tiles, n_tiles, order, x_div, out_order, glu)
+        ref.expert_gemm(x, unpack_groups(w), out, tiles, n_tiles, order, x_div, out_order, glu, relu2)
     return out

@@ -396,7 +396,7 @@ def table_route(tables, desc, ids, slots, T, tm, order, tiles, n_tiles):
         n_tiles[layer] = min(k, tmax)
 
 
-def expert_gemm(x, w, out, tiles, n_tiles, order, x_div, out_order, glu):
+def expert_gemm(x, w, out, tiles, n_tiles, order, x_div, out_order, glu, relu2=False):
     K = w.shape[2]
     for e, start, n, _ in tiles[:int(n_tiles[0])].tolist():
         p = torch.arange(start, start + n)
@@ -407,11 +407,13 @@ def expert_gemm(x, w, out, tiles, n_tiles, order, x_div, out_order, glu):
             y = y.view(n, -1, 2, 16)
             g, u = y[:, :, 0].reshape(n, -1).clamp(max=lim), y[:, :, 1].reshape(n, -1).clamp(-lim, lim)
             y = g * torch.sigmoid(alpha * (g + cubic * g ** 3)) * (u + bias)
+        if relu2:
+            y = y.clamp(min=0) ** 2
         out[order[p].long() if out_order else p, :y.shape[1]] = y.to(out.dtype)
 
 
 # ---------------------------------------------------------------------------
-# residual of several streams, windowed pooled attention, state-space layers, score routing (ops/hybrid.py)
+# residual of several streams, paged attention, recurrent layers, score routing (ops/hybrid.py)
 # ---------------------------------------------------------------------------
 
 
@@ -425,16 +427,31 @@ def yarn_frequencies(dims: int, base: float, factor: float, original: float, fas
     return f * (1 - ramp) + f / factor * ramp, 0.1 * math.log(factor) + 1
 
 
-def angle_table(max_pos: int, dims: int, base: float, yarn: Optional[dict] = None) -> torch.Tensor:
-    """fp32 [max_pos, dims]: cos | sin of the rotate-half pairs, YaRN-scaled if `yarn` (factor, original,
-    fast, slow) is given."""
-    f, m = yarn_frequencies(dims, base, **yarn) if yarn else \
-        (base ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims), 1.0)
+def slow_wave_frequencies(dims: int, base: float, factor: float, low: float, high: float, original: float):
+    """Angles per position of dims / 2 pairs, scaled by wavelength as in Llama 3.1: pairs that turn more than
+    `high` times within `original` positions keep theirs, those that turn less than `low` times are divided by
+    `factor`, and in between the two are mixed."""
+    f = base ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims)
+    turns = original * f / (2 * math.pi)
+    keep = ((turns - low) / (high - low)).clamp(0, 1) if high > low else (turns >= low).double()
+    return f * keep + f / factor * (1 - keep)
+
+
+def angle_table(max_pos: int, dims: int, base: float, yarn: Optional[dict] = None,
+                slow_waves: Optional[dict] = None) -> torch.Tensor:
+    """fp32 [max_pos, dims]: cos | sin of the rotate-half pairs, scaled if `yarn` (factor, original, fast, slow)
+    or `slow_waves` (factor, low, high, original) is given."""
+    if yarn:
+        f, m = yarn_frequencies(dims, base, **yarn)
+    elif slow_waves:
+        f, m = slow_wave_frequencies(dims, base, **slow_waves), 1.0
+    else:
+        f, m = base ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims), 1.0
     a = torch.arange(max_pos, dtype=torch.float64)[:, None] * f[None, :]
     return torch.cat([a.cos() * m, a.sin() * m], 1).float()
 
 
-def hyper_norm(x, eps, y, partials, y_weights, bias, mix, post, pre, emb, ids, w_next, out, rows):
+def hyper_norm(x, eps, y, partials, y_weights, y2, bias, mix, post, pre, emb, ids, w_next, out, rows):
     T, S, D = x.shape
     sel = torch.arange(T) if rows is None else rows.long()
     r = x[sel]
@@ -443,6 +460,8 @@ def hyper_norm(x, eps, y, partials, y_weights, bias, mix, post, pre, emb, ids, w
     if y is not None:
         v = y[:, :D].float().view(T, partials, D)[sel]
         v = (v * y_weights.view(T, partials)[sel][:, :, None]).sum(1) if y_weights is not None else v.sum(1)
+        if y2 is not None:
+            v = v + y2[:, :D].float()[sel]
         if bias is not None:
             v = v + bias
         r = torch.einsum("st,nsd->ntd", mix, r) + post[None, :, None] * v[:, None]
@@ -461,20 +480,30 @@ def _page_rows(pages, blocks, n):
     return pages[blocks.long()].permute(0, 3, 1, 2, 4).reshape(-1, G, d8 * 8)[:n].float()
 
 
-def paged_kv(x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_len, block_table, cos_sin, pool, num_seqs):
+def paged_kv(x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_len, block_table, cos_sin, pool, v_col,
+             q_norm, k_norm, norm_v, dim, vdim, eps, num_seqs):
     T, H, DK = q.shape
-    G, DV = kp.shape[1], vp.shape[2] * 8
-    r = x[:, :(H + G) * DK + G * DV].float()
+    G, GV, DV = kp.shape[1], vp.shape[1], vp.shape[2] * 8
+    at = (H + G) * DK if v_col < 0 else v_col
+    r = x[:, :max((H + G) * DK, at + GV * DV)].float()
     if bias is not None:
         r = r + bias
-    heads = _rotate_part(r[:, :(H + G) * DK].view(T, H + G, DK), positions[:T], cos_sin)
+    heads = r[:, :(H + G) * DK].view(T, H + G, DK)
+    mean_norm = lambda h, n: h * torch.rsqrt(h.pow(2).sum(-1, keepdim=True) / n + eps)  # noqa: E731
+    if q_norm is not None:
+        w = torch.cat([q_norm.expand(H, -1), k_norm.expand(G, -1)])
+        heads = mean_norm(heads, dim) * w
+    if cos_sin is not None:
+        heads = _rotate_part(heads, positions[:T], cos_sin)
     q.copy_(heads[:, :H].to(q.dtype))
-    k, v = heads[:, H:], r[:, (H + G) * DK:].view(T, G, DV)
+    k, v = heads[:, H:], r[:, at:at + GV * DV].view(T, GV, DV)
+    if norm_v:
+        v = mean_norm(v, vdim)
     for t in range(T):
         s = int(slots[t])
         if s >= 0:
             kp[s // 16, :, :, s % 16] = k[t].view(G, -1, 8).to(kp.dtype)
-            vp[s // 16, :, :, s % 16] = v[t].view(G, -1, 8).to(vp.dtype)
+            vp[s // 16, :, :, s % 16] = v[t].view(GV, -1, 8).to(vp.dtype)
     if pool <= 0:
         return
     for s in range(num_seqs):
@@ -490,32 +519,50 @@ def paged_kv(x, bias, q, kp, vp, pk, pv, positions, slots, q_start, q_len, ctx_l
             pv[int(blocks[page]), sub] = vr[b * pool:(b + 1) * pool].mean(0).to(pv.dtype)
 
 
-def window_attention(out, q, kp, vp, pk, pv, q_start, q_len, ctx_len, block_table, scale, window, pool, sink, num_seqs):
-    H, G = q.shape[1], kp.shape[1]
+def window_attention(out, q, kp, vp, pk, pv, q_start, q_len, ctx_len, block_table, scale, window, pool, keep, chunk,
+                     slopes, cap, sink, gate, gain, num_seqs):
+    H, G, GV = q.shape[1], kp.shape[1], vp.shape[1]
     for s in range(num_seqs):
         n, ctx, q0 = int(q_len[s]), int(ctx_len[s]), int(q_start[s])
         if n <= 0:
             continue
         blocks = block_table[s, :(ctx + 15) // 16]
         k, v = _page_rows(kp, blocks, ctx), _page_rows(vp, blocks, ctx)
-        pos = torch.arange(ctx - n, ctx)[:, None]
-        back = pos - torch.arange(ctx)[None, :]
-        seen = (back >= 0) & (back < window) if window > 0 else back >= 0
+        pos, key = torch.arange(ctx - n, ctx)[:, None], torch.arange(ctx)[None, :]
+        back = pos - key
+        seen = (back >= 0) & ((back < window) | (key < keep)) if window > 0 else back >= 0
+        if chunk > 0:
+            seen = seen & (pos // chunk == key // chunk)
         if pool > 0 and window > 0 and ctx // pool:
             ends = torch.arange(ctx // pool) * pool + pool - 1
             page = blocks[ends // 16].long()
             sub = torch.arange(ctx // pool) - ends // 16 * 16 // pool
             k, v = torch.cat([k, pk[page, sub].float()]), torch.cat([v, pv[page, sub].float()])
             seen = torch.cat([seen, ends[None, :] <= pos - window], 1)
-        k, v = k.repeat_interleave(H // G, 1), v.repeat_interleave(H // G, 1)
+        k, v = k.repeat_interleave(H // G, 1), v.repeat_interleave(H // GV, 1)
         sc = torch.einsum("thd,khd->htk", q[q0:q0 + n].float(), k) * scale
+        if cap > 0:
+            sc = cap * torch.tanh(sc / cap)
+        if slopes is not None:
+            sc = sc - slopes[:, None, None] * back.float()
         sc = sc.masked_fill(~seen, float("-inf"))
         m = sc.amax(-1, keepdim=True)
-        if sink > 0:
-            m = m.clamp(min=0)
+        if sink is not None:
+            m = torch.maximum(m, sink[:, None, None])
         p = torch.exp(sc - m)
-        p = p / (p.sum(-1, keepdim=True) + (sink * torch.exp(-m) if sink > 0 else 0))
-        out[q0:q0 + n] = torch.einsum("htk,khd->thd", p, v).to(out.dtype)
+        p = p / (p.sum(-1, keepdim=True) + (torch.exp(sink[:, None, None] - m) if sink is not None else 0))
+        o = torch.einsum("htk,khd->thd", p, v) * gain
+        if gate is not None:
+            o = o * torch.sigmoid(gate[q0:q0 + n].float().view(o.shape))
+        out[q0:q0 + n] = o.to(out.dtype)
+
+
+def head_difference(a, out, gate, groups, lam, gain, vdim, eps):
+    T, H2, D = a.shape
+    m = a.float().view(T, groups, 2, H2 // (2 * groups), D)
+    o = (m[:, :, 0] - lam * m[:, :, 1]).reshape(T, H2 // 2, D)
+    o = o * torch.rsqrt(o.pow(2).sum(-1, keepdim=True) / vdim + eps) * gain
+    out[:, :, :] = (o * torch.sigmoid(gate.float().view(o.shape))).to(out.dtype)
 
 
 def state_scan(proj, y, state, ring, conv_w, conv_b, dt_bias, a, d, q_start, q_len, ctx_len, state_slot, groups, num_seqs):
@@ -548,24 +595,63 @@ def state_scan(proj, y, state, ring, conv_w, conv_b, dt_bias, a, d, q_start, q_l
         state[slot] = S
 
 
-def gated_norm(y, z, w, heads, vdim, vpad, parts, eps):
+def matrix_memory(x, y, div, state, top, i_bias, f_bias, q_start, q_len, ctx_len, state_slot, cols, vdim, cap, q_scale,
+                  num_seqs):
+    H, V, N = state.shape[1:]
+    cq, ck, cv, ci, vin = cols
+    for s in range(num_seqs):
+        n, q0, slot = int(q_len[s]), int(q_start[s]), int(state_slot[s])
+        if n <= 0:
+            continue
+        r = x[q0:q0 + n].float()
+        q, k = r[:, cq:cq + H * N].view(n, H, N) * q_scale, r[:, ck:ck + H * N].view(n, H, N)
+        v = torch.zeros(n, H, V)
+        v[:, :, :vdim] = r[:, cv:cv + H * vin].view(n, H, vin)[:, :, :vdim]
+        v[:, :, vdim] = 1.0  # (the row that sums the keys)
+        i = cap * torch.tanh((r[:, ci:ci + H] + i_bias) / cap)
+        f = torch.nn.functional.logsigmoid(cap * torch.tanh((r[:, ci + H:ci + 2 * H] + f_bias) / cap))
+        fresh = int(ctx_len[s]) == n
+        S, m = (torch.zeros(H, V, N), torch.zeros(H)) if fresh else (state[slot].clone(), top[slot, :, 0].clone())
+        for t in range(n):
+            mn = torch.maximum(f[t] + m, i[t])
+            S = S * torch.exp(f[t] + m - mn)[:, None, None] + \
+                (torch.exp(i[t] - mn)[:, None] * v[t])[:, :, None] * k[t][:, None, :]
+            m = mn
+            o = (S * q[t][:, None, :]).sum(-1)
+            y[q0 + t, :H * vin].view(H, vin)[:, :vdim] = o[:, :vdim].to(y.dtype)
+            div[q0 + t] = torch.maximum(o[:, vdim].abs(), torch.exp(-m)) + 1e-6
+        state[slot], top[slot] = S, m[:, None]
+
+
+def gated_norm(y, z, w, heads, vdim, vpad, parts, eps, div, after):
     T = y.shape[0]
-    g, zf = (t[:, :heads * vpad].float().view(T, heads, vpad)[:, :, :vdim].reshape(T, -1) for t in (y, z))
-    g = (g * (zf * torch.sigmoid(zf))).view(T, parts, -1)
-    g = (_norm32(g, eps).view(T, -1) * w).view(T, heads, vdim)
+    g, zf = (t[:, :heads * vpad].float().reshape(T, heads, vpad)[:, :, :vdim] for t in (y, z))
+    if div is not None:
+        g = g / div[:, :, None]
+    g, zf = g.reshape(T, -1), zf.reshape(T, -1)
+    if not after:
+        g = g * (zf * torch.sigmoid(zf))
+    g = _norm32(g.view(T, parts, -1), eps).view(T, -1) * w
+    g = (g * torch.sigmoid(zf) if after else g).view(T, heads, vdim)
     y.zero_()
     y[:, :heads * vpad].view(T, heads, vpad)[:, :, :vdim] = g.to(y.dtype)
 
 
-def score_route(h, w, slots, weights, choice, order, tiles, n_tiles, E, top, groups, keep, always, tm):
+def score_route(h, w, slots, weights, choice, order, tiles, n_tiles, E, top, groups, keep, always, tm, softmax, correction,
+                share, scale):
     T = h.shape[0]
-    s = torch.sigmoid(h[:, :w.shape[1]].float() @ w[:E].float().T)
-    per = s.view(T, groups, E // groups)
+    z = h[:, :w.shape[1]].float() @ w[:E].float().T
+    s = torch.softmax(z, -1) if softmax else torch.sigmoid(z)
+    pick = s + correction if correction is not None else s
+    per = pick.view(T, groups, E // groups)
     best = per.topk(min(2, E // groups), -1).values.sum(-1).topk(keep, -1).indices
     ok = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True).repeat_interleave(E // groups, 1)
-    val, idx = s.masked_fill(~ok, -1).topk(top, -1)
+    idx = pick.masked_fill(~ok, float("-inf")).topk(top, -1).indices
+    val = s.gather(1, idx)
+    if share:
+        val = val / (val.sum(1, keepdim=True) + 1e-20)
     live = slots[:T] >= 0
-    weights[:, :top], weights[:, top:] = val, 1.0
+    weights[:, :top], weights[:, top:] = val * scale, 1.0
     weights[~live] = 0
     e = torch.cat([idx, torch.arange(E, E + always).expand(T, -1)], 1)
     choice.view(T, top + always).copy_(torch.where(live[:, None], e, -1))

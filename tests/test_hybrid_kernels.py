@@ -209,7 +209,7 @@ def run_attention(device, dt, H, G, dk, dv, reqs, W, P, sink=1.0, simple=False, 
     po, pm = torch.empty(mi * G * NB * 16 * dv, device=device), torch.empty(mi * G * NB * 32, device=device)
     d = lambda t: t.to(dt).to(device)  # noqa: E731
     ops.window_attention(out, po, pm, q.to(device), d(kp), d(vp), d(pk), d(pv), m["items"], m["n_items"], *(m[k] for k in SEQ),
-                         scale, W, P, sink, dec, tile, mi, num_seqs=len(reqs), simple=simple)
+                         scale, W, P, torch.full((H,), math.log(sink), device=device) if sink else None, dec, tile, mi, num_seqs=len(reqs), simple=simple)
     for i, (c, n) in enumerate(reqs):
         k, v = seqs[i]
         q0 = int(m["q_start"][i])
