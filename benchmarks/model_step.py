@@ -1,6 +1,6 @@
 """Step throughput of a served model design beside Llama layers of equal size (random weights).
 
-    python bench.py --design bozupel|mudepel [--steps K --warmup W]
+    python bench.py --design bozupel|mudepel|salipel [--steps K --warmup W]
 
 For each size the two engines hold the same width, layer count, heads and active feed-forward width.
 A case is one scheduler-built step (prompt portions or decode rows at a context), captured as the
@@ -26,12 +26,12 @@ CASES: List[Tuple[str, List[Tuple[int, int]]]] = [
     ("decode 256 at 1024", [(1024, 1)] * 256),
 ]
 
-DESIGNS = ("bozupel", "mudepel")
+DESIGNS = ("bozupel", "mudepel", "salipel")
 
 
 def pair(design: str):
     """[(size, design config, equal-size Llama config)]"""
-    from pilottai_amd.models import bozupel, mudepel
+    from pilottai_amd.models import bozupel, mudepel, salipel
     from pilottai_amd.models.llama import LlamaConfig
 
     if design not in DESIGNS:
@@ -42,6 +42,10 @@ def pair(design: str):
             c = bozupel.PRESETS[f"bozupel-{size}"]
             m, p = c.layers[0].mixer, c.layers[0].mlp
             heads, kv, ff = m.heads, m.heads // 4, p.top * p.ff
+        elif design == "salipel":  # half the layers dense, half experts of two matrices: the mean of their active widths
+            c = salipel.PRESETS[f"salipel-{size}"]
+            m, p = c.layers[0].mixer, c.layers[1].mlp
+            heads, kv, ff = m.heads, m.kv_heads, (3 * c.layers[0].mlp.ff + 2 * p.top * p.ff) // 6 // 256 * 256
         else:  # dense and expert layers in turn: the mean of their active widths
             c = mudepel.PRESETS[f"mudepel-{size}"]
             m, p = c.layers[0].mixer, c.layers[1].mlp
