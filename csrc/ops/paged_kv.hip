@@ -178,45 +178,74 @@ __global__ __launch_bounds__(256) void paged_kv_kernel(const Args A) {
   }
 }
 
-// With norms: a power of two of lanes per head, which sum its squares. Sections (queries and keys, then values) begin
-// at whole waves.
+// lanes of a head of D dimensions, as a power of two
+__host__ __device__ __forceinline__ int head_bits(int D) {
+  int b = 0;
+  while ((8 << b) < D) ++b;
+  return b;
+}
+// units of 8 dimensions: queries and keys, then, from a whole wave on, values
+__host__ __device__ __forceinline__ int normed_units(int heads, int values, int DK, int DV, int* nqk) {
+  *nqk = ((heads << head_bits(DK)) + 63) & ~63;
+  return *nqk + (values << head_bits(DV));
+}
+
+// With norms: a power of two of lanes per head, which sum its squares. A unit's loads go out together.
 template <typename T>
-__global__ __launch_bounds__(256) void normed_kv_kernel(const Args A) {
+__global__ __launch_bounds__(512) void normed_kv_kernel(const Args A) {
   const int t = token_of(blockIdx.x, A.T);
   if (t < 0) return;
   const int slot = A.slots[t], pos = A.positions[t];
   if (slot < 0) return;
   const T* row = (const T*)A.x + (size_t)t * A.ldx;
   const float* cs = A.cos_sin + (size_t)pos * A.rd;
-  const int ck = A.DK >> 3, cv = A.DV >> 3;
-  const int bk = 32 - __clz(ck - 1), bv = 32 - __clz(cv - 1);  // log2 of the lanes of a head (clz(0) is 32)
-  const int nqk = (((A.H + A.G) << bk) + 63) & ~63, total = nqk + (A.GV << bv);
-  for (int u0 = 0; u0 < total; u0 += 256) {
+  const int ck = A.DK >> 3, cv = A.DV >> 3, half = A.rd >> 1;
+  const int bk = head_bits(A.DK), bv = head_bits(A.DV);
+  int nqk;
+  const int total = normed_units(A.H + A.G, A.GV, A.DK, A.DV, &nqk);
+  for (int u0 = 0; u0 < total; u0 += blockDim.x) {
     const int u = u0 + threadIdx.x;
     const bool value = u >= nqk;
     const int w = value ? u - nqk : u, bits = value ? bv : bk, per = value ? cv : ck;
-    const int h = w >> bits, o = w & ((1 << bits) - 1);  // (query heads, then key heads)
-    const bool in = o < per && h < (value ? A.GV : A.H + A.G), query = !value && h < A.H;
+    const int h = w >> bits, d = (w & ((1 << bits) - 1)) * 8;  // (query heads, then key heads)
+    const bool in = d < per * 8 && h < (value ? A.GV : A.H + A.G), query = !value && h < A.H;
     const int off = value ? A.vcol + h * A.DV : h * A.DK;
     const float* nw = value ? nullptr : query ? A.qn : A.kn;
-    float inv = 1.f, v[8];
-    if (value ? A.norm_v != 0 : nw != nullptr) {
-      float ss = 0.f;
-      if (in) {
-        chunk<T, false>(A, row, off, o * 8, cs, false, v);
-#pragma unroll
-        for (int j = 0; j < 8; ++j) ss = fmaf(v[j], v[j], ss);
+    const bool normed = value ? A.norm_v != 0 : nw != nullptr;
+    const bool turn = in && !value && d < A.rd, whole = half % 8 == 0;
+    const int pd = d < half ? d + half : d - half, ci = d < half ? d : pd;
+    float v[8], p[8], c[8], s[8], wv[8], wp[8], ss = 0.f;
+    if (in) {
+      chunk<T, false>(A, row, off, d, cs, false, v);
+      if (nw) load8(nw + d, wv);
+      if (turn && whole) {
+        chunk<T, false>(A, row, off, pd, cs, false, p);
+        if (nw) load8(nw + pd, wp);
+        load8(cs + ci, c);
+        load8(cs + half + ci, s);
       }
-      for (int m = (1 << bits) >> 1; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
-      inv = 1.f / sqrtf(ss * (value ? A.ivdim : A.idim) + A.eps);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss = fmaf(v[j], v[j], ss);
     }
+    for (int m = (1 << bits) >> 1; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
     if (!in) continue;
-    chunk<T, true>(A, row, off, o * 8, cs, !value, v, inv, nw);
+    const float inv = normed ? 1.f / sqrtf(ss * (value ? A.ivdim : A.idim) + A.eps) : 1.f;
+    if (turn && !whole) {
+      chunk<T, true>(A, row, off, d, cs, true, v, inv, nw);
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] *= nw ? inv * wv[j] : inv;
+      if (turn) {
+        const float sign = d < half ? -inv : inv;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] = v[j] * c[j] + sign * (nw ? p[j] * wp[j] : p[j]) * s[j];
+      }
+    }
     if (query) {
-      put((T*)A.q + ((size_t)t * A.H + h) * A.DK + o * 8, v);
+      put((T*)A.q + ((size_t)t * A.H + h) * A.DK + d, v);
     } else {
       const int g = value ? h : h - A.H;
-      put((T*)(value ? A.vp : A.kp) + (((size_t)(slot >> 4) * (value ? A.GV : A.G) + g) * per + o) * 128 + (slot & 15) * 8, v);
+      put((T*)(value ? A.vp : A.kp) + (((size_t)(slot >> 4) * (value ? A.GV : A.G) + g) * per + (d >> 3)) * 128 + (slot & 15) * 8, v);
     }
   }
 }
@@ -271,8 +300,11 @@ extern "C" int pa_paged_kv(int fp32, const void* x, const float* bias, void* q, 
                        normed ? 1.f / dim : 0.f, normed ? 1.f / vdim : 0.f, eps};
   const dim3 grid((T + 7) / 8 * 8);
   if (normed) {
-    if (fp32) hipLaunchKernelGGL(pa::kv::normed_kv_kernel<float>, grid, dim3(256), 0, st, A);
-    else hipLaunchKernelGGL(pa::kv::normed_kv_kernel<pa::bf16>, grid, dim3(256), 0, st, A);
+    int nqk;
+    const int total = pa::kv::normed_units(H + G, GV, DK, DV, &nqk), rounds = (total + 511) / 512;
+    const dim3 wg(((total + rounds - 1) / rounds + 63) / 64 * 64);
+    if (fp32) hipLaunchKernelGGL(pa::kv::normed_kv_kernel<float>, grid, wg, 0, st, A);
+    else hipLaunchKernelGGL(pa::kv::normed_kv_kernel<pa::bf16>, grid, wg, 0, st, A);
     return (int)hipGetLastError();
   }
   const bool later = pool > 0 && T > 64, now = pool > 0 && !later;

@@ -73,17 +73,32 @@ __device__ __forceinline__ size_t pooled_row(const Args& A, const int* bt, int b
   return ((size_t)bt[page] * A.npb + (b - (page << 4) / A.pool)) * A.G + h;
 }
 
-// a score's cap and bias, in units of q . k, which the softmax's scale still multiplies
+// A score's cap and bias, in units of q . k, which the softmax's scale still multiplies. Within a tile the bias is
+// slope * (key - first key) on the scores and -slope * (distance to the first key) on all of a lane's scores alike.
+enum { NO_MODS = 0, CAP = 1, BIAS = 2 };  // BIAS: and a cap, if there is one
+
+template <int MODS>
 struct Mods {
-  float to_tanh, from_tanh, slope;
+  float to_tanh = 0.f, from_tanh = 0.f, slope = 0.f;
   __device__ __forceinline__ Mods(const Args& A, int head) {
-    to_tanh = A.cap > 0.f ? 2.f * LOG2E * A.scale / A.cap : 0.f;
-    from_tanh = A.cap / A.scale;
-    slope = A.slopes ? A.slopes[head] / A.scale : 0.f;
+    if (MODS != NO_MODS) {
+      to_tanh = A.cap > 0.f ? 2.f * LOG2E * A.scale / A.cap : 0.f;
+      from_tanh = A.cap / A.scale;
+    }
+    if (MODS == BIAS) slope = A.slopes[head] / A.scale;
   }
-  __device__ __forceinline__ float operator()(float s, int back) const {
-    if (to_tanh != 0.f) s = from_tanh * (1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s * to_tanh)));
-    return s - slope * (float)back;
+  __device__ __forceinline__ float capped(float s) const {  // from_tanh * tanh
+    const float r = __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s * to_tanh));
+    return fmaf(r, -2.f * from_tanh, from_tanh);
+  }
+  template <int N>
+  __device__ __forceinline__ void cap(f32x4 (&s)[N]) const {  // (one branch for all of them)
+    if (MODS == CAP || (MODS == BIAS && to_tanh != 0.f)) {
+#pragma unroll
+      for (int k = 0; k < N; ++k)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[k][r] = capped(s[k][r]);
+    }
   }
 };
 
@@ -198,11 +213,11 @@ __device__ __forceinline__ float final_scale(const Args& A, int head, float m, f
   return a / (l * a + exp2f(s - t));
 }
 
-template <int NK, int NV, bool MODS>
-__device__ __forceinline__ void split_item(const Args& A, const int4 it, char* smem) {
+template <int NK, int NV, int MODS>
+__device__ __forceinline__ void split_item(const Args& A, const int4 it, const int gk, char* smem) {
   constexpr int DK = 32 * NK, DV = 32 * NV;
   const int s = it.x, qb = it.y, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff, nparts = it.z >> 20, pidx = it.w;
-  const int cb = blockIdx.x, gk = blockIdx.z, gv = gk / (A.G / A.GV), cols = nq * A.R;
+  const int cb = blockIdx.x, gv = gk / (A.G / A.GV), cols = nq * A.R;
   if (cb * 16 >= cols) return;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, g = lane >> 4, c = lane & 15;
   const int ctx = A.ctx_len[s], ql = A.q_len[s];
@@ -215,7 +230,7 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
   auto row_of = [&](int col) { return (size_t)(A.q_start[s] + qb + tok_of(col)) * A.H + head_of(col); };  // q row of a column
   const int cpos = pos0 + tok_of(cb * 16 + c);  // this column's position
   const int klo = first_key(A, cpos), cnb = blocks_of(A, cpos);
-  const Mods mods(A, head_of(cb * 16 + c));
+  const Mods<MODS> mods(A, head_of(cb * 16 + c));
   // the item's tiles of 16: pooled blocks, then token pages (the kept ones before the window's); this partition's share
   const int last = pos0 + nq - 1, nb = blocks_of(A, last), np = (nb + 15) >> 4;
   const int p_lo = first_key(A, pos0) >> 4, nkeep = kept_tiles(A, 16, p_lo), total = np + nkeep + ((last + 16) >> 4) - p_lo;
@@ -259,7 +274,8 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
   const int toff = ((c & 3) >> 1) * 256 + (4 * g + (c >> 2)) * 16 + (c & 1) * 8;
 
   for (int t = t_begin + wid; t < t_end; t += NW) {
-    f32x4 sc = {0.f, 0.f, 0.f, 0.f};
+    f32x4 s1[1] = {f32x4{0.f, 0.f, 0.f, 0.f}};
+    f32x4& sc = s1[0];
 #pragma unroll
     for (int m = 0; m < NK; ++m) {
       const bf16x8 qf = *reinterpret_cast<const bf16x8*>(sq + m * 1024 + loff);
@@ -268,12 +284,13 @@ __device__ __forceinline__ void split_item(const Args& A, const int4 it, char* s
 #pragma unroll
     for (int m = 0; m < NV; ++m) *reinterpret_cast<bf16x8*>(my + m * 1024 + loff) = vf[m];
     if (t + NW < t_end) load(t + NW);
+    mods.cap(s1);
     float tmax = NEG_BIG;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int e = 4 * g + r, key = 16 * page_of(t) + e;
       const bool ok = t < np ? 16 * t + e < cnb : (key <= cpos && (key >= klo || key < A.keep));
-      if (MODS) sc[r] = mods(sc[r], t < np ? 0 : cpos - key);
+      if (MODS == BIAS && t >= np) sc[r] = fmaf(mods.slope, (float)(key - cpos), sc[r]);
       sc[r] = ok ? sc[r] * A.scale_log2 : NEG_BIG;
       tmax = fmaxf(tmax, sc[r]);
     }
@@ -405,12 +422,20 @@ __global__ __launch_bounds__(256) void merge_kernel(const Args A) {
 template <int NK, int NV>
 constexpr int tile_parts() { return NK + NV <= 8 ? 4 : 2; }  // 16-key parts of a tile
 
-template <int NK, int NV, bool MODS>
-__device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* smem) {
+// Tiles run in the order of the items, all KV heads of one after the other (a head stays on its XCDs), but every second
+// round of the 256 CUs from its end: the scheduler lists long items first, and a CU's workgroups then come to
+// about the same number of keys.
+__device__ __forceinline__ int tile_order(int i, int n, int G) {
+  const int per = max(1, 256 / G), round = i / per;
+  return round & 1 ? round * per + min(per, n - round * per) - 1 - (i - round * per) : i;
+}
+
+template <int NK, int NV, int MODS>
+__device__ __forceinline__ void tile_item(const Args& A, const int4 it, const int gk, char* smem) {
   constexpr int DK = 32 * NK, DV = 32 * NV, KT = tile_parts<NK, NV>(), KEYS = 16 * KT;
   constexpr int PART = (NK + NV) * 1024, TILE = KT * PART;  // a 16-key part: K, then V
   const int s = it.x, qb = it.y, nq = it.z & 0xff, part = (it.z >> 8) & 0xfff, nparts = it.z >> 20;
-  const int cols = nq * A.R, cw = blockIdx.x * (16 * NW), gk = blockIdx.z, gv = gk / (A.G / A.GV);
+  const int cols = nq * A.R, cw = blockIdx.x * (16 * NW), gv = gk / (A.G / A.GV);
   if (cw >= cols) return;
   const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), g = lane >> 4, c = lane & 15;
   const int ctx = A.ctx_len[s], ql = A.q_len[s];
@@ -418,13 +443,12 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
   const int* bt = A.block_table + (size_t)s * A.max_blocks;
   const int ci = cw + wid * 16 + c, cc = min(ci, cols - 1), ct = cc / A.R;
   const int cpos = pos0 + ct, klo = first_key(A, cpos), cnb = blocks_of(A, cpos);
-  const int head = gk * A.R + cc - ct * A.R;
-  const size_t tok = (size_t)(A.q_start[s] + qb + ct), row = tok * A.H + head;
-  const Mods mods(A, head);
+  const int row = (A.q_start[s] + qb + ct) * A.H + gk * A.R + cc - ct * A.R;  // of q
+  const Mods<MODS> mods(A, gk * A.R + cc - ct * A.R);
   const int loff = lane * 16;
   bf16x8 qf[NK];
 #pragma unroll
-  for (int m = 0; m < NK; ++m) qf[m] = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + row * DK + 32 * m + 8 * g);
+  for (int m = 0; m < NK; ++m) qf[m] = *reinterpret_cast<const bf16x8*>((const bf16*)A.q + (size_t)row * DK + 32 * m + 8 * g);
   // positions of the workgroup's columns -> its tiles: pooled blocks, then tokens (the kept before the window's)
   const int f = pos0 + cw / A.R, e = pos0 + min(cw + 16 * NW - 1, cols - 1) / A.R;
   const int nb = blocks_of(A, e), np = (nb + KEYS - 1) / KEYS;
@@ -501,11 +525,14 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
         sc[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[m], sc[k], 0, 0, 0);
       }
     const int key0 = KEYS * tile_of(t);  // wave-uniform
-    if (MODS) {
+    float off = 0.f;  // of all this lane's scores
+    mods.cap(sc);
+    if (MODS == BIAS && t >= np) {
+      off = mods.slope * (float)(key0 + 4 * g - cpos);
 #pragma unroll
       for (int k = 0; k < KT; ++k)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) sc[k][r] = mods(sc[k][r], t < np ? 0 : cpos - (key0 + 16 * k + 4 * g + r));
+        for (int r = 0; r < 4; ++r) sc[k][r] = fmaf(mods.slope, (float)(16 * k + r), sc[k][r]);
     }
     if (t < np ? KEYS * (t + 1) > full_nb
                : ((key0 < full_lo && key0 + KEYS > A.keep) || key0 + KEYS - 1 > full_hi)) {
@@ -522,6 +549,7 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
     for (int k = 0; k < KT; ++k)
 #pragma unroll
       for (int r = 0; r < 4; ++r) tmax = fmaxf(tmax, sc[k][r]);
+    if (MODS == BIAS) tmax += off;
     tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
     tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
     const float m_new = fmaxf(m_run, fmaxf(tmax * A.scale_log2, NEG_BIG));
@@ -533,7 +561,8 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
       m_run = m_new;
     }
     // a column that has seen no key yet (its window starts in a later tile): every weight is 0
-    const float nm = m_run < 0.01f * NEG_BIG ? 0.f : -m_run;
+    float nm = m_run < 0.01f * NEG_BIG ? 0.f : -m_run;
+    if (MODS == BIAS) nm = fmaf(off, A.scale_log2, nm);
     bf16x8 pf[KT / 2];
 #pragma unroll
     for (int k = 0; k < KT; ++k)
@@ -569,11 +598,12 @@ __device__ __forceinline__ void tile_item(const Args& A, const int4 it, char* sm
     if (g == 0) reinterpret_cast<float2*>(A.part_ml)[pc] = float2{m_run, l_run};
     return;
   }
+  const int tok = row / A.H, head = row - tok * A.H;
   const float fs = final_scale(A, head, m_run, l_run);
 #pragma unroll
   for (int n = 0; n < 2 * NV; ++n) {
     float v[4] = {o[n][0] * fs, o[n][1] * fs, o[n][2] * fs, o[n][3] * fs};
-    put_out<bf16>(A, tok, head, 16 * n + 4 * g, v);
+    put_out<bf16>(A, (size_t)tok, head, 16 * n + 4 * g, v);
   }
 }
 
@@ -586,23 +616,23 @@ constexpr int lds_bytes() {
 // run both in one launch, larger ones each in its own.
 enum { TILES = 1, SPLITS = 2 };
 
-template <int NK, int NV, int PATHS, bool MODS>
-__global__ __launch_bounds__(64 * NW, PATHS == TILES && NK + NV <= 8 ? 4 : 2) void mfma_kernel(const Args A) {
+template <int NK, int NV, int PATHS, int MODS>
+__global__ __launch_bounds__(64 * NW, (PATHS == TILES && NK + NV <= 8) || NK + NV <= 6 ? 4 : 2) void mfma_kernel(const Args A) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int n = A.n_items[0];
   // two passes over the workgroup's items, so that neither path's registers carry the other's
   if constexpr ((PATHS & TILES) != 0)
-    for (int item = blockIdx.y; item < n; item += gridDim.y) {
-      const int4 it = A.items[item];
+    for (int w = blockIdx.y; w < n * A.G; w += gridDim.y) {
+      const int4 it = A.items[tile_order(w / A.G, n, A.G)];
       if ((it.z & 0xff) <= A.dec_tokens) continue;
-      tile_item<NK, NV, MODS>(A, it, smem);
+      tile_item<NK, NV, MODS>(A, it, w % A.G, smem);
       __syncthreads();
     }
   if constexpr ((PATHS & SPLITS) != 0)
-    for (int item = blockIdx.y; item < n; item += gridDim.y) {
-      const int4 it = A.items[item];
+    for (int w = blockIdx.y; w < n * A.G; w += gridDim.y) {
+      const int4 it = A.items[w / A.G];
       if ((it.z & 0xff) > A.dec_tokens) continue;
-      split_item<NK, NV, MODS>(A, it, smem);
+      split_item<NK, NV, MODS>(A, it, w % A.G, smem);
       __syncthreads();
     }
 }
@@ -611,7 +641,8 @@ __global__ __launch_bounds__(64 * NW, PATHS == TILES && NK + NV <= 8 ? 4 : 2) vo
 }  // namespace pa
 
 // (key width, value width) in 32s with MFMA kernels, smallest first
-#define PA_WA_DIMS(X) X(1, 1) X(2, 1) X(2, 2) X(3, 3) X(4, 2) X(4, 4) X(6, 4) X(6, 6) X(8, 8)
+#define PA_WA_DIMS(X) \
+  X(1, 1) X(1, 2) X(2, 1) X(2, 2) X(2, 4) X(3, 3) X(4, 2) X(4, 4) X(4, 8) X(6, 4) X(6, 6) X(8, 8)
 
 // The padded widths for key size k and value size v: the first built pair that holds both, else whole
 // 32s (the simple kernel then runs).
@@ -646,8 +677,7 @@ extern "C" int pa_window_attention(int fp32, void* out, int out_f32, int ldo, fl
                  scale * pa::wa::LOG2E, sink, slopes, gate, scale, cap, gain, GV, keep, chunk, ldo, ldg, out_f32};
   if (!fp32 && !simple) {
     const int cw = 16 * pa::wa::NW, gt = (tile_tokens * R + cw - 1) / cw, gx = NB > gt ? NB : gt;
-    const int gy = std::min(max_items, std::max(256, 2048 / G));  // (workgroups loop over the rest)
-    const bool mods = cap > 0.f || slopes;
+    const int gi = std::min(max_items, std::max(256, 2048 / G)), gy = gi * G;  // (workgroups loop over the rest)
 #define PA_KERNELS(K, V, M)                                                                                   \
   do {                                                                                                        \
     constexpr int lds = lds_bytes<K, V>();                                                                    \
@@ -660,17 +690,19 @@ extern "C" int pa_window_attention(int fp32, void* out, int out_f32, int ldo, fl
     }                                                                                                         \
     const dim3 wg(64 * NW);                                                                                   \
     if (T <= 64) {                                                                                            \
-      hipLaunchKernelGGL((mfma_kernel<K, V, TILES | SPLITS, M>), dim3(gx, gy, G), wg, lds, st, A);            \
+      hipLaunchKernelGGL((mfma_kernel<K, V, TILES | SPLITS, M>), dim3(gx, gy), wg, lds, st, A);            \
     } else {                                                                                                  \
-      hipLaunchKernelGGL((mfma_kernel<K, V, TILES, M>), dim3(gt, gy, G), wg, lds, st, A);                     \
-      hipLaunchKernelGGL((mfma_kernel<K, V, SPLITS, M>), dim3(NB, gy, G), wg, lds, st, A);                    \
+      hipLaunchKernelGGL((mfma_kernel<K, V, TILES, M>), dim3(gt, gy), wg, lds, st, A);                     \
+      hipLaunchKernelGGL((mfma_kernel<K, V, SPLITS, M>), dim3(NB, gy), wg, lds, st, A);                    \
     }                                                                                                         \
   } while (0)
 #define PA_X(K, V)                                                                                            \
   if (DK == 32 * K && DV == 32 * V) {                                                                         \
     using namespace pa::wa;                                                                                   \
-    if (mods) PA_KERNELS(K, V, true); else PA_KERNELS(K, V, false);                                           \
-    hipLaunchKernelGGL((pa::wa::merge_kernel<V>), dim3(16, std::min(gy, 64), G), dim3(256), 0, st, A);        \
+    if (slopes) PA_KERNELS(K, V, BIAS);                                                                       \
+    else if (cap > 0.f) PA_KERNELS(K, V, CAP);                                                                \
+    else PA_KERNELS(K, V, NO_MODS);                                                                           \
+    hipLaunchKernelGGL((pa::wa::merge_kernel<V>), dim3(T <= 64 || T > 1024 ? 8 : 16, std::min(gi, 64), G), dim3(256), 0, st, A);        \
     return (int)hipGetLastError();                                                                            \
   }
     PA_WA_DIMS(PA_X)

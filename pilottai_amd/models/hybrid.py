@@ -207,6 +207,30 @@ def _heads(w: torch.Tensor, n: int, size: int, padded: int) -> torch.Tensor:
     return out.reshape(n * padded, *w.shape[1:])
 
 
+class SideStreams:
+    """Streams for branches of a step that do not depend on each other. They are used while a graph is captured, whose
+    replays then run the branches together; an eager step runs them one after the other. A branch's tensors are
+    its stream's: the next step of that stream waits for whoever has read them."""
+
+    def __init__(self, device, count: int):
+        self.streams = [torch.cuda.Stream(device) for _ in range(count)] if device.type == "cuda" else []
+
+    def run(self, first, *others, at: int = 0):
+        """Results of first() and others(), the latter on the streams from number `at` on."""
+        if not self.streams or not torch.cuda.is_current_stream_capturing():
+            return [f() for f in (first, *others)]
+        main, out = torch.cuda.current_stream(), []
+        used = self.streams[at:at + len(others)]
+        for s, f in zip(used, others):
+            s.wait_stream(main)
+            with torch.cuda.stream(s):
+                out.append(f())
+        out.insert(0, first())
+        for s in used:
+            main.wait_stream(s)
+        return out
+
+
 class AttentionRoom(NamedTuple):
     """What the engine's attention work items need: partial results and the tokens of an item."""
     part_o: torch.Tensor
@@ -375,15 +399,22 @@ class MixerBlock:
     def tensors(self):
         return [self.proj.w, self.o.w] + (self.mlp.tensors() if self.mlp else [])
 
-    def __call__(self, h, meta: StepMeta, caches, room: AttentionRoom):
-        x = self.proj(h)
+    def __call__(self, h, meta: StepMeta, caches, room: AttentionRoom, side: Optional[SideStreams] = None):
+        """`side`: streams 1 .. for the mixers behind the first, 0 for the feed-forward."""
         out = torch.empty(h.shape[0], self.o.K, dtype=self.dtype, device=self.device)
         if self.cols < self.o.K:
             out[:, self.cols:].zero_()
-        for m, a, b, cache in zip(self.mixers, self.at_in, self.at_out, caches):
-            m(x[:, a:], out[:, b:b + m.width], meta, cache, room)
-        if self.mlp is not None:
+
+        def mix():
+            x = self.proj(h)
+            each = [lambda m=m, a=a, b=b, c=c: m(x[:, a:], out[:, b:b + m.width], meta, c, room)
+                    for m, a, b, c in zip(self.mixers, self.at_in, self.at_out, caches)]
+            run(*each, at=1)
+
+        def feed():
             self.mlp.activate(h, out[:, self.at_out[-1]:self.at_out[-1] + self.mlp.fp])
+        run = side.run if side is not None else lambda *fs, at=0: [f() for f in fs]
+        run(mix, *([feed] if self.mlp is not None else []))
         return self.o(out), 1, None, self.bias
 
 

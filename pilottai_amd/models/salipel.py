@@ -37,7 +37,7 @@ from pilottai_amd import ops
 from pilottai_amd.models.cache import HybridCache, StepMeta
 from pilottai_amd.models.common import PackedLinear
 from pilottai_amd.models.hybrid import (GELU_TANH, AttentionSpec, DenseSpec, GatedMLP, HybridModel, MatrixMemory, MatrixMemorySpec,
-                                        MixerBlock, PagedAttention, ScoredExperts, ScoredExpertsSpec)
+                                        MixerBlock, PagedAttention, ScoredExperts, ScoredExpertsSpec, SideStreams)
 from pilottai_amd.ops.latent import pad_to
 from pilottai_amd.parallel.comm import TPGroup
 
@@ -106,7 +106,7 @@ def _feed_forward(p: Optional[dict]):
         raise ValueError(f"unknown feed-forward {p.get('kind')!r}")
     r = p["router"]
     return ScoredExpertsSpec(experts=int(r["experts"]), top=int(r["top"]), ff=int(p["expert"]["ff"]), act=None, softmax=True,
-                             correction=True, share=True, scale=float(r["scale"]))
+                             correction=True, share=True, scale=float(r.get("scale", 1.0)))
 
 
 MIXERS = {"parallel": _parallel, "attention": _chunked, "attention_2": _differential}
@@ -142,7 +142,7 @@ class SalipelConfig:
             except ValueError as e:
                 raise ValueError(f"layer {i}: {e}") from None
         return cls(name=name, vocab_size=int(d["vocab"]), hidden_size=int(d["width"]), layers=layers,
-                   eps=float(d["norm"]["eps"]), residual_mult=float(d["residual_mult"]))
+                   eps=float(d["norm"]["eps"]), residual_mult=float(d.get("residual_mult", 1.0)))
 
     def layer_shapes(self, i: int) -> Dict[str, tuple]:
         """Every tensor of layer i by its name behind "l<i>."."""
@@ -195,6 +195,7 @@ PRESETS: Dict[str, SalipelConfig] = {
 
 class SalipelModel(HybridModel):
     NAME = "Salipel"
+    SIDE_MAX_T = 2048  # largest captured step whose feed-forward and second mixer run beside the first mixer
 
     def __init__(self, cfg: SalipelConfig, device, dtype=torch.bfloat16, tp: Optional[TPGroup] = None, seed: int = 0,
                  weights_path: Optional[str] = None, max_len: int = 8192, **_):
@@ -220,6 +221,7 @@ class SalipelModel(HybridModel):
             dense = GatedMLP(L.mlp, sub("mlp."), d, dtype, dev, alone=False) if isinstance(L.mlp, DenseSpec) else None
             experts = ScoredExperts(L.mlp, sub("mlp."), d, dtype, dev) if isinstance(L.mlp, ScoredExpertsSpec) else None
             self.layers.append({"norm": self.f32(t["norm1"]), "mixer": MixerBlock(mixers, dtype, dev, dense), "mlp": experts})
+        self.side = SideStreams(dev, 2)
         self.finish()
 
     def _draw(self, part: str, rand: torch.Tensor, g: torch.Generator):
@@ -244,10 +246,13 @@ class SalipelModel(HybridModel):
         step = dict(emb=self.embed, ids=meta.input_ids[:T])
         for i, L in enumerate(self.layers):
             h = ops.hyper_norm(x, eps, pre=self.one, w_next=L["norm"], out=new_h(), **step)
-            y, _, _, _ = L["mixer"](h, meta, kv.layers[i], room)
+            side = self.side if T <= self.SIDE_MAX_T else None
+            mixer, mlp = lambda: L["mixer"](h, meta, kv.layers[i], room, side), lambda: L["mlp"](h, meta)  # noqa: E731, B023
+            both = [mixer] + ([mlp] if L["mlp"] is not None else [])
+            (y, *_), *more = side.run(*both) if side else [f() for f in both]
             step = dict(y=y, mix=self.keep, post=self.mult)
-            if L["mlp"] is not None:
-                part, k, w, _ = L["mlp"](h, meta)
+            if more:
+                part, k, w, _ = more[0]
                 step.update(y=part, partials=k, y_weights=w, y2=y)
             if residuals is not None:
                 after = x.clone()

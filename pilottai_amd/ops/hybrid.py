@@ -16,7 +16,7 @@ from .kernels import _on_gpu, require_hybrid
 from .latent import unpack_groups
 
 # (key width, value width) in 32s with MFMA kernels (window_attention.hip PA_WA_DIMS)
-WINDOW_TILES = ((1, 1), (2, 1), (2, 2), (3, 3), (4, 2), (4, 4), (6, 4), (6, 6), (8, 8))
+WINDOW_TILES = ((1, 1), (1, 2), (2, 1), (2, 2), (2, 4), (3, 3), (4, 2), (4, 4), (4, 8), (6, 4), (6, 6), (8, 8))
 SCAN_CHUNK = 64  # tokens of a scan item (state_scan.hip)
 SCAN_MIN = 8     # longer portions are scanned in chunks
 CONV_TAPS = (4, 8)  # built convolutions: shorter ones get zero taps in front
