@@ -583,10 +583,12 @@ int32_t Scheduler::emit(int32_t* buf) {
       const int32_t nq = c.c & 0xff;
       const int32_t keys = keys_of(c.keys, nq);
       const int32_t np = std::min(want, keys / 256);
-      if (np >= 2 && pslot + 8 * np <= L.max_items && total + np - 1 <= L.max_items) {
+      // slots of a partition: a portion's last few tokens fit the decode path, which holds them in one
+      const int32_t sl = nq <= tpw ? 1 : 8;
+      if (np >= 2 && pslot + sl * np <= L.max_items && total + np - 1 <= L.max_items) {
         for (int32_t q = 0; q < np; ++q)
-          split.push_back({keys / np, c.a, c.b, nq | (q << 8) | (np << 20), pslot + 8 * q});
-        pslot += 8 * np;
+          split.push_back({keys / np, c.a, c.b, nq | (q << 8) | (np << 20), pslot + sl * q});
+        pslot += sl * np;
         total += np - 1;
       } else {
         split.push_back(c);

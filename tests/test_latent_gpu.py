@@ -239,6 +239,8 @@ def test_latent_attention_bf16(gpu, H, R, r, step, window):
 def test_latent_attention_split_tiles(gpu, H, R, r, window):
     """Prompt portions cut over their keys: partitions of one item meet in the merge launch."""
     run_attention(gpu, torch.bfloat16, H, R, r, [(1500, 40), (900, 1), (0, 20), (700, 3)], window, tiles=64, part=256)
+    tile = 128 // min(H, 16)  # and portions whose rest is as short as a decode row's tokens
+    run_attention(gpu, torch.bfloat16, H, R, r, [(1500, tile + 1), (900, 2 * tile + 16 // min(H, 16))], window, tiles=64, part=256)
 
 
 @pytest.mark.parametrize("dt", DTYPES)

@@ -168,6 +168,34 @@ def test_attention_cut_over_keys(gpu, H, G, GV, dk, dv, kind):
     run_attention(gpu, BF16, H, G, GV, dk, dv, [(1500, 40), (900, 1), (0, 20), (700, 3)], tiles=64, part=64, split=2000, **kw)
 
 
+@pytest.mark.parametrize("group", [1, 2, 3, 4, 6, 16])
+def test_partition_slots(group):
+    """Portions cut over their keys: slots of their own for every partition, in a row: one where the portion's rest is no
+    longer than a decode row's tokens (the kernels take it for one), else eight."""
+    for tail in (1, 16 // group, 16 // group + 1):
+        n = 2 * (128 // group) + tail
+        _, m, dec, tile = fed_step("cpu", [(900, n), (700, 1), (1500, tail)], group, 1, part=64, tiles=64, split=2000)
+        used, parts = set(), {}
+        for seq, at, c, slot in m["items"][:int(m["n_items"])].tolist():
+            nq, k = c & 0xff, c >> 20
+            if k > 1:
+                own = set(range(slot, slot + (1 if nq <= dec else 8)))
+                assert not own & used and nq <= tile
+                used |= own
+                parts.setdefault((seq, at, nq, k), {})[c >> 8 & 0xfff] = slot
+        for (_, _, nq, k), slots in parts.items():
+            assert [slots[p] - slots[0] for p in range(k)] == [p * (1 if nq <= dec else 8) for p in range(k)]
+        assert (0, n - tail, tail) in {key[:3] for key in parts} and max(used) < m["items"].shape[0]
+
+
+@kinds
+@pytest.mark.parametrize("H,G,GV,dk,dv", [(6, 1, 1, 64, 64), (4, 4, 2, 32, 64), (4, 1, 1, 64, 32)])
+@pytest.mark.parametrize("mask", [{}, dict(window=300, keep=9), dict(chunk=1000)])
+def test_a_cut_portion_with_a_short_rest(device, dt, H, G, GV, dk, dv, mask):
+    tile = 128 // (H // G)
+    run_attention(device, dt, H, G, GV, dk, dv, [(1200, tile + 1), (600, tile + 16 // (H // G)), (0, 2 * tile + 1)], tiles=64, part=64, split=2000, **mask)
+
+
 @pytest.mark.gpu
 @pytest.mark.parametrize("dk,dv", [(32, 32), (64, 32), (96, 96), (128, 64), (192, 128), (256, 256), (288, 320)])
 def test_attention_every_width(gpu, dk, dv):
