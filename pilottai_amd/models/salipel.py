@@ -167,15 +167,15 @@ def _preset(name: str, width: int, heads: int, memory: MatrixMemorySpec, ff: int
                          window=1024, keep=16, qk_norm=True, keys_as_values=True, gate=True)
     chunked = AttentionSpec(**size, dim=128, scale=128 ** -0.5, chunk=2048, slopes=distance_slopes(heads), learned_sink=True,
                             v_norm=True)
-    twice = AttentionSpec(**size, dim=64, scale=64 ** -0.5, rot_base=500000.0, rot_dims=64, cap=50.0, diff=0.5, qk_norm=True, gate=True)
+    twice = AttentionSpec(**size, dim=64, scale=64 ** -0.5, rot_base=500000.0, rot_dims=64, cap=50.0, diff=0.4, qk_norm=True, gate=True)
     both = ParallelSpec(left, memory, 1.0, 1.0)
     layers = [SalipelLayer(chunked, DenseSpec(ff)), SalipelLayer(both, experts), SalipelLayer(twice, DenseSpec(ff)),
               SalipelLayer(both, experts)]
-    return SalipelConfig(name=name, vocab_size=vocab, hidden_size=width, layers=layers * repeat, residual_mult=0.7)
+    return SalipelConfig(name=name, vocab_size=vocab, hidden_size=width, layers=layers * repeat, residual_mult=0.5)
 
 
 def _experts(n: int, top: int, ff: int) -> ScoredExpertsSpec:
-    return ScoredExpertsSpec(experts=n, top=top, ff=ff, act=None, softmax=True, correction=True, share=True, scale=1.5)
+    return ScoredExpertsSpec(experts=n, top=top, ff=ff, act=None, softmax=True, correction=True, share=True, scale=2.0)
 
 
 PRESETS: Dict[str, SalipelConfig] = {

@@ -375,7 +375,7 @@ def test_norm_before_the_gate(device, dt, H, V, Vp):
 # ---- routing and experts ------------------------------------------------------------------------------
 @kinds
 @pytest.mark.parametrize("T", [1, 16, 17, 300])
-@pytest.mark.parametrize("E,top,scale", [(8, 2, 1.5), (6, 6, 1.0), (64, 6, 2.5), (5, 1, 0.7), (160, 5, 1.0), (1, 1, 3.0)])
+@pytest.mark.parametrize("E,top,scale", [(8, 2, 1.3), (6, 6, 1.0), (64, 6, 2.5), (5, 1, 0.7), (160, 5, 1.0), (1, 1, 3.0)])
 def test_softmax_route(device, dt, T, E, top, scale):
     """Choice by score + correction (of both signs), weights by the scores alone."""
     from pilottai_amd import ops
