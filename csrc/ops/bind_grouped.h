@@ -1,4 +1,4 @@
-// Shared by the bindings of the modules with grouped projections (_latent, _hybrid): operand checks and
+// Shared by the bindings of the modules with grouped projections (_latent, _hybrid, _latent_linear): operand checks and
 // the per-head and sorted projections of grouped_gemm.hip.
 #pragma once
 #include "bind_common.h"
@@ -7,7 +7,8 @@ extern "C" {
 int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out, long long wstride, int groups, int ldx, int xg,
                     int ldo, int og, int rows, int N16, int K32, const int* tiles, int max_tiles, const int* n_tiles,
                     const int* order, int x_div, int out_order, int tm, int epi, float limit, float alpha, float cubic, float bias,
-                    const int* positions, const float* cos_sin, int rskip, int r, int rp, int rd, hipStream_t st);
+                    const int* positions, const float* cos_sin, int rskip, int r, int rp, int rd, const float* row_w,
+                    const void* gate, int ldg, const void* table, const int* ids, int ldt, int tcol, int vocab, hipStream_t st);
 }
 
 namespace {
@@ -53,9 +54,10 @@ void dims(const at::Tensor& w, int f, int64_t* G, int64_t* N, int64_t* K) {
 }
 
 // every row of x through every group: x columns g * xg .. + K -> out columns g * og .. + N; with
-// positions / cos_sin also the rotated part: x columns g * xg + rskip .. + r -> out columns g * og + N .. + rp
+// positions / cos_sin also the rotated part: x columns g * xg + rskip .. + r -> out columns g * og + N .. + rp; with gate
+// times sigmoid(gate), whose columns are out's
 void head_gemm(at::Tensor x, int64_t xg, at::Tensor w, at::Tensor out, int64_t og, Opt positions, Opt cos_sin,
-               int64_t rskip, int64_t r, int64_t rp) {
+               int64_t rskip, int64_t r, int64_t rp, Opt gate) {
   const int f = is_f32(x, "x");
   check_rows(x, x.scalar_type(), "x");
   check_rows(out, x.scalar_type(), "out");
@@ -77,19 +79,45 @@ void head_gemm(at::Tensor x, int64_t xg, at::Tensor w, at::Tensor out, int64_t o
   } else {
     rp = 0;
   }
+  if (gate.has_value()) {
+    check_rows(*gate, x.scalar_type(), "gate");
+    TORCH_CHECK(gate->size(0) == x.size(0) && gate->size(1) >= (G - 1) * og + N && gate->stride(0) % 4 == 0 &&
+                    ((uintptr_t)gate->data_ptr() & 7) == 0, "head_gemm: gate must be [rows, >= out's columns]");
+  }
   TORCH_CHECK(f || (x.stride(0) % 8 == 0 && xg % 8 == 0 && out.stride(0) % 4 == 0 && og % 4 == 0),
               "head_gemm: 16-byte aligned operands");
   check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, G, x.stride(0), xg, out.stride(0), og,
-                           x.size(0), N / 16, K / 32, nullptr, 0, nullptr, nullptr, 0, 0, 0, 0, 0.f, 0.f, 0.f, 0.f,
-                           pos, cs, rskip, r, rp, rd, cur_stream()),
+                           x.size(0), N / 16, K / 32, nullptr, 0, nullptr, nullptr, 0, 0, 0, gate.has_value() ? 3 : 0, 0.f, 0.f,
+                           0.f, 0.f, pos, cs, rskip, r, rp, rd, nullptr, gate.has_value() ? gate->data_ptr() : nullptr,
+                           gate.has_value() ? gate->stride(0) : 0, nullptr, nullptr, 0, 0, 0, cur_stream()),
            "head_gemm");
 }
 
+// out = gated unit of (x w^T, the row's embedding): table [vocab, columns], from column tcol on
+void table_gemm(at::Tensor x, at::Tensor w, at::Tensor out, at::Tensor table, at::Tensor ids, int64_t tcol, double limit,
+                double alpha, double bias, double cubic) {
+  const int f = is_f32(x, "x");
+  for (auto* t : {&x, &out, &table}) check_rows(*t, x.scalar_type(), "table_gemm operand");
+  check_dtype(w, x.scalar_type(), "w");
+  int64_t G, N, K;
+  dims(w, f, &G, &N, &K);
+  TORCH_CHECK(G == 1 && out.size(0) == x.size(0) && K <= x.size(1) && N <= out.size(1) && tcol >= 0 &&
+                  tcol + N <= table.size(1) && table.size(0) > 0, "table_gemm sizes");
+  TORCH_CHECK(f || (x.stride(0) % 8 == 0 && out.stride(0) % 4 == 0 && table.stride(0) % 4 == 0 && tcol % 4 == 0 &&
+                    ((uintptr_t)x.data_ptr() & 15) == 0 && ((uintptr_t)out.data_ptr() & 7) == 0),
+              "table_gemm: 16-byte aligned operands");
+  check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, 1, x.stride(0), 0, out.stride(0), 0,
+                           x.size(0), N / 16, K / 32, nullptr, 0, nullptr, nullptr, 0, 0, 0, 4, (float)limit, (float)alpha,
+                           (float)cubic, (float)bias, nullptr, nullptr, 0, 0, 0, 0, nullptr, nullptr, 0, table.data_ptr(),
+                           ints(ids, x.size(0), "ids"), table.stride(0), (int)tcol, table.size(0), cur_stream()),
+           "table_gemm");
+}
+
 // rows sorted by group: x row = order[p] / x_div (x_div 0: p), out row = out_order ? order[p] : p; epi 1: the gated
-// unit, 2: the square of relu
+// unit, 2: the square of relu; row_w: weights of x's rows by order[p] (epi 1)
 void expert_gemm(at::Tensor x, at::Tensor w, at::Tensor out, at::Tensor tiles, at::Tensor n_tiles, at::Tensor order,
                  int64_t rows, int64_t x_div, bool out_order, int64_t tm, int64_t epi, double limit, double alpha,
-                 double bias, double cubic) {
+                 double bias, double cubic, Opt row_w) {
   const int f = is_f32(x, "x");
   check_rows(x, x.scalar_type(), "x");
   check_rows(out, x.scalar_type(), "out");
@@ -107,7 +135,8 @@ void expert_gemm(at::Tensor x, at::Tensor w, at::Tensor out, at::Tensor tiles, a
   check_rc(pa_grouped_gemm(f, x.data_ptr(), w.data_ptr(), out.data_ptr(), N * K, G, x.stride(0), 0, out.stride(0), 0, 0,
                            N / 16, K / 32, ints(tiles, 4, "tiles"), tiles.size(0), ints(n_tiles, 1, "n_tiles"),
                            ints(order, rows, "order"), x_div, out_order ? 1 : 0, tm, (int)epi, (float)limit,
-                           (float)alpha, (float)cubic, (float)bias, nullptr, nullptr, 0, 0, 0, 0, cur_stream()),
+                           (float)alpha, (float)cubic, (float)bias, nullptr, nullptr, 0, 0, 0, 0, opt_f32(row_w, rows, "row_w"),
+                           nullptr, 0, nullptr, nullptr, 0, 0, 0, cur_stream()),
            "expert_gemm");
 }
 

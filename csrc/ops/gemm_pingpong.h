@@ -441,11 +441,14 @@ __device__ __forceinline__ void pingpong_tile(const Args& A, const int bid, cons
   for (int j = 0; j < 4; ++j) {
     int m = row0 + wc * 64 + 16 * j + c;
     const bool ok = m < A.M;
-    if constexpr (GR)
+    float rs = 1.f;
+    if constexpr (GR) {
+      if constexpr (EPI == EP_GLU)
+        if (A.row_w && ok) rs = A.row_w[A.xmap[m]];
       if (A.ymap && ok) m = A.ymap[m];
+    }
     float sq = 0.f;
     if (ok) {
-      float rs = 1.f;
       if constexpr (NORM) rs = rsqrtf(A.ss_in[m] * inv_k + A.eps);
       if constexpr (pair_epi<EPI>()) {
 #pragma unroll

@@ -73,6 +73,7 @@ struct Args {
   const int* xmap = nullptr;
   const int* ymap = nullptr;
   int xdiv = 1;
+  const float* row_w = nullptr;  // by xmap: weight of x's row (gated pair)
   float limit = 0.f, alpha = 0.f, cubic = 0.f, bias = 0.f;
 };
 
@@ -726,8 +727,8 @@ extern "C" int pa_prefill_gemm(void* y, const void* x, const void* wp, const voi
 
 // Rows sorted by group (mixture-of-experts layers): tiles {group, first position, rows <= 256, 0}
 // on the ping-pong kernels, group g's packed weights at wp + g * wstride. x row of position p =
-// order[p] / x_div (x_div 0: p), y row = order[p] (out_order) or p. epi 0 plain, 5 gated
-// unit. K % 64 == 0, K >= 128, N % 128 == 0; y rows 16-byte aligned.
+// order[p] / x_div (x_div 0: p), times row_w[order[p]] if given; y row = order[p] (out_order) or p. epi 0 plain, 5
+// gated unit. K % 64 == 0, K >= 128, N % 128 == 0; y rows 16-byte aligned.
 namespace pa {
 namespace pf {
 template <int EPI, int F>
@@ -761,7 +762,7 @@ __global__ __launch_bounds__(512) void pingpong_grouped_kernel(Args A, const int
 extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long wstride, int N, int K, int ldx, int ldy,
                                const int* tiles, int max_tiles, const int* n_tiles, const int* order, int x_div,
                                int out_order, int epi, float limit, float alpha, float cubic, float bias,
-                               hipStream_t st) {
+                               const float* row_w, hipStream_t st) {
   using namespace pa::pf;
   if (K % 64 || K < 128 || N % 128 || ldx % 8 || ldy % 8 || (epi != EP_PLAIN && epi != EP_GLU && epi != EP_RELU2)) return -1;
   if (max_tiles <= 0) return 0;
@@ -773,6 +774,8 @@ extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long
   a.K = K;
   a.ldx = ldx;
   a.ldy = ldy;
+  if (row_w && !x_div) return -1;
+  a.row_w = row_w;
   a.limit = limit;
   a.alpha = alpha;
   a.cubic = cubic;

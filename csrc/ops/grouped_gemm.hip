@@ -12,12 +12,15 @@
 // rows share them; prompts with 256 rows and more per group run the ping-pong kernels instead
 // (gemm_prefill.hip pa_expert_tiles).
 //
-// Epilogues: plain, the gated unit of packed_epi.h (limit, alpha, cubic, bias), or the square of relu.
+// Epilogues: plain, the gated unit of packed_epi.h (limit, alpha, cubic, bias), or the square of relu; of dense rows
+// also the product times sigmoid(gate), and the gated unit whose second factor is the row's embedding in a table.
+// Sorted rows may have weights: the product is that of weight * x.
 #include "packed_epi.h"
 
 extern "C" int pa_expert_tiles(void* y, const void* x, const void* wp, long long wstride, int N, int K, int ldx, int ldy,
                                const int* tiles, int max_tiles, const int* n_tiles, const int* order, int x_div,
-                               int out_order, int epi, float limit, float alpha, float cubic, float bias, hipStream_t st);
+                               int out_order, int epi, float limit, float alpha, float cubic, float bias, const float* row_w,
+                               hipStream_t st);
 
 namespace pa {
 namespace gg {
@@ -41,6 +44,11 @@ struct Args {
   const float* cos_sin;
   int rskip, r, rp, rd;
   int wide;  // out rows and group offsets are multiples of 8 elements
+  const float* row_w;      // sorted, optional: by order[position], the weight of x's row
+  // dense, optional: gate [rows, ldg], columns as out's; table rows ids[row], its columns at tcol as out's
+  const void *gate, *table;
+  const int* ids;
+  int ldg, ldt, tcol, vocab;
 };
 
 // The rotated columns of `n` rows from `start` of group grp (one workgroup).
@@ -95,7 +103,19 @@ __device__ __forceinline__ float glu(float g, float u, const Args& A) {
   return pk::gated_unit(g, u, A.limit, A.alpha, A.cubic, A.bias);
 }
 
-enum { PLAIN = 0, GLU = 1, RELU2 = 2 };
+enum { PLAIN = 0, GLU = 1, RELU2 = 2, GATED = 3, TABLE = 4 };
+
+// where the second factor of a dense row's outputs lies (GATED, TABLE)
+template <typename T, int EPI>
+__device__ __forceinline__ const T* factor_row(const Args& A, int row, int grp) {
+  if constexpr (EPI == GATED) return (const T*)A.gate + (size_t)row * A.ldg + (size_t)grp * A.og;
+  return (const T*)A.table + (size_t)min(max(A.ids[row], 0), A.vocab - 1) * A.ldt + A.tcol;
+}
+template <int EPI>
+__device__ __forceinline__ float times(float a, float f, const Args& A) {
+  if constexpr (EPI == GATED) return a / (1.f + __expf(-f));
+  return glu(a, f, A);
+}
 
 template <int MT, int NT, int KU, int EPI>
 __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
@@ -173,13 +193,25 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
     const int orow = (A.tiles && A.out_order) ? A.order[pos[m]] : pos[m];
     bf16* o = (bf16*)A.out + (size_t)orow * A.ldo + (A.tiles ? 0 : (size_t)grp * A.og) + 4 * g;
     if constexpr (EPI == GLU) {
+      const float rw = A.row_w ? A.row_w[A.order[pos[m]]] : 1.f;
 #pragma unroll
       for (int i = 0; i + 1 < NT; i += 2) {
         if (nt0 + i >= A.N16) break;
         bf16x4 v;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = (bf16)glu(acc[m][i][j], acc[m][i + 1][j], A);
+        for (int j = 0; j < 4; ++j) v[j] = (bf16)glu(acc[m][i][j] * rw, acc[m][i + 1][j] * rw, A);
         *reinterpret_cast<bf16x4*>(o + (nt0 + i) * 8) = v;
+      }
+    } else if constexpr (EPI == GATED || EPI == TABLE) {
+      const bf16* f = factor_row<bf16, EPI>(A, pos[m], grp) + 4 * g;
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        if (nt0 + i >= A.N16) break;
+        const bf16x4 fv = *reinterpret_cast<const bf16x4*>(f + (nt0 + i) * 16);
+        bf16x4 v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = (bf16)times<EPI>(acc[m][i][j], (float)fv[j], A);
+        *reinterpret_cast<bf16x4*>(o + (nt0 + i) * 16) = v;
       }
     } else if (NT % 2 == 0 && A.N16 % 2 == 0 && A.wide) {
       // 16-byte stores: lanes of neighbouring lane groups trade halves
@@ -249,7 +281,14 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const Args A) {
   const int p = start + tm;
   const int orow = (A.tiles && A.out_order) ? A.order[p] : p;
   float* o = (float*)A.out + (size_t)orow * A.ldo + (A.tiles ? 0 : (size_t)grp * A.og) + bx * 16 + tn;
-  *o = PAIR ? glu(a0, a1, A) : EPI == RELU2 ? pk::relu2(a0) : a0;
+  if constexpr (PAIR) {
+    const float rw = A.row_w ? A.row_w[A.order[p]] : 1.f;
+    *o = glu(a0 * rw, a1 * rw, A);
+  } else if constexpr (EPI == GATED || EPI == TABLE) {
+    *o = times<EPI>(a0, factor_row<float, EPI>(A, p, grp)[bx * 16 + tn], A);
+  } else {
+    *o = EPI == RELU2 ? pk::relu2(a0) : a0;
+  }
 }
 
 // Routing by token id, for every expert layer of the model in one launch (workgroup = layer):
@@ -334,24 +373,29 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
                                int ldx, int xg, int ldo, int og, int rows, int N16, int K32, const int* tiles,
                                int max_tiles, const int* n_tiles, const int* order, int x_div, int out_order, int tm,
                                int epi, float limit, float alpha, float cubic, float bias, const int* positions,
-                               const float* cos_sin, int rskip, int r, int rp, int rd, hipStream_t st) {
+                               const float* cos_sin, int rskip, int r, int rp, int rd, const float* row_w, const void* gate,
+                               int ldg, const void* table, const int* ids, int ldt, int tcol, int vocab, hipStream_t st) {
   if (N16 <= 0 || K32 <= 0 || (epi == 1 && N16 % 2)) return -1;
+  if (row_w && (!tiles || epi != 1 || !x_div)) return -1;
+  if (tiles ? epi > 2 : (epi == 3 && !gate) || (epi == 4 && (!table || !ids))) return -1;
   if (tiles ? max_tiles <= 0 : rows <= 0) return 0;
   const pa::gg::Args A{x, w, out, wstride, ldx, xg, ldo, og, rows, N16, K32, (const int4*)tiles, n_tiles,
                        order, x_div, out_order, limit, alpha, cubic, bias, positions, cos_sin, rskip, r, rp, rd,
-                       ldo % 8 == 0 && og % 8 == 0 && ((uintptr_t)out & 15) == 0};
+                       ldo % 8 == 0 && og % 8 == 0 && ((uintptr_t)out & 15) == 0, row_w, gate, table, ids, ldg, ldt, tcol, vocab};
   const int rot = rp > 0 ? 1 : 0;  // one more column of workgroups
   if (fp32) {
     if (tiles && tm != 16) return -2;
     const dim3 grid((epi == 1 ? N16 / 2 : N16) + rot, tiles ? max_tiles : (rows + 15) / 16, tiles ? 1 : groups);
     if (epi == 1) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<pa::gg::GLU>), grid, dim3(256), 0, st, A);
     else if (epi == 2) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<pa::gg::RELU2>), grid, dim3(256), 0, st, A);
+    else if (epi == 3) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<pa::gg::GATED>), grid, dim3(256), 0, st, A);
+    else if (epi == 4) hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<pa::gg::TABLE>), grid, dim3(256), 0, st, A);
     else hipLaunchKernelGGL((pa::gg::gemm_f32_kernel<pa::gg::PLAIN>), grid, dim3(256), 0, st, A);
     return (int)hipGetLastError();
   }
   if (tiles && tm == 256)
     return pa_expert_tiles(out, x, w, wstride, N16 * 16, K32 * 32, ldx, ldo, tiles, max_tiles, n_tiles, order, x_div,
-                           out_order, epi == 1 ? pa::pk::EP_GLU : epi == 2 ? pa::pk::EP_RELU2 : pa::pk::EP_PLAIN, limit, alpha, cubic, bias, st);
+                           out_order, epi == 1 ? pa::pk::EP_GLU : epi == 2 ? pa::pk::EP_RELU2 : pa::pk::EP_PLAIN, limit, alpha, cubic, bias, row_w, st);
   // dense: 64-row tiles once they fill the chip
   if (!tiles) tm = (N16 + 15) / 16 * ((rows + 63) / 64) * groups < 256 ? 16 : 64;
   if (tm != 16 && tm != 64) return -2;
@@ -369,10 +413,14 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
   if (tm == 16) {
     if (epi == 1) PA_GGK(1, 2, pa::gg::GLU);
     else if (epi == 2) PA_GGK(1, 1, pa::gg::RELU2);
+    else if (epi == 3) PA_GGK(1, 1, pa::gg::GATED);
+    else if (epi == 4) PA_GGK(1, 1, pa::gg::TABLE);
     else PA_GGK(1, 1, pa::gg::PLAIN);
   } else {
     if (epi == 1) PA_GG(4, 4, 1, pa::gg::GLU);
     else if (epi == 2) PA_GG(4, 4, 1, pa::gg::RELU2);
+    else if (epi == 3) PA_GG(4, 4, 1, pa::gg::GATED);
+    else if (epi == 4) PA_GG(4, 4, 1, pa::gg::TABLE);
     else PA_GG(4, 4, 1, pa::gg::PLAIN);
   }
 #undef PA_GGK

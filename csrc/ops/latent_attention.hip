@@ -2,7 +2,7 @@
 // rows and mixed batches in one launch.
 //
 // The cache holds one row per token for all heads: [latent c (Rp) | rotated key part (rp)],
-// D = Rp + rp, pages of 16 tokens, fragment-major [D/8][16][8] (latent_cache.hip). With
+// D = Rp + rp (rp 0: a latent without positions), pages of 16 tokens, fragment-major [D/8][16][8] (latent_cache.hip). With
 //   q~_h = [W_uk,h^T q_h | rot(q_h)]          (absorbed before the launch)
 //   score_h(i, j) = q~_h(i) . row(j) * scale,  o~_h(i) = sum_j softmax_j score * c(j)
 // every head reads the same rows: keys are the whole row, values its first Rp dims, and the
@@ -554,7 +554,7 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
   pa::la::Args A{out, part_o, part_ml, q, pages, (const int4*)items, n_items, q_start, q_len, ctx_len,
                  block_table, max_blocks, H, NB, Rp, D, dec_tokens, window, scale_log2};
   const int RT = Rp / 32, PT = rp / 32;
-  if (!fp32 && !simple && PT >= 1 && PT <= 2) {
+  if (!fp32 && !simple && PT <= 2) {
 #define PA_LA(R, P)                                                                                           \
   do {                                                                                                        \
     constexpr int CT = 1;                                                                                     \
@@ -573,7 +573,7 @@ extern "C" int pa_latent_attention(int fp32, void* out, float* part_o, float* pa
     return (int)hipGetLastError();                                                                            \
   } while (0)
     switch (RT) {
-#define PA_X(N) case N: if (PT == 1) PA_LA(N, 1); else PA_LA(N, 2); break;
+#define PA_X(N) case N: if (PT == 0) PA_LA(N, 0); else if (PT == 1) PA_LA(N, 1); else PA_LA(N, 2); break;
       PA_LA_RT(PA_X)
 #undef PA_X
       default: break;

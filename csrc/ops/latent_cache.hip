@@ -1,9 +1,9 @@
 // Latent attention's down-projection output -> normed query latent + paged latent cache.
 //
 // Input row t: [query latent (NQ) | key-value latent (R) | shared key part (r)] of one projection.
-//   cq[t]        = norm(query latent) * w_q                      (columns NQ .. ldq zero)
+//   cq[t]        = norm(query latent) * w_q                      (columns NQ .. ldq zero; NQ 0: none)
 //   page[slot]   = norm(kv latent) * w_c, dims 0 .. R
-//                  rotate-half of the key part by the token's position, dims Rp .. Rp + r
+//                  rotate-half of the key part by the token's position, dims Rp .. Rp + r (r 0: none)
 // The page layout is fragment-major like the K pages of rope_cache.hip: [D/8][16 keys][8 dims],
 // D = Rp + rp, with R and r padded to whole MFMA chunks; the padding is written as zeros, so a
 // page needs no initialisation. One copy serves as keys and as values (latent_attention.hip).
@@ -29,7 +29,7 @@ __global__ __launch_bounds__(256) void latent_cache_kernel(
     const float v = (float)row[NQ + i];
     sc += v * v;
   }
-  const float iq = 1.f / sqrtf(block_sum<4>(sq, red) / (float)NQ + eps);
+  const float iq = 1.f / sqrtf(block_sum<4>(sq, red) / (float)max(NQ, 1) + eps);
   const float ic = 1.f / sqrtf(block_sum<4>(sc, red) / (float)R + eps);
   T* q = cq + (size_t)t * ldq;
   for (int i = threadIdx.x; i < ldq; i += 256) q[i] = i < NQ ? (T)((float)row[i] * iq * w_q[i]) : (T)0.f;
@@ -87,7 +87,7 @@ __global__ __launch_bounds__(256) void latent_cache_wave_kernel(
     if (i < NQ) sq += e;
     else sc += e;
   }
-  const float iq = 1.f / sqrtf(wave_sum(sq) / (float)NQ + eps);
+  const float iq = 1.f / sqrtf(wave_sum(sq) / (float)max(NQ, 1) + eps);
   const float ic = 1.f / sqrtf(wave_sum(sc) / (float)R + eps);
   T* q = cq + (size_t)t * ldq;
   for (int i = lane * 8; i < ldq; i += 512) {

@@ -1,6 +1,6 @@
 """In-tree builder for the native parts of pilottai_amd.
 
-Four shared objects are produced next to the Python sources so they travel with
+Five shared objects are produced next to the Python sources so they travel with
 the repository snapshot to the GPU box:
 
 * ``pilottai_amd/_C.so``       — CDNA4 HIP kernels (csrc/ops/*.hip, gfx950 only)
@@ -10,6 +10,7 @@ the repository snapshot to the GPU box:
                                   such a model needs no other kernel to run)
 * ``pilottai_amd/_hybrid.so`` — likewise for models with paged attention of many kinds, recurrent layers,
                                   score-routed experts and fp32 residuals
+* ``pilottai_amd/_latent_linear.so`` — likewise for models that mix latent attention with gated linear attention
 * ``pilottai_amd/_runtime.so`` — C++ serving runtime: paged-KV block manager,
                                   prefix cache, continuous-batching scheduler,
                                   grammar FSM + tokenizer (csrc/runtime/*.cpp),
@@ -44,8 +45,10 @@ HIP_FLAGS = ["-ffast-math", "-fno-gpu-rdc", "-Wno-unused-result", "-Xclang", "-t
 SHARED_HIP = ["gemm_decode.hip", "gemm_prefill.hip"]
 MODULES = {
     "latent": (["grouped_gemm.hip", "latent_attention.hip", "latent_cache.hip", "residual_norm.hip"], "bindings_latent.cpp"),
-    "hybrid": (["grouped_gemm.hip", "head_difference.hip", "hyper_norm.hip", "matrix_memory.hip", "paged_kv.hip",
+    "hybrid": (["gated_norm.hip", "grouped_gemm.hip", "head_difference.hip", "hyper_norm.hip", "matrix_memory.hip", "paged_kv.hip",
                 "score_route.hip", "state_scan.hip", "window_attention.hip"], "bindings_hybrid.cpp"),
+    "latent_linear": (["gated_norm.hip", "grouped_gemm.hip", "latent_attention.hip", "latent_cache.hip", "linear_attention.hip",
+                       "poly_norm.hip", "residual_norm.hip", "score_route.hip"], "bindings_latent_linear.cpp"),
 }
 FAMILY_HIP = {h for hips, _ in MODULES.values() for h in hips}
 FILE_FLAGS = {"gemm_mid.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"],
@@ -172,7 +175,7 @@ def _stale(so: Path, sources) -> bool:
 
 def ensure(kind: str, gpu: bool = True) -> None:
     """Build what running a model of `kind` needs, where it is missing or older than its sources: the
-    serving runtime and, for a GPU, the kernel module (_latent, _hybrid, or _C for "llama"). One process
+    serving runtime and, for a GPU, the kernel module (one of MODULES, or _C for "llama"). One process
     builds at a time; the others wait for it."""
     import fcntl
 

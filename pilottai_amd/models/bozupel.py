@@ -38,26 +38,13 @@ import torch
 from pilottai_amd import ops
 from pilottai_amd.models.cache import LatentKVCache, StepMeta
 from pilottai_amd.models.common import PackedLinear, checkpoint_reader, expert_tile_rows, layer_runs, parse_loop
-from pilottai_amd.ops import reference as ref
-from pilottai_amd.ops.latent import latent_pad, pad_to
+from pilottai_amd.models.hybrid import AttentionRoom, MixerBlock
+from pilottai_amd.models.latent import LatentAttention, LatentAttentionSpec
+from pilottai_amd.ops.latent import pad_to
 from pilottai_amd.parallel.comm import TPGroup
 
 GLU_ALPHA = 1.702  # the gated unit g * sigmoid(alpha g) * (u + bias)
 GLU_BIAS = 1.0
-
-
-@dataclass(frozen=True)
-class LatentAttentionSpec:
-    heads: int
-    dim: int          # unrotated query / key dimensions per head
-    rot_dim: int      # rotated dimensions per head (one key part shared by all heads)
-    vdim: int
-    q_rank: int
-    kv_rank: int
-    scale: float
-    rot_base: float
-    rot_dims: int     # rotated dimensions of rot_dim (rotate-half pairs)
-    window: int = 0   # keys a position sees, itself included; 0: all before it
 
 
 @dataclass(frozen=True)
@@ -102,13 +89,14 @@ class BozupelConfig:
             if L.get("type") != "latent_attention":
                 raise ValueError(f"layer {i}: unknown mixer {L.get('type')!r}")
             m = L["mixer"]
-            mixer = LatentAttentionSpec(
-                heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
-                q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]), scale=float(m["scale"]),
-                rot_base=float(m["rot"]["base"]), rot_dims=int(m["rot"].get("dims", m["rot_dim"])),
-                window=int((m.get("mask") or {}).get("size") or 0))
-            if mixer.rot_dims > mixer.rot_dim or mixer.rot_dims % 2:
-                raise ValueError(f"layer {i}: {mixer.rot_dims} rotated of {mixer.rot_dim} dimensions")
+            try:
+                mixer = LatentAttentionSpec(
+                    heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                    q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]), scale=float(m["scale"]),
+                    rot_base=float(m["rot"]["base"]), rot_dims=int(m["rot"].get("dims", m["rot_dim"])),
+                    window=int((m.get("mask") or {}).get("size") or 0))
+            except ValueError as e:
+                raise ValueError(f"layer {i}: {e}") from None
             p, mlp = L.get("mlp"), None
             if p is not None:
                 if p.get("kind") != "moe":
@@ -153,59 +141,6 @@ PRESETS: Dict[str, BozupelConfig] = {
                                                  scale=192 ** -0.5, rot_base=10000.0, rot_dims=64, window=4096),
                              TableExpertsSpec(experts=64, top=6, ff=2048, limit=7.0)),
 }
-
-
-class LatentAttention:
-    """Latent attention over the paged latent cache, queries absorbed into the latent space."""
-
-    def __init__(self, spec: LatentAttentionSpec, t: Dict[str, torch.Tensor], eps: float, dtype, device, cos_sin):
-        m = self.spec = spec
-        self.eps, self.dtype, self.device, self.cos_sin = eps, dtype, device, cos_sin
-        H, n, r, vd, R = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank
-        self.np, self.rp, self.vp = pad_to(n, 32), pad_to(r, 32), pad_to(vd, 16)
-        self.Rp = latent_pad(R)
-        self.D = self.Rp + self.rp
-        self.down = PackedLinear(torch.cat([t["dq"], t["dkv"]], 0), dtype, device)
-        self.w_q = t["dq.norm"].float().to(device)
-        self.w_c = t["dkv.norm"].float().to(device)
-        q = t["uq"].view(H, n + r, m.q_rank)
-        uq = torch.zeros(H, self.np + self.rp, m.q_rank, dtype=q.dtype, device=q.device)
-        uq[:, :n], uq[:, self.np:self.np + r] = q[:, :n], q[:, n:]
-        self.uq = PackedLinear(uq.view(-1, m.q_rank), dtype, device)
-        uk = torch.zeros(H, self.Rp, self.np, dtype=dtype, device=device)
-        uk[:, :R, :n] = t["uk"].to(device).view(H, n, R).transpose(1, 2)
-        self.uk = ops.pack_groups(uk, dtype)
-        uv = torch.zeros(H, self.vp, self.Rp, dtype=dtype, device=device)
-        uv[:, :vd, :R] = t["uv"].to(device).view(H, vd, R)
-        self.uv = ops.pack_groups(uv, dtype)
-        d = t["o"].shape[0]
-        o = torch.zeros(d, H, self.vp, dtype=t["o"].dtype, device=t["o"].device)
-        o[:, :, :vd] = t["o"].view(d, H, vd)
-        self.o = PackedLinear(o.view(d, -1), dtype, device)
-
-    def tensors(self):
-        return [self.down.w, self.uq.w, self.uk, self.uv, self.o.w]
-
-    def __call__(self, h, meta: StepMeta, pages, part_o, part_ml, dec_tokens: int, tile_tokens: int) -> torch.Tensor:
-        m, T, H = self.spec, h.shape[0], self.spec.heads
-        new = lambda *s: torch.empty(*s, dtype=self.dtype, device=self.device)  # noqa: E731
-        a = self.down(h)
-        cq = new(T, self.uq.K)
-        ops.latent_cache(a, m.q_rank, m.kv_rank, m.rot_dim, self.w_q, self.w_c, cq, pages, self.Rp, meta.positions,
-                         meta.slots, self.cos_sin, self.eps)
-        q = self.uq(cq)
-        qa = new(T, H, self.D)
-        ops.head_gemm(q, self.np + self.rp, self.uk, qa.view(T, -1), self.D,
-                      rot=(meta.positions, self.cos_sin, self.np, m.rot_dim, self.rp))
-        oc = new(T, H, self.Rp)
-        ops.latent_attention(oc, part_o, part_ml, qa, pages, meta.items, meta.n_items, meta.q_start,
-                             meta.q_len, meta.ctx_len, meta.block_table, m.scale, m.window, dec_tokens, tile_tokens,
-                             num_seqs=meta.num_seqs)
-        v = new(T, self.o.K)
-        if self.o.K > H * self.vp:
-            v[:, H * self.vp:] = 0
-        ops.head_gemm(oc.view(T, -1), self.Rp, self.uv, v, self.vp)
-        return self.o(v)
 
 
 class TableExperts:
@@ -279,13 +214,11 @@ class BozupelModel:
             m, p, pre = L.mixer, L.mlp, f"l{i}."
             key = (m.rot_dims, m.rot_base)
             if key not in rot:
-                rot[key] = ref.rope_cos_sin(self.max_len, m.rot_dims, m.rot_base).to(self.device)
-            shapes = {"dq": (m.q_rank, d), "dq.norm": (m.q_rank,), "uq": (m.heads * (m.dim + m.rot_dim), m.q_rank),
-                      "dkv": (m.kv_rank + m.rot_dim, d), "dkv.norm": (m.kv_rank,), "uk": (m.heads * m.dim, m.kv_rank),
-                      "uv": (m.heads * m.vdim, m.kv_rank), "o": (d, m.heads * m.vdim)}
-            layer = {"norm1": f32(pre + "norm1"), "norm1b": f32(pre + "norm1b"),
-                     "attn": LatentAttention(m, {k: get(f"{pre}mix.{k}", s) for k, s in shapes.items()}, eps, dtype,
-                                             self.device, rot[key]), "mlp": None}
+                rot[key] = m.angles(self.max_len).to(self.device)
+            attn = LatentAttention(m, {k: get(f"{pre}mix.{k}", s) for k, s in m.shapes(d).items()}, eps, dtype,
+                                   self.device, rot[key])
+            layer = {"norm1": f32(pre + "norm1"), "norm1b": f32(pre + "norm1b"), "mlp": None,
+                     "attn": attn, "block": MixerBlock([attn], dtype, self.device)}
             if p is not None:
                 layer["norm2"], layer["norm2b"] = f32(pre + "norm2"), f32(pre + "norm2b")
                 w = {}
@@ -328,7 +261,7 @@ class BozupelModel:
     def weight_bytes(self) -> int:
         ts = [self.embed, self.head.w]
         for L in self.layers:
-            ts += L["attn"].tensors() + (L["mlp"].tensors() if L["mlp"] else [])
+            ts += L["block"].tensors() + (L["mlp"].tensors() if L["mlp"] else [])
         return sum(t.numel() * t.element_size() for t in ts)
 
     # -- what the engine asks of every model ----------------------------------------
@@ -353,8 +286,9 @@ class BozupelModel:
 
     def attention_workspace(self, max_items: int) -> tuple:
         """(partial outputs, partial (max, sum) pairs) in floats, and tickets per sequence (none)."""
-        nb = [(self.dec_tokens * L["attn"].spec.heads + 15) // 16 for L in self.layers]
-        o = max(b * 16 * L["attn"].Rp for b, L in zip(nb, self.layers))
+        mixers = [L.mixer for L in self.cfg.layers]
+        nb = [(self.dec_tokens * m.heads + 15) // 16 for m in mixers]
+        o = max(b * 16 * m.out_width for b, m in zip(nb, mixers))
         return max_items * o, max_items * max(nb) * 32, 1
 
     def health_words(self) -> list:
@@ -400,11 +334,12 @@ class BozupelModel:
         new_h = lambda n=T: torch.empty(n, ldh, dtype=self.dtype, device=dev)  # noqa: E731
         rows = meta.logit_rows[:num_logit_rows]
         routes = self._route(meta, T)
+        room = AttentionRoom(part_o, part_ml, self.dec_tokens, self.tile_tokens, 0)
         resid = torch.empty(T, d, dtype=torch.float32, device=dev)
         h = ops.residual_norm(resid, eps, emb=self.embed, ids=ids, w_next=self.layers[self.runs[0][0]]["norm1"], out=new_h())
         for j, (i, _) in enumerate(self.runs):
             L = self.layers[i]
-            y = L["attn"](h, meta, kv.pages[j], part_o, part_ml, self.dec_tokens, self.tile_tokens)
+            y, *_ = L["block"](h, meta, [(kv.pages[j],)], room)
             post, k = L["norm1b"], 1
             if L["mlp"] is not None:
                 h = ops.residual_norm(resid, eps, y=y, w_post=post, w_next=L["norm2"], out=new_h())

@@ -7,9 +7,9 @@ manager (csrc/runtime) know nothing of what a page holds:
   LatentKVCache  one latent row per token for all heads (latent attention), one pool per layer RUN:
                  a layer that a looped stack runs several times has a pool for each pass, and
                  layers of different widths have pools of their own widths
-  HybridCache    per layer run, per-head keys and values with their pooled blocks, or the state slots
-                 of a recurrent layer, which belong to sequences (the scheduler hands them out) and
-                 not to pages
+  HybridCache    per layer run, per-head keys and values with their pooled blocks, latent rows (a run may
+                 read another's), or the state slots of a recurrent layer, which belong to sequences
+                 (the scheduler hands them out) and not to pages
 """
 from __future__ import annotations
 
@@ -86,8 +86,9 @@ class HybridCache:
     8], values alike, pooled keys [blocks, per page, G, DK], pooled values): a pooled block lies with the page of
     its last token (csrc/ops/paged_kv.hip); several key heads may share a value head. A state space has (state
     fp32 [slots, H, V, N], ring of the convolution's inputs [slots, rows, channels]), a matrix memory (state fp32
-    [slots, H, V, N], its running maximum at every row [slots, H, V]); a sequence that starts overwrites what its
-    slot held."""
+    [slots, H, V, N], its running maximum at every row [slots, H, V]), linear attention (state fp32 [slots, H, V, N]); a
+    sequence that starts overwrites what its slot held. Latent attention has (rows [blocks, D/8, 16, 8],), as LatentKVCache;
+    ("same", j) is the entry of run j."""
 
     def __init__(self, kinds: Sequence[Sequence[tuple]], num_blocks: int, slots: int, device, dtype=torch.bfloat16,
                  block_size: int = 16):
@@ -97,25 +98,35 @@ class HybridCache:
         zeros = lambda dt, *s: torch.zeros(*s, dtype=dt, device=device)  # noqa: E731
 
         def pools(kind, *n):
+            if kind == "same":
+                return self.layers[n[0]][0]
+            if kind == "latent":
+                return zeros(dtype, num_blocks, n[0] // 8, 16, 8),
             if kind == "attention":
                 G, dk, dv, per, gv = n
                 return (zeros(dtype, num_blocks, G, dk // 8, 16, 8), zeros(dtype, num_blocks, gv, dv // 8, 16, 8),
                         zeros(dtype, num_blocks if per else 0, per, G, dk), zeros(dtype, num_blocks if per else 0, per, gv, dv))
             H, V, N = n[:3]
             state = zeros(torch.float32, slots, H, V, N)
+            if kind == "linear":
+                return state,
             return state, zeros(torch.float32, slots, H, V) if kind == "memory" else zeros(dtype, slots, *n[3:])
-        self.layers: List[List[tuple]] = [[pools(*k) for k in run] for run in kinds]
+        self.layers: List[List[tuple]] = []
+        for run in kinds:
+            self.layers.append([pools(*k) for k in run])
 
     @staticmethod
     def bytes_per_block(kinds: Sequence[Sequence[tuple]], itemsize: int, block_size: int = 16) -> int:
-        return sum((n[0] * n[1] + n[4] * n[2]) * (block_size + n[3]) * itemsize
-                   for run in kinds for kind, *n in run if kind == "attention")
+        each = {"attention": lambda G, dk, dv, per, gv: (G * dk + gv * dv) * (block_size + per),
+                "latent": lambda D: D * block_size}
+        return itemsize * sum(each[kind](*n) for run in kinds for kind, *n in run if kind in each)
 
     @staticmethod
     def bytes_per_slot(kinds: Sequence[Sequence[tuple]], itemsize: int) -> int:
-        each = {"attention": lambda *n: 0, "state": lambda H, V, N, rows, ch: 4 * H * V * N + rows * ch * itemsize,
-                "memory": lambda H, V, N: 4 * H * V * (N + 1)}
-        return sum(each[kind](*n) for run in kinds for kind, *n in run)
+        each = {"state": lambda H, V, N, rows, ch: 4 * H * V * N + rows * ch * itemsize,
+                "memory": lambda H, V, N: 4 * H * V * (N + 1), "linear": lambda H, V, N: 4 * H * V * N}
+        return sum(each[kind](*n) for run in kinds for kind, *n in run if kind in each)
 
     def nbytes(self) -> int:
-        return sum(t.numel() * t.element_size() for run in self.layers for ts in run for t in ts)
+        pools = {id(t): t for run in self.layers for ts in run for t in ts}
+        return sum(t.numel() * t.element_size() for t in pools.values())

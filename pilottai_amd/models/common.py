@@ -30,8 +30,16 @@ class PackedLinear:
         return ops.prefill_gemm(x, self.w)
 
 
+def pad_heads(w: torch.Tensor, padded: int) -> torch.Tensor:
+    """[heads, size, k] -> [heads, padded, k], zeros behind every head."""
+    out = w.new_zeros(w.shape[0], padded, w.shape[2])
+    out[:, :w.shape[1]] = w
+    return out
+
+
 def checkpoint_reader(path: str) -> Callable:
-    """get(name, shape) over a folder's *.safetensors, checking that the tensor is there and has the shape."""
+    """get(name, shape) over a folder's *.safetensors, checking that the tensor is there and has the shape; get.shape(name)
+    for a size that no configuration gives."""
     from safetensors import safe_open
 
     where = {}
@@ -40,13 +48,17 @@ def checkpoint_reader(path: str) -> Callable:
             fh = safe_open(os.path.join(path, f), framework="pt")
             where.update({k: fh for k in fh.keys()})
 
-    def get(name, shape):
+    def file(name):
         if name not in where:
             raise ValueError(f"{path}: tensor {name!r} is missing")
-        t = where[name].get_tensor(name)
+        return where[name]
+
+    def get(name, shape):
+        t = file(name).get_tensor(name)
         if tuple(t.shape) != tuple(shape):
             raise ValueError(f"{path}: {name} has shape {tuple(t.shape)}, the configuration gives {tuple(shape)}")
         return t
+    get.shape = lambda name: tuple(file(name).get_slice(name).get_shape())
     return get
 
 

@@ -1,11 +1,11 @@
 """Sublayers of hybrid decoders: attention over paged keys and values, recurrent layers (Mamba-2, matrix
-memory), gated feed-forwards and score-routed experts, on the engine's pages, state slots and packed projections;
-and what the models made of them have in common.
+memory, gated linear attention), dense feed-forwards and score-routed experts, on the engine's pages, state slots and packed
+projections; and what the models made of them have in common.
 
 Every class takes its sizes and constants from a spec, its weights by short names, and pads every
 dimension with zero rows and columns to whole MFMA tiles at load, so any sizes run on the same kernels.
 
-A mixer (PagedAttention, StateSpace, MatrixMemory) reads its columns of a projection of the normed input and writes
+A mixer (PagedAttention, StateSpace, MatrixMemory, LinearAttention; models/latent.py LatentAttention) reads its columns of a projection of the normed input and writes
 columns that an output matrix takes: `rows` and `w_out` are its parts of those two matrices. A MixerBlock holds
 them for one mixer or several side by side, and, where a feed-forward reads the same input, for that one's
 second matrix too: one projection, one output product. Blocks and feed-forwards return (y, partials, weights,
@@ -89,6 +89,10 @@ class AttentionSpec:
     def rotation(self) -> tuple:
         return self.rot_dims, self.rot_base, self.yarn, self.slow_waves
 
+    @property
+    def out_width(self) -> int:
+        return ops.window_pad(self.dim, self.vdim)[1]
+
     def angles(self, max_len: int) -> torch.Tensor:
         named = lambda v, k: dict(zip(k, v)) if v else None  # noqa: E731
         return ops.angle_table(max_len, self.rot_dims, self.rot_base, named(self.yarn, ("factor", "original", "fast", "slow")),
@@ -159,6 +163,38 @@ class MatrixMemorySpec:
 
 
 @dataclass(frozen=True)
+class LinearAttentionSpec:
+    heads: int
+    dim: int
+    vdim: int
+    tau: float  # decays are sigmoid(z)^(1 / tau)
+    rank: int = 16  # of the map from the input to z
+
+    def __post_init__(self):
+        if self.tau <= 0:
+            raise ValueError(f"decays with tau {self.tau}")
+
+    @property
+    def padded(self) -> Tuple[int, int, int]:
+        """Widths of a key, a value and the decays' low-rank input."""
+        return pad_to(self.dim, 32), pad_to(self.vdim, 16), pad_to(self.rank, 32)
+
+    def shapes(self, d: int) -> Dict[str, tuple]:
+        N, V = self.heads * self.dim, self.heads * self.vdim
+        return {"q": (N, d), "k": (N, d), "v": (V, d), "g": (V, d), "o": (d, V), "norm": (self.vdim,), "a1": (self.rank, d),
+                "a2": (N, self.rank), "a2.b": (N,)}
+
+
+@dataclass(frozen=True)
+class PolySpec:
+    """A feed-forward without a gate whose activation is the polynomial norm of the token's vector."""
+    ff: int
+
+    def shapes(self, d: int) -> Dict[str, tuple]:
+        return {"up": (self.ff, d), "down": (d, self.ff), "act": (4,)}
+
+
+@dataclass(frozen=True)
 class DenseSpec:
     ff: int
     act: tuple = GELU_TANH
@@ -180,11 +216,14 @@ class ScoredExpertsSpec:
     correction: bool = False  # the choice is by score + tensor 'correction'
     share: bool = False  # weights: the chosen scores divided by their sum
     scale: float = 1.0   # of the weights
+    weigh_input: bool = False  # an expert's weight multiplies its input; else its output
 
     def __post_init__(self):
         if self.experts % self.groups or not 1 <= self.keep <= self.groups or \
                 not 1 <= self.top <= self.keep * (self.experts // self.groups):
             raise ValueError(f"{self.top} of {self.experts} experts from {self.keep} of {self.groups} groups")
+        if self.weigh_input and self.act is None:
+            raise ValueError("weights on the input of experts without a gate")
 
     @property
     def always(self) -> int:  # the shared expert, in pieces of the routed experts' width
@@ -362,7 +401,41 @@ class MatrixMemory:
                           meta.state_slot, meta.scan_items, meta.n_scan, self.cols, m.vdim, m.cap, m.dim ** -0.5,
                           num_seqs=meta.num_seqs)
         ops.gated_norm(out, x[:, self.g_col:], self.w_norm, meta.slots, m.heads, m.vdim, self.cols[4], m.heads, self.eps,
-                       div=div, after=True)
+                       div=div, after="sigmoid")
+
+
+class LinearAttention:
+    """Gated linear attention: an outer-product state per head whose key channels decay each by itself, its output normed
+    per head and gated. Projection rows [q | k | v | gate | low-rank inputs of the decays]."""
+
+    def __init__(self, spec: LinearAttentionSpec, t: Dict[str, torch.Tensor], eps: float, dtype, device):
+        m = self.spec = spec
+        self.eps, self.dtype, self.device = eps, dtype, device
+        H, (np_, vp, rp) = m.heads, m.padded
+        self.rows = torch.cat([_heads(t["q"], H, m.dim, np_), _heads(t["k"], H, m.dim, np_), _heads(t["v"], H, m.vdim, vp),
+                               _heads(t["g"], H, m.vdim, vp), t["a1"], t["a1"].new_zeros(rp - m.rank, t["a1"].shape[1])])
+        self.g_col = 2 * H * np_ + H * vp
+        self.cols = (0, H * np_, 2 * H * np_, self.g_col + H * vp)
+        self.a2 = torch.zeros(H * np_, rp, dtype=dtype, device=device)
+        self.a2[:, :m.rank] = _heads(t["a2"], H, m.dim, np_).to(device)
+        f32 = lambda x: x.float().to(device).contiguous()  # noqa: E731
+        self.bias, self.w_norm = f32(_heads(t["a2.b"], H, m.dim, np_)), f32(t["norm"].repeat(H))
+        self.w_out, self.out_bias, self.width = _heads(t["o"].T.contiguous(), H, m.vdim, vp).T, None, H * vp
+
+    def tensors(self):
+        return [self.a2]
+
+    def cache_kind(self) -> tuple:
+        np_, vp, _ = self.spec.padded
+        return ("linear", self.spec.heads, vp, np_)
+
+    def __call__(self, x, out, meta: StepMeta, cache, room):
+        m = self.spec
+        state, = cache
+        ops.linear_attention(x, out, state, self.a2, self.bias, meta.q_start, meta.q_len, meta.ctx_len, meta.state_slot,
+                             meta.scan_items, meta.n_scan, self.cols, m.dim ** -0.5, 1.0 / m.tau, num_seqs=meta.num_seqs)
+        ops.gated_norm(out, x[:, self.g_col:], self.w_norm, meta.slots, m.heads, m.vdim, m.padded[1], m.heads, self.eps,
+                       after="silu")
 
 
 class MixerBlock:
@@ -397,7 +470,8 @@ class MixerBlock:
             m.rows = m.w_out = None  # (packed here)
 
     def tensors(self):
-        return [self.proj.w, self.o.w] + (self.mlp.tensors() if self.mlp else [])
+        own = [t for m in self.mixers if hasattr(m, "tensors") for t in m.tensors()]
+        return [self.proj.w, self.o.w] + own + (self.mlp.tensors() if self.mlp else [])
 
     def __call__(self, h, meta: StepMeta, caches, room: AttentionRoom, side: Optional[SideStreams] = None):
         """`side`: streams 1 .. for the mixers behind the first, 0 for the feed-forward."""
@@ -459,6 +533,22 @@ class GatedMLP:
         return self.down(act), 1, None, None
 
 
+class PolyMLP:
+    """down(polynomial norm(up h))."""
+
+    def __init__(self, spec: PolySpec, t: Dict[str, torch.Tensor], eps: float, dtype, device):
+        self.spec, self.eps = spec, eps
+        self.up, self.down = PackedLinear(t["up"], dtype, device), PackedLinear(t["down"], dtype, device)
+        self.act = t["act"].float().to(device).contiguous()
+
+    def tensors(self):
+        return [self.up.w, self.down.w]
+
+    def __call__(self, h, meta: StepMeta):
+        z = self.up(h)[:, :self.down.K]
+        return self.down(ops.poly_norm(z, self.spec.ff, self.act, self.eps)), 1, None, None
+
+
 class ScoredExperts:
     """Experts chosen by the scores of a router, and a shared expert whose pieces are further experts that
     every token uses; one partial output per (token, expert) with its weight."""
@@ -510,10 +600,10 @@ class ScoredExperts:
                         s.groups, s.keep, s.always, tm, softmax=s.softmax, correction=self.correction, share=s.share, scale=s.scale)
         act = torch.empty(rows, self.fp, dtype=self.dtype, device=dev)
         ops.expert_gemm(h, self.w13, act, tiles, n_tiles, order, rows, x_div=K, out_order=False, tm=tm, glu=s.act,
-                        relu2=s.act is None)
+                        relu2=s.act is None, row_w=weights if s.weigh_input else None)
         y = torch.empty(rows, self.dn, dtype=self.dtype, device=dev)
         ops.expert_gemm(act, self.w2, y, tiles, n_tiles, order, rows, x_div=0, out_order=True, tm=tm)
-        return y, K, weights, None
+        return y, K, None if s.weigh_input else weights, None
 
 
 class HybridModel:
@@ -538,6 +628,8 @@ class HybridModel:
             raise ValueError(f"{self.NAME} models run on one GPU: tensor parallelism is not implemented for them")
         if dtype not in (torch.bfloat16, torch.float32):
             raise ValueError(f"unsupported dtype {dtype}")
+        if self.device.type == "cuda":  # (operations that several modules hold come from the one that is loaded)
+            ops.require_family(self.KERNELS)
         self.v_local, self.vocab_offset = cfg.vocab_size, 0
         self.attention = list(attention)
         self._group = min(max([m.group for m in self.attention], default=1), 16)
@@ -605,7 +697,7 @@ class HybridModel:
         o = ml = 1
         for m in self.attention:
             n = max_items * m.kv_heads * m.maps * ((self.dec_tokens * m.group + 15) // 16) * 16
-            o, ml = max(o, n * ops.window_pad(m.dim, m.vdim)[1]), max(ml, n * 2)
+            o, ml = max(o, n * m.out_width), max(ml, n * 2)
         return o, ml, 1
 
     def room(self, part_o, part_ml) -> AttentionRoom:

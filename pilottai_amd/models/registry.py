@@ -12,14 +12,14 @@ import json
 import os
 from typing import Dict, Optional
 
-from pilottai_amd.models import bozupel, llama, mudepel, salipel
+from pilottai_amd.models import bozupel, llama, mudepel, pusunex, salipel
 
 CONFIG_CLASSES: Dict[str, type] = {"Bozupel": bozupel.BozupelConfig, "Mudepel": mudepel.MudepelConfig,
-                                  "Salipel": salipel.SalipelConfig}
+                                  "Salipel": salipel.SalipelConfig, "Pusunex": pusunex.PusunexConfig}
 MODEL_CLASSES: Dict[type, type] = {llama.LlamaConfig: llama.LlamaModel, bozupel.BozupelConfig: bozupel.BozupelModel,
                                    mudepel.MudepelConfig: mudepel.MudepelModel,
-                                   salipel.SalipelConfig: salipel.SalipelModel}
-PRESETS = {**llama.PRESETS, **bozupel.PRESETS, **mudepel.PRESETS, **salipel.PRESETS}
+                                   salipel.SalipelConfig: salipel.SalipelModel, pusunex.PusunexConfig: pusunex.PusunexModel}
+PRESETS = {**llama.PRESETS, **bozupel.PRESETS, **mudepel.PRESETS, **salipel.PRESETS, **pusunex.PRESETS}
 
 
 def is_folder(name) -> bool:

@@ -2,7 +2,7 @@
 masks, biases and gates, state-space and matrix-memory layers, score-routed experts and fp32 residuals.
 
 Device tensors run the HIP kernels of csrc/ops/{hyper_norm, paged_kv, window_attention, head_difference,
-state_scan, matrix_memory, score_route}.hip and raise when the module is missing; CPU tensors run the fp32 references of
+state_scan, matrix_memory, gated_norm, score_route}.hip and raise when the module is missing; CPU tensors run the fp32 references of
 ops/reference.py. Every function takes its constants as arguments and works in bf16 or fp32.
 """
 from __future__ import annotations
@@ -12,13 +12,11 @@ from typing import Optional
 import torch
 
 from . import reference as ref
-from .kernels import _on_gpu, require_hybrid
-from .latent import unpack_groups
+from .kernels import MIXED, _on_gpu, require_family, require_hybrid
+from .latent import SCAN_CHUNK, SCAN_MIN, unpack_groups
 
 # (key width, value width) in 32s with MFMA kernels (window_attention.hip PA_WA_DIMS)
 WINDOW_TILES = ((1, 1), (1, 2), (2, 1), (2, 2), (2, 4), (3, 3), (4, 2), (4, 4), (4, 8), (6, 4), (6, 6), (8, 8))
-SCAN_CHUNK = 64  # tokens of a scan item (state_scan.hip)
-SCAN_MIN = 8     # longer portions are scanned in chunks
 CONV_TAPS = (4, 8)  # built convolutions: shorter ones get zero taps in front
 
 
@@ -160,12 +158,13 @@ def matrix_memory(x, y, div, state, top, i_bias, f_bias, q_start, q_len, ctx_len
 
 
 def gated_norm(y, z, w, slots, heads: int, vdim: int, vpad: int, parts: int, eps: float,
-               div: Optional[torch.Tensor] = None, after: bool = False):
-    """y (in place) = norm(y * silu(z)) * w, or with `after` norm(y) * w * sigmoid(z), normed in `parts` equal parts
-    of the heads * vdim real columns; column h * vpad + v holds head h's v. div [T, heads]: y is divided by it first
-    (csrc/ops/state_scan.hip)."""
+               div: Optional[torch.Tensor] = None, after: Optional[str] = None):
+    """y (in place) = norm(y * silu(z)) * w, or with `after` ("sigmoid", "silu") norm(y) * w * after(z), normed in `parts`
+    equal parts of the heads * vdim real columns; column h * vpad + v holds head h's v. div [T, heads]: y is divided by it
+    first (csrc/ops/gated_norm.hip)."""
     if _on_gpu(y):
-        require_hybrid().gated_norm(y, z, w, slots, int(heads), int(vdim), int(vpad), int(parts), float(eps), div, bool(after))
+        require_family(*MIXED).gated_norm(y, z, w, slots, int(heads), int(vdim), int(vpad), int(parts), float(eps), div,
+                                          (None, "sigmoid", "silu").index(after))
     else:
         ref.gated_norm(y, z, w, heads, vdim, vpad, parts, eps, div, after)
     return y
@@ -180,7 +179,7 @@ def score_route(h, w, slots, weights, choice, rank, counts, order, tiles, n_tile
     chosen s + 1e-20)); `always` more experts follow with weight 1. Writes weights [T, top + always] and the rows
     sorted by expert (csrc/ops/score_route.hip). counts: E + always zeros when there are more than 16 rows."""
     if _on_gpu(h):
-        require_hybrid().score_route(h, w, slots, weights, choice, rank, counts, order, tiles, n_tiles, int(E), int(top),
+        require_family(*MIXED).score_route(h, w, slots, weights, choice, rank, counts, order, tiles, n_tiles, int(E), int(top),
                                      int(groups), int(keep), int(always), int(tm), bool(softmax), correction, bool(share),
                                      float(scale))
     else:

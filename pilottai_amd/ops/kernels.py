@@ -60,25 +60,39 @@ def _require_family(name: str):
     return _FAMILY[name]
 
 
+# the modules that hold an operation, by what they are built for (_build.py MODULES)
+LATENT = ("latent", "latent_linear")
+MIXED = ("hybrid", "latent_linear")
+GROUPED = ("latent", "hybrid", "latent_linear")
+
+
+def require_family(*names: str):
+    """Of these modules the one that a model has loaded, else the first that is built."""
+    for name in _FAMILY:
+        if name in names:
+            return _FAMILY[name]
+    for name in names[:-1]:
+        try:
+            return _require_family(name)
+        except RuntimeError:
+            pass
+    return _require_family(names[-1])
+
+
 def require_latent():
-    """The _latent module (latent attention, expert tables, fp32 residual; csrc/ops/bindings_latent.cpp)."""
-    return _require_family("latent")
+    """A module with latent attention and its residual (csrc/ops/bind_latent.h)."""
+    return require_family(*LATENT)
 
 
 def require_hybrid():
     """The _hybrid module (paged attention, recurrent layers, score-routed experts, fp32 residuals;
     csrc/ops/bindings_hybrid.cpp)."""
-    return _require_family("hybrid")
+    return require_family("hybrid")
 
 
 def require_grouped():
-    """A module with the grouped projections: the one that is loaded, else the one that is built."""
-    for name in _FAMILY:
-        return _FAMILY[name]
-    try:
-        return require_latent()
-    except RuntimeError:
-        return require_hybrid()
+    """A module with the grouped projections."""
+    return require_family(*GROUPED)
 
 
 def _packed_module():

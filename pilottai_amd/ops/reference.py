@@ -308,20 +308,31 @@ def _norm32(x: torch.Tensor, eps: float) -> torch.Tensor:
     return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
 
 
-def residual_norm(resid, eps, y, partials, y_scale, w_post, emb, ids, emb_add, w_next, out, rows):
+def _group_norm32(x: torch.Tensor, eps: float, groups: int) -> torch.Tensor:
+    return _norm32(x.reshape(*x.shape[:-1], groups, -1), eps).reshape(x.shape)
+
+
+def residual_norm(resid, eps, y, partials, y_scale, w_post, emb, ids, emb_add, w_next, out, rows, post_groups=1, next_groups=1,
+                  mix=None, hist=None):
     T, D = resid.shape
     sel = torch.arange(T) if rows is None else rows.long()
     r = resid[sel]
     if y is not None:
         d = y[:, :D].float().view(T, partials, D).sum(1)[sel] * y_scale
-        r = r + (_norm32(d, eps) * w_post if w_post is not None else d)
+        r = r + (_group_norm32(d, eps, post_groups) * w_post if w_post is not None else d)
     if emb is not None:
         e = emb[ids[:T].long()[sel].clamp(0, emb.shape[0] - 1)].float()
-        r = r + e if emb_add else e  # (set: before any y)
+        if mix is not None:
+            n = mix.numel() - 1
+            if rows is None:
+                hist[n - 1, :T] = r
+            r = mix[0] * e + mix[n] * r + sum(mix[j] * hist[j - 1, :T][sel] for j in range(1, n))
+        else:
+            r = r + e if emb_add else e  # (set: before any y)
     if rows is None:
         resid.copy_(r)
     if out is not None:
-        out[:len(sel), :D] = (_norm32(r, eps) * w_next).to(out.dtype)
+        out[:len(sel), :D] = (_group_norm32(r, eps, next_groups) * w_next if w_next is not None else r).to(out.dtype)
         out[:len(sel), D:] = 0
     return out
 
@@ -339,12 +350,14 @@ def _rotate_part(x: torch.Tensor, positions: torch.Tensor, cos_sin: torch.Tensor
 def latent_cache(x, nq, R, r, w_q, w_c, cq, pages, Rp, positions, slots, cos_sin, eps):
     T = x.shape[0]
     xf = x.float()
-    cq.zero_()
-    cq[:, :nq] = (_norm32(xf[:, :nq], eps) * w_q).to(cq.dtype)
+    if nq:
+        cq.zero_()
+        cq[:, :nq] = (_norm32(xf[:, :nq], eps) * w_q).to(cq.dtype)
     D = pages.shape[1] * 8
     row = torch.zeros(T, D)
     row[:, :R] = _norm32(xf[:, nq:nq + R], eps) * w_c
-    row[:, Rp:Rp + r] = _rotate_part(xf[:, nq + R:nq + R + r], positions[:T], cos_sin)
+    if r:
+        row[:, Rp:Rp + r] = _rotate_part(xf[:, nq + R:nq + R + r], positions[:T], cos_sin)
     for t in range(T):
         s = int(slots[t])
         if s >= 0:
@@ -366,16 +379,30 @@ def latent_attention(out, q, pages, q_start, q_len, ctx_len, block_table, scale,
         out[q0:q0 + n] = torch.einsum("htk,kd->thd", p, rows[:, :Rp]).to(out.dtype)
 
 
-def head_gemm(x, x_step, w, out, out_step, rot):
+def head_gemm(x, x_step, w, out, out_step, rot, gate=None):
     N, K = w.shape[1:]
     for g in range(w.shape[0]):
         at = g * out_step
-        out[:, at:at + N] = (x[:, g * x_step:g * x_step + K].float() @ w[g].float().T).to(out.dtype)
+        y = x[:, g * x_step:g * x_step + K].float() @ w[g].float().T
+        if gate is not None:
+            y = y * torch.sigmoid(gate[:, at:at + N].float())
+        out[:, at:at + N] = y.to(out.dtype)
         if rot is not None:
             pos, cs, skip, r, rp = rot
             out[:, at + N:at + N + rp] = 0
             v = x[:, g * x_step + skip:g * x_step + skip + r].float()
             out[:, at + N:at + N + r] = _rotate_part(v, pos[:x.shape[0]], cs).to(out.dtype)
+
+
+def _gated_unit(g, u, lim, alpha, bias, cubic):
+    g, u = g.clamp(max=lim), u.clamp(-lim, lim)
+    return g * torch.sigmoid(alpha * (g + cubic * g ** 3)) * (u + bias)
+
+
+def table_gemm(x, w, out, table, ids, col, lim, alpha, bias, cubic):
+    N, K = w.shape
+    e = table[ids[:x.shape[0]].long().clamp(0, table.shape[0] - 1), col:col + N].float()
+    out[:, :N] = _gated_unit(x[:, :K].float() @ w.float().T, e, lim, alpha, bias, cubic).to(out.dtype)
 
 
 def table_route(tables, desc, ids, slots, T, tm, order, tiles, n_tiles):
@@ -396,17 +423,17 @@ def table_route(tables, desc, ids, slots, T, tm, order, tiles, n_tiles):
         n_tiles[layer] = min(k, tmax)
 
 
-def expert_gemm(x, w, out, tiles, n_tiles, order, x_div, out_order, glu, relu2=False):
+def expert_gemm(x, w, out, tiles, n_tiles, order, x_div, out_order, glu, relu2=False, row_w=None):
     K = w.shape[2]
     for e, start, n, _ in tiles[:int(n_tiles[0])].tolist():
         p = torch.arange(start, start + n)
         xr = order[p].long() // x_div if x_div else p
         y = x[xr, :K].float() @ w[e].float().T
+        if row_w is not None:
+            y = y * row_w.reshape(-1)[order[p].long()][:, None]
         if glu is not None:
-            lim, alpha, bias, cubic = (tuple(glu) + (0.0,))[:4]
             y = y.view(n, -1, 2, 16)
-            g, u = y[:, :, 0].reshape(n, -1).clamp(max=lim), y[:, :, 1].reshape(n, -1).clamp(-lim, lim)
-            y = g * torch.sigmoid(alpha * (g + cubic * g ** 3)) * (u + bias)
+            y = _gated_unit(y[:, :, 0].reshape(n, -1), y[:, :, 1].reshape(n, -1), *(tuple(glu) + (0.0,))[:4])
         if relu2:
             y = y.clamp(min=0) ** 2
         out[order[p].long() if out_order else p, :y.shape[1]] = y.to(out.dtype)
@@ -623,18 +650,44 @@ def matrix_memory(x, y, div, state, top, i_bias, f_bias, q_start, q_len, ctx_len
         state[slot], top[slot] = S, m[:, None]
 
 
+def linear_attention(x, y, state, a2, bias, q_start, q_len, ctx_len, state_slot, cols, q_scale, inv_tau, num_seqs):
+    H, V, N = state.shape[1:]
+    cq, ck, cv, ca = cols
+    for s in range(num_seqs):
+        n, q0, slot = int(q_len[s]), int(q_start[s]), int(state_slot[s])
+        if n <= 0:
+            continue
+        r = x[q0:q0 + n].float()
+        q, k = r[:, cq:cq + H * N].view(n, H, N) * q_scale, r[:, ck:ck + H * N].view(n, H, N)
+        v = r[:, cv:cv + H * V].view(n, H, V)
+        z = r[:, ca:ca + a2.shape[1]] @ a2.float().T + bias
+        d = torch.exp(torch.nn.functional.logsigmoid(z) * inv_tau).view(n, H, 1, N)
+        S = torch.zeros(H, V, N) if int(ctx_len[s]) == n else state[slot].clone()
+        for t in range(n):
+            S = S * d[t] + v[t][:, :, None] * k[t][:, None, :]
+            y[q0 + t, :H * V] = (S * q[t][:, None, :]).sum(-1).reshape(-1).to(y.dtype)
+        state[slot] = S
+
+
+def poly_norm(z, n, act, eps):
+    f = z[:, :n].float()
+    z[:, :n] = (sum(act[i] * _norm32(f ** (i + 1), eps) for i in range(3)) + act[3]).to(z.dtype)
+    z[:, n:] = 0
+
+
 def gated_norm(y, z, w, heads, vdim, vpad, parts, eps, div, after):
     T = y.shape[0]
     g, zf = (t[:, :heads * vpad].float().reshape(T, heads, vpad)[:, :, :vdim] for t in (y, z))
     if div is not None:
         g = g / div[:, :, None]
     g, zf = g.reshape(T, -1), zf.reshape(T, -1)
-    if not after:
+    if after is None:
         g = g * (zf * torch.sigmoid(zf))
     g = _norm32(g.view(T, parts, -1), eps).view(T, -1) * w
-    g = (g * torch.sigmoid(zf) if after else g).view(T, heads, vdim)
+    if after is not None:
+        g = g * torch.sigmoid(zf) * (zf if after == "silu" else 1.0)
     y.zero_()
-    y[:, :heads * vpad].view(T, heads, vpad)[:, :, :vdim] = g.to(y.dtype)
+    y[:, :heads * vpad].view(T, heads, vpad)[:, :, :vdim] = g.view(T, heads, vdim).to(y.dtype)
 
 
 def score_route(h, w, slots, weights, choice, order, tiles, n_tiles, E, top, groups, keep, always, tm, softmax, correction,

@@ -256,6 +256,7 @@ def test_latent_attention_module(folder, device):
     """The mixer alone, every branch of its sizes, against the oracle's."""
     from pilottai_amd.models.bozupel import BozupelConfig, LatentAttention
     from pilottai_amd.models.cache import StepMeta
+    from pilottai_amd.models.hybrid import AttentionRoom, MixerBlock
     from pilottai_amd.ops import reference as ref
     from pilottai_amd.ops.latent import pad_to
 
@@ -277,7 +278,7 @@ def test_latent_attention_module(folder, device):
                         iv(0), num_seqs=1)
         z = torch.zeros(len(items) * 64 * m.Rp, device=dev)
         pages = torch.zeros(5, m.D // 8, 16, 8, device=dev)
-        y = m(h.to(dev), meta, pages, z, z, dec, tile)
+        y = MixerBlock([m], torch.float32, dev)(h.to(dev), meta, [(pages,)], AttentionRoom(z, z, dec, tile, 0))[0]
         want = oracle.latent_attention(h[:, :d].double(), VARIED["layers"][i]["mixer"], {k: v.double() for k, v in w.items()}, 1e-4)
         torch.testing.assert_close(y.double().cpu()[:, :d], want, rtol=1e-4, atol=1e-4)
 

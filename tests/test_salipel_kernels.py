@@ -363,7 +363,7 @@ def test_norm_before_the_gate(device, dt, H, V, Vp):
     w, slots, div = torch.randn(H * V, generator=g), torch.arange(T, dtype=torch.int32), torch.rand(T, H, generator=g) * 3 + 0.01
     slots[4] = -1
     rows = y.to(device).clone()
-    ops.gated_norm(rows[:, :H * Vp], z.to(device)[:, 8:], w.to(device), slots.to(device), H, V, Vp, H, eps, div=div.to(device), after=True)
+    ops.gated_norm(rows[:, :H * Vp], z.to(device)[:, 8:], w.to(device), slots.to(device), H, V, Vp, H, eps, div=div.to(device), after="sigmoid")
     o = rows.double().cpu()
     pick = lambda t: t.double()[:, :H * Vp].reshape(T, H, Vp)[:, :, :V]  # noqa: E731
     want = oracle.rms(pick(y) / div.double()[:, :, None], eps).reshape(T, -1) * w.double() * torch.sigmoid(pick(z[:, 8:]).reshape(T, -1))
