@@ -120,9 +120,9 @@ def parse():
                          "the manager Serve, the control plane and all clients; ranks > 0 are CPU processes whose "
                          "agents answer with model-free schema LLMs after this many seconds per call (the measured "
                          "per-call latency of an 8-worker GPU rank). Use with PILOTTAI_DIST_BACKEND=gloo.")
-    ap.add_argument("--design", default=None, choices=["bozupel", "mudepel", "salipel"],
-                    help="instead of the workload: step throughput of this model design beside Llama layers of equal "
-                         "size, one JSON line per case (benchmarks/model_step.py)")
+    ap.add_argument("--design", default=None, choices=["bozupel", "mudepel", "salipel", "pusunex"],
+                    help="instead of the workload: step throughput of this model design beside the closest other model "
+                         "at equal size, one JSON line per case (benchmarks/model_step.py)")
     ap.add_argument("--design-cases", default="", help="with --design: only the cases whose name contains this")
     ap.add_argument("--design-sizes", default="", help="with --design: base, wide (default: both)")
     return ap.parse_args()

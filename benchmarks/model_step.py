@@ -1,6 +1,7 @@
-"""Step throughput of a served model design beside Llama layers of equal size (random weights).
+"""Step throughput of a served model design beside the closest other model at equal size (random weights): Llama layers,
+for Pusunex the latent attention and experts of Bozupel.
 
-    python bench.py --design bozupel|mudepel|salipel [--steps K --warmup W]
+    python bench.py --design bozupel|mudepel|salipel|pusunex [--steps K --warmup W]
 
 For each size the two engines hold the same width, layer count, heads and active feed-forward width.
 A case is one scheduler-built step (prompt portions or decode rows at a context), captured as the
@@ -26,18 +27,21 @@ CASES: List[Tuple[str, List[Tuple[int, int]]]] = [
     ("decode 256 at 1024", [(1024, 1)] * 256),
 ]
 
-DESIGNS = ("bozupel", "mudepel", "salipel")
+DESIGNS = ("bozupel", "mudepel", "salipel", "pusunex")
 
 
 def pair(design: str):
-    """[(size, design config, equal-size Llama config)]"""
-    from pilottai_amd.models import bozupel, mudepel, salipel
+    """[(size, design config, config of the other model at equal size)]"""
+    from pilottai_amd.models import bozupel, mudepel, pusunex, salipel
     from pilottai_amd.models.llama import LlamaConfig
 
     if design not in DESIGNS:
         raise ValueError(f"unknown design {design!r}; known: {DESIGNS}")
     out = []
     for size in ("base", "wide"):
+        if design == "pusunex":
+            out.append((size, pusunex.PRESETS[f"pusunex-{size}"], bozupel.PRESETS[f"bozupel-{size}"]))
+            continue
         if design == "bozupel":
             c = bozupel.PRESETS[f"bozupel-{size}"]
             m, p = c.layers[0].mixer, c.layers[0].mlp
@@ -130,10 +134,11 @@ def run(design: str, steps: int = 3, warmup: int = 1, only: str = "", sizes: str
             for t, i in zip(timers, ids):
                 t.unload(i)
             a, b = (statistics.median(m) for m in ms)
+            other = old.name.split("-")[0]
             row = {"metric": f"{design} step throughput", "case": name, "size": size, "tokens": T, "unit": "tokens/s",
-                   "value": round(T / a * 1e3), "ms_per_step": round(a, 4), "llama_equal_size": round(T / b * 1e3),
-                   "llama_ms_per_step": round(b, 4), "params_b": round(new.num_params() / 1e9, 2),
-                   "llama_params_b": round(old.num_params() / 1e9, 2), "dtype": "bf16", "data": "synthetic"}
+                   "value": round(T / a * 1e3), "ms_per_step": round(a, 4), f"{other}_equal_size": round(T / b * 1e3),
+                   f"{other}_ms_per_step": round(b, 4), "params_b": round(new.num_params() / 1e9, 2),
+                   f"{other}_params_b": round(old.num_params() / 1e9, 2), "dtype": "bf16", "data": "synthetic"}
             print(json.dumps(row), flush=True)
             out.append(row)
         del timers

@@ -202,7 +202,7 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
         for (int j = 0; j < 4; ++j) v[j] = (bf16)glu(acc[m][i][j] * rw, acc[m][i + 1][j] * rw, A);
         *reinterpret_cast<bf16x4*>(o + (nt0 + i) * 8) = v;
       }
-    } else if constexpr (EPI == GATED || EPI == TABLE) {
+    } else if constexpr (EPI == GATED) {
       const bf16* f = factor_row<bf16, EPI>(A, pos[m], grp) + 4 * g;
 #pragma unroll
       for (int i = 0; i < NT; ++i) {
@@ -231,6 +231,67 @@ __global__ __launch_bounds__(256) void gemm_kernel(const Args A) {
         *reinterpret_cast<bf16x4*>(o + (nt0 + i) * 16) = v;
       }
     }
+  }
+}
+
+// Dense rows through one group of few outputs (TABLE): 8 waves share a tile of 16 MT rows and 16 NT outputs, each every
+// eighth step of K, and add up through LDS.
+template <int MT, int NT>
+__global__ __launch_bounds__(512) void split_k_kernel(const Args A) {
+  extern __shared__ __attribute__((aligned(16))) f32x4 red[];  // [8][MT NT][64]
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
+  // tiles of the same rows next to each other on one XCD: they share its copy of x
+  const int cols = (A.N16 + NT - 1) / NT, tiles = cols * ((A.rows + 16 * MT - 1) / (16 * MT)), per = (tiles + 7) >> 3;
+  const int tile = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+  if ((int)(blockIdx.x >> 3) >= per || tile >= tiles) return;
+  const int nt0 = tile % cols * NT, start = tile / cols * (16 * MT), n = min(16 * MT, A.rows - start);
+  const bf16 *wt[NT], *xr[MT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) wt[i] = (const bf16*)A.w + (size_t)min(nt0 + i, A.N16 - 1) * A.K32 * 512 + lane * 8;
+#pragma unroll
+  for (int m = 0; m < MT; ++m) xr[m] = (const bf16*)A.x + (size_t)(start + min(16 * m + c, n - 1)) * A.ldx + 8 * g;
+  f32x4 acc[MT][NT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int i = 0; i < NT; ++i) acc[m][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  constexpr int U = MT * NT == 1 ? 8 : 4;  // steps whose loads go out together
+  for (int s = wid; s < A.K32; s += 8 * U) {
+    bf16x8 a[U][NT], b[U][MT];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = min(s + 8 * u, A.K32 - 1);
+#pragma unroll
+      for (int i = 0; i < NT; ++i) a[u][i] = *reinterpret_cast<const bf16x8*>(wt[i] + (size_t)k * 512);
+#pragma unroll
+      for (int m = 0; m < MT; ++m) b[u][m] = *reinterpret_cast<const bf16x8*>(xr[m] + (size_t)k * 32);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (s + 8 * u < A.K32) {
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+#pragma unroll
+          for (int i = 0; i < NT; ++i) acc[m][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u][i], b[u][m], acc[m][i], 0, 0, 0);
+      }
+  }
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int i = 0; i < NT; ++i) red[((wid * MT + m) * NT + i) * 64 + lane] = acc[m][i];
+  __syncthreads();
+  for (int t = wid; t < MT * NT; t += 8) {  // tile (m, i): the same lanes again
+    const int m = t / NT, i = t % NT, row = start + 16 * m + c;
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int w = 0; w < 8; ++w) v += red[((w * MT + m) * NT + i) * 64 + lane];
+    if (16 * m + c >= n || nt0 + i >= A.N16) continue;
+    const int col = (nt0 + i) * 16 + 4 * g;
+    const bf16x4 f = *reinterpret_cast<const bf16x4*>(factor_row<bf16, TABLE>(A, row, 0) + col);
+    bf16x4 o;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = (bf16)times<TABLE>(v[j], (float)f[j], A);
+    *reinterpret_cast<bf16x4*>((bf16*)A.out + (size_t)row * A.ldo + col) = o;
   }
 }
 
@@ -396,6 +457,26 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
   if (tiles && tm == 256)
     return pa_expert_tiles(out, x, w, wstride, N16 * 16, K32 * 32, ldx, ldo, tiles, max_tiles, n_tiles, order, x_div,
                            out_order, epi == 1 ? pa::pk::EP_GLU : epi == 2 ? pa::pk::EP_RELU2 : pa::pk::EP_PLAIN, limit, alpha, cubic, bias, row_w, st);
+  if (epi == 4) {  // tiles as large as leave most of the chip busy
+#define PA_SK(MT, NT)                                                                                                       \
+  do {                                                                                                                      \
+    constexpr int lds = 8 * MT * NT * 1024;                                                                                 \
+    static bool attr = false;                                                                                               \
+    if (!attr) {                                                                                                            \
+      (void)hipFuncSetAttribute((const void*)pa::gg::split_k_kernel<MT, NT>, hipFuncAttributeMaxDynamicSharedMemorySize, lds); \
+      attr = true;                                                                                                          \
+    }                                                                                                                       \
+    hipLaunchKernelGGL((pa::gg::split_k_kernel<MT, NT>), dim3(((N16 + NT - 1) / NT * ((rows + 16 * MT - 1) / (16 * MT)) + 7) / 8 * 8), \
+                       dim3(512), lds, st, A);                                                                              \
+  } while (0)
+    auto fills = [&](int t) { return (N16 + t - 1) / t * ((rows + 16 * t - 1) / (16 * t)) >= 192; };
+    if (groups != 1) return -1;
+    if (fills(4)) PA_SK(4, 4);
+    else if (fills(2)) PA_SK(2, 2);
+    else PA_SK(1, 1);
+#undef PA_SK
+    return (int)hipGetLastError();
+  }
   // dense: 64-row tiles once they fill the chip
   if (!tiles) tm = (N16 + 15) / 16 * ((rows + 63) / 64) * groups < 256 ? 16 : 64;
   if (tm != 16 && tm != 64) return -2;
@@ -414,13 +495,11 @@ extern "C" int pa_grouped_gemm(int fp32, const void* x, const void* w, void* out
     if (epi == 1) PA_GGK(1, 2, pa::gg::GLU);
     else if (epi == 2) PA_GGK(1, 1, pa::gg::RELU2);
     else if (epi == 3) PA_GGK(1, 1, pa::gg::GATED);
-    else if (epi == 4) PA_GGK(1, 1, pa::gg::TABLE);
     else PA_GGK(1, 1, pa::gg::PLAIN);
   } else {
     if (epi == 1) PA_GG(4, 4, 1, pa::gg::GLU);
     else if (epi == 2) PA_GG(4, 4, 1, pa::gg::RELU2);
     else if (epi == 3) PA_GG(4, 4, 1, pa::gg::GATED);
-    else if (epi == 4) PA_GG(4, 4, 1, pa::gg::TABLE);
     else PA_GG(4, 4, 1, pa::gg::PLAIN);
   }
 #undef PA_GGK

@@ -17,6 +17,8 @@
 // more than once, by padding).
 #include "common.h"
 
+#include <type_traits>
+
 namespace pa {
 namespace rn {
 
@@ -174,6 +176,168 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const Args A) {
   for (int i = D + threadIdx.x; i < A.ldo; i += 256) o[i] = (T)0.f;
 }
 
+// The same for rows of whole 8s whose groups are whole wave steps of 512 elements or a power of two of lanes: W waves a row
+// (4 / W rows a workgroup), NV vectors a thread in registers, all of a row's loads ahead of the first sum.
+template <typename T, int W, int NV>
+__global__ __launch_bounds__(256) void residual_norm_wave_kernel(const Args A, int n) {
+  constexpr int R = 4 / W;
+  __shared__ float slots[W > 1 ? R : 1][W > 1 ? W * NV : 1];
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, w = wid % W, r = wid / W;
+  const int b = blockIdx.x * R + r, D = A.D;
+  if (W == 1 && b >= n) return;  // (whole waves; with W > 1 all take the barriers)
+  const int t = A.rows ? A.rows[min(b, n - 1)] : min(b, n - 1);
+  auto at = [&](int s) { return ((s * W + w) * 64 + lane) * 8; };
+  auto in = [&](int s) { return min(at(s), D - 8); };  // (loads without branches; past the end they repeat the last 8)
+  // 1 / rms of the group of each of a thread's vectors
+  auto factors = [&](const float (&ss)[NV], int groups, float (&inv)[NV]) {
+    const int len = D / groups, width = groups == 1 ? 64 : min(64, len >> 3), units = groups == 1 ? W * NV : max(1, len >> 9);
+    float part[NV];
+#pragma unroll
+    for (int s = 0; s < NV; ++s) {
+      part[s] = ss[s];
+      for (int o = width >> 1; o > 0; o >>= 1) part[s] += __shfl_xor(part[s], o, 64);
+    }
+    if constexpr (W > 1) {
+      __syncthreads();
+      if (lane == 0) {
+#pragma unroll
+        for (int s = 0; s < NV; ++s) slots[r][s * W + w] = part[s];
+      }
+      __syncthreads();
+    }
+#pragma unroll
+    for (int s = 0; s < NV; ++s) {
+      float sum = 0.f;
+      if (units == 1) {
+        sum = part[s];
+      } else if constexpr (W > 1) {
+        const int u0 = (s * W + w) / units * units;
+        for (int u = u0; u < min(u0 + units, W * NV); ++u) sum += slots[r][u];
+      } else {
+#pragma unroll
+        for (int k = 0; k < NV; ++k) sum += k / units == s / units ? part[k] : 0.f;
+      }
+      inv[s] = 1.f / sqrtf(sum / (float)len + A.eps);
+    }
+  };
+  auto load = [](const auto* p, float (&v)[8]) {
+    using E = std::remove_cv_t<std::remove_pointer_t<decltype(p)>>;
+    E a[8];
+    __builtin_memcpy(a, __builtin_assume_aligned(p, sizeof(E) * 8), sizeof(a));
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = (float)a[j];
+  };
+  float* rr = A.resid + (size_t)t * D;
+  const T* er = A.emb ? (const T*)A.emb + (size_t)min(max(A.ids[t], 0), A.vocab - 1) * D : nullptr;
+  const bool set = er && !A.emb_add && !A.mix;
+  float y[NV][8], x[NV][8], ss[NV], inv[NV];
+#pragma unroll
+  for (int s = 0; s < NV; ++s) {
+    ss[s] = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[s][j] = y[s][j] = 0.f;
+    if (!set) load(rr + in(s), x[s]);
+  }
+  if (A.y) {
+    const T* yr = (const T*)A.y + (size_t)t * A.K * A.ldy;
+#pragma unroll 4
+    for (int k = 0; k < A.K; ++k)
+#pragma unroll
+      for (int s = 0; s < NV; ++s) {
+        float v[8];
+        load(yr + (size_t)k * A.ldy + in(s), v);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) y[s][j] += v[j];
+      }
+#pragma unroll
+    for (int s = 0; s < NV; ++s) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        y[s][j] *= A.y_scale;
+        ss[s] = fmaf(y[s][j], y[s][j], ss[s]);
+      }
+      if (at(s) >= D) ss[s] = 0.f;
+    }
+    if (A.w_post) {
+      float g[NV][8];  // (on their way during the sum)
+#pragma unroll
+      for (int s = 0; s < NV; ++s) load(A.w_post + in(s), g[s]);
+      factors(ss, A.post_groups, inv);
+#pragma unroll
+      for (int s = 0; s < NV; ++s)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[s][j] = fmaf(y[s][j] * inv[s], g[s][j], x[s][j]);
+    } else {
+#pragma unroll
+      for (int s = 0; s < NV; ++s)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[s][j] += y[s][j];
+    }
+  }
+  const bool keep = !A.rows && b < n;
+  auto store = [&](float* p, const float (&v)[8]) { __builtin_memcpy(__builtin_assume_aligned(p, 32), v, 32); };
+  if (A.mix) {
+    float* hr = A.hist + (size_t)t * D;
+    const float a0 = A.mix[0], an = A.mix[A.n_hist];
+#pragma unroll
+    for (int s = 0; s < NV; ++s) {
+      if (keep && at(s) < D) store(hr + (A.n_hist - 1) * A.hist_step + at(s), x[s]);
+      float e[8];
+      load(er + in(s), e);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[s][j] = a0 * e[j] + an * x[s][j];
+    }
+#pragma unroll 4
+    for (int k = 1; k < A.n_hist; ++k) {
+      const float ak = A.mix[k];
+#pragma unroll
+      for (int s = 0; s < NV; ++s) {
+        float v[8];
+        load(hr + (k - 1) * A.hist_step + in(s), v);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[s][j] = fmaf(ak, v[j], x[s][j]);
+      }
+    }
+  } else if (er) {
+#pragma unroll
+    for (int s = 0; s < NV; ++s) {
+      float e[8];
+      load(er + in(s), e);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[s][j] += e[j];
+    }
+  }
+  if (keep && (A.y || er)) {
+#pragma unroll
+    for (int s = 0; s < NV; ++s)
+      if (at(s) < D) store(rr + at(s), x[s]);
+  }
+  if (!A.out) return;  // (all of them)
+  if (A.w_next) {
+#pragma unroll
+    for (int s = 0; s < NV; ++s) {
+      ss[s] = 0.f;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss[s] = fmaf(x[s][j], x[s][j], ss[s]);
+      if (at(s) >= D) ss[s] = 0.f;
+    }
+    factors(ss, A.next_groups, inv);
+  }
+  if (b >= n) return;
+  T* o = (T*)A.out + (size_t)b * A.ldo;
+#pragma unroll
+  for (int s = 0; s < NV; ++s) {
+    if (at(s) >= A.ldo) continue;
+    T a[8];
+    float g[8];
+    if (A.w_next && at(s) < D) load(A.w_next + at(s), g);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) a[j] = (T)(at(s) >= D ? 0.f : A.w_next ? x[s][j] * inv[s] * g[j] : x[s][j]);
+    __builtin_memcpy(__builtin_assume_aligned(o + at(s), sizeof(a)), a, sizeof(a));
+  }
+  for (int i = W * NV * 512 + (w * 64 + lane); i < A.ldo; i += 64 * W) o[i] = (T)0.f;
+}
+
 }  // namespace rn
 }  // namespace pa
 
@@ -188,6 +352,26 @@ extern "C" int pa_residual_norm(int fp32, float* resid, const void* y, int K, in
   if (post_groups < 1 || next_groups < 1 || D % post_groups || D % next_groups || (mix && (!emb || !hist || n_hist < 1))) return -1;
   const Args A{resid, y, w_post, emb, ids, mix, hist, w_next, out, rows, hist_step, K, ldy, vocab, emb_add, n_hist, ldo, D,
                post_groups, next_groups, y_scale, eps};
+  // whole 8s, and groups that are lanes of a wave (a power of two) or whole wave steps
+  auto lanes = [&](int g) { const int len = D / g, l = len / 8; return g == 1 || len % 512 == 0 || (len % 8 == 0 && l <= 64 && (l & (l - 1)) == 0); };
+  const int steps = (D + 511) / 512;
+  if (D % 8 == 0 && ldy % 8 == 0 && ldo % 8 == 0 && lanes(post_groups) && lanes(next_groups) && steps <= 16) {
+    // many rows: as few waves a row as hold it in 4 vectors a thread; few: 4 waves
+    const int w = n >= 1024 ? (steps <= 4 ? 1 : steps <= 8 ? 2 : 4) : 4, nv = (steps + w - 1) / w;
+#define PA_RW(T, W, N) hipLaunchKernelGGL((residual_norm_wave_kernel<T, W, N>), dim3((n + 4 / W - 1) / (4 / W)), dim3(256), 0, st, A, n)
+#define PA_RW_N(T, W)                       \
+  do {                                      \
+    if (nv == 1) PA_RW(T, W, 1);            \
+    else if (nv == 2) PA_RW(T, W, 2);       \
+    else PA_RW(T, W, 4);                    \
+  } while (0)
+#define PA_RW_T(T) do { if (w == 1) PA_RW_N(T, 1); else if (w == 2) PA_RW(T, 2, 4); else PA_RW_N(T, 4); } while (0)
+    if (fp32) PA_RW_T(float); else PA_RW_T(pa::bf16);
+#undef PA_RW_T
+#undef PA_RW_N
+#undef PA_RW
+    return (int)hipGetLastError();
+  }
   const int most = post_groups > next_groups ? post_groups : next_groups;
   // vectors that divide the groups, so that each lies in one
   auto fits = [&](int v) {

@@ -127,7 +127,7 @@ def table_route(tables, desc, desc_host, ids, slots, T: int, tm: int, order, til
     """Sort every layer's (token, choice) pairs by expert, from the layers' token tables, in one launch
     (grouped_gemm.hip table_route_kernel)."""
     if _on_gpu(ids):
-        require_latent().table_route(tables, desc, desc_host, ids, slots, int(T), int(tm), order, tiles, n_tiles)
+        require_family("latent").table_route(tables, desc, desc_host, ids, slots, int(T), int(tm), order, tiles, n_tiles)
     else:
         ref.table_route(tables, desc_host, ids, slots, T, tm, order, tiles, n_tiles)
 
