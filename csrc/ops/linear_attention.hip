@@ -179,15 +179,20 @@ __device__ __forceinline__ float log_decay_fast(const Args& A, float z) {
   return (fminf(z, 0.f) - (t < 0.01f ? series : log)) * A.inv_tau;
 }
 
-// 4 waves, 16 tokens each; a lane holds token 16 w + c and 8 channels of 32. Two barriers per 32 channels.
-__global__ __launch_bounds__(256, 3) void prepare_kernel(const Args A) {
+// 4 waves a part, 16 tokens each; a lane holds token 16 w + c and 8 channels of 32. P parts take every P-th 32 channels. Two
+// barriers per 32 channels.
+template <int P>
+__global__ __launch_bounds__(256 * P, 2) void prepare_kernel(const Args A) {
   constexpr int KL = 40;  // LDS row of 32 channels
-  __shared__ __attribute__((aligned(16))) bf16 kt[2][2][48][KL];  // [turn][value, remainder]: keys to the end of their block
-  __shared__ float tot[2][4][32];                                  // a wave's sum of g
-  __shared__ float dg[4][16][17];
+  __shared__ __attribute__((aligned(16))) bf16 kts[P][2][2][48][KL];  // [turn][value, remainder]: keys to the end of their block
+  __shared__ float tots[P][2][4][32];                                  // [turn]: a wave's sum of g
+  __shared__ float dg[P][4][16][17];
+  __shared__ f32x4 others[P > 1 ? P - 1 : 1][4][3][64];
   const int h = blockIdx.x, n_items = A.n_items[0], N = A.N;
-  const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lg = lane >> 4, c = lane & 15;
-  const int i = 16 * w + c;
+  const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int part = wid >> 2, w = wid & 3, lg = lane >> 4, c = lane & 15, i = 16 * w + c;
+  auto &kt = kts[part];
+  auto &tot = tots[part];
   const size_t HN = (size_t)A.H * N, plane = (size_t)A.T * HN;
   const float past[3] = {w > 0 ? 1.f : 0.f, w > 1 ? 1.f : 0.f, w > 2 ? 1.f : 0.f};
   for (int item = blockIdx.y; item < n_items; item += gridDim.y) {
@@ -205,25 +210,36 @@ __global__ __launch_bounds__(256, 3) void prepare_kernel(const Args A) {
     for (int a = 0; a < 3; ++a) blk[a] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int s = 0; s < 16; ++s) d[s] = 0.f;
-    bf16x8 qn = *reinterpret_cast<const bf16x8*>(xq), kn = *reinterpret_cast<const bf16x8*>(xk);
-    for (int m = 0; m < N / 32; ++m) {
-      const bf16x8 qb = qn, kb = kn;
-      if (m + 1 < N / 32) {
-        qn = *reinterpret_cast<const bf16x8*>(xq + 32 * (m + 1));
-        kn = *reinterpret_cast<const bf16x8*>(xk + 32 * (m + 1));
+    // the next channels are on their way: q, k, W_a2's first 32 columns, the bias
+    bf16x8 qn, kn, wn[2];
+    f32x4 bn[2];
+    const bf16* wr = (const bf16*)A.a2 + (size_t)(h * N + 8 * (c >> 2) + (c & 3)) * A.rp + 8 * lg;
+    const float* br = A.bias + h * N + 8 * lg;
+    auto load = [&](int m) {
+      qn = *reinterpret_cast<const bf16x8*>(xq + 32 * m);
+      kn = *reinterpret_cast<const bf16x8*>(xk + 32 * m);
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+        wn[half] = *reinterpret_cast<const bf16x8*>(wr + (size_t)(32 * m + 4 * half) * A.rp);
+        bn[half] = *reinterpret_cast<const f32x4*>(br + 32 * m + 4 * half);
       }
+    };
+    load(part);
+    for (int m = part, turn = 0; m < N / 32; m += P, turn ^= 1) {  // (all parts take as many: N / 32 is a multiple of P)
+      const bf16x8 qb = qn, kb = kn, wb[2] = {wn[0], wn[1]};
+      const f32x4 bb[2] = {bn[0], bn[1]};
+      if (m + P < N / 32) load(m + P);
       // z^T = W_a2 a^T; the rows of W_a2 in the order that gives a lane its 8 channels in two results
       float g[8], q[8], k[8];
 #pragma unroll
       for (int half = 0; half < 2; ++half) {
-        const bf16* wr = (const bf16*)A.a2 + (size_t)(h * N + 32 * m + 8 * (c >> 2) + 4 * half + (c & 3)) * A.rp + 8 * lg;
-        f32x4 z = {0.f, 0.f, 0.f, 0.f};
-        z = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(wr), a0, z, 0, 0, 0);
+        f32x4 z = bb[half];
+        z = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wb[half], a0, z, 0, 0, 0);
         for (int r = 32; r < A.rp; r += 32)
-          z = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(wr + r), *reinterpret_cast<const bf16x8*>(xa + r), z, 0, 0, 0);
-        const f32x4 b = *reinterpret_cast<const f32x4*>(A.bias + h * N + 32 * m + 8 * lg + 4 * half);
+          z = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(wr + (size_t)(32 * m + 4 * half) * A.rp + r),
+                                                      *reinterpret_cast<const bf16x8*>(xa + r), z, 0, 0, 0);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) g[4 * half + r] = log_decay_fast(A, z[r] + b[r]) * on;
+        for (int r = 0; r < 4; ++r) g[4 * half + r] = log_decay_fast(A, z[r]) * on;
       }
       float l[8], al[8];
 #pragma unroll
@@ -240,14 +256,14 @@ __global__ __launch_bounds__(256, 3) void prepare_kernel(const Args A) {
       }
       if (c == 15) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) tot[m & 1][w][8 * lg + e] = l[e];
+        for (int e = 0; e < 8; ++e) tot[turn][w][8 * lg + e] = l[e];
       }
       __syncthreads();
       // sums up to this wave's block, and of the chunk (the same order of additions everywhere)
       float base[8], L[8];
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        const float* t = &tot[m & 1][0][8 * lg + e];
+        const float* t = &tot[turn][0][8 * lg + e];
         const float t0 = t[0], t1 = t[32], t2 = t[64];
         base[e] = fmaf(t2, past[2], fmaf(t1, past[1], t0 * past[0]));
         L[e] = t0 + t1 + t2 + t[96];
@@ -259,10 +275,10 @@ __global__ __launch_bounds__(256, 3) void prepare_kernel(const Args A) {
       bf16x8 hi, lo;
       if (w < 3) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) v[e] = k[e] * __expf(base[e] + tot[m & 1][w][8 * lg + e] - l[e]);
+        for (int e = 0; e < 8; ++e) v[e] = k[e] * __expf(base[e] + tot[turn][w][8 * lg + e] - l[e]);
         split8(v, hi, lo);
-        *reinterpret_cast<bf16x8*>(&kt[m & 1][0][i][8 * lg]) = hi;
-        *reinterpret_cast<bf16x8*>(&kt[m & 1][1][i][8 * lg]) = lo;
+        *reinterpret_cast<bf16x8*>(&kt[turn][0][i][8 * lg]) = hi;
+        *reinterpret_cast<bf16x8*>(&kt[turn][1][i][8 * lg]) = lo;
       }
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] = q[e] * A.qs * __expf(l[e]);
@@ -307,12 +323,12 @@ __global__ __launch_bounds__(256, 3) void prepare_kernel(const Args A) {
         if (a < w) {  // wave-uniform
 #pragma unroll
           for (int e = 0; e < 8; ++e) {
-            R[e] += tot[m & 1][a][8 * lg + e];
+            R[e] += tot[turn][a][8 * lg + e];
             v[e] = q[e] * A.qs * __expf(l[e] - R[e]);
           }
           split8(v, hi, lo);
-          const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(&kt[m & 1][0][16 * a + c][8 * lg]);
-          const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(&kt[m & 1][1][16 * a + c][8 * lg]);
+          const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(&kt[turn][0][16 * a + c][8 * lg]);
+          const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(&kt[turn][1][16 * a + c][8 * lg]);
           blk[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, hi, blk[a], 0, 0, 0);
           blk[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, lo, blk[a], 0, 0, 0);
           blk[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, hi, blk[a], 0, 0, 0);
@@ -323,9 +339,19 @@ __global__ __launch_bounds__(256, 3) void prepare_kernel(const Args A) {
     for (int s = 0; s < 16; ++s) {
       d[s] += __shfl_xor(d[s], 16, 64);
       d[s] += __shfl_xor(d[s], 32, 64);
-      if (lg == (s & 3) && c + s < 16) dg[w][c + s][c] = d[s] * A.qs;
+      if (lg == (s & 3) && c + s < 16) dg[part][w][c + s][c] = d[s] * A.qs;
+    }
+    if (P > 1 && part > 0) {
+#pragma unroll
+      for (int a = 0; a < 3; ++a) others[part - 1][w][a][lane] = blk[a];
     }
     __syncthreads();
+    if (P > 1 && part == 0) {
+#pragma unroll
+      for (int o = 0; o < P - 1; ++o)
+#pragma unroll
+        for (int a = 0; a < 3; ++a) blk[a] += others[o][w][a][lane];
+    }
     bf16* o = A.sc + ((size_t)row * A.H + h) * LC + 4 * lg;
     const size_t low = (size_t)A.T * A.H * LC;
 #pragma unroll
@@ -335,13 +361,16 @@ __global__ __launch_bounds__(256, 3) void prepare_kernel(const Args A) {
       for (int r = 0; r < 4; ++r) {
         float v = 0.f;
         if (a < 3 && a < w) v = blk[a < 3 ? a : 0][r];
-        if (a == w && 4 * lg + r <= c) v = dg[w][c][4 * lg + r];
+        if (a == w && 4 * lg + r <= c) {
+#pragma unroll
+          for (int o = 0; o < P; ++o) v += dg[o][w][c][4 * lg + r];
+        }
         bf16 x, y;
         split(v, x, y);
         hi[r] = x;
         lo[r] = y;
       }
-      if (live) {
+      if (live && part == 0) {
         *reinterpret_cast<bf16x4*>(o + 16 * a) = hi;
         *reinterpret_cast<bf16x4*>(o + low + 16 * a) = lo;
       }
@@ -600,7 +629,9 @@ extern "C" int pa_linear_attention(int fp32, const void* x, int ldx, void* y, in
       set = true;                                                                                        \
     }                                                                                                    \
   } while (0)
-  hipLaunchKernelGGL(prepare_kernel, dim3(H, gy), dim3(256), 0, st, A);
+  // (few chunks: a head's channels over twice the waves)
+  if (N % 64 == 0 && H * gy <= 1024) hipLaunchKernelGGL(prepare_kernel<2>, dim3(H, gy), dim3(512), 0, st, A);
+  else hipLaunchKernelGGL(prepare_kernel<1>, dim3(H, gy), dim3(256), 0, st, A);
   PA_ATTR(chunk_state_kernel);
   hipLaunchKernelGGL(chunk_state_kernel, dim3(H * vts * ((N + NT - 1) / NT), gy), dim3(256), lds_s, st, A);
   hipLaunchKernelGGL(state_pass_kernel, dim3((V * N / 4 + 255) / 256, std::min(max_items, 16), H), dim3(256), 0, st, A);
